@@ -101,3 +101,11 @@ def _safurax(d):
 
 
 register_architecture("Safurax", _safurax)
+
+
+def _busadra(d):
+    from .busadra import BusadraConfig
+    return BusadraConfig.from_dict(d)
+
+
+register_architecture("Busadra", _busadra)

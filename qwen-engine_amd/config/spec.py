@@ -169,11 +169,14 @@ class RopeHalfAnglesSpec:
     """Half-split rotation of the first ``rotary_dim`` numbers of a head (number i < rotary_dim / 2 pairs with
     i + rotary_dim / 2) by ``position * theta ** (-2 i / rotary_dim)``; the rest of the head passes unchanged.
     The kernels form angle, sine and cosine in 32-bit from the frequencies: no table, no limit of positions.
-    ``scaling_factor``: every frequency is divided by it (positions stretched linearly)."""
+    ``scaling_factor``: every frequency is divided by it (positions stretched linearly).  ``band_scaling``: None, or
+    (factor, low, high, original): a frequency whose wavelength is above original / low is divided by factor, one below
+    original / high stays, those between are blended linearly in original / wavelength."""
     theta: float
     rotary_dim: int
     kind: str = "rope_half_angles"
     scaling_factor: float = 1.0
+    band_scaling: Optional[Tuple[float, float, float, float]] = None
 
 
 @dataclass(frozen=True)
@@ -183,6 +186,8 @@ class ConvAttentionSpec:
     ``head_dim`` numbers, values ``v_head_dim``.  ``window`` None: all earlier keys; else the last ``window`` keys
     (the query's own included) and, wherever the window stands, the request's first ``keep_first`` keys.
     ``sink``: the softmax's denominator has a 1 added (one more entry of score 0 that carries no value).
+    ``softcap`` not None: the scaled scores pass softcap * tanh(. / softcap).  ``out_bias``: the output projection has
+    a bias too.
     ``names``: the tensors' names inside the part for q, k, v and the output projection; a bias is the
     projection's name + ``bias_suffix``, a convolution's weights [channels, taps] its name + ``conv_suffix``."""
     num_heads: int
@@ -200,6 +205,8 @@ class ConvAttentionSpec:
     bias_suffix: str = ".b"
     conv_suffix: str = ".conv"
     kind: str = "conv_attention"
+    softcap: Optional[float] = None
+    out_bias: bool = False
 
 
 @dataclass(frozen=True)
@@ -313,6 +320,21 @@ class DecayedLinearSpec:
 
 
 @dataclass(frozen=True)
+class ForgetGateLinearSpec:
+    """HGRN2: linear attention whose forget gate also decides what is written.  q = silu(W_q x) with ``head_dim``
+    numbers a head, v = W_v x with ``v_head_dim``; per head and channel f = l + (1 - l) sigmoid(W_f x + b) with l a tensor
+    of the layer (the lower bound); S <- diag(f) S + (1 - f) v^T, o = S^T q; every head's o RMS-normed with one weight of
+    ``v_head_dim`` numbers, then the output projection.  ``names``: q, forget gate, its bias, lower bound, v, norm,
+    output projection."""
+    num_heads: int
+    head_dim: int
+    v_head_dim: int
+    norm_eps: float
+    names: Tuple[str, str, str, str, str, str, str] = ("q", "f", "f.b", "lower", "v", "norm", "o")
+    kind: str = "forget_gate_linear"
+
+
+@dataclass(frozen=True)
 class SideBySideMixerSpec:
     """Two mixers that read the same input; the result is left_scale * left + right_scale * right.  Their tensors
     lie under ``names`` inside the mixer.  At most one of them keeps keys and values and at most one a state."""
@@ -338,6 +360,14 @@ class LogitSoftcapSpec:
     cap: float
     prefix: str = ""
     kind: str = "logit_softcap"
+
+
+@dataclass(frozen=True)
+class LogitScaleSpec:
+    """logits <- scale * logits; no tensors."""
+    scale: float
+    prefix: str = ""
+    kind: str = "logit_scale"
 
 
 @dataclass(frozen=True)
@@ -388,6 +418,54 @@ class TopSoftmaxMoESpec:
     shared_intermediate_size: Optional[int] = None
     shared_gate: bool = False
     kind: str = "top_softmax_moe"
+
+
+@dataclass(frozen=True)
+class SigmoidMoESpec:
+    """A routed mixture of small gated feed-forwards down(silu(gate x) * up x) without biases.  The ``top`` largest of
+    the router's 32-bit logits (plus a bias tensor if ``router_bias``) are chosen; their weights are the sigmoids of
+    their logits, not renormalised.  ``weigh_input``: a weight multiplies what its expert reads, not what it gives.
+    The shared expert as in TopSoftmaxMoESpec."""
+    num_experts: int
+    top: int
+    intermediate_size: int
+    weigh_input: bool = False
+    router_bias: bool = False
+    shared_intermediate_size: Optional[int] = None
+    shared_gate: bool = False
+    kind: str = "sigmoid_moe"
+
+
+@dataclass(frozen=True)
+class DepthAverageSpec:
+    """After layer ``index`` the stream becomes sum_j c[j] X_j over j = 0 .. index + 1, X_0 the embedding output and
+    X_(j + 1) the result of layer j before its own average; c is a tensor of the layer.  ``layers``: how many layers of
+    the model keep results."""
+    index: int
+    layers: int
+
+
+@dataclass(frozen=True)
+class ScaledLayerSpec:
+    """A pre-norm block x <- x + s1 * mixer(c1(norm(x))); x <- x + s2 * ffn(c2(norm(x))).  c1, c2 (``mixer_conv``,
+    ``ffn_conv``): None or a causal convolution over time added to its input, a state of its own each; s1, s2
+    (``layer_scale``): a learned factor per channel on each sublayer's result; ``depth_average``: what goes on to the next
+    layer is a weighted sum over all results so far.  ``ffn`` None: the layer is its mixer alone (the folder may still
+    hold the tensors around the missing feed-forward)."""
+    prefix: str
+    mixer_norm: object
+    mixer: object
+    ffn_norm: object
+    ffn: Optional[object]
+    mixer_conv: Optional[object] = None
+    ffn_conv: Optional[object] = None
+    layer_scale: bool = False
+    depth_average: Optional[DepthAverageSpec] = None
+    part_names: Tuple[str, str, str, str] = ("norm1", "mix", "norm2", "mlp")
+    conv_names: Tuple[str, str] = ("canon1", "canon2")
+    scale_names: Tuple[str, str] = ("ls1", "ls2")
+    average_name: str = "dwa"
+    kind: str = "scaled_prenorm_block"
 
 
 @dataclass(frozen=True)

@@ -12,13 +12,14 @@
 // current one is computed, and the split's page ids are read before the loop.
 // (Merging the splits in this same kernel, by the wave that finishes last, was tried: the
 // device-wide fences it needs cost several times what the separate merge kernel costs.)
-template <int D, int SPLIT>
+// CAP: a soft cap on the scores (scale then holds 2 log2(e) / cap, see attn_tile_step).
+template <int D, int SPLIT, bool CAP>
 __global__ __launch_bounds__(64) void attention_decode_split_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ cache,
     const int* __restrict__ dec_tokens, const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ shared_keys,
     float* __restrict__ part_acc, float* __restrict__ part_ml,
-    int Hq, int Hkv, int P, float scale, int window, int keep_first, int num_splits) {
+    int Hq, int Hkv, int P, float scale, int window, int keep_first, int num_splits, float cap) {
     constexpr int TILES = SPLIT / 16;
     const int lane = threadIdx.x, g = lane >> 4, n = lane & 15;
     const int split = blockIdx.x, kvh = blockIdx.y, di = blockIdx.z;
@@ -70,7 +71,7 @@ __global__ __launch_bounds__(64) void attention_decode_split_kernel(
 #define TILE_OF(i_) ((i_) < first_tiles ? (i_) : (i_) + gap)
 #define LOAD(buf_, i_) load_tile<D>(buf_, cache, __builtin_amdgcn_readlane(my_page, TILE_OF(i_)), page_stride, kvh, Hkv, P, \
                                     (split * SPLIT + TILE_OF(i_) * 16) % P, g, n, stream)
-#define STEP(buf_, i_) attn_tile_step<D>(st, buf_, qreg, scale, split * SPLIT + TILE_OF(i_) * 16, g, k_begin, k_end, k_begin, k_end, kf)
+#define STEP(buf_, i_) attn_tile_step<D, CAP>(st, buf_, qreg, scale, split * SPLIT + TILE_OF(i_) * 16, g, k_begin, k_end, k_begin, k_end, kf, cap)
     KVTile<D> ta, tb;
     int i = walk0;
     const int walk1 = tile1 - gap;
@@ -417,7 +418,7 @@ size_t qe_attention_decode_workspace(int n_dec, int Hq, int D, int num_splits) {
 int qe_attention_decode(const void* q, void* out, const void* cache, const int* dec_tokens, int n_dec,
                         const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                         const int* shared_keys, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first,
-                        int sink, int max_position, int split_keys, void* workspace, size_t workspace_bytes,
+                        int sink, float softcap, int max_position, int split_keys, void* workspace, size_t workspace_bytes,
                         hipStream_t stream) {
     QE_REQUIRE(qe_attention_decode_ok(Hq, Hkv, D, P, QE_BF16), "decode attention: sizes not taken");
     QE_REQUIRE(split_keys == 128 || split_keys == 256, "decode attention: splits of 128 or 256 keys, not %d", split_keys);
@@ -431,11 +432,15 @@ int qe_attention_decode(const void* q, void* out, const void* cache, const int* 
     (void)qe_cdiv;
     dim3 grid(num_splits, Hkv, n_dec);
     dim3 mgrid(n_dec, Hq);
+    if (softcap > 0.f) scale = scale * 2.f * 1.4426950408889634f / softcap;
+#define QE_DECODE_SPLIT(D_, S_, CAP_)                                                                   \
+        attention_decode_split_kernel<D_, S_, CAP_><<<grid, 64, 0, stream>>>(                           \
+            (const bf16_t*)q, (const bf16_t*)cache, dec_tokens, positions, tok_seq, block_table,        \
+            max_blocks, shared_keys, part_acc, part_ml, Hq, Hkv, P, scale, window, keep_first, num_splits, softcap)
 #define QE_DECODE(D_, S_)                                                                               \
     do {                                                                                                \
-        attention_decode_split_kernel<D_, S_><<<grid, 64, 0, stream>>>(                                 \
-            (const bf16_t*)q, (const bf16_t*)cache, dec_tokens, positions, tok_seq, block_table,        \
-            max_blocks, shared_keys, part_acc, part_ml, Hq, Hkv, P, scale, window, keep_first, num_splits); \
+        if (softcap > 0.f) QE_DECODE_SPLIT(D_, S_, true);                                               \
+        else QE_DECODE_SPLIT(D_, S_, false);                                                            \
         attention_decode_merge_kernel<D_><<<mgrid, 256, 0, stream>>>(part_acc, part_ml, dec_tokens,     \
                                                                      (bf16_t*)out, Hq, num_splits, sink); \
     } while (0)
@@ -444,6 +449,7 @@ int qe_attention_decode(const void* q, void* out, const void* cache, const int* 
     else if (split_keys == 128) QE_DECODE(64, 128);
     else QE_DECODE(64, 256);
 #undef QE_DECODE
+#undef QE_DECODE_SPLIT
     QE_LAUNCH_CHECK();
     return 0;
 }

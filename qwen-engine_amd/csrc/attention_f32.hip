@@ -38,7 +38,7 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
     const float* __restrict__ q, float* __restrict__ out, const float* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tokens,
-    int Hq, int Hkv, int P, float scale, int window, int keep_first, int sink) {
+    int Hq, int Hkv, int P, float scale, int window, int keep_first, int sink, float softcap) {
     constexpr int D = DB * 16;
     extern __shared__ float merge_lds[];                  // [F32_WAVES][DB * 4 + 2][64]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, n = lane & 15;
@@ -96,7 +96,9 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
         for (int i = 0; i < 4; ++i) {
             const int key = kk + 4 * g + i;
             ok[i] = (key >= lo || key < kf) && key <= p;
-            s[i] = ok[i] ? s[i] * scale : -INFINITY;
+            s[i] *= scale;
+            if (softcap > 0.f) s[i] = softcap * tanhf(s[i] / softcap);
+            if (!ok[i]) s[i] = -INFINITY;
             tmax = fmaxf(tmax, s[i]);
         }
         tmax = max_over_rows_of_lanes(tmax);
@@ -183,7 +185,7 @@ bool qe_attention_f32_ok(int Hq, int Hkv, int D, int P) {
 
 int qe_attention_f32(const float* q, float* out, const float* cache, const int* positions, const int* tok_seq,
                      const int* block_table, int max_blocks, const int* tokens, int T, int Hq, int Hkv, int D,
-                     int P, float scale, int window, int keep_first, int sink, hipStream_t stream) {
+                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream) {
     QE_REQUIRE(qe_attention_f32_ok(Hq, Hkv, D, P), "attention (32-bit): sizes not taken");
     const int groups16 = (Hq / Hkv + 15) / 16;
     QE_REQUIRE((long)Hkv * groups16 <= 65535, "attention (32-bit): too many heads");
@@ -201,7 +203,7 @@ int qe_attention_f32(const float* q, float* out, const float* cache, const int* 
             }                                                                                         \
         }                                                                                             \
         attention_f32_kernel<DB_><<<grid, 64 * F32_WAVES, lds, stream>>>(q, out, cache, positions, tok_seq, \
-                                                    block_table, max_blocks, tokens, Hq, Hkv, P, scale, window, keep_first, sink); \
+                                                    block_table, max_blocks, tokens, Hq, Hkv, P, scale, window, keep_first, sink, softcap); \
         break;                                                                                        \
     }
     switch (D / 16) {

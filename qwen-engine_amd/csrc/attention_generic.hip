@@ -24,7 +24,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     const TA* __restrict__ q, TA* __restrict__ out, const TA* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tokens,
-    int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink) {
+    int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink, float softcap) {
     extern __shared__ float smem[];
     float* qs = smem;            // D
     float* ps = smem + D;        // 64 probabilities of the current chunk
@@ -63,6 +63,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
             float dot = 0.f;
             for (int d = 0; d < D; ++d) dot = fmaf(qs[d], Elem<TA>::load(krow + d), dot);
             sc = dot * scale;
+            if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
         }
         const float mn = fmaxf(m, wave_max(sc));   // finite: key j0 is always seen
         const float alpha = expf(m - mn);          // exp(-inf) = 0 on the first chunk
@@ -97,7 +98,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
 bool qe_attention_f32_ok(int Hq, int Hkv, int D, int P);
 int qe_attention_f32(const float* q, float* out, const float* cache, const int* positions, const int* tok_seq,
                      const int* block_table, int max_blocks, const int* tokens, int T, int Hq, int Hkv, int D,
-                     int P, float scale, int window, int keep_first, int sink, hipStream_t stream);
+                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream);
 
 // 32-bit attention goes to the kernel on the matrix units (attention_f32.hip) where it takes the
 // sizes, unless qe_use_matrix_f32(0) has switched that off.
@@ -106,10 +107,10 @@ extern int g_qe_matrix_f32;
 int qe_attention_generic(const void* q, void* out, const void* cache, const int* positions,
                          const int* tok_seq, const int* block_table, int max_blocks, const int* tokens,
                          int T, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink,
-                         int dt_a, hipStream_t stream) {
+                         float softcap, int dt_a, hipStream_t stream) {
     if (dt_a == QE_F32 && g_qe_matrix_f32 && qe_attention_f32_ok(Hq, Hkv, D, P))
         return qe_attention_f32((const float*)q, (float*)out, (const float*)cache, positions, tok_seq, block_table,
-                                max_blocks, tokens, T, Hq, Hkv, D, P, scale, window, keep_first, sink, stream);
+                                max_blocks, tokens, T, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, stream);
     QE_REQUIRE(D <= ATTN_MAX_D, "attention: head_dim=%d exceeds %d", D, ATTN_MAX_D);
     QE_REQUIRE(Hq <= 65535, "attention: too many heads");
     dim3 grid(T, Hq);
@@ -117,11 +118,11 @@ int qe_attention_generic(const void* q, void* out, const void* cache, const int*
     if (dt_a == QE_F32)
         attention_generic_kernel<float><<<grid, 64, shmem, stream>>>(
             (const float*)q, (float*)out, (const float*)cache, positions, tok_seq, block_table,
-            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink);
+            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap);
     else if (dt_a == QE_BF16)
         attention_generic_kernel<bf16_t><<<grid, 64, shmem, stream>>>(
             (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, tok_seq, block_table,
-            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink);
+            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap);
     else
         QE_REQUIRE(false, "attention: unknown dtype %d", dt_a);
     QE_LAUNCH_CHECK();

@@ -107,13 +107,15 @@ __device__ __forceinline__ void store_columns(bf16_t* __restrict__ out, const fl
 
 // Two waves per SIMD (at most 256 registers a lane), as two blocks of one group or one block of
 // two: while one wave waits for its next tile or at its barrier, the other computes.
-template <int D, int NG>
+// CAP: the scaled scores pass cap * tanh(. / cap): cap_in is the scores' scale times 2 log2(e) / cap, cap_out the cap
+// in the base-2 domain, and scale_log2 is 1.
+template <int D, int NG, bool CAP>
 __global__ __launch_bounds__(256 * NG, NG == 1 ? 2 : 1) void attention_prefill_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ tiles, const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks,
     int Hq, int Hkv, int P, int log2P, float scale_log2, int window, int R, int seg_param, int keys_row,
-    float* __restrict__ part, int keep_first, int sink) {
+    float* __restrict__ part, int keep_first, int sink, float cap_in, float cap_out) {
     constexpr int KROW = D * 2 + 16;                 // bytes of a staged key row
     constexpr int KBYTES = 32 * KROW, VBYTES = 2 * D * VROW, BUF = KBYTES + VBYTES;
     constexpr int KP = 32 * (D / 8) / 256;           // 16-byte key pieces per thread (2 for D = 128)
@@ -316,6 +318,10 @@ __global__ __launch_bounds__(256 * NG, NG == 1 ? 2 : 1) void attention_prefill_k
 #pragma unroll
             for (int ks = 0; ks < D / 16; ++ks)
                 s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[ks], qreg[ks], s, 0, 0, 0);
+            if (CAP) {
+#pragma unroll
+                for (int e = 0; e < 16; ++e) s[e] = soft_capped(s[e] * cap_in, cap_out);
+            }
             PackV vf[D / 32][2];
 #pragma unroll
             for (int db = 0; db < D / 32; ++db)
@@ -567,7 +573,7 @@ int qe_attention_prefill(const void* q, void* out, const void* cache, const int*
                          const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                          int Hq, int Hkv, int D, int P, float scale, int window, int groups,
                          int seg_keys, int max_keys, int keys_row, void* workspace, size_t workspace_bytes,
-                         hipStream_t stream, int keep_first, int sink) {
+                         hipStream_t stream, int keep_first, int sink, float softcap) {
     QE_REQUIRE(seg_keys == 0 || (keep_first == 0 && !sink),
                "prefill attention: kept first keys and a sink go with uncut walks only");
     QE_REQUIRE((D == 64 || D == 128) && P >= 16 && (P & (P - 1)) == 0 && Hq % Hkv == 0,
@@ -596,18 +602,22 @@ int qe_attention_prefill(const void* q, void* out, const void* cache, const int*
     QE_REQUIRE(num_tiles / 4 <= 65535, "prefill attention: %d tiles are too many for one launch", num_tiles);
     dim3 grid(Hkv * waves_per_kv, segments, num_tiles / 4);
     dim3 mgrid(Hkv * waves_per_kv, D / 32, num_tiles / 4);
-    const float scale_log2 = scale * 1.4426950408889634f;
+    const float scale_log2 = softcap > 0.f ? 1.f : scale * 1.4426950408889634f;
+    const float cap_in = softcap > 0.f ? scale * 2.f * 1.4426950408889634f / softcap : 0.f, cap_out = softcap * 1.4426950408889634f;
     // two groups a block where the blocks do not fill the compute units twice anyway
     // (groups: 0 = choose, 1 or 2)
     if (groups == 0) groups = (long)grid.x * grid.z <= qe_compute_units() ? 2 : 1;
     QE_REQUIRE(groups == 1 || groups == 2, "prefill attention: %d groups a block", groups);
-#define QE_PREFILL(D_, NG_)                                                                         \
-    attention_prefill_kernel<D_, NG_><<<grid, 256 * NG_, 0, stream>>>(                              \
+#define QE_PREFILL_CAP(D_, NG_, CAP_)                                                               \
+    attention_prefill_kernel<D_, NG_, CAP_><<<grid, 256 * NG_, 0, stream>>>(                        \
         (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, tiles, positions, tok_seq, block_table, \
-        max_blocks, Hq, Hkv, P, log2P, scale_log2, window, R, seg_keys, keys_row, (float*)workspace, keep_first, sink)
+        max_blocks, Hq, Hkv, P, log2P, scale_log2, window, R, seg_keys, keys_row, (float*)workspace, keep_first, sink, \
+        cap_in, cap_out)
+#define QE_PREFILL(D_, NG_) do { if (softcap > 0.f) QE_PREFILL_CAP(D_, NG_, true); else QE_PREFILL_CAP(D_, NG_, false); } while (0)
     if (D == 128) { if (groups == 2) QE_PREFILL(128, 2); else QE_PREFILL(128, 1); }
     else          { if (groups == 2) QE_PREFILL(64, 2); else QE_PREFILL(64, 1); }
 #undef QE_PREFILL
+#undef QE_PREFILL_CAP
     if (seg_keys != 0) {
         if (D == 128)
             attention_prefill_merge_kernel<128><<<mgrid, 256, 0, stream>>>((const float*)workspace, (bf16_t*)out, tiles,

@@ -80,9 +80,11 @@ struct AttnState {
 // The tile's keys are kk .. kk + 15; this lane's column sees the keys in [lo, hi); [vlo, vhi) is
 // the range that any column of the wave sees (keys outside it may be unwritten memory).  Keys below
 // kf are seen as well, by every column (a request's kept first keys, where a window is given).
-template <int D>
+// CAP: the scaled scores pass cap * tanh(. / cap); scale is then the scores' scale times 2 log2(e) / cap.
+template <int D, bool CAP = false>
 __device__ __forceinline__ void attn_tile_step(AttnState<D>& st, const KVTile<D>& tile, const bf16x8 (&qreg)[D / 32],
-                                               float scale, int kk, int g, int lo, int hi, int vlo, int vhi, int kf = 0) {
+                                               float scale, int kk, int g, int lo, int hi, int vlo, int vhi, int kf = 0,
+                                               float cap = 0.f) {
     floatx4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int c = 0; c < D / 32; ++c) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile.k[c], qreg[c], s, 0, 0, 0);
@@ -92,7 +94,7 @@ __device__ __forceinline__ void attn_tile_step(AttnState<D>& st, const KVTile<D>
     for (int j = 0; j < 4; ++j) {
         const int key = kk + g * 4 + j;
         ok[j] = (key >= lo && key < hi) || key < kf;
-        s[j] = ok[j] ? s[j] * scale : -INFINITY;
+        s[j] = ok[j] ? (CAP ? soft_capped(s[j] * scale, cap) : s[j] * scale) : -INFINITY;
         tmax = fmaxf(tmax, s[j]);
     }
     tmax = max_over_lane_rows(tmax);

@@ -45,6 +45,12 @@ __device__ __forceinline__ int first_seen_key(int p, int window) {
     return 0;
 }
 
+// cap * tanh(x / cap) from y = x * 2 log2(e) / cap: the scores of an attention with a soft cap, in the kernels whose
+// operands are bfloat16 (two hardware transcendentals; the error is some 1e-7 of the cap)
+__device__ __forceinline__ float soft_capped(float y, float cap) {
+    return cap - 2.f * cap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(y) + 1.f);
+}
+
 template <typename T> struct Elem;
 template <> struct Elem<float> {
     static __device__ __forceinline__ float load(const float* p) { return *p; }

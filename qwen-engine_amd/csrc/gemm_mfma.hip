@@ -61,6 +61,10 @@ struct QkvTail {
     float act_limit, act_slope;
     // Without SILU: the result is relu(.)^2 instead of the product itself.
     int relu_sq;
+    // With SILU over grouped rows: sorted row i is row_w[perm[i]] times its row of x (null: that row itself); the
+    // factor meets gate and up in 32-bit.
+    const float* row_w;
+    const int* perm;
 };
 
 // BIG (256 x 256 by four waves, one wave a SIMD, a wave's part 128 x 128): the accumulators fill the
@@ -106,6 +110,7 @@ __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
     if (tail.tiles) {
         if (tile_m >= tail.n_tiles[0]) return;
         const int expert = tail.tiles[3 * tile_m], first = tail.tiles[3 * tile_m + 1];
+        if (SILU && tail.row_w) tail.perm += first;        // (from here on by the tile's own rows)
         M = tail.tiles[3 * tile_m + 2];
         x += (long)first * K;
         w += (long)expert * N * K;
@@ -506,6 +511,11 @@ __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
 #pragma unroll
     for (int i = 0; i < MI; ++i) {
         __builtin_amdgcn_sched_barrier(0);   // one strip after the other: nothing of the next is computed early
+        float row_w = 1.f;
+        if (SILU && tail.row_w) {
+            const int m = wm + i * 32 + (lane & 31);       // (a grouped tile starts at row 0 of its rows)
+            row_w = tail.row_w[tail.perm[m < M ? m : M - 1]];
+        }
 #pragma unroll
         for (int j = 0; j < NJ; j += (SILU ? 2 : 1))
 #pragma unroll
@@ -517,6 +527,7 @@ __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
                     if (SILU) {
                         float gt = acc[i][j][4 * bq + r], up = acc[i][j + (SILU ? 1 : 0)][4 * bq + r];
                         float slope = 1.f;
+                        if (tail.row_w) { gt *= row_w; up *= row_w; }
                         if (tail.act_limit > 0.f) {
                             gt = fminf(gt, tail.act_limit);
                             up = fminf(fmaxf(up, -tail.act_limit), tail.act_limit) + 1.f;
@@ -599,7 +610,8 @@ static int launch_mfma(const void* x, const void* w, const float* bias, void* ou
 // Rows grouped by expert against one matrix per expert (see QkvTail): tiles of 128 x 128.
 template <typename TO, bool SILU>
 static int launch_grouped(const void* x, const void* w, void* out, const int* tiles, const int* n_tiles,
-                          int max_tiles, int N, int K, float limit, float slope, hipStream_t stream, int relu_sq = 0) {
+                          int max_tiles, int N, int K, float limit, float slope, hipStream_t stream, int relu_sq = 0,
+                          const float* row_w = nullptr, const int* perm = nullptr) {
     constexpr int BM = 128, BN = 128, BK = 64, NW = 4;
     const int tiles_n = qe_cdiv(N, BN);
     const long blocks = (long)max_tiles * tiles_n;
@@ -617,6 +629,8 @@ static int launch_grouped(const void* x, const void* w, void* out, const int* ti
     tail.act_limit = limit;
     tail.act_slope = slope;
     tail.relu_sq = relu_sq;
+    tail.row_w = row_w;
+    tail.perm = perm;
     gemm_mfma_kernel<TO, BM, BN, BK, NW, 2, SILU, false><<<dim3((unsigned)blocks, 1), 64 * NW, shmem, stream>>>(
         (const bf16_t*)x, (const bf16_t*)w, nullptr, (TO*)out, 0, N, K, max_tiles, tiles_n, K, 0, 0, 0, tail);
     QE_LAUNCH_CHECK();
@@ -624,12 +638,14 @@ static int launch_grouped(const void* x, const void* w, void* out, const int* ti
 }
 
 // x [rows, K] in the order of the tiles (an expert's rows side by side), w [E, N, K], out [rows, N] (silu: w's
-// gate and up rows interleaved in blocks of 32, out [rows, N / 2], with the clamped activation when limit > 0).
+// gate and up rows interleaved in blocks of 32, out [rows, N / 2], with the clamped activation when limit > 0; row i of
+// x is then taken row_w[perm[i]] times, if row_w is given).
 extern "C" int qe_gemm_mfma_grouped(const void* x, const void* w, void* out, const int* tiles, const int* n_tiles,
                                     int max_tiles, int N, int K, int silu, float limit, float slope, int dt_o,
-                                    hipStream_t stream) {
+                                    const float* row_w, const int* perm, hipStream_t stream) {
     QE_REQUIRE(K % 8 == 0 && K >= 64, "mfma gemm (grouped): K=%d", K);
     QE_REQUIRE(silu != 1 || N % 64 == 0, "mfma gemm (grouped): gate|up rows in blocks of 32");
+    QE_REQUIRE(!row_w || (silu == 1 && perm), "mfma gemm (grouped): row factors go with gate|up rows and the rows' order");
     if (max_tiles == 0) return 0;
     if (silu == 2) {       // one matrix an expert, the result relu(.)^2
         QE_REQUIRE(dt_o == QE_BF16, "mfma gemm (grouped): the activation is stored in bfloat16");
@@ -637,7 +653,7 @@ extern "C" int qe_gemm_mfma_grouped(const void* x, const void* w, void* out, con
     }
     if (silu) {
         QE_REQUIRE(dt_o == QE_BF16, "mfma gemm (grouped): the activation is stored in bfloat16");
-        return launch_grouped<bf16_t, true>(x, w, out, tiles, n_tiles, max_tiles, N, K, limit, slope, stream);
+        return launch_grouped<bf16_t, true>(x, w, out, tiles, n_tiles, max_tiles, N, K, limit, slope, stream, 0, row_w, perm);
     }
     if (dt_o == QE_F32) return launch_grouped<float, false>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);
     return launch_grouped<bf16_t, false>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);

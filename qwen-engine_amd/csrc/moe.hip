@@ -19,9 +19,10 @@
 //   qe_moe_gemm    for every tile, rows . W_e^T:
 //                    first product  (dual): x row of the pair's token against gate and up rows of
 //                      W_e [2 F, K]; g = min(g, limit), u = clamp(u, -limit, limit),
-//                      a = g sigmoid(slope g) (u + 1), stored at the sorted row
-//                    second product (weighted): a's sorted row against W_e [N, K], times the pair's
-//                      weight, to parts[j][t] (32-bit): the norm that follows adds a token's ``top``
+//                      a = g sigmoid(slope g) (u + 1), stored at the sorted row; with weights the expert
+//                      reads weight times the row (gate and up are multiplied by it in 32-bit)
+//                    second product: a's sorted row against W_e [N, K], times the pair's
+//                      weight (if weights are given), to parts[j][t] (32-bit): the norm that follows adds a token's ``top``
 //                      parts in the order of j.
 //                    dual == 2: one matrix W_e [F, K] and a = relu(W_e x)^2 instead.
 //                  Any sizes, every multiply-add in IEEE 32-bit.
@@ -110,12 +111,14 @@ extern "C" int qe_moe_route(const float* logits, int* ids, float* weights, int T
 // One token's routing by one wave: softmax over all E outputs, choice by score + correction, weights from the
 // scores alone.  Without a correction (null) the choice goes by the logits themselves and the weights are the
 // softmax over the chosen logits alone (the scores stay unnormalised: the largest is 1, so the chosen ones' sum
-// is at least 1 however far the others lie below).  sc: the wave's own 2 E + top floats of shared memory.  Every wave of the block calls it together
+// is at least 1 however far the others lie below).  sigmoid: the scores are sigmoids, each output's by itself; the
+// choice goes by the logits (or, with a correction, by score + correction) and the weights are the chosen scores as
+// they are, times scale.  sc: the wave's own 2 E + top floats of shared memory.  Every wave of the block calls it together
 // (the barriers are the block's); a wave without a token (z null) only keeps step.
 __device__ __forceinline__ void route_biased_token(const float* __restrict__ z, const float* __restrict__ correction,
                                                    float* sc, int* __restrict__ ids, float* __restrict__ weights, int E,
                                                    int top, float scale, int lane, long zs = 1,
-                                                   const float* __restrict__ zbias = nullptr) {
+                                                   const float* __restrict__ zbias = nullptr, int sigmoid = 0) {
     float* ch = sc + E;
     float* picked = ch + E;
     if (z) {                                             // (zs: the distance between a token's logits; zbias: added to them)
@@ -128,13 +131,13 @@ __device__ __forceinline__ void route_biased_token(const float* __restrict__ z, 
         mx = wave_max(mx);
         float sum = 0.f;
         for (int e = lane; e < E; e += 64) {
-            const float ex = expf(ch[e] - mx);
+            const float ex = sigmoid ? 1.f / (1.f + expf(-ch[e])) : expf(ch[e] - mx);
             sc[e] = ex;
             sum += ex;
         }
         sum = wave_sum(sum);
         for (int e = lane; e < E; e += 64) {
-            float v = correction ? sc[e] / sum : sc[e];
+            float v = correction && !sigmoid ? sc[e] / sum : sc[e];
             if (!(v == v)) v = 0.f;            // (a row of garbage still gets experts inside the table)
             sc[e] = v;
             float c = correction ? v + correction[e] : ch[e];
@@ -161,29 +164,29 @@ __device__ __forceinline__ void route_biased_token(const float* __restrict__ z, 
     if (z && lane == 0) {
         float tot = 0.f;
         for (int r = 0; r < top; ++r) tot += picked[r];
-        for (int r = 0; r < top; ++r) weights[r] = picked[r] / (tot + 1e-20f) * scale;
+        for (int r = 0; r < top; ++r) weights[r] = sigmoid ? picked[r] * scale : picked[r] / (tot + 1e-20f) * scale;
     }
 }
 
 __global__ __launch_bounds__(64) void moe_route_biased_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
                                                               int* __restrict__ ids, float* __restrict__ weights, int E, int top,
                                                               float scale, int transposed, const float* __restrict__ zbias,
-                                                              int ld) {
+                                                              int ld, int sigmoid) {
     extern __shared__ float sc[];          // E scores, E choice scores, top chosen scores
     const long t = blockIdx.x;
     // (transposed: logits [E, T], as a product of the router's few rows against the tokens' many leaves them)
     route_biased_token(transposed ? logits + t : logits + t * ld, correction, sc, ids + t * top, weights + t * top, E, top,
-                       scale, threadIdx.x, transposed ? (long)gridDim.x : 1L, zbias);
+                       scale, threadIdx.x, transposed ? (long)gridDim.x : 1L, zbias, sigmoid);
 }
 
 extern "C" int qe_moe_route_biased(const float* logits, const float* correction, int* ids, float* weights, int T, int E,
-                                   int top, float scale, int transposed, const float* zbias, int ld, hipStream_t stream) {
+                                   int top, float scale, int transposed, const float* zbias, int ld, int sigmoid, hipStream_t stream) {
     if (ld <= 0) ld = E;                   // (ld: the distance between two tokens' logits where they are not transposed)
     QE_REQUIRE(ld >= E, "moe_route_biased: rows of %d logits for %d experts", ld, E);
     QE_REQUIRE(T >= 0 && E > 0 && top >= 1 && top <= E, "moe_route_biased: top %d of %d experts", top, E);
     QE_REQUIRE((2 * E + top) * sizeof(float) <= 60000, "moe_route_biased: too many experts");
     if (T == 0) return 0;
-    moe_route_biased_kernel<<<T, 64, (2 * E + top) * sizeof(float), stream>>>(logits, correction, ids, weights, E, top, scale, transposed, zbias, ld);
+    moe_route_biased_kernel<<<T, 64, (2 * E + top) * sizeof(float), stream>>>(logits, correction, ids, weights, E, top, scale, transposed, zbias, ld, sigmoid);
     QE_LAUNCH_CHECK();
     return 0;
 }
@@ -275,7 +278,7 @@ __global__ __launch_bounds__(1024) void moe_front_small_kernel(
     const float* __restrict__ logits, const float* __restrict__ correction, const TA* __restrict__ x, int* __restrict__ ids,
     float* __restrict__ weights, int* __restrict__ perm, int* __restrict__ inv, int* __restrict__ tiles,
     int* __restrict__ n_tiles, float* __restrict__ parts, int T, int H, int E, int E_real, int top, float scale, int tile_rows,
-    const float* __restrict__ zbias, int ld) {
+    const float* __restrict__ zbias, int ld, int sigmoid) {
     extern __shared__ int sm[];
     const int n = T * top;
     int* ids_s = sm;                                     // n
@@ -286,7 +289,7 @@ __global__ __launch_bounds__(1024) void moe_front_small_kernel(
     for (int t0 = 0; t0 < T; t0 += waves) {
         const int t = t0 + wave;
         route_biased_token(t < T ? logits + (long)t * ld : nullptr, correction, wave_sc + (long)wave * (2 * E + top),
-                           ids_s + (t < T ? t : 0) * top, w_s + (t < T ? t : 0) * top, E, top, scale, lane, 1L, zbias);
+                           ids_s + (t < T ? t : 0) * top, w_s + (t < T ? t : 0) * top, E, top, scale, lane, 1L, zbias, sigmoid);
     }
     __syncthreads();
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
@@ -316,7 +319,7 @@ extern "C" int qe_moe_front_small_supported(int T, int E, int top) {
 extern "C" int qe_moe_front_small(const float* logits, const float* correction, const void* x, int* ids, float* weights,
                                   int* perm, int* inv, int* tiles, int* n_tiles, float* parts, int max_tiles, int T, int H,
                                   int E, int E_real, int top, float scale, int tile_rows, int dt_a, const float* zbias, int ld,
-                                  hipStream_t stream) {
+                                  int sigmoid, hipStream_t stream) {
     if (ld <= 0) ld = E;
     QE_REQUIRE(qe_moe_front_small_supported(T, E, top), "moe_front_small: %d tokens, %d outputs, top %d", T, E, top);
     QE_REQUIRE(E_real >= 1 && E_real <= E && top <= E && tile_rows > 0 && H > 0, "moe_front_small: bad sizes");
@@ -324,9 +327,9 @@ extern "C" int qe_moe_front_small(const float* logits, const float* correction, 
     QE_REQUIRE(max_tiles >= (n + tile_rows - 1) / tile_rows + (E_real < n ? E_real : n), "moe_front_small: %d tiles may not be enough", max_tiles);
     const size_t lds = ((size_t)2 * n + 2 * E + 16 * (2 * E + top)) * 4;
     if (dt_a == QE_BF16)
-        moe_front_small_kernel<bf16_t><<<1, 1024, lds, stream>>>(logits, correction, (const bf16_t*)x, ids, weights, perm, inv, tiles, n_tiles, parts, T, H, E, E_real, top, scale, tile_rows, zbias, ld);
+        moe_front_small_kernel<bf16_t><<<1, 1024, lds, stream>>>(logits, correction, (const bf16_t*)x, ids, weights, perm, inv, tiles, n_tiles, parts, T, H, E, E_real, top, scale, tile_rows, zbias, ld, sigmoid);
     else if (dt_a == QE_F32)
-        moe_front_small_kernel<float><<<1, 1024, lds, stream>>>(logits, correction, (const float*)x, ids, weights, perm, inv, tiles, n_tiles, parts, T, H, E, E_real, top, scale, tile_rows, zbias, ld);
+        moe_front_small_kernel<float><<<1, 1024, lds, stream>>>(logits, correction, (const float*)x, ids, weights, perm, inv, tiles, n_tiles, parts, T, H, E, E_real, top, scale, tile_rows, zbias, ld, sigmoid);
     else
         QE_REQUIRE(false, "moe_front_small: unknown type %d", dt_a);
     QE_LAUNCH_CHECK();
@@ -424,6 +427,11 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
             }
         } else if (DUAL) {
             TA* o = (TA*)out_ + (long)(r0 + m) * N;
+            if (weights) {                             // (the expert reads weight times the row)
+                const float wgt = weights[perm[r0 + m]];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) { acc[i][j] *= wgt; acu[DUAL ? i : 0][j] *= wgt; }
+            }
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int n = n0 + tx * 4 + j;
@@ -439,7 +447,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
             }
         } else {
             const int pair = perm[r0 + m];
-            const float wgt = weights[pair];
+            const float wgt = weights ? weights[pair] : 1.f;
             float* o = (float*)out_ + ((long)(pair % top) * T + pair / top) * N;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
@@ -505,7 +513,7 @@ __global__ void moe_combine_kernel(const TY* __restrict__ y, const int* __restri
     const long t = blockIdx.x;
     for (int c = threadIdx.x; c < H; c += blockDim.x) {
         float a = 0.f;
-        for (int j = 0; j < top; ++j) a = fmaf(weights[t * top + j], Elem<TY>::load(y + (long)inv[t * top + j] * H + c), a);
+        for (int j = 0; j < top; ++j) a = fmaf(weights ? weights[t * top + j] : 1.f, Elem<TY>::load(y + (long)inv[t * top + j] * H + c), a);
         out[t * H + c] = a;
     }
 }

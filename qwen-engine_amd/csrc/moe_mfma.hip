@@ -68,6 +68,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(
             if (DUAL) au[0] += part[v][1][lane];
         }
     }
+    // (weights with the first product: gate and up of weight times the row; without any, the second product's rows as they are)
     // lane (g, nn) holds the row m = i * 16 + nn at the features n_base + g * 4 + j
     const int n0 = n_base + g * 4;
 #pragma unroll
@@ -84,6 +85,11 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(
             }
         } else if (DUAL) {
             bf16_t* o = (bf16_t*)out_ + (long)(r0 + m) * N + n0;
+            if (weights) {
+                const float wgt = weights[perm[r0 + m]];
+                ag[i] *= wgt;
+                au[i] *= wgt;
+            }
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 if (n0 + j >= N) break;
@@ -98,7 +104,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(
             }
         } else {
             const int pair = perm[r0 + m];
-            const float wgt = weights[pair];
+            const float wgt = weights ? weights[pair] : 1.f;
             float* o = (float*)out_ + ((long)(pair % top) * T + pair / top) * N + n0;
 #pragma unroll
             for (int j = 0; j < 4; ++j)

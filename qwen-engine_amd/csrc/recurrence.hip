@@ -8,6 +8,9 @@
 //                           mode 1 (a decay per key channel, a bonus for the token itself):
 //                                 o_t = (S + diag(u) k_t v_t^T)^T q_t;   S <- diag(w_t) S + k_t v_t^T
 //                                 with w_t = exp(-exp(x_t + w0)) from the projected x_t
+//                           mode 2 (a forget gate per key channel that also decides what is written):
+//                                 S <- diag(f_t) S + (1 - f_t) v_t^T;   o_t = S^T q_t
+//                                 with f_t = l + (1 - l) sigmoid(z_t + b) from the projected z_t
 //   qe_gated_norm         y = o / rms(o) * weight * act(gate) * scale, the root mean square over each of
 //                         `groups` equal pieces of a row (one: the whole row)
 //
@@ -20,6 +23,15 @@
 
 __device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+// f = l + (1 - l) sigmoid(z) and 1 - f, neither by a difference
+__device__ __forceinline__ void forget_gate(float z, float l, float& f, float& kf) {
+    const float e = expf(-fabsf(z));
+    const float big = 1.f / (1.f + e), small = e * big;
+    f = fmaf(1.f - l, z >= 0.f ? big : small, l);
+    kf = (1.f - l) * (z >= 0.f ? small : big);
+}
+// log f, from whichever of f and 1 - f is small
+__device__ __forceinline__ float log_forget(float f, float kf) { return kf < 0.5f ? log1pf(-kf) : logf(f); }
 
 // ---- blends with the token before ---------------------------------------------------------------------
 // grid (T); mode 0: read the state, write y; mode 1: the rows that are their request's last write the state;
@@ -76,6 +88,7 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
     const float* __restrict__ wx, long w_stride, const float* __restrict__ w0, const float* __restrict__ u,
     const float* __restrict__ decay, int act_silu, float* __restrict__ state, long state_stride,
     const int* __restrict__ tok_seq, float* __restrict__ out, int T, int H, int D, int Dv) {
+    // (MODE 2: k holds the forget gate's logits, w0 its bias, u its lower bound; act_silu means q alone)
     const int t0 = blockIdx.x;
     const int seq = tok_seq[t0];
     if (t0 > 0 && tok_seq[t0 - 1] == seq) return;          // not a request's first row (the whole block leaves)
@@ -113,7 +126,8 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
                 const long r = (long)(tb + tt) * row_stride + h * D + d;
                 a = Elem<TA>::load(q + r);
                 b = Elem<TA>::load(k + r);
-                if (act_silu) { a = silu_f(a); b = silu_f(b); }
+                if (act_silu) { a = silu_f(a); if (MODE != 2) b = silu_f(b); }
+                if (MODE == 2) { const float z = b + w0[h * D + d]; forget_gate(z, u[h * D + d], c, b); }
                 if (MODE == 1) c = expf(-expf(wx[(long)(tb + tt) * w_stride + h * D + d] + w0[h * D + d]));
             }
             sq[tt][d] = a; sk[tt][d] = b; sw[tt][d] = c;
@@ -124,7 +138,7 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
             vv[tt] = 0.f;
             if (tt < nb && col_ok) {
                 vv[tt] = Elem<TA>::load(v + (long)(tb + tt) * row_stride + (long)h * Dv + col);
-                if (act_silu) vv[tt] = silu_f(vv[tt]);
+                if (act_silu && MODE != 2) vv[tt] = silu_f(vv[tt]);
             }
         }
         __syncthreads();
@@ -138,6 +152,9 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
                     const float kv = sk[tt][d0 + i] * vt;
                     if (MODE == 0) {
                         S[i] = fmaf(dec, S[i], kv);
+                        o = fmaf(sq[tt][d0 + i], S[i], o);
+                    } else if (MODE == 2) {
+                        S[i] = fmaf(sw[tt][d0 + i], S[i], kv);
                         o = fmaf(sq[tt][d0 + i], S[i], o);
                     } else {
                         o = fmaf(sq[tt][d0 + i], fmaf(uu[i], kv, S[i]), o);
@@ -168,7 +185,8 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
 
 // q, k: row t at + t * row_stride, H * D numbers; v likewise (v's own pointer), H * Dv numbers.  mode 1: q is what
 // multiplies the state (the receptance), wx float32 [T, w_stride] the decays before their exponentials, w0 and u float32
-// [H * D]; mode 0: decay float32 [H].  act_silu: q, k and v pass silu first.  state: row tok_seq[t] at
+// [H * D]; mode 0: decay float32 [H]; mode 2: k the forget gate's logits, w0 their bias, u the gate's lower bound
+// (float32 [H * D]).  act_silu: q, k and v (mode 2: q) pass silu first.  state: row tok_seq[t] at
 // + tok_seq[t] * state_stride, H * D * Dv floats.  out float32 [T, H, Dv].
 extern "C" int qe_linear_recurrence(const void* q, const void* k, const void* v, long row_stride, const float* wx,
                                     long w_stride, const float* w0, const float* u, const float* decay, int mode,
@@ -176,7 +194,7 @@ extern "C" int qe_linear_recurrence(const void* q, const void* k, const void* v,
                                     int T, int H, int D, int Dv, int dt_a, hipStream_t stream) {
     QE_REQUIRE(T >= 0 && H > 0 && D > 0 && Dv > 0, "linear_recurrence: bad sizes");
     QE_REQUIRE(D <= 256, "linear_recurrence: heads of %d key channels (at most 256)", D);
-    QE_REQUIRE(mode == 0 ? decay != nullptr : (mode == 1 && wx && w0 && u), "linear_recurrence: mode %d lacks operands", mode);
+    QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "linear_recurrence: mode %d lacks operands", mode);
     QE_REQUIRE(state_stride >= (long)H * D * Dv, "linear_recurrence: state rows overlap");
     if (T == 0) return 0;
     dim3 grid(T, H, (Dv + 63) / 64);
@@ -184,7 +202,7 @@ extern "C" int qe_linear_recurrence(const void* q, const void* k, const void* v,
 #define QE_LR3(TA_, DPG_, MODE_) linear_recurrence_kernel<TA_, DPG_, MODE_><<<grid, REC_DG * 64, 0, stream>>>(              \
         (const TA_*)q, (const TA_*)k, (const TA_*)v, row_stride, wx, w_stride, w0, u, decay, act_silu, state, \
         state_stride, tok_seq, out, T, H, D, Dv)
-#define QE_LR2(TA_, DPG_) do { if (mode == 0) QE_LR3(TA_, DPG_, 0); else QE_LR3(TA_, DPG_, 1); } while (0)
+#define QE_LR2(TA_, DPG_) do { if (mode == 0) QE_LR3(TA_, DPG_, 0); else if (mode == 1) QE_LR3(TA_, DPG_, 1); else QE_LR3(TA_, DPG_, 2); } while (0)
 #define QE_LR(TA_) do { if (dpg == 8) QE_LR2(TA_, 8); else if (dpg == 16) QE_LR2(TA_, 16); else if (dpg == 32) QE_LR2(TA_, 32); else QE_LR2(TA_, 64); } while (0)
     if (dt_a == QE_F32) QE_LR(float);
     else if (dt_a == QE_BF16) QE_LR(bf16_t);
@@ -321,6 +339,8 @@ extern "C" int qe_scaled_sum(const void* a, float sa, const void* b, float sb, i
 //   a decay per key channel:  with L_t the running sum of log w (= -exp(x + w0)) up to row t, in 64-bit:
 //       g_s = exp(L_(n-1) - L_s), gamma = exp(L_(n-1)), a_t = exp(L_(t-1)),
 //       A[t][s] = sum_d q_t[d] k_s[d] exp(L_(t-1)[d] - L_s[d]) (s < t),  A[t][t] = sum_d q_t[d] u[d] k_t[d]
+//   a forget gate per key channel: k_s = 1 - f_s, L_t the running sum of log f, a_t = exp(L_t),
+//       A[t][s] = sum_d q_t[d] k_s[d] exp(L_t[d] - L_s[d]) (s <= t)
 //   (every exponent is <= 0: nothing overflows however strong the decays; log w is kept above -200, below which
 //   w is 0 in 32-bit anyway, so that the running sums keep their small terms)
 // Three launches: every chunk's sum_s diag(g_s) k_s v_s^T and gamma (parallel over chunks, heads and blocks of 64
@@ -343,7 +363,7 @@ __host__ __device__ __forceinline__ RecChunkLayout rec_chunk_layout(int C, int D
     L.s = L.a + C * C;
     L.pw = L.s + L.d4 * 64;
     L.l = L.pw + ((C + 1 + 3) & ~3);
-    L.total = L.l + (mode == 1 ? 2 * C * L.d4 : 0);
+    L.total = L.l + (mode != 0 ? 2 * C * L.d4 : 0);
     return L;
 }
 
@@ -377,19 +397,25 @@ __global__ __launch_bounds__(RC_THREADS) void recurrence_chunk_kernel(
             const long r = (long)(row0 + t) * row_stride + h * D + d;
             b = Elem<TA>::load(k + r);
             if (PHASE == 1) a = Elem<TA>::load(q + r);
-            if (act_silu) { a = silu_f(a); b = silu_f(b); }
+            if (act_silu) { a = silu_f(a); if (MODE != 2) b = silu_f(b); }
+            if (MODE == 2) {
+                float f;
+                const float z = b + w0[h * D + d];
+                forget_gate(z, u[h * D + d], f, b);
+                lw = (double)fmaxf(log_forget(f, b), -200.f);
+            }
             if (MODE == 1) lw = -(double)fminf(expf(wx[(long)(row0 + t) * w_stride + h * D + d] + w0[h * D + d]), 200.f);   // (exp(-200) is 0 in 32-bit)
         }
         qs[t * L.ld + d] = a;
         ks[t * L.ld + d] = b;
-        if (MODE == 1) Ld[t * L.d4 + d] = lw;
+        if (MODE != 0) Ld[t * L.d4 + d] = lw;
     }
     for (int i = tid; i < C * 64; i += RC_THREADS) {
         const int t = i >> 6, cc = i & 63;
         float x = 0.f;
         if (t < n && col0 + cc < Dv) {
             x = Elem<TA>::load(v + (long)(row0 + t) * row_stride + (long)h * Dv + col0 + cc);
-            if (act_silu) x = silu_f(x);
+            if (act_silu && MODE != 2) x = silu_f(x);
         }
         vs[i] = x;
     }
@@ -399,7 +425,7 @@ __global__ __launch_bounds__(RC_THREADS) void recurrence_chunk_kernel(
         for (int i = 0; i <= C; ++i) { pw[i] = x; x *= dec; }
     }
     __syncthreads();
-    if (MODE == 1) {
+    if (MODE != 0) {
         for (int d = tid; d < L.d4; d += RC_THREADS) {
             double run = 0.0;
             for (int t = 0; t < C; ++t) { run += Ld[t * L.d4 + d]; Ld[t * L.d4 + d] = run; }     // (rows from n on add nothing)
@@ -461,10 +487,10 @@ __global__ __launch_bounds__(RC_THREADS) void recurrence_chunk_kernel(
                     x = fmaf(e.x, f.x, x); y = fmaf(e.y, f.y, y); x = fmaf(e.z, f.z, x); y = fmaf(e.w, f.w, y);
                 }
                 a = (x + y) * pw[t - s];
-            } else if (s == t) {
+            } else if (MODE == 1 && s == t) {
                 for (int d = 0; d < D; ++d) a = fmaf(qs[t * L.ld + d] * u[h * D + d], ks[s * L.ld + d], a);
             } else {
-                const double* lt = Ld + (t - 1) * L.d4;
+                const double* lt = Ld + (MODE == 1 ? t - 1 : t) * L.d4;
                 const double* ls = Ld + s * L.d4;
                 for (int d = 0; d < D; ++d)
                     a = fmaf(qs[t * L.ld + d] * ks[s * L.ld + d], expf((float)(lt[d] - ls[d])), a);
@@ -477,6 +503,7 @@ __global__ __launch_bounds__(RC_THREADS) void recurrence_chunk_kernel(
         const int t = i / L.d4, d = i - t * L.d4;
         float a;
         if (MODE == 0) a = pw[t + 1];
+        else if (MODE == 2) a = expf((float)Ld[t * L.d4 + d]);
         else a = t == 0 ? 1.f : expf((float)Ld[(t - 1) * L.d4 + d]);
         qs[t * L.ld + d] *= a;
     }
@@ -544,7 +571,7 @@ extern "C" int qe_linear_recurrence_chunked(const void* q, const void* k, const 
                                             int H, int D, int Dv, int dt_a, hipStream_t stream) {
     QE_REQUIRE(n_chunks >= 0 && n_portions >= 0 && H > 0 && D > 0 && Dv > 0, "linear_recurrence: bad sizes");
     QE_REQUIRE(D <= 256, "linear_recurrence: heads of %d key channels (at most 256)", D);
-    QE_REQUIRE(mode == 0 ? decay != nullptr : (mode == 1 && wx && w0 && u), "linear_recurrence: mode %d lacks operands", mode);
+    QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "linear_recurrence: mode %d lacks operands", mode);
     QE_REQUIRE(state_stride >= (long)H * D * Dv, "linear_recurrence: state rows overlap");
     if (n_chunks == 0) return 0;
     QE_REQUIRE(ws && chunks && portions, "linear_recurrence: chunks without a workspace");
@@ -563,7 +590,7 @@ extern "C" int qe_linear_recurrence_chunked(const void* q, const void* k, const 
             (const TA_*)q, (const TA_*)k, (const TA_*)v, row_stride, wx, w_stride, w0, u, decay, act_silu, chunks,   \
             ws_s, ws_g, out, C, H, D, Dv);                                                                           \
     } while (0)
-#define QE_RC2(TA_, PHASE_) do { if (mode == 0) QE_RC(TA_, 0, PHASE_); else QE_RC(TA_, 1, PHASE_); } while (0)
+#define QE_RC2(TA_, PHASE_) do { if (mode == 0) QE_RC(TA_, 0, PHASE_); else if (mode == 1) QE_RC(TA_, 1, PHASE_); else QE_RC(TA_, 2, PHASE_); } while (0)
     QE_REQUIRE(dt_a == QE_F32 || dt_a == QE_BF16, "linear_recurrence: unknown element type %d", dt_a);
     if (dt_a == QE_F32) QE_RC2(float, 0); else QE_RC2(bf16_t, 0);
     recurrence_scan_kernel<<<dim3(n_portions, H, (D * Dv + 255) / 256), 256, 0, stream>>>(portions, tok_seq, ws_s, ws_g, state,

@@ -44,6 +44,8 @@ def load_library():
     sigs = {
         "qe_embedding": [vp, vp, vp, i32, i32, i32, i32, vp],
         "qe_rmsnorm": [vp, vp, i32, i32, i64, vp, vp, vp, i32, i32, f32, i32, i32, vp],
+        "qe_stream_norm": [vp, vp, i32, i32, vp, vp, i32, vp, vp, i32, vp, vp, vp, i32, i32, f32, i32, i32, vp, vp, vp, i32, vp],
+        "qe_norm_conv": [vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, vp],
         "qe_residual_add": [vp, vp, i64, i32, vp],
         "qe_scatter_int": [vp, vp, vp, i32, i64, vp],
         "qe_silu_mul": [vp, vp, i32, i32, i32, i32, vp],
@@ -59,7 +61,7 @@ def load_library():
         "qe_attention_decode_supported": [i32, i32, i32, i32, i32],
         "qe_attention_prefill_supported": [i32, i32, i32, i32, i32],
         "qe_attention_prefill_rows": [i32, i32],
-        "qe_attention_prefill_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, i32, i32, i32,
+        "qe_attention_prefill_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, i32, i32,
                                      i32, vp, i64, vp],
         "qe_attention_prefill_plan_segments": [i32, i32, i32],
         "qe_attention_prefill_tiles_run": [vp, i32, i32, vp, i32, vp],
@@ -67,7 +69,7 @@ def load_library():
         "qe_attention_prefill_plan": [i32, i32, i32, i32],
         "qe_attention_prefill_plan_uncut_keys": [],
         "qe_attention_prefill_workspace_bytes": [i32, i32, i32, i32, i32, i32],
-        "qe_attention_decode_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, i32, i32, f32, i32, i32, i32, i32, i32, vp, i64, vp],
+        "qe_attention_decode_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, i32, vp, i64, vp],
         "qe_attention_decode_fused_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, vp, vp, vp, f32, vp,
                                           i32, i32, i32, i32, f32, i32, i32, i32, vp, i64, vp],
         "qe_qk_rope_store": [vp, vp, vp, vp, f32, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp],
@@ -75,12 +77,12 @@ def load_library():
         "qe_qk_rope_store_parts_supported": [i32, i32],
         "qe_gemm_partial_preferred": [i32, i32, i32, i32, i32],
         "qe_gemm_branch_splits": [i32, i32, i32, i32, i32],
-        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, i32, vp],
+        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, vp],
         "qe_qkv_conv_rope_store": [vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp],
         "qe_scale_f32": [vp, i64, f32, vp],
-        "qe_moe_route_biased": [vp, vp, vp, vp, i32, i32, i32, f32, i32, vp, i32, vp],
+        "qe_moe_route_biased": [vp, vp, vp, vp, i32, i32, i32, f32, i32, vp, i32, i32, vp],
         "qe_moe_front_small_supported": [i32, i32, i32],
-        "qe_moe_front_small": [vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, i32, i32, vp, i32, vp],
+        "qe_moe_front_small": [vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, i32, i32, vp, i32, i32, vp],
         "qe_moe_row_gate": [vp, vp, i32, vp, i64, i32, i32, i32, vp],
         "qe_diff_heads": [vp, vp, vp, i64, i32, i32, i32, i32, i32, f32, f32, f32, i32, vp],
         "qe_moe_identity": [vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp],
@@ -117,7 +119,7 @@ def load_library():
         "qe_moe_gemm": [vp, vp, i32, vp, vp, vp, vp, vp, i32, i32, i32, i32, f32, f32, i32, i32, i32, i32, vp],
         "qe_moe_gather": [vp, vp, i32, vp, i32, i32, i32, vp],
         "qe_moe_combine": [vp, vp, vp, vp, i32, i32, i32, i32, vp],
-        "qe_gemm_mfma_grouped": [vp, vp, vp, vp, vp, i32, i32, i32, i32, f32, f32, i32, vp],
+        "qe_gemm_mfma_grouped": [vp, vp, vp, vp, vp, i32, i32, i32, i32, f32, f32, i32, vp, vp, vp],
         "qe_gemm_mfma_grouped_tile_rows": [],
         "qe_moe_tile_rows": [],
         "qe_moe_gemm_mfma_supported": [i32],
@@ -252,6 +254,75 @@ def rmsnorm(h: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.
     _need(out, "out", out_dtype, (n, H), h.device)
     _check(lib.qe_rmsnorm(h.data_ptr(), _ptr(delta), n_delta, dt_d, T, _ptr(rows), weight.data_ptr(),
                           out.data_ptr(), n, H, float(eps), _DT[out_dtype], int(bool(center)), _stream()), "rmsnorm")
+    return out
+
+
+def stream_norm(h: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, center: bool = False,
+                delta: Optional[torch.Tensor] = None, scale: Optional[torch.Tensor] = None,
+                kept: Optional[torch.Tensor] = None, index: int = 0, coef: Optional[torch.Tensor] = None,
+                rows: Optional[torch.Tensor] = None, conv_w: Optional[torch.Tensor] = None,
+                state: Optional[torch.Tensor] = None, tok_seq: Optional[torch.Tensor] = None,
+                single_rows: bool = False) -> Optional[torch.Tensor]:
+    """The residual sum, the average over depth, the norm and the convolution between two sublayers, on the 32-bit
+    stream h [T, H]:
+      v = h + scale * (sum of delta)          delta [T, H] or float32 [S, T, H], added in order; scale float32 [H] or None
+      kept[index] = v                         with ``kept`` float32 [n, T, H]
+      h <- sum_j coef[j] kept[j] (j <= index) with ``coef`` float32 [index + 1]; else h <- v
+      out = norm(h) * weight                  RMS norm, or with ``center`` layer norm
+      out_t += sum_j conv_w[j] norm_(t - taps + 1 + j)    with conv_w float32 [taps, H]; the inputs before a request's rows
+                                              are state[tok_seq[t]] (float32 [slots, taps - 1, H]), brought up to date
+    With ``rows`` (int32 [R]) only those rows are normed and nothing is written back.  ``single_rows``: every row is the
+    only row of its request (everything is one launch).  ``weight`` None: the sums alone."""
+    lib = load_library()
+    _need(h, "h", torch.float32, (None, None))
+    T, H = h.shape
+    dev = h.device
+    n_delta, dt_d = 0, F32
+    if delta is not None:
+        if delta.dim() == 3:
+            _need(delta, "delta", torch.float32, (None, T, H), dev)
+            n_delta = delta.shape[0]
+        else:
+            _need(delta, "delta", _ACT, (T, H), dev)
+            n_delta, dt_d = 1, _DT[delta.dtype]
+    if scale is not None:
+        _need(scale, "scale", torch.float32, (H,), dev)
+    if kept is not None:
+        _need(kept, "kept", torch.float32, (None, T, H), dev)
+        if not 0 <= index < kept.shape[0]:
+            raise KernelError(f"stream_norm: result {index} of {kept.shape[0]}")
+    if coef is not None:
+        _need(coef, "coef", torch.float32, (index + 1,), dev)
+    n = T
+    if rows is not None:
+        _need(rows, "rows", torch.int32, (None,), dev)
+        n = rows.shape[0]
+    out = stats = None
+    taps = 1
+    if weight is not None:
+        _need(weight, "weight", torch.float32, (H,), dev)
+        out = torch.empty((n, H), dtype=out_dtype, device=dev)
+    if conv_w is not None:
+        _need(conv_w, "conv_w", torch.float32, (None, H), dev)
+        taps = conv_w.shape[0]
+        _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
+        if rows is not None or weight is None:
+            raise KernelError("stream_norm: a convolution goes over all rows, after a norm")
+        if taps > 1:
+            if state is None:
+                raise KernelError(f"stream_norm: {taps} taps need a state")
+            _need(state, "state", torch.float32, (None, taps - 1, H), dev)
+        if not single_rows:
+            stats = torch.empty((T, 2), dtype=torch.float32, device=dev)
+    first_out = out if stats is None else None
+    fused = conv_w is not None and stats is None
+    _check(lib.qe_stream_norm(h.data_ptr(), _ptr(delta), n_delta, dt_d, _ptr(scale), _ptr(kept), int(index), _ptr(coef),
+                              _ptr(rows), n, _ptr(weight), _ptr(first_out), _ptr(stats), T, H, float(eps), _DT[out_dtype],
+                              int(bool(center)), _ptr(conv_w) if fused else None, _ptr(state) if fused else None,
+                              _ptr(tok_seq) if fused else None, taps, _stream()), "stream_norm")
+    if stats is not None:
+        _check(lib.qe_norm_conv(h.data_ptr(), stats.data_ptr(), weight.data_ptr(), conv_w.data_ptr(), _ptr(state),
+                                tok_seq.data_ptr(), out.data_ptr(), T, H, taps, _DT[out_dtype], _stream()), "norm_conv")
     return out
 
 
@@ -633,7 +704,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
               other_tiles: Optional[torch.Tensor] = None, prefill_groups: int = 0,
               max_other_keys: int = 0, prefill_segment_keys: int = -1,
               other_keys_row: Optional[int] = None, shared_keys: Optional[torch.Tensor] = None,
-              keep_first: int = 0, sink: bool = False, chunk: int = 0) -> torch.Tensor:
+              keep_first: int = 0, sink: bool = False, chunk: int = 0, softcap: float = 0.0) -> torch.Tensor:
     """q [T, Hq, D]; cache [pages, 2, Hkv, P, D] (key tiles [P][D], value tiles transposed [D][P]);
     positions, tok_seq int32 [T]; block_table int32 [B, max_blocks].  Token t sees the keys at
     positions max(0, p - window + 1) .. p of request tok_seq[t] (window 0: all).  The caller
@@ -655,7 +726,8 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
     Without the lists every row is treated alike.
 
     ``chunk`` (instead of a window): positions are cut into chunks of that many, counted from the request's
-    start, and a token sees the keys of its own chunk up to itself.
+    start, and a token sees the keys of its own chunk up to itself.  ``softcap`` > 0: the scaled scores pass
+    softcap * tanh(. / softcap) before the softmax.
 
     shared_keys (int32, an entry per row of block_table, or None): how many of a request's first keys
     other requests read too.  A hint for the decode kernel's loads; results do not depend on it."""
@@ -683,6 +755,9 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
     keep_first, sink = int(keep_first) if window > 0 else 0, int(bool(sink))
     if keep_first < 0:
         raise KernelError("attention: negative keep_first")
+    softcap = float(softcap)
+    if softcap < 0:
+        raise KernelError(f"attention: a soft cap of {softcap}")
     if keep_first or sink or chunk:
         prefill_segment_keys = 0    # (no segments of keys: such walks are short)
 
@@ -690,7 +765,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
         n = T if tokens is None else tokens.shape[0]
         _check(lib.qe_attention(q.data_ptr(), out.data_ptr(), cache.data_ptr(), positions.data_ptr(),
                                 tok_seq.data_ptr(), block_table.data_ptr(), max_blocks, _ptr(tokens), n,
-                                Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, _DT[q.dtype], _stream()),
+                                Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap, _DT[q.dtype], _stream()),
                "attention")
 
     if dec_tokens is None and other_tokens is None:
@@ -706,7 +781,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
                                                dec_tokens.data_ptr(), n_dec, positions.data_ptr(),
                                                tok_seq.data_ptr(), block_table.data_ptr(), max_blocks,
                                                _ptr(shared_keys), Hq, Hkv,
-                                               D, P, float(scale), int(window), keep_first, sink, int(max_dec_position),
+                                               D, P, float(scale), int(window), keep_first, sink, softcap, int(max_dec_position),
                                                DECODE_SPLIT_KEYS, ws.data_ptr(), nbytes, _stream()),
                    "attention (decode)")
         else:
@@ -739,7 +814,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
             _check(lib.qe_attention_prefill_run(q.data_ptr(), out.data_ptr(), cache.data_ptr(),
                                                 other_tiles.data_ptr(), n_tiles,
                                                 positions.data_ptr(), tok_seq.data_ptr(), block_table.data_ptr(),
-                                                max_blocks, Hq, Hkv, D, P, float(scale), int(window), keep_first, sink,
+                                                max_blocks, Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap,
                                                 int(prefill_groups), seg, max_keys, keys_row, _ptr(ws), nbytes,
                                                 _stream()),
                    "attention (prefill)")
@@ -1092,13 +1167,15 @@ def moe_route(logits: torch.Tensor, groups: int, keep: int, top: int):
 
 
 def moe_route_biased(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, scale: float,
-                     transposed: bool = False, logit_bias: Optional[torch.Tensor] = None, experts: int = 0):
+                     transposed: bool = False, logit_bias: Optional[torch.Tensor] = None, experts: int = 0,
+                     sigmoid: bool = False):
     """logits float32 [T, E] (``transposed``: [E, T]), correction float32 [E] -> (ids int32 [T, top], weights float32 [T, top]): softmax
     over all experts; the ``top`` largest of score + correction are chosen (the lower index on ties); their
     weights are their scores without the correction, divided by the chosen scores' sum (+ 1e-20), times scale.
     Without a correction (None) the ``top`` largest logits are chosen and weighed by the softmax over them alone.
     ``logit_bias`` (float32 [E]) is added to the logits first.  ``experts``: only the first so many outputs of the
-    logits are the router's (the rest belongs to the caller); 0: all."""
+    logits are the router's (the rest belongs to the caller); 0: all.  ``sigmoid``: an output's score is its sigmoid;
+    the choice goes by the logits (or score + correction), the weights are the chosen scores as they are, times scale."""
     lib = load_library()
     _need(logits, "logits", torch.float32, (None, None))
     T, ld = (logits.shape[1], 0) if transposed else logits.shape
@@ -1112,8 +1189,8 @@ def moe_route_biased(logits: torch.Tensor, correction: Optional[torch.Tensor], t
     ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _check(lib.qe_moe_route_biased(logits.data_ptr(), _ptr(correction), ids.data_ptr(), weights.data_ptr(), T, E,
-                                   int(top), float(scale), int(bool(transposed)), _ptr(logit_bias), int(ld), _stream()),
-           "moe_route_biased")
+                                   int(top), float(scale), int(bool(transposed)), _ptr(logit_bias), int(ld),
+                                   int(bool(sigmoid)), _stream()), "moe_route_biased")
     return ids, weights
 
 
@@ -1173,7 +1250,8 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
                 w_down: torch.Tensor, limit: float = 0.0, slope: float = 1.0, interleaved: bool = False,
                 algo: int = ALGO_AUTO, act: str = "gated", identity: int = 0,
                 rows_dtype: torch.dtype = torch.float32, biased_route=None,
-                parts_out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                parts_out: Optional[torch.Tensor] = None, sigmoid_route: bool = False,
+                weigh_input: bool = False) -> torch.Tensor:
     """The chosen experts' outputs, weighted: float32 [S, T, H] whose sum over S, in order, is the mixture's
     output (S = top: a token's choices in their order; or S = 1: already added up in that order).
     x [T, K]; w_gate_up [E, 2 F, K] (gate rows, then up rows; or, ``interleaved``, in alternating blocks of
@@ -1189,7 +1267,8 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
     a bias float32 [E + identity] that is added to the logits, and how many of the logits' outputs are the router's
     where they are the first of more): a step of few tokens then
     routes, sorts and writes the identity experts' rows in one launch.  ``limit`` 0: the plain silu(g) u.  ``parts_out``: float32 [top, T, H] to take the
-    parts (the paths of fewer than 1024 pairs only).
+    parts (the paths of fewer than 1024 pairs only).  ``sigmoid_route``: the routing's scores are sigmoids, see
+    moe_route_biased.  ``weigh_input``: a pair's weight multiplies what its expert reads instead of what it gives.
 
     The (token, choice) pairs are grouped by expert on the device.  bfloat16 with many pairs: their rows are
     gathered side by side and both products run on the tiled kernel of the dense products, a tile of 128
@@ -1226,6 +1305,8 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
     if act not in ("gated", "relu_sq"):
         raise KernelError(f"moe_experts: activation {act!r}")
     single = act == "relu_sq"
+    if weigh_input and (single or identity):
+        raise KernelError("moe_experts: weighed inputs go with gated experts")
     first_mode = 2 if single else 1
     Fd = F2 if single else F2 // 2
     _need(w_down, "w_down", x.dtype, (E, None, Fd), dev)
@@ -1267,12 +1348,13 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
             _check(lib.qe_moe_front_small(r_logits.data_ptr(), _ptr(r_corr), x.data_ptr(), ids.data_ptr(),
                                           weights.data_ptr(), perm.data_ptr(), inv.data_ptr(), tiles.data_ptr(),
                                           n_tiles.data_ptr(), parts.data_ptr(), max_tiles, T, Hout, E + identity, E, top,
-                                          float(r_scale), tile_rows, _DT[x.dtype], _ptr(r_bias), r_width, _stream()),
+                                          float(r_scale), tile_rows, _DT[x.dtype], _ptr(r_bias), r_width,
+                                          int(bool(sigmoid_route)), _stream()),
                    "moe_front_small")
             fused_front = True
         else:
             ids, weights = moe_route_biased(r_logits, r_corr, top, r_scale, transposed=r_transposed, logit_bias=r_bias,
-                                            experts=r_outputs)
+                                            experts=r_outputs, sigmoid=sigmoid_route)
     # (identity experts are buckets of the sort like the others, behind them, and get no tiles)
     if not fused_front:
         _check(lib.qe_moe_sort(ids.data_ptr(), n, E + identity, E, tile_rows, perm.data_ptr(), inv.data_ptr(), tiles.data_ptr(),
@@ -1284,39 +1366,41 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
                                        _ptr(rows_), T, top, Hout, E, _DT[x.dtype],
                                        int(rows_ is not None and rows_.dtype == x.dtype and x.dtype != torch.float32),
                                        _stream()), "moe_identity")
+    w_in, w_out = (weights.data_ptr(), None) if weigh_input else (None, weights.data_ptr())
     a = torch.empty((n, Fd), dtype=x.dtype, device=dev)
     if tiled:
         xs = torch.empty((n, K), dtype=x.dtype, device=dev)
         _check(lib.qe_moe_gather(x.data_ptr(), perm.data_ptr(), top, xs.data_ptr(), n, K, _DT[x.dtype], _stream()), "moe_gather")
         _check(lib.qe_gemm_mfma_grouped(xs.data_ptr(), w_gate_up.data_ptr(), a.data_ptr(), tiles.data_ptr(),
                                         n_tiles.data_ptr(), max_tiles, Fd if single else 2 * Fd, K, first_mode, float(limit),
-                                        float(slope), BF16, _stream()), "grouped gemm (gate, up)")
+                                        float(slope), BF16, w_in, perm.data_ptr() if weigh_input else None, _stream()),
+               "grouped gemm (gate, up)")
         if rows_dtype not in (torch.float32, torch.bfloat16):
             raise KernelError(f"moe_experts: rows in {rows_dtype}")
         y = torch.empty((n, Hout), dtype=rows_dtype, device=dev)
         _check(lib.qe_gemm_mfma_grouped(a.data_ptr(), w_down.data_ptr(), y.data_ptr(), tiles.data_ptr(),
-                                        n_tiles.data_ptr(), max_tiles, Hout, Fd, 0, 0.0, 1.0, _DT[rows_dtype], _stream()),
+                                        n_tiles.data_ptr(), max_tiles, Hout, Fd, 0, 0.0, 1.0, _DT[rows_dtype], None, None, _stream()),
                "grouped gemm (down)")
         identity(None, y)
         out = torch.empty((1, T, Hout), dtype=torch.float32, device=dev)
-        _check(lib.qe_moe_combine(y.data_ptr(), inv.data_ptr(), weights.data_ptr(), out.data_ptr(), T, top, Hout,
+        _check(lib.qe_moe_combine(y.data_ptr(), inv.data_ptr(), w_out, out.data_ptr(), T, top, Hout,
                                   _DT[rows_dtype], _stream()), "moe_combine")
         return out
     if parts is None:
         parts = torch.empty((top, T, Hout), dtype=torch.float32, device=dev)
     if mfma:
-        _check(lib.qe_moe_gemm_mfma(x.data_ptr(), perm.data_ptr(), top, w_gate_up.data_ptr(), a.data_ptr(), None,
+        _check(lib.qe_moe_gemm_mfma(x.data_ptr(), perm.data_ptr(), top, w_gate_up.data_ptr(), a.data_ptr(), w_in,
                                     tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, T, Fd, K, float(limit),
                                     float(slope), first_mode, int(interleaved), _stream()), "moe_gemm (gate, up; mfma)")
         _check(lib.qe_moe_gemm_mfma(a.data_ptr(), perm.data_ptr(), top, w_down.data_ptr(), parts.data_ptr(),
-                                    weights.data_ptr(), tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, T,
+                                    w_out, tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, T,
                                     Hout, Fd, 0.0, 0.0, 0, 0, _stream()), "moe_gemm (down; mfma)")
         identity(parts, None)
         return parts
-    _check(lib.qe_moe_gemm(x.data_ptr(), perm.data_ptr(), top, w_gate_up.data_ptr(), a.data_ptr(), None,
+    _check(lib.qe_moe_gemm(x.data_ptr(), perm.data_ptr(), top, w_gate_up.data_ptr(), a.data_ptr(), w_in,
                            tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, T, Fd, K, float(limit), float(slope), first_mode,
                            int(interleaved), _DT[x.dtype], _DT[w_gate_up.dtype], _stream()), "moe_gemm (gate, up)")
-    _check(lib.qe_moe_gemm(a.data_ptr(), perm.data_ptr(), top, w_down.data_ptr(), parts.data_ptr(), weights.data_ptr(),
+    _check(lib.qe_moe_gemm(a.data_ptr(), perm.data_ptr(), top, w_down.data_ptr(), parts.data_ptr(), w_out,
                            tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, T, Hout, Fd, 0.0, 0.0, 0, 0,
                            _DT[x.dtype], _DT[w_down.dtype], _stream()), "moe_gemm (down)")
     identity(parts, None)
@@ -1476,13 +1560,16 @@ def recurrence_chunks(portions, chunk_len: int):
 def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, tok_seq: torch.Tensor,
                       heads: int, decay: Optional[torch.Tensor] = None, decay_x: Optional[torch.Tensor] = None,
                       decay_bias: Optional[torch.Tensor] = None, bonus: Optional[torch.Tensor] = None,
-                      silu: bool = False, chunks=None) -> torch.Tensor:
+                      silu: bool = False, chunks=None, forget_bias: Optional[torch.Tensor] = None,
+                      lower: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per head, with a 32-bit state S [D][Dv] per request (state[tok_seq[t]], float32 [slots, >= H D Dv]):
     with ``decay`` (float32 [H]):  S <- decay_h S + k_t v_t^T, o_t = S^T q_t;
     with ``decay_x`` float32 [T, H D], ``decay_bias`` and ``bonus`` (float32 [H D]):  o_t = (S + diag(bonus) k_t v_t^T)^T q_t,
     then S <- diag(w_t) S + k_t v_t^T with w_t = exp(-exp(decay_x_t + decay_bias)).
+    with ``forget_bias`` and ``lower`` (float32 [H D]) k holds the logits of a forget gate f = lower + (1 - lower)
+    sigmoid(k + forget_bias):  S <- diag(f_t) S + (1 - f_t) v_t^T, o_t = S^T q_t.
     q, k [T, H D], v [T, H Dv] (column slices of one wider tensor are taken as they are, all with one row stride);
-    ``silu``: the three pass silu first.  Returns o float32 [T, H, Dv].
+    ``silu``: the three (with a forget gate: q) pass silu first.  Returns o float32 [T, H, Dv].
     ``chunks`` (recurrence_chunks() of all rows' portions, on the device, for recurrence_chunk_len(D)): the rows are
     taken chunk by chunk, the chunks in parallel, instead of row by row: for long portions."""
     lib = load_library()
@@ -1499,6 +1586,11 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     mode, sw = 0, 0
     if decay is not None:
         _need(decay, "decay", torch.float32, (H,), dev)
+    elif lower is not None:
+        mode = 2
+        _need(forget_bias, "forget_bias", torch.float32, (H * D,), dev)
+        _need(lower, "lower", torch.float32, (H * D,), dev)
+        decay_bias, bonus = forget_bias, lower
     else:
         mode = 1
         if decay_x is None or decay_x.dtype != torch.float32:

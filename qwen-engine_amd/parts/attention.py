@@ -143,7 +143,7 @@ class PagedAttention:
         self.window = int(spec.window) if spec.window else 0
         self.qk_eps = spec.qk_norm_eps
         self.position = build_part(spec.position, hidden_size) if spec.position is not None else None
-        self.w_qkv = self.b_qkv = self.w_o = self.q_norm = self.k_norm = None
+        self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.q_norm = self.k_norm = None
 
     @property
     def graph_safe(self) -> bool:
@@ -274,8 +274,8 @@ class PagedAttention:
         if splits:
             # the product is cut along K (few rows: to fill the chip; a narrow matrix: to give every
             # compute unit blocks to overlap); the norm that follows adds the parts
-            return ops.gemm(o, self.w_o, epilogue=ops.EPI_PARTIAL, splits=splits)
-        return ops.gemm(o, self.w_o)
+            return ops.gemm(o, self.w_o, self.b_o, epilogue=ops.EPI_PARTIAL, splits=splits)
+        return ops.gemm(o, self.w_o, self.b_o)
 
 
 def common_head_dim(k_dim: int, v_dim: int) -> int:
@@ -291,11 +291,11 @@ def common_head_dim(k_dim: int, v_dim: int) -> int:
 
 
 class ConvAttention(PagedAttention):
-    """Grouped-query attention with a short causal convolution over time on every channel of the projected q, k
-    and v (``ConvAttentionSpec``): one product for q | k | v with the biases, then one kernel that convolves (a
+    """Grouped-query attention, with a short causal convolution over time on every channel of the projected q, k
+    and v if asked for (``ConvAttentionSpec``): one product for q | k | v with the biases, then one kernel that convolves (a
     request's last ``conv_taps - 1`` projected rows are its state), rotates the first numbers of every q and k head
-    and writes q and the cache, then the attention kernels of PagedAttention with the window's kept first keys and
-    the sink, then the output projection.  Keys and values of different sizes share the cache under one head size
+    and writes q and the cache, then the attention kernels of PagedAttention with the window's kept first keys,
+    the sink and the soft cap, then the output projection.  Keys and values of different sizes share the cache under one head size
     (``common_head_dim``), and the output projection's columns beyond a value head's own numbers are zeros."""
     takes_stream = False
 
@@ -311,9 +311,10 @@ class ConvAttention(PagedAttention):
         self.window = int(spec.window) if spec.window else 0
         self.keep_first = int(spec.keep_first) if self.window else 0
         self.sink = bool(spec.sink)
+        self.softcap = float(spec.softcap) if spec.softcap is not None else 0.0
         self.taps = int(spec.conv_taps)
         self.position = build_part(spec.position, hidden_size) if spec.position is not None else None
-        self.w_qkv = self.b_qkv = self.w_o = self.conv_w = self.conv_w_t = None
+        self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.conv_w = self.conv_w_t = None
 
     graph_safe = True        # every launch's grid follows the rows alone; the state is device memory
 
@@ -334,6 +335,8 @@ class ConvAttention(PagedAttention):
             if spec.conv_taps >= 1:
                 t[name + spec.conv_suffix] = TensorInfo((n, int(spec.conv_taps)), "normal", "vector")
         t[no] = TensorInfo((hidden, spec.num_heads * spec.v_head_dim))
+        if spec.out_bias:
+            t[no + spec.bias_suffix] = TensorInfo((hidden,), "zeros", "vector")
         return t
 
     @staticmethod
@@ -356,6 +359,8 @@ class ConvAttention(PagedAttention):
         self.w_qkv = rt.place_matrix(torch.cat(mats, dim=0))
         if s.qkv_bias:
             self.b_qkv = rt.place_vector(torch.cat([tensors[n + s.bias_suffix].float() for n in (nq, nk, nv)]))
+        if s.out_bias:
+            self.b_o = rt.place_vector(tensors[no + s.bias_suffix])
         if self.taps >= 1:
             self.conv_w = rt.place_vector(torch.cat([tensors[n + s.conv_suffix].float() for n in (nq, nk, nv)], dim=0))
         else:                                              # no convolution: one tap of weight 1
@@ -398,12 +403,12 @@ class ConvAttention(PagedAttention):
                           other_tokens=ex["other_tokens"],
                           other_tiles=self._other_tiles(ctx) if ex["other_tokens"] is not None else None,
                           max_other_keys=ex.get("max_other_keys", 0), other_keys_row=ex.get("other_keys_row"),
-                          shared_keys=ctx.shared_keys, keep_first=self.keep_first, sink=self.sink)
+                          shared_keys=ctx.shared_keys, keep_first=self.keep_first, sink=self.sink, softcap=self.softcap)
         o = o.view(T, self.hq * self.d)
         if parts_out is not None:
-            return ops.gemm(o, self.w_o, epilogue=ops.EPI_PARTIAL, splits=parts_out.shape[0], out=parts_out)
+            return ops.gemm(o, self.w_o, self.b_o, epilogue=ops.EPI_PARTIAL, splits=parts_out.shape[0], out=parts_out)
         if add_to is not None and not ops.gemm_branch_splits(o, self.w_o) and ops.gemm_fused_supported(o, self.w_o):
-            ops.gemm(o, self.w_o, epilogue=ops.EPI_RESIDUAL, out=add_to)
+            ops.gemm(o, self.w_o, self.b_o, epilogue=ops.EPI_RESIDUAL, out=add_to)
             return None
         return self._project_out(o)
 

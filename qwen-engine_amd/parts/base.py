@@ -4,7 +4,8 @@ model it is in: each gets its sizes and constants from its spec.
 Norm          forward(h, rt, delta=None, rows=None) -> x
               h is the 32-bit residual stream [T, H]; with ``delta`` (a branch output, see
               below) the sum h + delta is normed and written back to h; with ``rows`` only
-              those rows are normed.
+              those rows are normed.  ``delta`` may be a BranchSum: a branch output with a scale per
+              channel and an average over depth on the way.
 Mixer         forward(x, ctx, binding) -> y      x, y [T, H] in the activation type
               cache_need(spec) -> KVNeed | None, state_need(spec, hidden) -> StateNeed | None
 FeedForward   forward(x, ctx) -> y
@@ -125,6 +126,40 @@ class Stream:
 
 
 @dataclass
+class DepthAverage:
+    """Where a layer's result is kept for the averages over depth, and the average that follows it."""
+    kept: torch.Tensor               # float32 [n, T, H]: the results so far, entry 0 the embedding output
+    index: int                       # this result's place
+    coef: Optional[torch.Tensor]     # float32 [index + 1]: the stream becomes sum_j coef[j] kept[j]; None: it stays as it is
+
+
+@dataclass
+class BranchSum:
+    """A branch output that is still to be added to the stream, with what its layer does to it on the way: handed on in
+    the place of the plain branch output, and resolved by the norm that follows (or by ``add_pending``)."""
+    parts: Optional[torch.Tensor]    # [T, H] in the activation type, or float32 [S, T, H]; None: nothing is added
+    scale: Optional[torch.Tensor] = None     # float32 [H]: multiplies the branch's sum
+    average: Optional[DepthAverage] = None
+
+    def kernel_args(self) -> dict:
+        a = self.average
+        d = dict(delta=self.parts, scale=self.scale)
+        if a is not None:
+            d.update(kept=a.kept, index=a.index, coef=a.coef)
+        return d
+
+
+def add_pending(h: torch.Tensor, pending) -> None:
+    """A pending branch output of any form into the stream, by a kernel of its own (for blocks whose first step is not a
+    norm of the stream)."""
+    from ..kernels import ops
+    if isinstance(pending, BranchSum):
+        ops.stream_norm(h, None, 0.0, torch.float32 if pending.parts is None else pending.parts.dtype, **pending.kernel_args())
+    elif pending is not None:
+        ops.residual_add(h, pending)
+
+
+@dataclass
 class StreamInput:
     """The input of a part as (stream, what is still to be added to it, norm before the part)
     instead of the normed rows."""
@@ -143,6 +178,8 @@ class StreamInput:
         """True if a product can take the residual sum and the norm as its prologue at all: nothing to
         add, or float32 partial products and a second buffer for the sums."""
         d = self.delta
+        if isinstance(d, BranchSum):
+            return False
         return d is None or (d.dim() == 3 and d.dtype == torch.float32 and self.stream.spare is not None)
 
     def prefers_prologue(self, ops, w: torch.Tensor) -> bool:

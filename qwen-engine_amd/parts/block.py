@@ -8,7 +8,8 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import CacheBinding, Runtime, Stream, StreamInput, TensorInfo, join_name, named_tensors, sub_tensors
+from .base import (BranchSum, CacheBinding, DepthAverage, Runtime, Stream, StreamInput, TensorInfo, add_pending, join_name,
+                   named_tensors, sub_tensors)
 from ..kernels import ops
 from .registry import build_part, part_class, register_part
 
@@ -188,8 +189,7 @@ class PostNormBlock:
         kind before this one left to be added.  Returns None: nothing is left to add."""
         x = h.h if isinstance(h, Stream) else h
         rt = ctx.rt
-        if pending is not None:
-            ops.residual_add(x, pending)
+        add_pending(x, pending)
         binding = bindings[0]
         kept = ctx.memo.pop(self._COPY, None) if pending is None else None
         if self.conv is not None:
@@ -290,6 +290,103 @@ class ParallelBlock:
         return y
 
 
+class ScaledPreNormBlock(PreNormBlock):
+    """A pre-norm block with, each if asked for, a causal convolution on what a sublayer reads, a factor per channel on
+    what it gives, and a weighted sum over all layers' results after it (``ScaledLayerSpec``).  The factor, the residual
+    sum, the average and the norm that follows are one kernel (with single new tokens the convolution too): the block
+    hands its branch on as a BranchSum.  Cache users: the mixer, then the convolutions.  The results of the layers
+    travel in ctx.memo, one tensor for the step."""
+    _KEPT = "depth_average.kept"
+
+    def __init__(self, spec, hidden_size: int):
+        super().__init__(spec, hidden_size)
+        self.mixer_conv = build_part(spec.mixer_conv, hidden_size) if spec.mixer_conv is not None else None
+        self.ffn_conv = build_part(spec.ffn_conv, hidden_size) if spec.ffn_conv is not None and self.ffn is not None else None
+        self.mixer_scale = self.ffn_scale = self.coef = None
+
+    def parts(self):
+        return super().parts() + tuple(p for p in (self.mixer_conv, self.ffn_conv) if p is not None)
+
+    @property
+    def graph_safe_with_state(self) -> bool:
+        return all(getattr(p, "graph_safe", False) is True for p in (self.mixer, self.mixer_conv, self.ffn_conv)
+                   if p is not None)
+
+    @staticmethod
+    def cache_needs(spec, hidden: int):
+        needs = PreNormBlock.cache_needs(spec, hidden)
+        for conv in (spec.mixer_conv, spec.ffn_conv if spec.ffn is not None else None):
+            if conv is not None:
+                needs.append((None, part_class(conv.kind).state_need(conv, hidden)))
+        return needs
+
+    @staticmethod
+    def _vectors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        """The block's own tensors."""
+        t: Dict[str, TensorInfo] = {}
+        if spec.layer_scale:
+            t[spec.scale_names[0]] = TensorInfo((hidden,), "ones", "vector")
+            t[spec.scale_names[1]] = TensorInfo((hidden,), "ones", "vector", optional=spec.ffn is None)
+        if spec.depth_average is not None:
+            t[spec.average_name] = TensorInfo((int(spec.depth_average.index) + 2,), "normal", "vector")
+        return t
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        out = PreNormBlock.expected_tensors(spec, hidden)
+        around = [(spec.conv_names[0], spec.mixer_conv, False), (spec.conv_names[1], spec.ffn_conv, spec.ffn is None)]
+        if spec.ffn is None:               # (what stands around a missing feed-forward may be there and is not used)
+            around.append((_names(spec)[2], spec.ffn_norm, True))
+        for name, sub, optional in around:
+            if sub is not None:
+                for rel, info in part_class(sub.kind).expected_tensors(sub, hidden).items():
+                    out[join_name(name, rel)] = info._replace(optional=True) if optional else info
+        out.update(ScaledPreNormBlock._vectors(spec, hidden))
+        return out
+
+    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        s = self.spec
+        super().load(tensors, rt)
+        for name, sub, part in ((s.conv_names[0], s.mixer_conv, self.mixer_conv), (s.conv_names[1], s.ffn_conv, self.ffn_conv)):
+            if part is not None:
+                part.load(named_tensors(tensors, name, type(part).expected_tensors(sub, self.hidden)), rt)
+        if s.layer_scale:
+            self.mixer_scale = rt.place_vector(tensors[s.scale_names[0]])
+            if self.ffn is not None:
+                self.ffn_scale = rt.place_vector(tensors[s.scale_names[1]])
+        if s.depth_average is not None:
+            self.coef = rt.place_vector(tensors[s.average_name])
+
+    def forward(self, h, pending, ctx, bindings):
+        x = h.h if isinstance(h, Stream) else h
+        bind = iter(bindings[1:])
+        avg = self.spec.depth_average
+        kept = None
+        if avg is not None:
+            key = (self._KEPT, int(avg.layers))
+            kept = ctx.memo.get(key)
+            if kept is None:
+                kept = ctx.memo[key] = torch.empty((int(avg.layers) + 1, *x.shape), dtype=torch.float32, device=x.device)
+            if avg.index == 0:             # (the stream is the embedding output: the first result)
+                add_pending(x, pending)
+                pending = BranchSum(None, average=DepthAverage(kept, 0, None))
+        u = self._sublayer_input(self.mixer_norm, self.mixer_conv, x, pending, ctx, bind)
+        last = BranchSum(self.mixer.forward(u, ctx, bindings[0]), self.mixer_scale)
+        if self.ffn is not None:
+            u = self._sublayer_input(self.ffn_norm, self.ffn_conv, x, last, ctx, bind)
+            last = BranchSum(self.ffn.forward(u, ctx), self.ffn_scale)
+        if avg is not None:
+            last.average = DepthAverage(kept, int(avg.index) + 1, self.coef)
+        return last
+
+    @staticmethod
+    def _sublayer_input(norm, conv, x: torch.Tensor, pending, ctx, bind) -> torch.Tensor:
+        if conv is None:
+            return norm.forward(x, ctx.rt, delta=pending)
+        return conv.after_norm(norm, x, pending, ctx, next(bind).state)
+
+
 register_part("prenorm_block", PreNormBlock)
+register_part("scaled_prenorm_block", ScaledPreNormBlock)
 register_part("parallel_block", ParallelBlock)
 register_part("postnorm_block", PostNormBlock)

@@ -232,6 +232,10 @@ class TopSoftmaxMoE:
             total += (self.shared.w_gu.numel() + self.shared.w_down.numel()) * self.shared.w_down.element_size()
         return total
 
+    def _routing(self) -> dict:
+        """How ops.moe_experts scores and weighs, where it differs from a softmax over the chosen logits."""
+        return {}
+
     def forward(self, x: torch.Tensor, ctx) -> torch.Tensor:
         T = x.shape[0]
         outputs = self.w_router.shape[0]
@@ -240,12 +244,14 @@ class TopSoftmaxMoE:
         logits = ops.gemm(self.w_router, x, out_dtype=torch.float32) if transposed else \
             ops.gemm(x, self.w_router, out_dtype=torch.float32)
         route = (logits, None, self.top, 1.0, transposed, self.router_bias, self.e)
+        how = self._routing()
         if self.shared is None:
-            return ops.moe_experts(x, None, None, self.w_gate_up, self.w_down, interleaved=self.interleaved, biased_route=route)
+            return ops.moe_experts(x, None, None, self.w_gate_up, self.w_down, interleaved=self.interleaved, biased_route=route,
+                                   **how)
         few = T * self.top < 1024          # (the paths of ops.moe_experts that leave a part per choice)
         parts = torch.empty((self.top + 1, T, self.hidden), dtype=torch.float32, device=x.device) if few else None
         out = ops.moe_experts(x, None, None, self.w_gate_up, self.w_down, interleaved=self.interleaved, biased_route=route,
-                              parts_out=parts[:self.top] if few else None)
+                              parts_out=parts[:self.top] if few else None, **how)
         a = self.shared.activation(x)
         if not self.shared_gate:
             if few:
@@ -262,7 +268,17 @@ class TopSoftmaxMoE:
         return out
 
 
+class SigmoidMoE(TopSoftmaxMoE):
+    """The same mixture with sigmoid scores (``SigmoidMoESpec``): the largest logits chosen, each weighed by its own
+    sigmoid; with ``weigh_input`` the weight multiplies the expert's input: gate and up are linear in it, so the first
+    product's epilogue multiplies both by the pair's weight in 32-bit before the activation."""
+
+    def _routing(self) -> dict:
+        return dict(sigmoid_route=True, weigh_input=bool(self.spec.weigh_input))
+
+
 register_part("polynorm_mlp", PolyNormMLP)
+register_part("sigmoid_moe", SigmoidMoE)
 register_part("top_softmax_moe", TopSoftmaxMoE)
 register_part("biased_moe", BiasedMoE)
 register_part("grouped_moe", GroupedMoE)

@@ -7,11 +7,20 @@ from typing import Dict, Optional
 import torch
 
 from ..kernels import ops
-from .base import Runtime, TensorInfo
+from .base import BranchSum, Runtime, TensorInfo
 from .registry import register_part
 
 
+def _norm(h: torch.Tensor, weight: torch.Tensor, eps: float, rt: Runtime, delta, rows, center: bool) -> torch.Tensor:
+    """A norm of the stream with whatever is pending before it."""
+    if isinstance(delta, BranchSum):
+        return ops.stream_norm(h, weight, eps, rt.dtype, center=center, rows=rows, **delta.kernel_args())
+    return ops.rmsnorm(h, weight, eps, rt.dtype, delta=delta, rows=rows, center=center)
+
+
 class RMSNorm:
+    center = False           # (a layer norm takes the mean off first)
+
     def __init__(self, spec, size: int):
         self.eps = float(spec.eps)
         self.size = int(size)
@@ -30,7 +39,7 @@ class RMSNorm:
 
     def forward(self, h: torch.Tensor, rt: Runtime, delta: Optional[torch.Tensor] = None,
                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-        return ops.rmsnorm(h, self.weight, self.eps, rt.dtype, delta=delta, rows=rows)
+        return _norm(h, self.weight, self.eps, rt, delta, rows, self.center)
 
     def after_sum(self, x: torch.Tensor, delta: Optional[torch.Tensor], alpha: float, rt: Runtime):
         """The norm of a post-norm block: x <- w * z / rms(z) with z = alpha * x + delta, on the 32-bit stream in
@@ -43,6 +52,7 @@ class ScalarRMSNorm:
     ``forward`` is the norm interface of ``parts.base`` (the model's last norm, on the wanted rows);
     ``after_sum`` is the norm of a post-norm block: x <- g * z / rms(z) with z = alpha * x + delta, on the
     32-bit stream in place, returning the new x in the activation type where that is not 32-bit."""
+    center = False
 
     def __init__(self, spec, size: int):
         self.eps = float(spec.eps)
@@ -60,7 +70,7 @@ class ScalarRMSNorm:
 
     def forward(self, h: torch.Tensor, rt: Runtime, delta: Optional[torch.Tensor] = None,
                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-        return ops.rmsnorm(h, self.weight, self.eps, rt.dtype, delta=delta, rows=rows)
+        return _norm(h, self.weight, self.eps, rt, delta, rows, self.center)
 
     def after_sum(self, x: torch.Tensor, delta: Optional[torch.Tensor], alpha: float, rt: Runtime):
         return ops.postnorm(x, delta, alpha, self.gain, self.eps, rt.dtype)
@@ -81,6 +91,7 @@ class BareLayerNorm:
     """Layer norm with a weight and no bias, (v - mean) * rsqrt(mean of the squared deviations + eps) * w, the weight
     tensor named as the part itself.  The residual sum that stands before it is formed in the same kernel, as in the
     RMS norms; it is no product's prologue (no ``fusable_weight``)."""
+    center = True
 
     def __init__(self, spec, size: int):
         self.eps = float(spec.eps)
@@ -96,7 +107,7 @@ class BareLayerNorm:
 
     def forward(self, h: torch.Tensor, rt: Runtime, delta: Optional[torch.Tensor] = None,
                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-        return ops.rmsnorm(h, self.weight, self.eps, rt.dtype, delta=delta, rows=rows, center=True)
+        return _norm(h, self.weight, self.eps, rt, delta, rows, self.center)
 
 
 class StreamScale:
@@ -135,7 +146,26 @@ class LogitSoftcap:
         return ops.unary(logits, ops.UNARY_SOFTCAP, cap=self.cap, inplace=True)
 
 
+class LogitScale:
+    """logits <- scale * logits, in place on the 32-bit logits."""
+
+    def __init__(self, spec, hidden_size: int = 0):
+        self.scale = float(spec.scale)
+
+    @staticmethod
+    def expected_tensors(spec, hidden_size: int) -> Dict[str, TensorInfo]:
+        return {}
+
+    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        pass
+
+    def forward(self, logits: torch.Tensor, ctx) -> torch.Tensor:
+        ops.scale_(logits, self.scale)
+        return logits
+
+
 register_part("rmsnorm", RMSNorm)
+register_part("logit_scale", LogitScale)
 register_part("logit_softcap", LogitSoftcap)
 register_part("rmsnorm_bare", BareRMSNorm)
 register_part("layernorm_bare", BareLayerNorm)

@@ -146,6 +146,61 @@ class DecayedLinearMixer:
         return ops.gemm(z, self.w_o, out_dtype=torch.float32)
 
 
+class ForgetGateLinearMixer:
+    """``ForgetGateLinearSpec`` (HGRN2): one product for q | f | v that stays 32-bit (the gate enters the recurrence), the
+    recurrence (silu on q, the gate and what it leaves to be written formed as they are read), a norm per head, the
+    output projection."""
+    graph_safe = True
+
+    def __init__(self, spec, hidden_size: int):
+        self.spec = spec
+        self.hidden = int(hidden_size)
+        self.h, self.d, self.dv = int(spec.num_heads), int(spec.head_dim), int(spec.v_head_dim)
+        self.eps = float(spec.norm_eps)
+        self.w_in = self.w_o = self.norm = self.forget_bias = self.lower = None
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        nk, nv = spec.num_heads * spec.head_dim, spec.num_heads * spec.v_head_dim
+        q, f, fb, low, v, norm, o = spec.names
+        return {q: TensorInfo((nk, hidden)), f: TensorInfo((nk, hidden)), fb: TensorInfo((nk,), "zeros", "vector"),
+                low: TensorInfo((nk,), "zeros", "vector"), v: TensorInfo((nv, hidden)),
+                norm: TensorInfo((int(spec.v_head_dim),), "ones", "vector"), o: TensorInfo((hidden, nv))}
+
+    @staticmethod
+    def cache_need(spec):
+        return None
+
+    @staticmethod
+    def state_need(spec, hidden: int) -> Optional[StateNeed]:
+        return StateNeed(shape=(spec.num_heads * spec.head_dim * spec.v_head_dim,), dtype="float32")
+
+    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        q, f, fb, low, v, norm, o = self.spec.names
+        mats = [tensors[n] for n in (q, f, v)]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        self.w_in = rt.place_matrix(torch.cat(mats, dim=0))
+        self.w_o = rt.place_matrix(tensors[o])
+        self.forget_bias = rt.place_vector(tensors[fb])
+        self.lower = rt.place_vector(tensors[low])
+        self.norm = rt.place_vector(tensors[norm]).repeat(self.h)
+
+    def forward(self, x: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+        if binding.state is None:
+            raise RuntimeError("the recurrence was given no state")
+        T = x.shape[0]
+        nk, nv = self.h * self.d, self.h * self.dv
+        y = ops.gemm(x, self.w_in, out_dtype=torch.float32)
+        o = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:], binding.state, ctx.tok_seq, self.h, silu=True,
+                                  forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.d))
+        z = ops.gated_norm(o.view(T, nv), self.norm, self.eps, self.h, ctx.rt.dtype)
+        splits = ops.gemm_branch_splits(z, self.w_o)
+        if splits:
+            return ops.gemm(z, self.w_o, epilogue=ops.EPI_PARTIAL, splits=splits)
+        return ops.gemm(z, self.w_o)
+
+
 class SideBySideMixer:
     """``SideBySideMixerSpec``: two mixers read the same rows; their outputs are added with weights, in 32-bit.  The
     two share the block's one cache binding: the keys and values of the one that has any, the state of the one that
@@ -208,4 +263,5 @@ class SideBySideMixer:
 
 register_part("shifted_decay", ShiftedDecayMixer)
 register_part("decayed_linear", DecayedLinearMixer)
+register_part("forget_gate_linear", ForgetGateLinearMixer)
 register_part("side_by_side", SideBySideMixer)

@@ -3,6 +3,7 @@ it (src/models/qwen3/model.py:75-86): 32-bit inverse frequencies 1 / theta^(2i/D
 32-bit outer product with the positions, then cos and sin, row = [cos | sin]."""
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional
 
 import torch
@@ -62,10 +63,22 @@ class RotaryPairs:
         return self._inv_freq
 
 
+def banded_frequencies(f: torch.Tensor, factor: float, low: float, high: float, original: float) -> torch.Tensor:
+    """Frequencies f (64-bit) for longer contexts: with r = original / wavelength, f where r > high, f / factor where
+    r < low, and between the two (1 - s) f / factor + s f with s = (r - low) / (high - low)."""
+    turns = original * f / (2.0 * math.pi)
+    if high > low:
+        s = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+    else:                                     # (no band between: either side of the one edge)
+        s = (turns > high).to(f.dtype)
+    return (1.0 - s) * f / factor + s * f
+
+
 class RotaryHalfAngles:
     """Half-split rotation of a head's first ``rotary_dim`` numbers (number i pairs with i + rotary_dim / 2) by
     position * theta^(-2i / rotary_dim).  The kernels that rotate form the angle, its sine and cosine in 32-bit from
-    ``inv_freq()``; the frequencies are computed in 64-bit, divided by the spec's scaling factor and rounded once.
+    ``inv_freq()``; the frequencies are computed in 64-bit, divided by the spec's scaling factor, scaled by bands of
+    wavelengths if the spec asks for it (``banded_frequencies``), and rounded once.
     No table: no limit of positions."""
 
     def __init__(self, spec, hidden_size: int = 0):
@@ -76,6 +89,7 @@ class RotaryHalfAngles:
         self.scaling_factor = float(getattr(spec, "scaling_factor", 1.0))
         if not self.scaling_factor > 0:
             raise ValueError(f"a scaling factor of {self.scaling_factor}")
+        self.band_scaling = getattr(spec, "band_scaling", None)
         self._inv_freq: Optional[torch.Tensor] = None
 
     @staticmethod
@@ -86,6 +100,8 @@ class RotaryHalfAngles:
         d = self.rotary_dim
         i = torch.arange(0, d, 2, dtype=torch.float64)
         f = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -i / d) / self.scaling_factor
+        if self.band_scaling is not None:
+            f = banded_frequencies(f, *(float(v) for v in self.band_scaling))
         self._inv_freq = f.to(torch.float32).to(rt.device)
 
     def inv_freq(self) -> torch.Tensor:
