@@ -35,9 +35,11 @@ Other sizes and workloads (not what the default line reports):
                             recorded graph of repetitions over weights that do not fit the caches, and its rate
                             against the nominal and the measured peaks (the counterpart of the reference's
                             per-operator benchmarks, src/layers/ops/linear.py:204-249)
-  --design zarorax|nufavik|potatar|safurax
+  --design zarorax|nufavik|potatar|safurax|busadra
                             another design beside the closest Qwen3 model of equal sizes (safurax: beside the Zarorax
-                            model of equal sizes, the engine's other design of latent attention and routed experts) (width, layers, heads, and a
+                            model of equal sizes, the engine's other design of latent attention and routed experts;
+                            busadra: beside the Potatar and the Nufavik model of equal sizes, the engine's other designs
+                            of recurrences and of windowed attention with routed experts) (width, layers, heads, and a
                             feed-forward as wide as the experts a token uses, or of as many weights): prefill (one prompt of --prefill-tokens
                             in one step) and decode (batch 1 and --batch at --context) of both, at the sizes of
                             --design-sizes (small, medium); one JSON line of its own.  The default line is unchanged.
@@ -96,7 +98,7 @@ def parse():
                     help="run steps of single new tokens beside a prompt portion as they come, not from a recorded graph")
     ap.add_argument("--requests", type=int, default=None, help="requests of the serving workloads")
     ap.add_argument("--kernels", action="store_true", help="time each kernel of a layer alone over a range of rows")
-    ap.add_argument("--design", default=None, choices=["zarorax", "nufavik", "potatar", "safurax"],
+    ap.add_argument("--design", default=None, choices=["zarorax", "nufavik", "potatar", "safurax", "busadra"],
                     help="measure this design beside the closest Qwen3 model of equal sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="small,medium", help="which of the design's sizes (small, medium), with commas")
     ap.add_argument("--warmup-passes", type=int, default=2,
@@ -453,6 +455,42 @@ def safurax_config(z, layers, vocab):
             "layers": ls}
 
 
+# Layer sizes for --design busadra: heads and sizes of the recurrence, query and key/value heads, key and value size,
+# window, rotated numbers, taps, experts, chosen, expert ff
+BUSADRA_SIZES = {
+    "small": dict(width=1024, rec_heads=16, rec_dim=64, heads=16, kv_heads=4, dim=64, vdim=64, window=1024, rot_dims=32,
+                  taps=4, experts=32, top=4, expert_ff=768),
+    "medium": dict(width=2048, rec_heads=16, rec_dim=128, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, rot_dims=64,
+                   taps=4, experts=32, top=4, expert_ff=1024),
+}
+
+
+def busadra_config(z, layers, vocab):
+    """Recurrence, attention, recurrence, recurrence, in turn, each with a mixture."""
+    moe = {"kind": "moe", "expert": {"ff": z["expert_ff"]}, "router": {"experts": z["experts"], "top": z["top"]}}
+    rec = {"type": "hgrn2", "mlp": moe, "mixer": {"heads": z["rec_heads"], "dim": z["rec_dim"], "vdim": z["rec_dim"]}}
+    att = {"type": "attention", "mlp": moe,
+           "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"], "softcap": 30.0,
+                     "scale": z["dim"] ** -0.5, "mask": {"size": z["window"]},
+                     "rot": {"base": 10000.0, "dims": z["rot_dims"],
+                             "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    order = [rec, att, rec, rec]
+    return {"architecture": "Busadra", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-5}, "logit_scale": 0.5,
+            "canon": {"taps": z["taps"]}, "layers": [order[i % 4] for i in range(layers)]}
+
+
+def busadra_neighbours(z, layers, vocab):
+    """The Potatar model of the same width, head and recurrence sizes with a dense feed-forward of as many weights as a
+    token's experts have, and the Nufavik model of the same attention and experts."""
+    pz = dict(POTATAR_SIZES["small"], width=z["width"], heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["vdim"],
+              rot_dims=z["rot_dims"], chunk=z["window"], rec_heads=z["rec_heads"], rec_dim=z["rec_dim"],
+              ff=z["top"] * z["expert_ff"] * 3 // 2)
+    nz = dict(NUFAVIK_SIZES["small"], width=z["width"], heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["vdim"],
+              conv=z["taps"], window=z["window"], rot_dims=z["rot_dims"], experts=z["experts"], identity=0, top=z["top"],
+              expert_ff=z["expert_ff"])
+    return {"potatar": potatar_config(pz, layers, vocab), "nufavik": nufavik_config(nz, layers, vocab)}
+
+
 def design_compare(args) -> int:
     """Prefill and decode of another design beside the Qwen3 model of equal sizes, through the same step
     function.  A "step" is one decode step; the line's value is the design's decode rate at --batch, first size."""
@@ -520,12 +558,19 @@ def design_compare(args) -> int:
     out = {}
     design = args.design
     title = design.capitalize()
-    other, other_title = ("zarorax", "Zarorax") if design == "safurax" else ("qwen3", "Qwen3")
+    other, other_title = {"safurax": ("zarorax", "Zarorax"), "busadra": ("potatar", "Potatar and Nufavik")}.get(design, ("qwen3", "Qwen3"))
     for name in [n for n in args.design_sizes.split(",") if n]:
         if design == "safurax":
             z = SAFURAX_SIZES[name]
             out[name] = {"sizes": dict(z, layers=layers, vocab=V), design: measure(config_from_dict(safurax_config(z, layers, V))),
                          other: measure(config_from_dict(zarorax_config(z, layers, V)))}
+            print(f"[bench] {name}: {out[name]}", file=sys.stderr, flush=True)
+            continue
+        if design == "busadra":
+            z = BUSADRA_SIZES[name]
+            out[name] = {"sizes": dict(z, layers=layers, vocab=V), design: measure(config_from_dict(busadra_config(z, layers, V)))}
+            for other_design, c in busadra_neighbours(z, layers, V).items():
+                out[name][other_design] = measure(config_from_dict(c))
             print(f"[bench] {name}: {out[name]}", file=sys.stderr, flush=True)
             continue
         if design == "potatar":

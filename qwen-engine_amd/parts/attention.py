@@ -41,6 +41,7 @@ def prefill_tiles(portions, rows_per_tile: int) -> List[int]:
 
 class PagedAttention:
     takes_stream = True       # forward may get a StreamInput: residual sum and norm are then the q|k|v product's prologue
+    b_o: Optional[torch.Tensor] = None     # the output projection's bias, for the kinds that have one
 
     # ---- what the step function prepares for this part (parts.base) --------------------------
     @staticmethod
@@ -143,7 +144,7 @@ class PagedAttention:
         self.window = int(spec.window) if spec.window else 0
         self.qk_eps = spec.qk_norm_eps
         self.position = build_part(spec.position, hidden_size) if spec.position is not None else None
-        self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.q_norm = self.k_norm = None
+        self.w_qkv = self.b_qkv = self.w_o = self.q_norm = self.k_norm = None
 
     @property
     def graph_safe(self) -> bool:
