@@ -22,8 +22,8 @@ import copy
 from typing import Any, Dict, List, Optional
 
 from .qwen3 import ConfigError
-from .spec import (BareLayerNormSpec, ConvAttentionSpec, DepthAverageSpec, ForgetGateLinearSpec, LogitScaleSpec, ModelSpec,
-                   RopeHalfAnglesSpec, ScaledLayerSpec, ScheduleEntry, ShortConvSpec, SigmoidMoESpec)
+from .spec import (BareLayerNormSpec, ConvAttentionSpec, DepthAverageSpec, ForgetGateLinearSpec, ModelSpec, RopeHalfAnglesSpec,
+                   ScaledLayerSpec, ScheduleEntry, ShortConvSpec, SigmoidMoESpec)
 
 ARCHITECTURE = "Busadra"
 MIXER_TYPES = ("hgrn2", "attention")
@@ -143,9 +143,8 @@ class BusadraConfig:
             for i, layer in enumerate(self.layers))
         spec = ModelSpec(
             architecture=self.architecture, vocab_size=self.vocab, hidden_size=self.width, layers=layers,
-            schedule=tuple(ScheduleEntry(layer=i) for i in range(len(layers))), final_norm=norm,
+            schedule=tuple(ScheduleEntry(layer=i) for i in range(len(layers))), final_norm=BareLayerNormSpec(eps=self.eps, gain=self.logit_scale),
             embed_name="embed", final_norm_name="final.norm", head_name="head", tie_head=False,
-            max_positions=self.max_positions,
-            logit_epilogue=LogitScaleSpec(scale=self.logit_scale) if self.logit_scale != 1.0 else None)
+            max_positions=self.max_positions)
         spec.validate()
         return spec

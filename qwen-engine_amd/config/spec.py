@@ -363,19 +363,13 @@ class LogitSoftcapSpec:
 
 
 @dataclass(frozen=True)
-class LogitScaleSpec:
-    """logits <- scale * logits; no tensors."""
-    scale: float
-    prefix: str = ""
-    kind: str = "logit_scale"
-
-
-@dataclass(frozen=True)
 class BareLayerNormSpec:
     """y = (x - mean(x)) * rsqrt(mean((x - mean(x))^2) + eps) * w over the last dimension, no bias; the weight tensor
-    carries the part's own name."""
+    carries the part's own name.  ``gain``: one more factor on the result, multiplied into the weight in 32-bit (a model
+    whose logits have a factor puts it on its last norm: the logits are linear in the normed row)."""
     eps: float
     kind: str = "layernorm_bare"
+    gain: float = 1.0
 
 
 @dataclass(frozen=True)

@@ -40,13 +40,15 @@ struct StreamNorm {
 };
 
 // One block per row, the row in registers: NV pieces of four a thread.  FEW: few rows, whose time is the latency of
-// their loads: eight parts (or kept results) are asked for at a time from addresses that are always valid, before the
-// first is added; many rows are bound by the memory's rate and take two at a time.
+// their loads: everything a row needs (the first SB parts, the first SB kept results, the weights, the convolution's taps
+// and the state's rows, up to four taps) is asked for before anything is waited for, from addresses that are always valid
+// (a part beyond the last reads another again and is not used); further parts and results come SB at a time.  Many rows
+// are bound by the memory's rate and take two at a time.
 template <typename TA, typename TD, int NV, bool FEW>
-__global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
-    constexpr int SB = !FEW ? 2 : (NV <= 4 ? 8 : 4);
-    constexpr int ST = 3;                                  // state rows asked for ahead
-    __shared__ float red[16];
+__global__ __launch_bounds__(FEW ? 512 : 256) void stream_norm_kernel(StreamNorm a) {
+    constexpr int SB = !FEW ? 2 : (NV <= 1 ? 8 : (NV <= 2 ? 4 : 2));
+    constexpr int ST = 3;                                  // state rows and taps asked for ahead: up to ST, ST + 1
+    __shared__ float red[2][16];
     const long r = blockIdx.x;
     const long src = a.rows ? (long)a.rows[r] : r;
     const int H = a.H;
@@ -59,50 +61,81 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
         ok[i] = c < H;
         cs[i] = ok[i] ? c : 0;
     }
-    float v[NV][4];
+    const int n1 = a.taps - 1;
+    const bool ahead = FEW && a.conv_w && n1 <= ST;        // (the same for the whole grid, as all conditions on a's fields)
+    float* st = a.conv_w ? a.state + (long)a.tok_seq[src] * n1 * H : nullptr;
+    const TD* parts = (const TD*)a.delta + src * H;
+    float* kr = a.kept + src * H;
+    const bool averages = a.coef != nullptr && a.k > 0;
+
+    float v[NV][4], d0[SB][NV][4], k0[SB][NV][4], c0[SB], sc[NV][4], wv[NV][4];
+    float sv[FEW ? ST : 1][NV][4], uv[FEW ? ST + 1 : 1][NV][4];
+    auto load_parts = [&](int s0, float (&d)[SB][NV][4]) {
+#pragma unroll
+        for (int s = 0; s < SB; ++s) {
+            const TD* part = parts + (long)min(s0 + s, a.n_delta - 1) * a.delta_stride;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) Vec4<TD>::load(part + cs[i], d[s][i]);
+        }
+    };
+    auto load_kept = [&](int s0, float (&d)[SB][NV][4], float (&c)[SB]) {
+#pragma unroll
+        for (int s = 0; s < SB; ++s) {
+            const int at = min(s0 + s, a.k - 1);
+            c[s] = a.coef[at];
+#pragma unroll
+            for (int i = 0; i < NV; ++i) Vec4<float>::load(kr + (long)at * a.kept_stride + cs[i], d[s][i]);
+        }
+    };
 #pragma unroll
     for (int i = 0; i < NV; ++i) Vec4<float>::load(xr + cs[i], v[i]);
-    const int n1 = a.taps - 1;
-    float* st = a.conv_w ? a.state + (long)a.tok_seq[src] * n1 * H : nullptr;
-    float sv[FEW ? ST : 1][NV][4];
-    if (FEW && st) {
+    if (a.delta) load_parts(0, d0);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        sc[i][0] = sc[i][1] = sc[i][2] = sc[i][3] = 1.f;
+        if (a.scale) Vec4<float>::load(a.scale + cs[i], sc[i]);
+    }
+    float ck = 1.f;
+    if (a.coef) ck = a.coef[a.k];
+    if (FEW && averages) load_kept(0, k0, c0);
+    if (a.out) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) Vec4<float>::load(a.w + cs[i], wv[i]);
+    }
+    if (ahead) {
+#pragma unroll
+        for (int j = 0; j <= ST; ++j)
+            if (j <= n1) {
+#pragma unroll
+                for (int i = 0; i < NV; ++i) Vec4<float>::load(a.conv_w + (long)j * H + cs[i], uv[FEW ? j : 0][i]);
+            }
 #pragma unroll
         for (int j = 0; j < ST; ++j)
             if (j < n1) {
 #pragma unroll
-                for (int i = 0; i < NV; ++i) Vec4<float>::load(st + (long)j * H + cs[i], sv[j][i]);
+                for (int i = 0; i < NV; ++i) Vec4<float>::load(st + (long)j * H + cs[i], sv[FEW ? j : 0][i]);
             }
     }
     if (a.delta) {
         float sum[NV][4] = {};
         for (int s0 = 0; s0 < a.n_delta; s0 += SB) {
-            float d[SB][NV][4];
-#pragma unroll
-            for (int s = 0; s < SB; ++s) {
-                const TD* part = (const TD*)a.delta + src * H + (long)min(s0 + s, a.n_delta - 1) * a.delta_stride;
-#pragma unroll
-                for (int i = 0; i < NV; ++i) Vec4<TD>::load(part + cs[i], d[s][i]);
-            }
+            if (s0 > 0) load_parts(s0, d0);
 #pragma unroll
             for (int s = 0; s < SB; ++s)
                 if (s0 + s < a.n_delta) {
 #pragma unroll
                     for (int i = 0; i < NV; ++i)
 #pragma unroll
-                        for (int e = 0; e < 4; ++e) sum[i][e] += d[s][i][e];
+                        for (int e = 0; e < 4; ++e) sum[i][e] += d0[s][i][e];
                 }
         }
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            float sc[4] = {1.f, 1.f, 1.f, 1.f};
-            if (a.scale) Vec4<float>::load(a.scale + cs[i], sc);
+        for (int i = 0; i < NV; ++i)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[i][e] = fmaf(sc[e], sum[i][e], v[i][e]);
-        }
+            for (int e = 0; e < 4; ++e) v[i][e] = fmaf(sc[i][e], sum[i][e], v[i][e]);
     }
     const bool write = !a.rows;
     if (a.kept) {
-        float* kr = a.kept + src * H;
         if (write) {
 #pragma unroll
             for (int i = 0; i < NV; ++i)
@@ -111,24 +144,16 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
         if (a.coef) {
             float acc[NV][4] = {};
             for (int s0 = 0; s0 < a.k; s0 += SB) {
-                float d[SB][NV][4], c[SB];
-#pragma unroll
-                for (int s = 0; s < SB; ++s) {
-                    const int at = min(s0 + s, a.k - 1);
-                    c[s] = a.coef[at];
-#pragma unroll
-                    for (int i = 0; i < NV; ++i) Vec4<float>::load(kr + (long)at * a.kept_stride + cs[i], d[s][i]);
-                }
+                if (!FEW || s0 > 0) load_kept(s0, k0, c0);
 #pragma unroll
                 for (int s = 0; s < SB; ++s)
                     if (s0 + s < a.k) {
 #pragma unroll
                         for (int i = 0; i < NV; ++i)
 #pragma unroll
-                            for (int e = 0; e < 4; ++e) acc[i][e] = fmaf(c[s], d[s][i][e], acc[i][e]);
+                            for (int e = 0; e < 4; ++e) acc[i][e] = fmaf(c0[s], k0[s][i][e], acc[i][e]);
                     }
             }
-            const float ck = a.coef[a.k];
 #pragma unroll
             for (int i = 0; i < NV; ++i)
 #pragma unroll
@@ -141,11 +166,6 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
             if (ok[i]) Vec4<float>::store(xr + cs[i], v[i]);
     }
     if (!a.out && !a.stats) return;                        // (the sums alone; the same for the whole grid)
-    float wv[NV][4];
-    if (a.out) {
-#pragma unroll
-        for (int i = 0; i < NV; ++i) Vec4<float>::load(a.w + cs[i], wv[i]);
-    }
     float mean = 0.f;
     if (a.center) {
         float sm = 0.f;
@@ -155,7 +175,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
 #pragma unroll
                 for (int e = 0; e < 4; ++e) sm += v[i][e];
             }
-        mean = block_sum(sm, red) / (float)H;
+        mean = block_sum(sm, red[0]) / (float)H;
     }
     float ss = 0.f;
 #pragma unroll
@@ -164,7 +184,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) ss += (v[i][e] - mean) * (v[i][e] - mean);
         }
-    ss = block_sum(ss, red);
+    ss = block_sum(ss, red[1]);
     const float rstd = rsqrtf(ss / (float)H + a.eps);
     if (a.stats && threadIdx.x == 0) {
         a.stats[2 * r] = mean;
@@ -178,20 +198,25 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(StreamNorm a) {
         float h[4], o[4];
 #pragma unroll
         for (int e = 0; e < 4; ++e) o[e] = h[e] = (v[i][e] - mean) * rstd * wv[i][e];
-        if (a.conv_w) {
-            float u[4];
-            for (int j = 0; j < n1; ++j) {                 // oldest input first
-                float p[4];
-                if (FEW && j < ST) {
+        if (ahead) {                                       // oldest input first
 #pragma unroll
-                    for (int q = 0; q < ST; ++q)
-                        if (q == j) {
+            for (int j = 0; j < ST; ++j)
+                if (j < n1) {
 #pragma unroll
-                            for (int e = 0; e < 4; ++e) p[e] = sv[FEW ? q : 0][i][e];
-                        }
-                } else {
-                    Vec4<float>::load(st + (long)j * H + c, p);
+                    for (int e = 0; e < 4; ++e) o[e] = fmaf(uv[FEW ? j : 0][i][e], sv[FEW ? j : 0][i][e], o[e]);
+                    if (j > 0) Vec4<float>::store(st + (long)(j - 1) * H + c, sv[FEW ? j : 0][i]);
                 }
+#pragma unroll
+            for (int j = 0; j <= ST; ++j)
+                if (j == n1) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) o[e] = fmaf(uv[FEW ? j : 0][i][e], h[e], o[e]);
+                }
+            if (n1 > 0) Vec4<float>::store(st + (long)(n1 - 1) * H + c, h);
+        } else if (a.conv_w) {
+            float u[4], p[4];
+            for (int j = 0; j < n1; ++j) {
+                Vec4<float>::load(st + (long)j * H + c, p);
                 Vec4<float>::load(a.conv_w + (long)j * H + c, u);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) o[e] = fmaf(u[e], p[e], o[e]);
@@ -270,7 +295,8 @@ template <typename TA, typename TD>
 static void launch_stream_norm(const StreamNorm& a, int n_rows, hipStream_t stream) {
     if (a.H % 4 == 0 && a.H <= 8192) {
         int threads = ((a.H / 4 + 63) / 64) * 64;
-        if (threads > 256) threads = 256;
+        const int most = n_rows <= 512 ? 512 : 256;
+        if (threads > most) threads = most;
         const int nv = (a.H / 4 + threads - 1) / threads;
 #define QE_SN(NV_)                                                                                  \
     do {                                                                                            \
@@ -280,7 +306,7 @@ static void launch_stream_norm(const StreamNorm& a, int n_rows, hipStream_t stre
         if (nv <= 1) QE_SN(1);
         else if (nv <= 2) QE_SN(2);
         else if (nv <= 4) QE_SN(4);
-        else QE_SN(8);
+        else stream_norm_kernel<TA, TD, 8, false><<<n_rows, threads, 0, stream>>>(a);   // (few rows have at most four pieces a thread)
 #undef QE_SN
         return;
     }
@@ -418,10 +444,13 @@ __global__ __launch_bounds__(256) void norm_conv_state_kernel(const float* __res
                                                               const int* __restrict__ tok_seq, int T, int H, int taps) {
     const int c = blockIdx.x * blockDim.x + threadIdx.x;
     const int n1 = taps - 1;
-    const int t_end = min(T, (int)(blockIdx.y + 1) * NC_STATE_ROWS);
-    for (int t = blockIdx.y * NC_STATE_ROWS; t < t_end; ++t) {
+    // every lane looks at one row: few are among their request's last taps - 1 (a request's rows are consecutive)
+    const int mine = blockIdx.y * NC_STATE_ROWS + (threadIdx.x & (NC_STATE_ROWS - 1));
+    const bool last = mine < T && !(mine + n1 < T && tok_seq[mine + n1] == tok_seq[mine]);
+    unsigned long todo = __ballot(last) & ((1UL << NC_STATE_ROWS) - 1);
+    for (; todo; todo &= todo - 1) {
+        const int t = blockIdx.y * NC_STATE_ROWS + __builtin_ctzl(todo);
         const int s = tok_seq[t];
-        if (t + n1 < T && tok_seq[t + n1] == s) continue;  // (a request's rows are consecutive)
         int before = 0, after = 0;
         while (before < n1 && t - 1 - before >= 0 && tok_seq[t - 1 - before] == s) ++before;
         while (after < n1 && t + 1 + after < T && tok_seq[t + 1 + after] == s) ++after;

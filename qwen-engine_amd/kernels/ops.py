@@ -97,8 +97,11 @@ def load_library():
         "qe_attention_talk_splits": [i32, i32],
         "qe_token_shift": [vp, vp, i32, vp, i64, vp, vp, i32, i32, i32, i32, vp],
         "qe_recurrence_chunk_len": [i32],
-        "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, vp, vp,
+        "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, i32, vp, vp,
                                          i32, i32, i32, i32, vp],
+        "qe_recurrence_single_supported": [i32, i32],
+        "qe_recurrence_single": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, f32, vp, i32, i32, i32,
+                                 i32, i32, i32, vp],
         "qe_linear_recurrence": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, i32, i32, i32,
                                  i32, vp],
         "qe_gated_norm": [vp, vp, vp, i64, i32, i32, f32, f32, vp, i64, i32, i32, i32, i32, vp],
@@ -1546,22 +1549,24 @@ def recurrence_chunk_len(head_dim: int) -> int:
 
 
 def recurrence_chunks(portions, chunk_len: int):
-    """For portions given as (first row, rows) on the host: the ``chunks`` of linear_recurrence(), a pair of int32
-    tensors (on the host) [n, 2] = (first row, rows <= chunk_len) and [m, 3] = (first chunk, chunks, first row)."""
+    """For portions given as (first row, rows) on the host: the ``chunks`` of linear_recurrence(), two int32 tensors (on
+    the host), [n, 3] = (first row, rows <= chunk_len, 1 if the portion is this chunk alone) and [m, 3] = (first chunk,
+    chunks, first row)."""
     chunks, ports = [], []
     for start, n in portions:
         if n <= 0:
             continue
         ports.append((len(chunks), -(-n // chunk_len), start))
-        chunks += [(start + r, min(chunk_len, n - r)) for r in range(0, n, chunk_len)]
-    return (torch.tensor(chunks, dtype=torch.int32).view(-1, 2), torch.tensor(ports, dtype=torch.int32).view(-1, 3))
+        chunks += [(start + r, min(chunk_len, n - r), int(n <= chunk_len)) for r in range(0, n, chunk_len)]
+    return (torch.tensor(chunks, dtype=torch.int32).view(-1, 3), torch.tensor(ports, dtype=torch.int32).view(-1, 3))
 
 
 def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, tok_seq: torch.Tensor,
                       heads: int, decay: Optional[torch.Tensor] = None, decay_x: Optional[torch.Tensor] = None,
                       decay_bias: Optional[torch.Tensor] = None, bonus: Optional[torch.Tensor] = None,
                       silu: bool = False, chunks=None, forget_bias: Optional[torch.Tensor] = None,
-                      lower: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      lower: Optional[torch.Tensor] = None, norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0,
+                      norm_dtype: Optional[torch.dtype] = None, single_rows: bool = False) -> torch.Tensor:
     """Per head, with a 32-bit state S [D][Dv] per request (state[tok_seq[t]], float32 [slots, >= H D Dv]):
     with ``decay`` (float32 [H]):  S <- decay_h S + k_t v_t^T, o_t = S^T q_t;
     with ``decay_x`` float32 [T, H D], ``decay_bias`` and ``bonus`` (float32 [H D]):  o_t = (S + diag(bonus) k_t v_t^T)^T q_t,
@@ -1571,7 +1576,10 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     q, k [T, H D], v [T, H Dv] (column slices of one wider tensor are taken as they are, all with one row stride);
     ``silu``: the three (with a forget gate: q) pass silu first.  Returns o float32 [T, H, Dv].
     ``chunks`` (recurrence_chunks() of all rows' portions, on the device, for recurrence_chunk_len(D)): the rows are
-    taken chunk by chunk, the chunks in parallel, instead of row by row: for long portions."""
+    taken chunk by chunk, the chunks in parallel, instead of row by row: for long portions.
+    ``norm_weight`` (float32 [H Dv]): every head's o is divided by its root mean square (norm_eps inside) and multiplied
+    by the weight; the result is [T, H Dv] in norm_dtype.  ``single_rows``: no two rows belong to one request (the norm
+    is then part of the one launch)."""
     lib = load_library()
     T, dev, H = q.shape[0], q.device, int(heads)
     if q.dtype not in _ACT or k.dtype != q.dtype or v.dtype != q.dtype:
@@ -1598,16 +1606,32 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         sw = _rows_view(decay_x, "decay_x", H * D, T)
         _need(decay_bias, "decay_bias", torch.float32, (H * D,), dev)
         _need(bonus, "bonus", torch.float32, (H * D,), dev)
+    if norm_weight is not None:
+        _need(norm_weight, "norm_weight", torch.float32, (H * Dv,), dev)
+        norm_dtype = norm_dtype or q.dtype
+        if single_rows and lib.qe_recurrence_single_supported(D, Dv):
+            y = torch.empty((T, H * Dv), dtype=norm_dtype, device=dev)
+            _check(lib.qe_recurrence_single(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw, _ptr(decay_bias),
+                                            _ptr(bonus), _ptr(decay), mode, int(bool(silu)), state.data_ptr(),
+                                            state.stride(0), tok_seq.data_ptr(), norm_weight.data_ptr(), float(norm_eps),
+                                            y.data_ptr(), T, H, D, Dv, _DT[q.dtype], _DT[norm_dtype], _stream()),
+                   "recurrence_single")
+            return y
+        o = linear_recurrence(q, k, v, state, tok_seq, heads, decay=decay, decay_x=decay_x,
+                              decay_bias=decay_bias if mode == 1 else None, bonus=bonus if mode == 1 else None, silu=silu,
+                              chunks=chunks, forget_bias=forget_bias, lower=lower)
+        return gated_norm(o.view(T, H * Dv), norm_weight, norm_eps, H, norm_dtype)
     out = torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
     if chunks is not None and chunks[0].shape[0]:
         ch, po = chunks
-        _need(ch, "chunks", torch.int32, (None, 2), dev)
+        _need(ch, "chunks", torch.int32, (None, 3), dev)
         _need(po, "portions", torch.int32, (None, 3), dev)
-        ws = torch.empty((ch.shape[0] * H * (D * Dv + D),), dtype=torch.float32, device=dev)
+        all_single = ch.shape[0] == po.shape[0]
+        ws = None if all_single else torch.empty((ch.shape[0] * H * (D * Dv + D),), dtype=torch.float32, device=dev)
         _check(lib.qe_linear_recurrence_chunked(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw,
                                                 _ptr(decay_bias), _ptr(bonus), _ptr(decay), mode, int(bool(silu)),
                                                 state.data_ptr(), state.stride(0), tok_seq.data_ptr(), ch.data_ptr(),
-                                                ch.shape[0], po.data_ptr(), po.shape[0], ws.data_ptr(), out.data_ptr(),
+                                                ch.shape[0], po.data_ptr(), po.shape[0], int(all_single), _ptr(ws), out.data_ptr(),
                                                 H, D, Dv, _DT[q.dtype], _stream()), "linear_recurrence (chunked)")
         return out
     _check(lib.qe_linear_recurrence(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw, _ptr(decay_bias),

@@ -95,6 +95,7 @@ class BareLayerNorm:
 
     def __init__(self, spec, size: int):
         self.eps = float(spec.eps)
+        self.gain = float(spec.gain)
         self.size = int(size)
         self.weight: Optional[torch.Tensor] = None
 
@@ -103,7 +104,7 @@ class BareLayerNorm:
         return {"": TensorInfo((size,), "ones", "vector")}
 
     def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
-        self.weight = rt.place_vector(tensors[""])
+        self.weight = rt.place_vector(tensors[""].to(torch.float32) * self.gain)
 
     def forward(self, h: torch.Tensor, rt: Runtime, delta: Optional[torch.Tensor] = None,
                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -146,26 +147,7 @@ class LogitSoftcap:
         return ops.unary(logits, ops.UNARY_SOFTCAP, cap=self.cap, inplace=True)
 
 
-class LogitScale:
-    """logits <- scale * logits, in place on the 32-bit logits."""
-
-    def __init__(self, spec, hidden_size: int = 0):
-        self.scale = float(spec.scale)
-
-    @staticmethod
-    def expected_tensors(spec, hidden_size: int) -> Dict[str, TensorInfo]:
-        return {}
-
-    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
-        pass
-
-    def forward(self, logits: torch.Tensor, ctx) -> torch.Tensor:
-        ops.scale_(logits, self.scale)
-        return logits
-
-
 register_part("rmsnorm", RMSNorm)
-register_part("logit_scale", LogitScale)
 register_part("logit_softcap", LogitSoftcap)
 register_part("rmsnorm_bare", BareRMSNorm)
 register_part("layernorm_bare", BareLayerNorm)

@@ -20,7 +20,7 @@ def _single_rows(ctx, T: int) -> bool:
 
 # From this many rows of one request in a step, the recurrences take the step's rows chunk by chunk (the chunks in
 # parallel) instead of row by row.
-CHUNKED_FROM_ROWS = 64
+CHUNKED_FROM_ROWS = 8
 
 
 def _chunks(ctx, head_dim: int):
@@ -148,8 +148,8 @@ class DecayedLinearMixer:
 
 class ForgetGateLinearMixer:
     """``ForgetGateLinearSpec`` (HGRN2): one product for q | f | v that stays 32-bit (the gate enters the recurrence), the
-    recurrence (silu on q, the gate and what it leaves to be written formed as they are read), a norm per head, the
-    output projection."""
+    recurrence (silu on q, the gate and what it leaves to be written formed as they are read) with the norm per head
+    behind it (one launch for single new tokens), the output projection."""
     graph_safe = True
 
     def __init__(self, spec, hidden_size: int):
@@ -190,11 +190,12 @@ class ForgetGateLinearMixer:
         if binding.state is None:
             raise RuntimeError("the recurrence was given no state")
         T = x.shape[0]
-        nk, nv = self.h * self.d, self.h * self.dv
+        nk = self.h * self.d
         y = ops.gemm(x, self.w_in, out_dtype=torch.float32)
-        o = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:], binding.state, ctx.tok_seq, self.h, silu=True,
-                                  forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.d))
-        z = ops.gated_norm(o.view(T, nv), self.norm, self.eps, self.h, ctx.rt.dtype)
+        z = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:], binding.state, ctx.tok_seq, self.h, silu=True,
+                                  forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.d),
+                                  norm_weight=self.norm, norm_eps=self.eps, norm_dtype=ctx.rt.dtype,
+                                  single_rows=_single_rows(ctx, T))
         splits = ops.gemm_branch_splits(z, self.w_o)
         if splits:
             return ops.gemm(z, self.w_o, epilogue=ops.EPI_PARTIAL, splits=splits)
