@@ -19,11 +19,16 @@
 //   mode 1 (a decay per channel, a bonus for the token itself): row t sees the state before it: F_t and A's products stop
 //   before row t, and A[t][t] = sum_d q_t[d] u[d] k_t[d]
 //
+// Preparing 16 rows is vector arithmetic, using them is matrix arithmetic: between two barriers every wave prepares the
+// next 16 rows and uses the last, half of the waves in the one order and half in the other, so that the two waves that
+// share a SIMD keep both of its units busy.
 // Wave w prepares 16 key channels (a lane holds row r = lane % 16 of channels 4 g + j, g = lane / 16: the operand layout of
 // the matrix instruction, in which a level's matrix is both operands; products along the rows run over the 16 lanes by
 // register moves), leaves q F, k B, G and its share of A in shared memory (two buffers in turn, one barrier per 16 rows),
-// then takes 16 value columns: the state of those columns stays in its registers, as accumulators of the state's update
+// and takes 16 value columns of the rows prepared before: the state of those columns stays in its registers, as accumulators of the state's update
 // and, as they lie, as the operand of the output's product.
+// With a norm behind it (a head's columns in one block), the waves leave the squares' sums of 16 rows in shared memory
+// before the barrier and write the rows, normed, after it.
 // chunks: int32 [n][3] = (first row, rows, 1 if the portion is this chunk alone); portions: int32 [m][3] = (first chunk,
 // chunks, first row); a portion's state row is tok_seq of its first row, read on the device (a recorded step serves
 // another request at every replay).  The order of all sums depends on a row's place in its portion alone.
@@ -49,8 +54,12 @@ struct RecArgs {
     float* state;
     long state_stride;
     const int* tok_seq;
-    float* out;                     // [T][H][Dv]
+    float* out;                     // [T][H][Dv]; null with a norm
     int H, D, Dv;
+    const float* norm_w;            // [H * Dv] or null
+    float norm_eps;
+    void* y;                        // [T][H * Dv] normed rows
+    int y_bf16;
 };
 
 // the value of the lane's partner in the other half of an aligned group of 2 H lanes of its 16 (for H = 4, 8 of some lane
@@ -78,6 +87,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
     __shared__ __align__(16) float kt[2][16][LD];
     __shared__ __align__(16) float gt[2][DP];
     __shared__ __align__(16) float at[PHASE == 1 ? 2 : 1][8][16][20];
+    __shared__ __align__(16) float sq[PHASE == 1 ? 2 : 1][8][16];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6, g = lane >> 4, r = lane & 15;
     const int c = blockIdx.x, h = blockIdx.y;
     const int row0 = a.chunks[3 * c], n = a.chunks[3 * c + 1], single = a.chunks[3 * c + 2];
@@ -125,7 +135,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
     }
 
     RecRaw raw[NPT];
-    float vr[4];
+    float vr[4], vv[4];                                    // value rows: of the rows prepared next, of the rows used now
     auto fetch = [&](int base) {
         const int nb = n - base < 16 ? n - base : 16;
 #pragma unroll
@@ -138,13 +148,17 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
                 if (MODE == 1) load4<float>(a.wx + (long)(row0 + base + r) * a.w_stride + (long)h * D + d0, D - d0, vec, raw[p].w);
             }
         }
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-            vr[j] = (col_ok && 4 * g + j < nb) ? Elem<TA>::load(v + (long)(row0 + base + 4 * g + j) * a.row_stride + (long)h * Dv + col) : 0.f;
     };
-    fetch(0);
-#pragma unroll 1
-    for (int base = 0, buf = 0; base < n; base += 16, buf ^= 1) {
+    auto fetch_values = [&](int base) {
+        const int nb = n - base < 16 ? n - base : 16;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int row = 4 * g + j < nb ? 4 * g + j : 0;
+            const float x = Elem<TA>::load(v + (long)(row0 + base + row) * a.row_stride + (long)h * Dv + (col_ok ? col : 0));
+            vr[j] = col_ok && 4 * g + j < nb ? x : 0.f;
+        }
+    };
+    auto prepare = [&](int base, int buf) {
         const int nb = n - base < 16 ? n - base : 16;
         const int qb = PHASE == 1 ? buf : 0;
         floatx4 ga = {0.f, 0.f, 0.f, 0.f};
@@ -156,17 +170,19 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
             float qv[4], kv[4], F[4], B[4], tot[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
+                const bool in = r < nb && d0 + j < D;
                 float f = 1.f;
                 qv[j] = kv[j] = 0.f;
-                if (r < nb && d0 + j < D) {
-                    if (PHASE == 1) qv[j] = a.act_silu ? silu_f(raw[p].q[j]) : raw[p].q[j];
-                    if (MODE == 2) {
-                        forget_gate(raw[p].k[j] + bias[p][j], low[p][j], f, kv[j]);
-                    } else {
-                        kv[j] = a.act_silu ? silu_f(raw[p].k[j]) : raw[p].k[j];
-                        f = MODE == 0 ? dec : expf(-expf(raw[p].w[j] + bias[p][j]));
-                    }
+                if (PHASE == 1) qv[j] = a.act_silu ? silu_f(raw[p].q[j]) : raw[p].q[j];
+                if (MODE == 2) {
+                    forget_gate(raw[p].k[j] + bias[p][j], low[p][j], f, kv[j]);
+                } else {
+                    kv[j] = a.act_silu ? silu_f(raw[p].k[j]) : raw[p].k[j];
+                    f = MODE == 0 ? dec : expf(-expf(raw[p].w[j] + bias[p][j]));
                 }
+                qv[j] = in ? qv[j] : 0.f;                  // (what lies beyond the rows and channels changes nothing)
+                kv[j] = in ? kv[j] : 0.f;
+                f = in ? f : 1.f;
                 F[j] = MODE == 1 ? 1.f : f;
                 B[j] = 1.f;
                 tot[j] = f;
@@ -227,36 +243,92 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) at[qb][wave][4 * g + i][r] = ga[i];
         }
-        float vv[4];
+    };
+    floatx4 o_held = {0.f, 0.f, 0.f, 0.f};                 // (with a norm: the outputs of the last 16 rows)
+    auto use = [&](int base, int buf) {
+        const int nb = n - base < 16 ? n - base : 16;
+        const int qb = PHASE == 1 ? buf : 0;
+        if (PHASE == 1) {
+            floatx4 av = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
+            for (int w = 0; w < preparers; ++w) av += *(const floatx4*)&at[qb][w][r][4 * g];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) vv[j] = (a.act_silu && MODE != 2) ? silu_f(vr[j]) : vr[j];     // (silu(0) = 0)
-        if (base + 16 < n) fetch(base + 16);               // (the next rows travel while these are computed)
-        __syncthreads();
-        if (has_cols) {
-            if (PHASE == 1) {
-                floatx4 av = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
-                for (int w = 0; w < preparers; ++w) av += *(const floatx4*)&at[qb][w][r][4 * g];
+            for (int ct = 0; ct < DT; ++ct) {
+                const floatx4 x = *(const floatx4*)&qt[qb][r][ct * 16 + 4 * g];
 #pragma unroll
-                for (int ct = 0; ct < DT; ++ct) {
-                    const floatx4 x = *(const floatx4*)&qt[qb][r][ct * 16 + 4 * g];
+                for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], S[ct][j], o, 0, 0, 0);
+            }
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], S[ct][j], o, 0, 0, 0);
+            for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(av[j], vv[j], o, 0, 0, 0);
+            if (a.norm_w) {
+                o_held = o;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {              // (columns beyond the head's are zeros)
+                    const float q2 = row16_sum(o[i] * o[i]);
+                    if (r == 0) sq[qb][wave][4 * g + i] = q2;
                 }
-#pragma unroll
-                for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(av[j], vv[j], o, 0, 0, 0);
+            } else {
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
                     if (col_ok && 4 * g + i < nb) a.out[((long)(row0 + base + 4 * g + i) * H + h) * Dv + col] = o[i];
             }
+        }
 #pragma unroll
-            for (int ct = 0; ct < DT; ++ct) {
-                S[ct] *= *(const floatx4*)&gt[buf][ct * 16 + 4 * g];
+        for (int ct = 0; ct < DT; ++ct) {
+            S[ct] *= *(const floatx4*)&gt[buf][ct * 16 + 4 * g];
 #pragma unroll
-                for (int j = 0; j < 4; ++j)
-                    S[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[buf][4 * g + j][ct * 16 + r], vv[j], S[ct], 0, 0, 0);
+            for (int j = 0; j < 4; ++j)
+                S[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[buf][4 * g + j][ct * 16 + r], vv[j], S[ct], 0, 0, 0);
+        }
+    };
+    const int col_waves = (Dv + 15) / 16 < 8 ? (Dv + 15) / 16 : 8;
+    const float nw = PHASE == 1 && a.norm_w && col_ok ? a.norm_w[h * Dv + col] : 0.f;
+    auto write_normed = [&](int base, int buf) {           // rows whose squares' sums the last barrier has made whole
+        const int nb = n - base < 16 ? n - base : 16;
+        const int qb = PHASE == 1 ? buf : 0;
+        floatx4 all = {0.f, 0.f, 0.f, 0.f};
+        for (int w = 0; w < col_waves; ++w) all += *(const floatx4*)&sq[qb][w][4 * g];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float x = o_held[i] * rsqrtf(all[i] / (float)Dv + a.norm_eps) * nw;
+            if (col_ok && 4 * g + i < nb) {
+                const long to = (long)(row0 + base + 4 * g + i) * H * Dv + (long)h * Dv + col;
+                if (a.y_bf16) ((bf16_t*)a.y)[to] = float_to_bf16(x);
+                else ((float*)a.y)[to] = x;
             }
         }
+    };
+
+    // (SILU of the values: silu(0) = 0)
+    auto values = [&]() {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) vv[j] = (a.act_silu && MODE != 2) ? silu_f(vr[j]) : vr[j];
+    };
+    const bool prepares_first = (wave & 4) == 0;
+    fetch(0);
+    if (has_cols) fetch_values(0);
+    prepare(0, 0);
+    if (n > 16) fetch(16);
+    __syncthreads();
+#pragma unroll 1
+    for (int base = 0, buf = 0; base < n; base += 16, buf ^= 1) {
+        const bool more = base + 16 < n;
+        if (has_cols) {
+            values();
+            if (more) fetch_values(base + 16);
+            if (PHASE == 1 && a.norm_w && base > 0) write_normed(base - 16, buf ^ 1);
+        }
+        if (more && prepares_first) {
+            prepare(base + 16, buf ^ 1);
+            if (base + 32 < n) fetch(base + 32);
+        }
+        if (has_cols) use(base, buf);
+        if (more && !prepares_first) {
+            prepare(base + 16, buf ^ 1);
+            if (base + 32 < n) fetch(base + 32);
+        }
+        __syncthreads();
     }
+    if (PHASE == 1 && a.norm_w && has_cols) write_normed((n - 1) / 16 * 16, ((n - 1) / 16) & 1);
     if (PHASE == 0 || single) {
         float* to = PHASE == 0 ? mine : slot;
 #pragma unroll
@@ -343,12 +415,15 @@ static int launch_phases(const RecArgs& a, int n_chunks, const int* portions, in
 }
 
 // As qe_linear_recurrence (recurrence.hip), for rows cut into chunks on the host.  ws: float32, n_chunks * H *
-// (D * Dv + D) numbers (not read if all_single: every portion is one chunk).  Rows that no chunk names are left alone.
+// (D * Dv + D) numbers (not read if all_single: every portion is one chunk).  norm_w (float32 [H * Dv], or null; heads
+// of at most 128 value columns): every head's output divided by its root mean square (norm_eps inside) and multiplied by
+// the weight goes to y [T, H * Dv] in dt_y instead of out.  Rows that no chunk names are left alone.
 extern "C" int qe_linear_recurrence_chunked(const void* q, const void* k, const void* v, long row_stride, const float* wx,
                                             long w_stride, const float* w0, const float* u, const float* decay, int mode,
                                             int act_silu, float* state, long state_stride, const int* tok_seq,
                                             const int* chunks, int n_chunks, const int* portions, int n_portions, int all_single,
-                                            float* ws, float* out, int H, int D, int Dv, int dt_a, hipStream_t stream) {
+                                            float* ws, float* out, const float* norm_w, float norm_eps, void* y, int dt_y,
+                                            int H, int D, int Dv, int dt_a, hipStream_t stream) {
     QE_REQUIRE(n_chunks >= 0 && n_portions >= 0 && H > 0 && H <= 65535 && D > 0 && Dv > 0, "linear_recurrence: bad sizes");
     QE_REQUIRE(D <= 256, "linear_recurrence: heads of %d key channels (at most 256)", D);
     QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "linear_recurrence: mode %d lacks operands", mode);
@@ -356,8 +431,9 @@ extern "C" int qe_linear_recurrence_chunked(const void* q, const void* k, const 
     QE_REQUIRE(dt_a == QE_F32 || dt_a == QE_BF16, "linear_recurrence: unknown element type %d", dt_a);
     if (n_chunks == 0) return 0;
     QE_REQUIRE(chunks && portions && (all_single || ws), "linear_recurrence: chunks without a workspace");
+    QE_REQUIRE(norm_w ? (y && Dv <= 128 && (dt_y == QE_F32 || dt_y == QE_BF16)) : out != nullptr, "linear_recurrence: no place for the outputs, or heads too wide for the norm inside");
     RecArgs a{q, k, v, row_stride, wx, w_stride, w0, u, decay, act_silu, chunks, ws, ws + (long)n_chunks * H * D * Dv,
-              state, state_stride, tok_seq, out, H, D, Dv};
+              state, state_stride, tok_seq, out, H, D, Dv, norm_w, norm_eps, y, dt_y == QE_BF16};
 #define QE_RP(TA_) (mode == 0 ? launch_phases<TA_, 0>(a, n_chunks, portions, n_portions, all_single, stream)   \
                   : mode == 1 ? launch_phases<TA_, 1>(a, n_chunks, portions, n_portions, all_single, stream)   \
                               : launch_phases<TA_, 2>(a, n_chunks, portions, n_portions, all_single, stream))

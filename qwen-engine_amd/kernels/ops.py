@@ -97,7 +97,7 @@ def load_library():
         "qe_attention_talk_splits": [i32, i32],
         "qe_token_shift": [vp, vp, i32, vp, i64, vp, vp, i32, i32, i32, i32, vp],
         "qe_recurrence_chunk_len": [i32],
-        "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, i32, vp, vp,
+        "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, i32, vp, vp, vp, f32, vp, i32,
                                          i32, i32, i32, i32, vp],
         "qe_recurrence_single_supported": [i32, i32],
         "qe_recurrence_single": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, f32, vp, i32, i32, i32,
@@ -1363,7 +1363,7 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
         _check(lib.qe_moe_sort(ids.data_ptr(), n, E + identity, E, tile_rows, perm.data_ptr(), inv.data_ptr(), tiles.data_ptr(),
                                n_tiles.data_ptr(), max_tiles, _stream()), "moe_sort")
 
-    def identity(parts_, rows_):
+    def write_identity_rows(parts_, rows_):
         if identity and not fused_front:
             _check(lib.qe_moe_identity(x.data_ptr(), ids.data_ptr(), weights.data_ptr(), inv.data_ptr(), _ptr(parts_),
                                        _ptr(rows_), T, top, Hout, E, _DT[x.dtype],
@@ -1384,7 +1384,7 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
         _check(lib.qe_gemm_mfma_grouped(a.data_ptr(), w_down.data_ptr(), y.data_ptr(), tiles.data_ptr(),
                                         n_tiles.data_ptr(), max_tiles, Hout, Fd, 0, 0.0, 1.0, _DT[rows_dtype], None, None, _stream()),
                "grouped gemm (down)")
-        identity(None, y)
+        write_identity_rows(None, y)
         out = torch.empty((1, T, Hout), dtype=torch.float32, device=dev)
         _check(lib.qe_moe_combine(y.data_ptr(), inv.data_ptr(), w_out, out.data_ptr(), T, top, Hout,
                                   _DT[rows_dtype], _stream()), "moe_combine")
@@ -1398,7 +1398,7 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
         _check(lib.qe_moe_gemm_mfma(a.data_ptr(), perm.data_ptr(), top, w_down.data_ptr(), parts.data_ptr(),
                                     w_out, tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, T,
                                     Hout, Fd, 0.0, 0.0, 0, 0, _stream()), "moe_gemm (down; mfma)")
-        identity(parts, None)
+        write_identity_rows(parts, None)
         return parts
     _check(lib.qe_moe_gemm(x.data_ptr(), perm.data_ptr(), top, w_gate_up.data_ptr(), a.data_ptr(), w_in,
                            tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, T, Fd, K, float(limit), float(slope), first_mode,
@@ -1406,7 +1406,7 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
     _check(lib.qe_moe_gemm(a.data_ptr(), perm.data_ptr(), top, w_down.data_ptr(), parts.data_ptr(), w_out,
                            tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, T, Hout, Fd, 0.0, 0.0, 0, 0,
                            _DT[x.dtype], _DT[w_down.dtype], _stream()), "moe_gemm (down)")
-    identity(parts, None)
+    write_identity_rows(parts, None)
     return parts
 
 
@@ -1617,11 +1617,16 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
                                             y.data_ptr(), T, H, D, Dv, _DT[q.dtype], _DT[norm_dtype], _stream()),
                    "recurrence_single")
             return y
+    fused_norm = norm_weight is not None and chunks is not None and chunks[0].shape[0] > 0 and Dv <= 128
+    if norm_weight is not None and not fused_norm:
         o = linear_recurrence(q, k, v, state, tok_seq, heads, decay=decay, decay_x=decay_x,
                               decay_bias=decay_bias if mode == 1 else None, bonus=bonus if mode == 1 else None, silu=silu,
                               chunks=chunks, forget_bias=forget_bias, lower=lower)
         return gated_norm(o.view(T, H * Dv), norm_weight, norm_eps, H, norm_dtype)
-    out = torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
+    if fused_norm:
+        out = torch.empty((T, H * Dv), dtype=norm_dtype, device=dev)
+    else:
+        out = torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
     if chunks is not None and chunks[0].shape[0]:
         ch, po = chunks
         _need(ch, "chunks", torch.int32, (None, 3), dev)
@@ -1631,7 +1636,9 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         _check(lib.qe_linear_recurrence_chunked(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw,
                                                 _ptr(decay_bias), _ptr(bonus), _ptr(decay), mode, int(bool(silu)),
                                                 state.data_ptr(), state.stride(0), tok_seq.data_ptr(), ch.data_ptr(),
-                                                ch.shape[0], po.data_ptr(), po.shape[0], int(all_single), _ptr(ws), out.data_ptr(),
+                                                ch.shape[0], po.data_ptr(), po.shape[0], int(all_single), _ptr(ws),
+                                                None if fused_norm else out.data_ptr(), _ptr(norm_weight), float(norm_eps),
+                                                out.data_ptr() if fused_norm else None, _DT[out.dtype],
                                                 H, D, Dv, _DT[q.dtype], _stream()), "linear_recurrence (chunked)")
         return out
     _check(lib.qe_linear_recurrence(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw, _ptr(decay_bias),
