@@ -70,11 +70,18 @@ __device__ __forceinline__ float other_half(float v) {
     return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xf, 0xf, true));
 }
 
-template <typename TA>
-__device__ __forceinline__ void load4(const TA* __restrict__ p, int left, bool vec, float (&v)[4]) {
-    if (vec && left >= 4) { Vec4<TA>::load(p, v); return; }
+// four neighbouring elements from an address of any alignment (an element's own)
+__device__ __forceinline__ void load4(const float* __restrict__ p, float (&v)[4]) {
+    typedef float float4_any __attribute__((ext_vector_type(4), aligned(4)));
+    const float4_any t = *(const float4_any*)p;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = j < left ? Elem<TA>::load(p + j) : 0.f;
+    for (int j = 0; j < 4; ++j) v[j] = t[j];
+}
+__device__ __forceinline__ void load4(const bf16_t* __restrict__ p, float (&v)[4]) {
+    typedef unsigned short ushort4_any __attribute__((ext_vector_type(4), aligned(2)));
+    const ushort4_any t = *(const ushort4_any*)p;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = bf16_bits_to_float(t[j]);
 }
 
 // What a lane brings of one tile of 16 channels for 16 rows: channels d .. d + 3 of its row.
@@ -96,13 +103,10 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
     const int col0 = blockIdx.z * 128 + wave * 16, col = col0 + r;
     const bool has_cols = wave < 8 && col0 < Dv && wave * 16 < 128;
     const bool col_ok = has_cols && col < Dv;
-    const int preparers = waves < DT ? waves : DT;
+    constexpr int PREP = DT < 8 ? DT : 8;                  // waves that prepare channels (the launch has at least as many)
     const TA* q = (const TA*)a.q;
     const TA* k = (const TA*)a.k;
     const TA* v = (const TA*)a.v;
-    const bool vec = D % 4 == 0 && a.row_stride % 4 == 0 && (((unsigned long)q | (unsigned long)k) & 15) == 0 &&
-                     (MODE != 1 || (a.w_stride % 4 == 0 && ((unsigned long)a.wx & 15) == 0));
-
     floatx4 S[DT];
     float* slot = a.state + (long)a.tok_seq[row0] * a.state_stride + (long)h * D * Dv;
     float* mine = a.ws_s + ((long)c * H + h) * D * Dv;
@@ -127,35 +131,60 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
         const int d0 = (wave + p * waves) * 16 + 4 * g;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const bool in = MODE != 0 && wave + p * waves < DT && d0 + j < D;
-            bias[p][j] = in ? a.w0[h * D + d0 + j] : 0.f;
-            low[p][j] = in ? a.u[h * D + d0 + j] : 0.f;
+            const int d = min(d0 + j, D - 1);              // (what stands beyond the head's channels is not used)
+            bias[p][j] = MODE != 0 ? a.w0[h * D + d] : 0.f;
+            low[p][j] = MODE != 0 ? a.u[h * D + d] : 0.f;
             whole[p][j] = 1.f;
         }
     }
 
-    RecRaw raw[NPT];
-    float vr[4], vv[4];                                    // value rows: of the rows prepared next, of the rows used now
+    // Loads are asked for a whole round ahead (the raw numbers of the rows prepared next round, the values of the rows
+    // used next round) and moved to the registers that this round reads before the next ones are asked for: no wait in
+    // the middle of a round meets a load that was just issued.  They have no branches: rows beyond the chunk read its last
+    // one again, channels beyond the head its last four; what is read there is not used.
+    RecRaw raw[NPT], raw_next[NPT];
+    float vv[4], v_next[4];
+    const TA* qc = q + (long)row0 * a.row_stride + (long)h * D;
+    const TA* kc = k + (long)row0 * a.row_stride + (long)h * D;
+    const TA* vc = v + (long)row0 * a.row_stride + (long)h * Dv + (col_ok ? col : 0);
+    const float* wc = MODE == 1 ? a.wx + (long)row0 * a.w_stride + (long)h * D : nullptr;
+    const int stride = (int)a.row_stride, w_stride = (int)a.w_stride;
     auto fetch = [&](int base) {
-        const int nb = n - base < 16 ? n - base : 16;
+        const int row = min(base + r, n - 1);
 #pragma unroll
         for (int p = 0; p < NPT; ++p) {
-            const int d0 = (wave + p * waves) * 16 + 4 * g;
-            if (wave + p * waves < DT && r < nb && d0 < D) {
-                const long at_ = (long)(row0 + base + r) * a.row_stride + (long)h * D + d0;
-                if (PHASE == 1) load4<TA>(q + at_, D - d0, vec, raw[p].q);
-                load4<TA>(k + at_, D - d0, vec, raw[p].k);
-                if (MODE == 1) load4<float>(a.wx + (long)(row0 + base + r) * a.w_stride + (long)h * D + d0, D - d0, vec, raw[p].w);
+            const int d = min((wave + p * waves) * 16 + 4 * g, D - 4);
+            if (PHASE == 1) load4(qc + row * stride + d, raw_next[p].q);
+            load4(kc + row * stride + d, raw_next[p].k);
+            if (MODE == 1) load4(wc + row * w_stride + d, raw_next[p].w);
+        }
+    };
+    auto shift = [](float (&x)[4], int by) {               // x[j] <- x[j + by] where there is one
+        const float y[4] = {x[0], x[1], x[2], x[3]};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) x[j] = by == 0 ? y[j] : (by == 1 ? y[j < 3 ? j + 1 : 3] : (by == 2 ? y[j < 2 ? j + 2 : 3] : y[3]));
+    };
+    auto take = [&]() {
+#pragma unroll
+        for (int p = 0; p < NPT; ++p) {
+            raw[p] = raw_next[p];
+            if (D % 4) {                                   // (the head's last channels were read from its last four)
+                const int d0 = (wave + p * waves) * 16 + 4 * g, by = d0 > D - 4 ? min(d0 - (D - 4), 3) : 0;
+                if (PHASE == 1) shift(raw[p].q, by);
+                shift(raw[p].k, by);
+                if (MODE == 1) shift(raw[p].w, by);
             }
         }
     };
     auto fetch_values = [&](int base) {
-        const int nb = n - base < 16 ? n - base : 16;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v_next[j] = Elem<TA>::load(vc + min(base + 4 * g + j, n - 1) * stride);
+    };
+    auto take_values = [&](int base) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const int row = 4 * g + j < nb ? 4 * g + j : 0;
-            const float x = Elem<TA>::load(v + (long)(row0 + base + row) * a.row_stride + (long)h * Dv + (col_ok ? col : 0));
-            vr[j] = col_ok && 4 * g + j < nb ? x : 0.f;
+            const float x = (a.act_silu && MODE != 2) ? silu_quick(v_next[j]) : v_next[j];
+            vv[j] = col_ok && base + 4 * g + j < n ? x : 0.f;
         }
     };
     auto prepare = [&](int base, int buf) {
@@ -173,11 +202,11 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
                 const bool in = r < nb && d0 + j < D;
                 float f = 1.f;
                 qv[j] = kv[j] = 0.f;
-                if (PHASE == 1) qv[j] = a.act_silu ? silu_f(raw[p].q[j]) : raw[p].q[j];
+                if (PHASE == 1) qv[j] = a.act_silu ? silu_quick(raw[p].q[j]) : raw[p].q[j];
                 if (MODE == 2) {
                     forget_gate(raw[p].k[j] + bias[p][j], low[p][j], f, kv[j]);
                 } else {
-                    kv[j] = a.act_silu ? silu_f(raw[p].k[j]) : raw[p].k[j];
+                    kv[j] = a.act_silu ? silu_quick(raw[p].k[j]) : raw[p].k[j];
                     f = MODE == 0 ? dec : expf(-expf(raw[p].w[j] + bias[p][j]));
                 }
                 qv[j] = in ? qv[j] : 0.f;                  // (what lies beyond the rows and channels changes nothing)
@@ -239,26 +268,35 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
             *(floatx4*)&kt[buf][r][d0] = wk;
             if (r == 0) *(floatx4*)&gt[buf][d0] = wg;
         }
-        if (PHASE == 1 && wave < preparers) {
+        if (PHASE == 1 && wave < PREP) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) at[qb][wave][4 * g + i][r] = ga[i];
         }
     };
+    const int out_stride = H * Dv;
+    const long out0 = (long)row0 * out_stride + (long)h * Dv + col;
+    if (PHASE == 1)
+        for (int i = threadIdx.x; i < 256; i += blockDim.x) (&sq[0][0][0])[i] = 0.f;      // (waves without columns leave no sums)
     floatx4 o_held = {0.f, 0.f, 0.f, 0.f};                 // (with a norm: the outputs of the last 16 rows)
     auto use = [&](int base, int buf) {
         const int nb = n - base < 16 ? n - base : 16;
         const int qb = PHASE == 1 ? buf : 0;
         if (PHASE == 1) {
-            floatx4 av = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
-            for (int w = 0; w < preparers; ++w) av += *(const floatx4*)&at[qb][w][r][4 * g];
+            floatx4 av = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f}, o2 = {0.f, 0.f, 0.f, 0.f};   // (two chains)
+#pragma unroll
+            for (int w = 0; w < PREP; ++w) av += *(const floatx4*)&at[qb][w][r][4 * g];
 #pragma unroll
             for (int ct = 0; ct < DT; ++ct) {
                 const floatx4 x = *(const floatx4*)&qt[qb][r][ct * 16 + 4 * g];
 #pragma unroll
-                for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], S[ct][j], o, 0, 0, 0);
+                for (int j = 0; j < 4; ++j) {
+                    if (ct & 1) o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], S[ct][j], o2, 0, 0, 0);
+                    else o = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], S[ct][j], o, 0, 0, 0);
+                }
             }
 #pragma unroll
             for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(av[j], vv[j], o, 0, 0, 0);
+            o += o2;
             if (a.norm_w) {
                 o_held = o;
 #pragma unroll
@@ -269,7 +307,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
             } else {
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
-                    if (col_ok && 4 * g + i < nb) a.out[((long)(row0 + base + 4 * g + i) * H + h) * Dv + col] = o[i];
+                    if (col_ok && 4 * g + i < nb) a.out[out0 + (base + 4 * g + i) * out_stride] = o[i];
             }
         }
 #pragma unroll
@@ -280,52 +318,44 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
                 S[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[buf][4 * g + j][ct * 16 + r], vv[j], S[ct], 0, 0, 0);
         }
     };
-    const int col_waves = (Dv + 15) / 16 < 8 ? (Dv + 15) / 16 : 8;
+    const float inv_dv = 1.f / (float)Dv;
     const float nw = PHASE == 1 && a.norm_w && col_ok ? a.norm_w[h * Dv + col] : 0.f;
     auto write_normed = [&](int base, int buf) {           // rows whose squares' sums the last barrier has made whole
         const int nb = n - base < 16 ? n - base : 16;
         const int qb = PHASE == 1 ? buf : 0;
         floatx4 all = {0.f, 0.f, 0.f, 0.f};
-        for (int w = 0; w < col_waves; ++w) all += *(const floatx4*)&sq[qb][w][4 * g];
+#pragma unroll
+        for (int w = 0; w < 8; ++w) all += *(const floatx4*)&sq[qb][w][4 * g];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const float x = o_held[i] * rsqrtf(all[i] / (float)Dv + a.norm_eps) * nw;
+            const float x = o_held[i] * rsqrtf(fmaf(all[i], inv_dv, a.norm_eps)) * nw;
             if (col_ok && 4 * g + i < nb) {
-                const long to = (long)(row0 + base + 4 * g + i) * H * Dv + (long)h * Dv + col;
+                const long to = out0 + (base + 4 * g + i) * out_stride;
                 if (a.y_bf16) ((bf16_t*)a.y)[to] = float_to_bf16(x);
                 else ((float*)a.y)[to] = x;
             }
         }
     };
-
-    // (SILU of the values: silu(0) = 0)
-    auto values = [&]() {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) vv[j] = (a.act_silu && MODE != 2) ? silu_f(vr[j]) : vr[j];
-    };
     const bool prepares_first = (wave & 4) == 0;
     fetch(0);
-    if (has_cols) fetch_values(0);
+    take();
+    fetch(16);
+    fetch_values(0);
     prepare(0, 0);
-    if (n > 16) fetch(16);
     __syncthreads();
 #pragma unroll 1
     for (int base = 0, buf = 0; base < n; base += 16, buf ^= 1) {
         const bool more = base + 16 < n;
-        if (has_cols) {
-            values();
-            if (more) fetch_values(base + 16);
-            if (PHASE == 1 && a.norm_w && base > 0) write_normed(base - 16, buf ^ 1);
-        }
-        if (more && prepares_first) {
-            prepare(base + 16, buf ^ 1);
-            if (base + 32 < n) fetch(base + 32);
-        }
+        take();
+        take_values(base);
+        __builtin_amdgcn_sched_barrier(0);
+        fetch(base + 32);
+        fetch_values(base + 16);
+        __builtin_amdgcn_sched_barrier(0);
+        if (PHASE == 1 && a.norm_w && base > 0 && has_cols) write_normed(base - 16, buf ^ 1);
+        if (more && prepares_first) prepare(base + 16, buf ^ 1);
         if (has_cols) use(base, buf);
-        if (more && !prepares_first) {
-            prepare(base + 16, buf ^ 1);
-            if (base + 32 < n) fetch(base + 32);
-        }
+        if (more && !prepares_first) prepare(base + 16, buf ^ 1);
         __syncthreads();
     }
     if (PHASE == 1 && a.norm_w && has_cols) write_normed((n - 1) / 16 * 16, ((n - 1) / 16) & 1);
@@ -381,10 +411,6 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(const int* __restr
     *sp = S;
 }
 
-// Rows of a chunk: many enough that the states between chunks (written, read, written and read again) cost little
-// beside the rows, few enough that a prompt's chunks and heads fill the chip.
-extern "C" int qe_recurrence_chunk_len(int D) { (void)D; return 128; }
-
 template <typename TA, int MODE, int PHASE>
 static int launch_chunks(const RecArgs& a, int n_chunks, hipStream_t stream) {
     const int tiles = (a.D + 15) / 16, vt = a.Dv >= 128 ? 8 : (a.Dv + 15) / 16;
@@ -425,12 +451,13 @@ extern "C" int qe_linear_recurrence_chunked(const void* q, const void* k, const 
                                             float* ws, float* out, const float* norm_w, float norm_eps, void* y, int dt_y,
                                             int H, int D, int Dv, int dt_a, hipStream_t stream) {
     QE_REQUIRE(n_chunks >= 0 && n_portions >= 0 && H > 0 && H <= 65535 && D > 0 && Dv > 0, "linear_recurrence: bad sizes");
-    QE_REQUIRE(D <= 256, "linear_recurrence: heads of %d key channels (at most 256)", D);
+    QE_REQUIRE(D >= 4 && D <= 256, "linear_recurrence: heads of %d key channels (4 to 256 in chunks)", D);
     QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "linear_recurrence: mode %d lacks operands", mode);
     QE_REQUIRE(state_stride >= (long)H * D * Dv, "linear_recurrence: state rows overlap");
     QE_REQUIRE(dt_a == QE_F32 || dt_a == QE_BF16, "linear_recurrence: unknown element type %d", dt_a);
     if (n_chunks == 0) return 0;
     QE_REQUIRE(chunks && portions && (all_single || ws), "linear_recurrence: chunks without a workspace");
+    QE_REQUIRE(row_stride < (1L << 23) && w_stride < (1L << 23) && (long)H * Dv < (1L << 23), "linear_recurrence: rows too long");
     QE_REQUIRE(norm_w ? (y && Dv <= 128 && (dt_y == QE_F32 || dt_y == QE_BF16)) : out != nullptr, "linear_recurrence: no place for the outputs, or heads too wide for the norm inside");
     RecArgs a{q, k, v, row_stride, wx, w_stride, w0, u, decay, act_silu, chunks, ws, ws + (long)n_chunks * H * D * Dv,
               state, state_stride, tok_seq, out, H, D, Dv, norm_w, norm_eps, y, dt_y == QE_BF16};

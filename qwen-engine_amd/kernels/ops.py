@@ -96,7 +96,6 @@ def load_library():
                               f32, i32, i32, vp, i32, vp],
         "qe_attention_talk_splits": [i32, i32],
         "qe_token_shift": [vp, vp, i32, vp, i64, vp, vp, i32, i32, i32, i32, vp],
-        "qe_recurrence_chunk_len": [i32],
         "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, i32, vp, vp, vp, f32, vp, i32,
                                          i32, i32, i32, i32, vp],
         "qe_recurrence_single_supported": [i32, i32],
@@ -1543,9 +1542,14 @@ def _rows_view(t: torch.Tensor, name: str, n: int, T: int):
     return t.stride(0) if T > 1 else n
 
 
-def recurrence_chunk_len(head_dim: int) -> int:
-    """Rows of a chunk of the chunked recurrence for heads of this many key channels."""
-    return load_library().qe_recurrence_chunk_len(int(head_dim))
+def recurrence_chunk_len(rows: int, heads: int) -> int:
+    """Rows of a chunk of the chunked recurrence, for the longest portion's rows and the heads: the longest of 64, 128 and
+    256 that still gives every compute unit a block (the states between chunks cost less the longer the chunks are; a
+    chunk is walked by one block a head)."""
+    for length in (256, 128):
+        if int(rows) * int(heads) >= 256 * length:
+            return length
+    return 64
 
 
 def recurrence_chunks(portions, chunk_len: int):
@@ -1575,7 +1579,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     sigmoid(k + forget_bias):  S <- diag(f_t) S + (1 - f_t) v_t^T, o_t = S^T q_t.
     q, k [T, H D], v [T, H Dv] (column slices of one wider tensor are taken as they are, all with one row stride);
     ``silu``: the three (with a forget gate: q) pass silu first.  Returns o float32 [T, H, Dv].
-    ``chunks`` (recurrence_chunks() of all rows' portions, on the device, for recurrence_chunk_len(D)): the rows are
+    ``chunks`` (recurrence_chunks() of all rows' portions, on the device): the rows are
     taken chunk by chunk, the chunks in parallel, instead of row by row: for long portions.
     ``norm_weight`` (float32 [H Dv]): every head's o is divided by its root mean square (norm_eps inside) and multiplied
     by the weight; the result is [T, H Dv] in norm_dtype.  ``single_rows``: no two rows belong to one request (the norm
@@ -1591,6 +1595,8 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
     if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < H * D * Dv or state.stride(1) != 1:
         raise KernelError("linear_recurrence: the state is float32 [slots, >= H D Dv]")
+    if D < 4:
+        chunks = None                # (the chunked kernels read four channels at a time)
     mode, sw = 0, 0
     if decay is not None:
         _need(decay, "decay", torch.float32, (H,), dev)

@@ -23,12 +23,13 @@ def _single_rows(ctx, T: int) -> bool:
 CHUNKED_FROM_ROWS = 8
 
 
-def _chunks(ctx, head_dim: int):
+def _chunks(ctx, heads: int):
     """The step's rows cut into chunks for the chunked recurrence, if a request brings many rows: built and sent to the
     device once per step and chunk length, shared by the layers.  None: row by row."""
-    if max((s.q_len for s in ctx.seqs), default=0) < CHUNKED_FROM_ROWS:
+    longest = max((s.q_len for s in ctx.seqs), default=0)
+    if longest < CHUNKED_FROM_ROWS:
         return None
-    C = ops.recurrence_chunk_len(head_dim)
+    C = ops.recurrence_chunk_len(longest, heads)
     key = ("recurrence.chunks", C)
     if key not in ctx.memo:
         ch, po = ops.recurrence_chunks([(s.q_start, s.q_len) for s in ctx.seqs], C)
@@ -90,7 +91,7 @@ class ShiftedDecayMixer:
         low = ops.unary(ops.gemm(m[4], self.w_1, out_dtype=torch.float32), ops.UNARY_TANH, out_dtype=ctx.rt.dtype)
         decay_x = ops.gemm(low, self.w_2, out_dtype=torch.float32)      # (exponentials of the decay: in the recurrence, 32-bit)
         o = ops.linear_recurrence(r, k, v, st[:, W:], ctx.tok_seq, self.h, decay_x=decay_x, decay_bias=self.w0,
-                                  bonus=self.u, chunks=_chunks(ctx, self.d))
+                                  bonus=self.u, chunks=_chunks(ctx, self.h))
         y = ops.gated_norm(o.view(T, self.h * self.d), self.norm, self.eps, self.h, ctx.rt.dtype, gate=gate,
                            gate_act=ops.GATE_SILU)
         return ops.gemm(y, self.w_o, out_dtype=torch.float32)
@@ -140,7 +141,7 @@ class DecayedLinearMixer:
         nk, nv = self.h * self.d, self.h * self.dv
         y = ops.gemm(x, self.w_in)
         o = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], binding.state, ctx.tok_seq,
-                                  self.h, decay=self.decay, silu=True, chunks=_chunks(ctx, self.d))
+                                  self.h, decay=self.decay, silu=True, chunks=_chunks(ctx, self.h))
         z = ops.gated_norm(o.view(T, nv), self.norm, self.eps, 1, ctx.rt.dtype, gate=y[:, 2 * nk + nv:],
                            gate_act=ops.GATE_SIGMOID)
         return ops.gemm(z, self.w_o, out_dtype=torch.float32)
@@ -193,7 +194,7 @@ class ForgetGateLinearMixer:
         nk = self.h * self.d
         y = ops.gemm(x, self.w_in, out_dtype=torch.float32)
         z = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:], binding.state, ctx.tok_seq, self.h, silu=True,
-                                  forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.d),
+                                  forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.h),
                                   norm_weight=self.norm, norm_eps=self.eps, norm_dtype=ctx.rt.dtype,
                                   single_rows=_single_rows(ctx, T))
         splits = ops.gemm_branch_splits(z, self.w_o)

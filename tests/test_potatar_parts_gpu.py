@@ -322,7 +322,7 @@ def _chunks_of(portions, head_dim, chunked):
     chunks in parallel), or None for the path that walks row by row."""
     if not chunked:
         return None
-    ch, po = ops().recurrence_chunks(portions, ops().recurrence_chunk_len(head_dim))
+    ch, po = ops().recurrence_chunks(portions, 64)
     return ch.to(DEV), po.to(DEV)
 
 
