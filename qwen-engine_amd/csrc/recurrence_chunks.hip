@@ -138,10 +138,10 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(RecArgs a) {
         }
     }
 
-    // Loads are asked for a whole round ahead (the raw numbers of the rows prepared next round, the values of the rows
-    // used next round) and moved to the registers that this round reads before the next ones are asked for: no wait in
-    // the middle of a round meets a load that was just issued.  They have no branches: rows beyond the chunk read its last
-    // one again, channels beyond the head its last four; what is read there is not used.
+    // Loads are asked for 16 rows ahead of their use (the raw numbers of the rows prepared next, the values of the rows
+    // used next) and moved to the registers that are read before the following ones are asked for: no wait between two
+    // barriers meets a load that was just issued.  They have no branches: rows beyond the chunk read its last one again,
+    // channels beyond the head its last four; what is read there is not used.
     RecRaw raw[NPT], raw_next[NPT];
     float vv[4], v_next[4];
     const TA* qc = q + (long)row0 * a.row_stride + (long)h * D;
