@@ -109,3 +109,11 @@ def _busadra(d):
 
 
 register_architecture("Busadra", _busadra)
+
+
+def _vuzinex(d, shapes=None):
+    from .vuzinex import VuzinexConfig
+    return VuzinexConfig.from_dict(d, shapes)
+
+
+register_architecture("Vuzinex", _vuzinex, tensor_shapes=True)

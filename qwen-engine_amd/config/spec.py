@@ -57,10 +57,13 @@ class AttentionSpec:
 
 @dataclass(frozen=True)
 class SwiGLUSpec:
-    """down(silu(gate(x)) * up(x)), no biases.  ``names``: the tensors of gate, up and down inside the part."""
+    """down(silu(gate(x)) * up(x)), with biases on all three if ``bias``.  ``names``: the tensors of gate, up and down inside
+    the part; a bias is its name + ``bias_suffix``."""
     intermediate_size: int
     kind: str = "swiglu"
     names: Tuple[str, str, str] = ("gate_proj.weight", "up_proj.weight", "down_proj.weight")
+    bias: bool = False
+    bias_suffix: str = ".b"
 
 
 @dataclass(frozen=True)
@@ -73,10 +76,15 @@ class ScalarRMSNormSpec:
 @dataclass(frozen=True)
 class RopePairsSpec:
     """Rotary position encoding over neighbouring pairs: the pair (2i, 2i + 1), i < rotary_dim / 2, is
-    turned by ``position * theta ** (-2 i / rotary_dim)``; features from rotary_dim on pass unchanged."""
+    turned by ``position * theta ** (-2 i / rotary_dim)``; features from rotary_dim on pass unchanged.
+    ``band_scaling``: as in RopeHalfAnglesSpec.  ``yarn``: None, or (factor, original, fast, slow): with at(t) = rotary_dim
+    ln(original / (2 pi t)) / (2 ln theta), frequency i goes from itself to itself / factor along a ramp from
+    max(floor(at(fast)), 0) to min(ceil(at(slow)), rotary_dim - 1), and cosine and sine are multiplied by 0.1 ln(factor) + 1."""
     theta: float
     rotary_dim: int
     kind: str = "rope_pairs"
+    band_scaling: Optional[Tuple[float, float, float, float]] = None
+    yarn: Optional[Tuple[float, float, float, float]] = None
 
 
 @dataclass(frozen=True)
@@ -239,9 +247,12 @@ class ParallelLayerSpec:
 
 @dataclass(frozen=True)
 class BareRMSNormSpec:
-    """RMSNorm whose weight tensor carries the part's own name (no ``.weight`` behind it)."""
+    """RMSNorm whose weight tensor carries the part's own name (no ``.weight`` behind it).  ``offset`` is added to the stored
+    weight (1 for weights stored around zero); ``gain``: one more factor on the result (see BareLayerNormSpec)."""
     eps: float
     kind: str = "rmsnorm_bare"
+    offset: float = 0.0
+    gain: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -256,7 +267,10 @@ class StreamScaleSpec:
 class ChunkAttentionSpec:
     """Grouped-query attention inside chunks of positions: with ``chunk`` = c, a query at position i sees the keys
     j <= i with i // c == j // c, chunks counted from the request's start (None: all earlier keys).  Keys have
-    ``head_dim`` numbers, values ``v_head_dim``; all four projections have biases if ``bias``.
+    ``head_dim`` numbers, values ``v_head_dim``; all four projections have biases if ``bias`` (the output projection: if
+    ``out_bias``, where that is given).  ``head_sink``: a learned number per head whose exponential joins the softmax's
+    denominator and carries no value.  ``output_gate``: the heads' outputs are multiplied by sigmoid of a projection of the
+    mixer's input, a number per output.
     ``qk_norm``: None, "head" (RMS norm of every q and k head with one weight of the head's size for all heads) or
     "whole" (RMS norm over all heads of q, and of k, at once, a weight per coordinate), before the rotation.
     ``values_from_keys``: there is no value projection; the values are the keys as projected, before their norm.
@@ -290,6 +304,11 @@ class ChunkAttentionSpec:
     distance_bias_name: str = "rel"
     talk_name: str = "talk"
     kind: str = "chunk_attention"
+    out_bias: Optional[bool] = None
+    head_sink: bool = False
+    output_gate: bool = False
+    sink_name: str = "sink"
+    gate_name: str = "g"
 
 
 @dataclass(frozen=True)
@@ -332,6 +351,69 @@ class ForgetGateLinearSpec:
     norm_eps: float
     names: Tuple[str, str, str, str, str, str, str] = ("q", "f", "f.b", "lower", "v", "norm", "o")
     kind: str = "forget_gate_linear"
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec:
+    """Gated linear attention: q = W_q x * head_dim^(-1/2), k = W_k x, v = W_v x; a decay per key channel
+    sigmoid(W_2 (W_1 x) + b)^(1 / tau) (W_1 has ``decay_rank`` rows); S <- diag(decay) S + k v^T, o = S^T q; every head's o
+    RMS-normed with one weight of ``v_head_dim`` numbers, times silu(W_g x), then the output projection.  ``names``: q, k, v,
+    gate, output projection, norm, W_1, W_2, b."""
+    num_heads: int
+    head_dim: int
+    v_head_dim: int
+    decay_rank: int
+    tau: float
+    norm_eps: float
+    names: Tuple[str, ...] = ("q", "k", "v", "g", "o", "norm", "a1", "a2", "a2.b")
+    kind: str = "gated_linear"
+
+
+@dataclass(frozen=True)
+class MatrixMemorySpec:
+    """The matrix memory of xLSTM (mLSTM).  q = W_q x * head_dim^(-1/2), k = W_k x, v = W_v x; per head the log gates
+    i = cap tanh((W_i x + b_i) / cap) and f = log sigmoid(cap tanh((W_f x + b_f) / cap)); with the running maximum m <- max(f +
+    m, i) from 0: S <- exp(f + m' - m) S + exp(i - m) k v^T, n likewise with k alone, o = S^T q / (max(|n . q|, exp(-m)) +
+    1e-6).  Every head's o divided by its root mean square, times a weight over all heads, times sigmoid(W_g x), then the
+    output projection.  ``names``: q, k, v, gate, output projection, norm, input gate, its bias, forget gate, its bias."""
+    num_heads: int
+    head_dim: int
+    v_head_dim: int
+    gate_cap: float
+    norm_eps: float
+    names: Tuple[str, ...] = ("q", "k", "v", "g", "o", "norm", "i", "i.b", "f", "f.b")
+    kind: str = "matrix_memory"
+
+
+@dataclass(frozen=True)
+class StateSpaceSpec:
+    """Mamba-2.  One projection [z | x | B | C | dt]: ``num_heads`` heads of ``head_dim`` numbers in z and x, ``groups`` groups of
+    ``state_dim`` in B and C, a number per head in dt.  x, B and C pass a causal convolution of ``taps`` taps per channel with
+    a bias, and silu.  dt = softplus(dt + bias); S <- exp(-exp(A) dt) S + dt B x^T, y = S^T C + D x (head h uses group
+    h // (heads / groups)); y * silu(z) RMS-normed in ``norm_groups`` equal parts, times a weight, then the output projection.
+    ``names``: projection, convolution, its bias, dt's bias, A, D, norm, output projection."""
+    num_heads: int
+    head_dim: int
+    state_dim: int
+    groups: int
+    taps: int
+    norm_groups: int
+    norm_eps: float
+    names: Tuple[str, ...] = ("in", "conv", "conv.b", "dt_bias", "A_log", "D", "norm", "o")
+    kind: str = "state_space"
+
+
+@dataclass(frozen=True)
+class PairEmbeddingSpec:
+    """The stream begins as scale * embed[token] + pairs[row], row = (previous token * mul_prev + token * mul_cur) mod buckets
+    of the tensor ``name`` [buckets + 1, hidden]; a request's first token takes the last row."""
+    scale: float
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+    name: str = "bigram"
+    prefix: str = ""
+    kind: str = "pair_embedding"
 
 
 @dataclass(frozen=True)
@@ -463,6 +545,23 @@ class ScaledLayerSpec:
 
 
 @dataclass(frozen=True)
+class SandwichLayerSpec:
+    """A block that norms before and after each sublayer: x <- x + mult * mixer_post(mixer(mixer_norm(x))), then
+    x <- x + mult * ffn_post(ffn(ffn_norm(x))).  ``ffn`` None: the first of the two alone.  ``names``: the checkpoint names
+    inside ``prefix`` of mixer norm, mixer, norm behind it, feed-forward norm, feed-forward, norm behind it."""
+    prefix: str
+    mixer_norm: object
+    mixer: object
+    mixer_post: object
+    ffn_norm: object
+    ffn: Optional[object]
+    ffn_post: object
+    mult: float = 1.0
+    names: Tuple[str, str, str, str, str, str] = ("norm1", "mix", "norm1b", "norm2", "mlp", "norm2b")
+    kind: str = "sandwich_block"
+
+
+@dataclass(frozen=True)
 class LayerSpec:
     """One pre-norm residual block: x += mixer(norm(x)); x += ffn(norm(x)).  ``ffn`` None: the layer is its mixer alone
     (its second norm is then used only if ``ffn_norm`` is given and the folder holds its tensors).
@@ -508,7 +607,7 @@ class ModelSpec:
     max_positions: int
     eos_token_ids: Tuple[int, ...] = field(default_factory=tuple)
     # optional parts around the layers: a spec with a ``kind`` (and a ``prefix`` for its tensors' names)
-    stream_prologue: Optional[object] = None   # changes the stream right after the embedding
+    stream_prologue: Optional[object] = None   # changes the stream right after the embedding, or makes it
     logit_epilogue: Optional[object] = None    # changes the logits after the head
 
     def validate(self) -> None:

@@ -10,20 +10,36 @@
 int qe_attention_generic(const void* q, void* out, const void* cache, const int* positions,
                          const int* tok_seq, const int* block_table, int max_blocks, const int* tokens,
                          int T, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink,
-                         float softcap, int dt_a, hipStream_t stream);
+                         float softcap, int dt_a, hipStream_t stream, const AttnTail& tail);
 bool qe_attention_decode_ok(int Hq, int Hkv, int D, int P, int dt_a);
 size_t qe_attention_decode_workspace(int n_dec, int Hq, int D, int num_splits);
 int qe_attention_decode(const void* q, void* out, const void* cache, const int* dec_tokens, int n_dec,
                         const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                         const int* shared_keys, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first,
                         int sink, float softcap, int max_position, int split_keys, void* workspace, size_t workspace_bytes,
-                        hipStream_t stream);
+                        hipStream_t stream, const AttnTail& tail);
 
 int qe_attention_prefill(const void* q, void* out, const void* cache, const int* tiles, int num_tiles,
                          const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                          int Hq, int Hkv, int D, int P, float scale, int window, int groups,
                          int seg_keys, int max_keys, int keys_row, void* workspace, size_t workspace_bytes,
-                         hipStream_t stream, int keep_first = 0, int sink = 0, float softcap = 0.f);
+                         hipStream_t stream, int keep_first, int sink, float softcap, const AttnTail& tail);
+static AttnTail make_tail(int Hq, int D, const void* out, long out_stride, int dv, const float* sink_heads, const void* gate,
+                          long gate_stride, int dt_g) {
+    AttnTail t{};
+    t.dv = dv > 0 ? dv : D;
+    t.out_stride = out_stride > 0 ? out_stride : (long)Hq * t.dv;
+    t.sink = sink_heads;
+    t.gate = gate;
+    t.gate_stride = gate_stride;
+    t.gate_f32 = dt_g == QE_F32;
+    t.plain = !gate && t.dv == D && t.out_stride % 4 == 0 && (((unsigned long)out) & 15) == 0;
+    return t;
+}
+#define QE_TAIL_CHECK()                                                                                                  \
+    QE_REQUIRE(dv >= 0 && dv <= D && (out_stride == 0 || out_stride >= (long)Hq * (dv ? dv : D)), "attention: rows of the result overlap"); \
+    QE_REQUIRE(!gate || (gate_stride >= (long)Hq * (dv ? dv : D) && (dt_g == QE_F32 || dt_g == QE_BF16)), "attention: gate rows overlap")
+
 int qe_attention_prefill_segment_keys(long blocks, int max_keys);
 int qe_attention_prefill_segments(long blocks);
 int qe_attention_prefill_uncut_keys();
@@ -90,26 +106,33 @@ extern "C" int qe_attention_prefill_run(const void* q, void* out, const void* ca
                                         const int* block_table, int max_blocks, int Hq, int Hkv, int D, int P,
                                         float scale, int window, int keep_first, int sink, float softcap, int groups, int seg_keys,
                                         int max_keys, int keys_row, void* workspace, long workspace_bytes,
-                                        hipStream_t stream) {
+                                        long out_stride, int dv, const float* sink_heads, const void* gate,
+                                        long gate_stride, int dt_g, hipStream_t stream) {
+    QE_TAIL_CHECK();
     QE_REQUIRE(num_tiles >= 0 && Hq > 0 && Hkv > 0 && max_blocks > 0 && keep_first >= 0 &&
                workspace_bytes >= 0, "prefill attention: bad sizes");
     return qe_attention_prefill(q, out, cache, tiles, num_tiles, positions, tok_seq, block_table, max_blocks,
                                 Hq, Hkv, D, P, scale, window, groups, seg_keys, max_keys, keys_row, workspace,
-                                (size_t)workspace_bytes, stream, keep_first, sink, softcap);
+                                (size_t)workspace_bytes, stream, keep_first, sink, softcap,
+                                make_tail(Hq, D, out, out_stride, dv, sink_heads, gate, gate_stride, dt_g));
 }
 
-// tokens: null for all T rows of q, else n_tokens row indices.  keep_first: the first keys of a request
+// out_stride, dv, sink_heads, gate, gate_stride, dt_g, here and below: see AttnTail (0, 0, null, null: plain rows of Hq * D
+// numbers, a sink of score 0).  tokens: null for all T rows of q, else n_tokens row indices.  keep_first: the first keys of a request
 // that every later query sees wherever its window stands; sink: a 1 is added to the softmax's denominator.
 extern "C" int qe_attention(const void* q, void* out, const void* cache, const int* positions,
                             const int* tok_seq, const int* block_table, int max_blocks, const int* tokens,
                             int n_tokens, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first,
-                            int sink, float softcap, int dt_a, hipStream_t stream) {
+                            int sink, float softcap, int dt_a, long out_stride, int dv, const float* sink_heads,
+                            const void* gate, long gate_stride, int dt_g, hipStream_t stream) {
+    QE_TAIL_CHECK();
     QE_REQUIRE(n_tokens >= 0 && Hq > 0 && Hkv > 0 && D > 0 && P > 0 && max_blocks > 0, "attention: bad sizes");
     QE_REQUIRE(Hq % Hkv == 0, "attention: %d query heads are no multiple of %d key/value heads", Hq, Hkv);
     QE_REQUIRE(keep_first >= 0 && (window >= 0 || keep_first == 0), "attention: kept first keys go with a window of the last keys");
     if (n_tokens == 0) return 0;
     return qe_attention_generic(q, out, cache, positions, tok_seq, block_table, max_blocks, tokens, n_tokens,
-                                Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, dt_a, stream);
+                                Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, dt_a, stream,
+                                make_tail(Hq, D, out, out_stride, dv, sink_heads, gate, gate_stride, dt_g));
 }
 
 extern "C" int qe_attention_decode_supported(int Hq, int Hkv, int D, int P, int dt_a) {
@@ -155,10 +178,13 @@ extern "C" int qe_attention_decode_run(const void* q, void* out, const void* cac
                                        const int* block_table, int max_blocks, const int* shared_keys,
                                        int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink, float softcap,
                                        int max_position, int split_keys, void* workspace, long workspace_bytes,
-                                       hipStream_t stream) {
+                                       long out_stride, int dv, const float* sink_heads, const void* gate,
+                                       long gate_stride, int dt_g, hipStream_t stream) {
+    QE_TAIL_CHECK();
     QE_REQUIRE(Hq > 0 && Hkv > 0 && max_blocks > 0 && keep_first >= 0 && max_position >= 0,
                "decode attention: bad sizes");
     return qe_attention_decode(q, out, cache, dec_tokens, n_dec, positions, tok_seq, block_table, max_blocks,
                                shared_keys, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, max_position, split_keys,
-                               workspace, (size_t)workspace_bytes, stream);
+                               workspace, (size_t)workspace_bytes, stream,
+                               make_tail(Hq, D, out, out_stride, dv, sink_heads, gate, gate_stride, dt_g));
 }

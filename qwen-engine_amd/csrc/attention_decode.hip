@@ -333,7 +333,7 @@ __global__ __launch_bounds__(64) void attention_decode_fused_split_kernel(
 template <int D>
 __global__ __launch_bounds__(256) void attention_decode_merge_kernel(
     const float* __restrict__ part_acc, const float* __restrict__ part_ml, const int* __restrict__ dec_tokens,
-    bf16_t* __restrict__ out, int Hq, int num_splits, int sink) {
+    bf16_t* __restrict__ out, int Hq, int num_splits, int sink, AttnTail tail) {
     constexpr int PER = (D + 63) / 64;
     __shared__ float red_o[4][D];
     __shared__ float red_l[4];
@@ -343,6 +343,7 @@ __global__ __launch_bounds__(256) void attention_decode_merge_kernel(
     const float* pacc = part_acc + ((long)di * Hq + head) * num_splits * D;
     // (the largest maximum is reduced only after the first eight splits' loads have been issued: its
     // own loads were issued before them, so waiting for those does not wait for these)
+    const float sk = sink ? tail.sink_of(head) : 0.f;
     float M = -INFINITY;
     for (int s = lane; s < num_splits; s += 64) M = fmaxf(M, pml[2 * s]);
     bool reduced = false;
@@ -371,8 +372,8 @@ __global__ __launch_bounds__(256) void attention_decode_merge_kernel(
                 a[k][i] = d < D ? pacc[(long)(s < num_splits ? s : num_splits - 1) * D + d] : 0.f;
             }
         }
-        // (sink: one more entry of score 0 that carries no value)
-        if (!reduced) { M = wave_max(M); if (sink) M = fmaxf(M, 0.f); reduced = true; }
+        // (sink: one more entry that carries no value)
+        if (!reduced) { M = wave_max(M); if (sink) M = fmaxf(M, sk); reduced = true; }
 #pragma unroll
         for (int k = 0; k < 8; ++k) {
             if (ms[k] == -INFINITY) continue;
@@ -390,12 +391,12 @@ __global__ __launch_bounds__(256) void attention_decode_merge_kernel(
     if (lane == 0) red_l[wave] = denom;
     __syncthreads();
     if (wave == 0) {
-        const float inv = 1.f / (red_l[0] + red_l[1] + red_l[2] + red_l[3] + (sink ? __expf(-M) : 0.f));
-        bf16_t* orow = out + ((long)(dec_tokens ? dec_tokens[di] : di) * Hq + head) * D;
+        const float inv = 1.f / (red_l[0] + red_l[1] + red_l[2] + red_l[3] + (sink ? __expf(sk - M) : 0.f));
+        const long row = dec_tokens ? dec_tokens[di] : di;
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
             const int d = lane + i * 64;
-            if (d < D) orow[d] = float_to_bf16((red_o[0][d] + red_o[1][d] + red_o[2][d] + red_o[3][d]) * inv);
+            if (d < D) tail.store(out, row, head, d, (red_o[0][d] + red_o[1][d] + red_o[2][d] + red_o[3][d]) * inv);
         }
     }
 }
@@ -419,7 +420,7 @@ int qe_attention_decode(const void* q, void* out, const void* cache, const int* 
                         const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                         const int* shared_keys, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first,
                         int sink, float softcap, int max_position, int split_keys, void* workspace, size_t workspace_bytes,
-                        hipStream_t stream) {
+                        hipStream_t stream, const AttnTail& tail) {
     QE_REQUIRE(qe_attention_decode_ok(Hq, Hkv, D, P, QE_BF16), "decode attention: sizes not taken");
     QE_REQUIRE(split_keys == 128 || split_keys == 256, "decode attention: splits of 128 or 256 keys, not %d", split_keys);
     if (n_dec == 0) return 0;
@@ -442,7 +443,7 @@ int qe_attention_decode(const void* q, void* out, const void* cache, const int* 
         if (softcap > 0.f) QE_DECODE_SPLIT(D_, S_, true);                                               \
         else QE_DECODE_SPLIT(D_, S_, false);                                                            \
         attention_decode_merge_kernel<D_><<<mgrid, 256, 0, stream>>>(part_acc, part_ml, dec_tokens,     \
-                                                                     (bf16_t*)out, Hq, num_splits, sink); \
+                                                                     (bf16_t*)out, Hq, num_splits, sink, tail); \
     } while (0)
     if (D == 128 && split_keys == 128) QE_DECODE(128, 128);
     else if (D == 128) QE_DECODE(128, 256);
@@ -474,6 +475,9 @@ int qe_attention_decode_fused(const void* qkv, void* out, void* cache, const int
     float* part_ml = part_acc + (size_t)n_dec * Hq * num_splits * D;
     dim3 grid(num_splits, Hkv, n_dec);
     dim3 mgrid(n_dec, Hq);
+    AttnTail tail{};
+    tail.out_stride = (long)Hq * D;
+    tail.dv = D;
     const bool few = (long)num_splits * Hkv * n_dec <= 1024;   // at most a wave per SIMD: loads further ahead
 #define QE_DECODE_FUSED(D_, S_)                                                                         \
     do {                                                                                                \
@@ -488,7 +492,7 @@ int qe_attention_decode_fused(const void* qkv, void* out, void* cache, const int
             shared_keys, slots, q_w, k_w, eps, table, part_acc, part_ml, Hq, Hkv, P, scale, window,     \
             num_splits);                                                                                \
         attention_decode_merge_kernel<D_><<<mgrid, 256, 0, stream>>>(part_acc, part_ml, dec_tokens,     \
-                                                                     (bf16_t*)out, Hq, num_splits, 0);  \
+                                                                     (bf16_t*)out, Hq, num_splits, 0, tail); \
     } while (0)
     if (D == 128 && split_keys == 128) QE_DECODE_FUSED(128, 128);
     else if (D == 128) QE_DECODE_FUSED(128, 256);

@@ -38,7 +38,7 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
     const float* __restrict__ q, float* __restrict__ out, const float* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tokens,
-    int Hq, int Hkv, int P, float scale, int window, int keep_first, int sink, float softcap) {
+    int Hq, int Hkv, int P, float scale, int window, int keep_first, int sink, float softcap, AttnTail tail) {
     constexpr int D = DB * 16;
     extern __shared__ float merge_lds[];                  // [F32_WAVES][DB * 4 + 2][64]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, n = lane & 15;
@@ -151,10 +151,11 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
     mine[(DB * 4 + 1) * 64] = l;
     __syncthreads();
     if (wave != 0) return;
-    float M = sink ? 0.f : -INFINITY;                     // (the sink: one more entry of score 0 without a value)
+    const float sk = sink && head_ok ? tail.sink_of(head) : 0.f;
+    float M = sink ? sk : -INFINITY;                      // (the sink: one more entry without a value)
 #pragma unroll
     for (int w = 0; w < F32_WAVES; ++w) M = fmaxf(M, merge_lds[((long)w * (DB * 4 + 2) + DB * 4) * 64 + lane]);
-    float wgt[F32_WAVES], lsum = sink ? expf(-M) : 0.f;
+    float wgt[F32_WAVES], lsum = sink ? expf(sk - M) : 0.f;
 #pragma unroll
     for (int w = 0; w < F32_WAVES; ++w) {
         const float mw = merge_lds[((long)w * (DB * 4 + 2) + DB * 4) * 64 + lane];
@@ -163,7 +164,6 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
     }
     if (head_ok) {
         const float inv = 1.f / lsum;
-        float* orow = out + (t * Hq + head) * D + g * 4;
 #pragma unroll
         for (int db = 0; db < DB; ++db) {
             floatx4 o;
@@ -174,7 +174,10 @@ __global__ __launch_bounds__(64 * F32_WAVES) void attention_f32_kernel(
                 for (int w = 0; w < F32_WAVES; ++w) a += wgt[w] * merge_lds[((long)w * (DB * 4 + 2) + db * 4 + i) * 64 + lane];
                 o[i] = a * inv;
             }
-            *(floatx4*)(orow + db * 16) = o;
+            if (tail.plain) *(floatx4*)(out + t * tail.out_stride + (long)head * D + g * 4 + db * 16) = o;
+            else
+#pragma unroll
+                for (int i = 0; i < 4; ++i) tail.store(out, t, head, db * 16 + g * 4 + i, o[i]);
         }
     }
 }
@@ -185,7 +188,7 @@ bool qe_attention_f32_ok(int Hq, int Hkv, int D, int P) {
 
 int qe_attention_f32(const float* q, float* out, const float* cache, const int* positions, const int* tok_seq,
                      const int* block_table, int max_blocks, const int* tokens, int T, int Hq, int Hkv, int D,
-                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream) {
+                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream, const AttnTail& tail) {
     QE_REQUIRE(qe_attention_f32_ok(Hq, Hkv, D, P), "attention (32-bit): sizes not taken");
     const int groups16 = (Hq / Hkv + 15) / 16;
     QE_REQUIRE((long)Hkv * groups16 <= 65535, "attention (32-bit): too many heads");
@@ -203,7 +206,7 @@ int qe_attention_f32(const float* q, float* out, const float* cache, const int* 
             }                                                                                         \
         }                                                                                             \
         attention_f32_kernel<DB_><<<grid, 64 * F32_WAVES, lds, stream>>>(q, out, cache, positions, tok_seq, \
-                                                    block_table, max_blocks, tokens, Hq, Hkv, P, scale, window, keep_first, sink, softcap); \
+                                                    block_table, max_blocks, tokens, Hq, Hkv, P, scale, window, keep_first, sink, softcap, tail); \
         break;                                                                                        \
     }
     switch (D / 16) {

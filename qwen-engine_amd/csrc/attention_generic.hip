@@ -10,8 +10,8 @@
 // taken 64 at a time, the kept first keys behind the window first, then from lo upwards, with
 // an online softmax, so the order of the sums depends on p, the window and keep_first only:
 // not on how the request's tokens were cut into steps, nor on what else is in the batch.
-// With sink the softmax has one more entry of score 0 that carries no value (a 1 in the
-// denominator): the running maximum starts at 0 with a sum of 1.
+// With sink the softmax has one more entry that carries no value, of the head's score in AttnTail or of score 0:
+// the running maximum starts there with a sum of 1.
 //
 // cache of one layer: [page][2 (k, v)][Hkv][P * D]; a key tile is [P][D], a value tile is
 // stored transposed, [D][P] (the layout the MFMA kernels read without a shuffle).
@@ -24,7 +24,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     const TA* __restrict__ q, TA* __restrict__ out, const TA* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tokens,
-    int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink, float softcap) {
+    int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink, float softcap, AttnTail tail) {
     extern __shared__ float smem[];
     float* qs = smem;            // D
     float* ps = smem + D;        // 64 probabilities of the current chunk
@@ -42,7 +42,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     for (int d = lane; d < D; d += 64) qs[d] = Elem<TA>::load(qrow + d);
     __syncthreads();
 
-    float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+    float m = sink ? tail.sink_of(h) : -INFINITY, l = sink ? 1.f : 0.f;
     float acc[ATTN_MAX_D / 64];
 #pragma unroll
     for (int i = 0; i < ATTN_MAX_D / 64; ++i) acc[i] = 0.f;
@@ -86,19 +86,18 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
         }
         __syncthreads();
     }
-    TA* orow = out + (t * Hq + h) * D;
     const float inv = 1.f / l;
 #pragma unroll
     for (int i = 0; i < ATTN_MAX_D / 64; ++i) {
         const int d = lane + i * 64;
-        if (d < D) Elem<TA>::store(orow + d, acc[i] * inv);
+        if (d < D) tail.store(out, t, h, d, acc[i] * inv);
     }
 }
 
 bool qe_attention_f32_ok(int Hq, int Hkv, int D, int P);
 int qe_attention_f32(const float* q, float* out, const float* cache, const int* positions, const int* tok_seq,
                      const int* block_table, int max_blocks, const int* tokens, int T, int Hq, int Hkv, int D,
-                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream);
+                     int P, float scale, int window, int keep_first, int sink, float softcap, hipStream_t stream, const AttnTail& tail);
 
 // 32-bit attention goes to the kernel on the matrix units (attention_f32.hip) where it takes the
 // sizes, unless qe_use_matrix_f32(0) has switched that off.
@@ -107,10 +106,10 @@ extern int g_qe_matrix_f32;
 int qe_attention_generic(const void* q, void* out, const void* cache, const int* positions,
                          const int* tok_seq, const int* block_table, int max_blocks, const int* tokens,
                          int T, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first, int sink,
-                         float softcap, int dt_a, hipStream_t stream) {
+                         float softcap, int dt_a, hipStream_t stream, const AttnTail& tail) {
     if (dt_a == QE_F32 && g_qe_matrix_f32 && qe_attention_f32_ok(Hq, Hkv, D, P))
         return qe_attention_f32((const float*)q, (float*)out, (const float*)cache, positions, tok_seq, block_table,
-                                max_blocks, tokens, T, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, stream);
+                                max_blocks, tokens, T, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, stream, tail);
     QE_REQUIRE(D <= ATTN_MAX_D, "attention: head_dim=%d exceeds %d", D, ATTN_MAX_D);
     QE_REQUIRE(Hq <= 65535, "attention: too many heads");
     dim3 grid(T, Hq);
@@ -118,11 +117,11 @@ int qe_attention_generic(const void* q, void* out, const void* cache, const int*
     if (dt_a == QE_F32)
         attention_generic_kernel<float><<<grid, 64, shmem, stream>>>(
             (const float*)q, (float*)out, (const float*)cache, positions, tok_seq, block_table,
-            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap);
+            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, tail);
     else if (dt_a == QE_BF16)
         attention_generic_kernel<bf16_t><<<grid, 64, shmem, stream>>>(
             (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, tok_seq, block_table,
-            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap);
+            max_blocks, tokens, Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, tail);
     else
         QE_REQUIRE(false, "attention: unknown dtype %d", dt_a);
     QE_LAUNCH_CHECK();

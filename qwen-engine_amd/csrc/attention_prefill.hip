@@ -92,16 +92,44 @@ __device__ __forceinline__ int segment_keys(int seg_param, const int* __restrict
 // 32 db + 8 b + 4 g + j.
 template <int D>
 __device__ __forceinline__ void store_columns(bf16_t* __restrict__ out, const floatx16 (&acc)[D / 32], float inv,
-                                              int row, int head, int Hq, int g) {
-    bf16_t* orow = out + ((long)row * Hq + head) * D + 4 * g;
+                                              int row, int head, int g, const AttnTail& tail) {
+    if (tail.plain) {
+        bf16_t* orow = out + (long)row * tail.out_stride + (long)head * D + 4 * g;
+#pragma unroll
+        for (int db = 0; db < D / 32; ++db)
+#pragma unroll
+            for (int b = 0; b < 4; ++b) {
+                bf16x4 o;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) o[j] = (__bf16)(acc[db][4 * b + j] * inv);
+                *(bf16x4*)(orow + db * 32 + 8 * b) = o;
+            }
+        return;
+    }
+    // (the pieces of four whose gates and places are whole pieces too go as such)
+    const bool four = tail.dv % 4 == 0 && tail.out_stride % 4 == 0 && (((unsigned long)out) & 7) == 0 &&
+                      (!tail.gate || (!tail.gate_f32 && tail.gate_stride % 4 == 0 && (((unsigned long)tail.gate) & 7) == 0));
 #pragma unroll
     for (int db = 0; db < D / 32; ++db)
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
-            bf16x4 o;
+            const int d = db * 32 + 8 * b + 4 * g;
+            if (four) {
+                if (d >= tail.dv) continue;
+                float v[4];
 #pragma unroll
-            for (int j = 0; j < 4; ++j) o[j] = (__bf16)(acc[db][4 * b + j] * inv);
-            *(bf16x4*)(orow + db * 32 + 8 * b) = o;
+                for (int j = 0; j < 4; ++j) v[j] = acc[db][4 * b + j] * inv;
+                if (tail.gate) {
+                    float z[4];
+                    Vec4<bf16_t>::load((const bf16_t*)tail.gate + (long)row * tail.gate_stride + (long)head * tail.dv + d, z);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) v[j] *= __builtin_amdgcn_rcpf(1.f + __expf(-z[j]));
+                }
+                Vec4<bf16_t>::store(out + (long)row * tail.out_stride + (long)head * tail.dv + d, v);
+            } else {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) tail.store(out, row, head, d + j, acc[db][4 * b + j] * inv);
+            }
         }
 }
 
@@ -115,7 +143,7 @@ __global__ __launch_bounds__(256 * NG, NG == 1 ? 2 : 1) void attention_prefill_k
     const int* __restrict__ tiles, const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks,
     int Hq, int Hkv, int P, int log2P, float scale_log2, int window, int R, int seg_param, int keys_row,
-    float* __restrict__ part, int keep_first, int sink, float cap_in, float cap_out) {
+    float* __restrict__ part, int keep_first, int sink, float cap_in, float cap_out, AttnTail tail) {
     constexpr int KROW = D * 2 + 16;                 // bytes of a staged key row
     constexpr int KBYTES = 32 * KROW, VBYTES = 2 * D * VROW, BUF = KBYTES + VBYTES;
     constexpr int KP = 32 * (D / 8) / 256;           // 16-byte key pieces per thread (2 for D = 128)
@@ -428,9 +456,9 @@ __global__ __launch_bounds__(256 * NG, NG == 1 ? 2 : 1) void attention_prefill_k
         }
         return;
     }
-    // (sink: one more entry of score 0 that carries no value; m is the scaled reference of the weights)
-    if (sink) l += __builtin_amdgcn_exp2f(fminf(-m, 126.f));
-    if (col_ok) store_columns<D>(out, acc, 1.f / l, row, head, Hq, g);
+    // (sink: one more entry that carries no value; m is the scaled reference of the weights)
+    if (sink) l += __builtin_amdgcn_exp2f(fminf(tail.sink_of(head) * 1.4426950408889634f - m, 126.f));
+    if (col_ok) store_columns<D>(out, acc, 1.f / l, row, head, g, tail);
 }
 
 // The segments' partial results of the blocks that left some: the same first two grid dimensions
@@ -439,7 +467,7 @@ __global__ __launch_bounds__(256 * NG, NG == 1 ? 2 : 1) void attention_prefill_k
 template <int D>
 __global__ __launch_bounds__(256) void attention_prefill_merge_kernel(
     const float* __restrict__ part, bf16_t* __restrict__ out, const int* __restrict__ tiles,
-    const int* __restrict__ positions, int Hq, int Hkv, int window, int R, int seg_param, int keys_row) {
+    const int* __restrict__ positions, int Hq, int Hkv, int window, int R, int seg_param, int keys_row, AttnTail tail) {
     constexpr int NV = 2 + (D / 32) * 16;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 5, r = lane & 31;
     const int G = Hq / Hkv, GH = 32 / R;
@@ -480,13 +508,16 @@ __global__ __launch_bounds__(256) void attention_prefill_merge_kernel(
         for (int e = 0; e < 16; ++e) acc[e] += wgt * src[z * zstride + (2 + db * 16 + e) * 64];
     }
     const float inv = 1.f / l;
-    bf16_t* orow = out + ((long)row * Hq + head) * D + 4 * g + db * 32;
+    bf16_t* orow = out + (long)row * tail.out_stride + (long)head * D + 4 * g + db * 32;
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
         bf16x4 o;
 #pragma unroll
         for (int j = 0; j < 4; ++j) o[j] = (__bf16)(acc[4 * b + j] * inv);
-        *(bf16x4*)(orow + 8 * b) = o;
+        if (tail.plain) *(bf16x4*)(orow + 8 * b) = o;
+        else
+#pragma unroll
+            for (int j = 0; j < 4; ++j) tail.store(out, row, head, db * 32 + 8 * b + 4 * g + j, acc[4 * b + j] * inv);
     }
 }
 
@@ -573,7 +604,7 @@ int qe_attention_prefill(const void* q, void* out, const void* cache, const int*
                          const int* positions, const int* tok_seq, const int* block_table, int max_blocks,
                          int Hq, int Hkv, int D, int P, float scale, int window, int groups,
                          int seg_keys, int max_keys, int keys_row, void* workspace, size_t workspace_bytes,
-                         hipStream_t stream, int keep_first, int sink, float softcap) {
+                         hipStream_t stream, int keep_first, int sink, float softcap, const AttnTail& tail) {
     QE_REQUIRE(seg_keys == 0 || (keep_first == 0 && !sink),
                "prefill attention: kept first keys and a sink go with uncut walks only");
     QE_REQUIRE((D == 64 || D == 128) && P >= 16 && (P & (P - 1)) == 0 && Hq % Hkv == 0,
@@ -612,7 +643,7 @@ int qe_attention_prefill(const void* q, void* out, const void* cache, const int*
     attention_prefill_kernel<D_, NG_, CAP_><<<grid, 256 * NG_, 0, stream>>>(                        \
         (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, tiles, positions, tok_seq, block_table, \
         max_blocks, Hq, Hkv, P, log2P, scale_log2, window, R, seg_keys, keys_row, (float*)workspace, keep_first, sink, \
-        cap_in, cap_out)
+        cap_in, cap_out, tail)
 #define QE_PREFILL(D_, NG_) do { if (softcap > 0.f) QE_PREFILL_CAP(D_, NG_, true); else QE_PREFILL_CAP(D_, NG_, false); } while (0)
     if (D == 128) { if (groups == 2) QE_PREFILL(128, 2); else QE_PREFILL(128, 1); }
     else          { if (groups == 2) QE_PREFILL(64, 2); else QE_PREFILL(64, 1); }
@@ -621,10 +652,10 @@ int qe_attention_prefill(const void* q, void* out, const void* cache, const int*
     if (seg_keys != 0) {
         if (D == 128)
             attention_prefill_merge_kernel<128><<<mgrid, 256, 0, stream>>>((const float*)workspace, (bf16_t*)out, tiles,
-                                                                           positions, Hq, Hkv, window, R, seg_keys, keys_row);
+                                                                           positions, Hq, Hkv, window, R, seg_keys, keys_row, tail);
         else
             attention_prefill_merge_kernel<64><<<mgrid, 256, 0, stream>>>((const float*)workspace, (bf16_t*)out, tiles,
-                                                                          positions, Hq, Hkv, window, R, seg_keys, keys_row);
+                                                                          positions, Hq, Hkv, window, R, seg_keys, keys_row, tail);
     }
     QE_LAUNCH_CHECK();
     return 0;

@@ -86,6 +86,32 @@ template <> struct Vec4<bf16_t> {
     }
 };
 
+// What the attention kernels do with a head's result o[0 .. D) before they store it: only the first dv numbers are
+// stored (a value head smaller than the common head size of the cache), head h of row t at out + t * out_stride +
+// h * dv; with a gate they are multiplied by sigmoid(gate[t * gate_stride + h * dv + d]) first, in 32-bit.  sink: per query
+// head, the score of one more entry of the softmax that carries no value (null: 0, where a sink is asked for at all).
+// plain: nothing of it applies beyond out_stride, and whole 8-byte pieces may be stored.
+struct AttnTail {
+    long out_stride;
+    int dv;
+    int plain;
+    const float* sink;
+    const void* gate;
+    long gate_stride;
+    int gate_f32;
+    __device__ __forceinline__ float sink_of(int head) const { return sink ? sink[head] : 0.f; }
+    __device__ __forceinline__ float gated(float v, long row, int head, int d) const {
+        if (!gate) return v;
+        const long at = row * gate_stride + (long)head * dv + d;
+        const float z = gate_f32 ? ((const float*)gate)[at] : bf16_to_float(((const bf16_t*)gate)[at]);
+        return v / (1.f + __expf(-z));
+    }
+    template <typename TA>
+    __device__ __forceinline__ void store(TA* out, long row, int head, int d, float v) const {
+        if (d < dv) Elem<TA>::store(out + row * out_stride + (long)head * dv + d, gated(v, row, head, d));
+    }
+};
+
 // v of this lane and of its partner across the wave's halves (lane ^ 32) or across odd and even
 // rows of 16 lanes (lane ^ 16), by a swap between two vector registers.  (The two results are
 // taken out of the returned pair into plain integers first: a bit cast applied to an element of

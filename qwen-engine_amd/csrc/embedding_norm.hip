@@ -27,6 +27,72 @@ extern "C" int qe_embedding(const int* ids, const void* table, float* out, int T
     return 0;
 }
 
+// out[t, :] = scale * table[ids[t], :] + pairs[row, :] with row = (prev * mul_prev + ids[t] * mul_cur) mod buckets, prev
+// the token before in the same request; a request's first token (position 0) takes row number `buckets`.  The token before
+// a request's rows in this step is its state (last[slot]), which then takes the request's last token.
+// mode 0: state read only; 2: read and brought up to date (no two rows belong to one request).  One block per token.
+template <typename TW>
+__global__ void embedding_pairs_kernel(const int* __restrict__ ids, const int* __restrict__ positions,
+                                       const int* __restrict__ tok_seq, int* __restrict__ last,
+                                       const TW* __restrict__ table, const TW* __restrict__ pairs, float scale,
+                                       long mul_prev, long mul_cur, long buckets, float* __restrict__ out, int H, int mode) {
+    const long t = blockIdx.x;
+    const int id = ids[t], s = tok_seq[t];
+    long row = buckets;
+    if (positions[t] > 0) {
+        const int prev = (mode == 0 && t > 0 && tok_seq[t - 1] == s) ? ids[t - 1] : last[s];
+        row = (prev * mul_prev + id * mul_cur) % buckets;
+        if (row < 0) row += buckets;
+    }
+    if (mode == 2) {
+        __syncthreads();                                   // (everyone has read the state)
+        if (threadIdx.x == 0) last[s] = id;
+    }
+    const TW* a = table + (long)id * H;
+    const TW* b = pairs + row * H;
+    float* o = out + t * H;
+    if (H % 4 == 0) {
+        for (int c = threadIdx.x * 4; c < H; c += blockDim.x * 4) {
+            float x[4], y[4];
+            Vec4<TW>::load(a + c, x);
+            Vec4<TW>::load(b + c, y);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[e] = fmaf(scale, x[e], y[e]);
+            Vec4<float>::store(o + c, x);
+        }
+    } else {
+        for (int c = threadIdx.x; c < H; c += blockDim.x) o[c] = fmaf(scale, Elem<TW>::load(a + c), Elem<TW>::load(b + c));
+    }
+}
+
+__global__ void embedding_pairs_state_kernel(const int* __restrict__ ids, const int* __restrict__ tok_seq,
+                                             int* __restrict__ last, int T) {
+    const int t = blockIdx.x * blockDim.x + threadIdx.x;
+    if (t < T && (t + 1 == T || tok_seq[t + 1] != tok_seq[t])) last[tok_seq[t]] = ids[t];
+}
+
+extern "C" int qe_embedding_pairs(const int* ids, const int* positions, const int* tok_seq, int* last, const void* table,
+                                  const void* pairs, float scale, long mul_prev, long mul_cur, long buckets, float* out,
+                                  int T, int H, int single_rows, int dt_w, hipStream_t stream) {
+    QE_REQUIRE(T >= 0 && H > 0 && buckets > 0, "embedding_pairs: bad sizes T=%d H=%d buckets=%ld", T, H, buckets);
+    if (T == 0) return 0;
+    const int threads = H >= 1024 ? 256 : (H >= 256 ? 128 : 64);
+    if (dt_w == QE_F32)
+        embedding_pairs_kernel<float><<<T, threads, 0, stream>>>(ids, positions, tok_seq, last, (const float*)table,
+            (const float*)pairs, scale, mul_prev, mul_cur, buckets, out, H, single_rows ? 2 : 0);
+    else if (dt_w == QE_BF16)
+        embedding_pairs_kernel<bf16_t><<<T, threads, 0, stream>>>(ids, positions, tok_seq, last, (const bf16_t*)table,
+            (const bf16_t*)pairs, scale, mul_prev, mul_cur, buckets, out, H, single_rows ? 2 : 0);
+    else
+        QE_REQUIRE(false, "embedding_pairs: unknown table dtype %d", dt_w);
+    QE_LAUNCH_CHECK();
+    if (!single_rows) {
+        embedding_pairs_state_kernel<<<qe_cdiv(T, 256), 256, 0, stream>>>(ids, tok_seq, last, T);
+        QE_LAUNCH_CHECK();
+    }
+    return 0;
+}
+
 // One block per output row r.  src row = rows ? rows[r] : r.
 //   v = h[src] (+ delta_0[src] + delta_1[src] + ...);  if delta and !rows: h[src] = v  (the residual sum, 32-bit)
 //   out[r] = v * rsqrt(mean(v^2) + eps) * w        (all in 32-bit, one rounding at the store)

@@ -104,7 +104,8 @@ extern "C" int qe_gemm_branch_splits(int M, int N, int K, int dt_a, int dt_w) {
 }
 
 // out[M, N] = x[M, K] . w[N, K]^T (+ bias).  epilogue 0: store in dt_o.  1: add into out, the
-// 32-bit stream.  2: w is [2 N, K], gate rows then up rows; out = silu(x.gate^T) * (x.up^T).
+// 32-bit stream.  2: w is [2 N, K], gate rows then up rows; out = silu(x.gate^T) * (x.up^T)
+// (a bias then has 2 N numbers, in the order of w's rows).
 // 3: out is float [splits, M, N], partial products along K to be summed over the first index.
 // 4: as 2 with the gate and up rows of w interleaved in blocks of 32 (gate 0..31, up 0..31, ...);
 //    taken by the kernel for few rows and by the tiled one.

@@ -527,6 +527,11 @@ __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
                     if (SILU) {
                         float gt = acc[i][j][4 * bq + r], up = acc[i][j + (SILU ? 1 : 0)][4 * bq + r];
                         float slope = 1.f;
+                        if (bias) {                        // (as W's rows lie; a column beyond the output is never stored: any bias does)
+                            const int n = no0 + nl + r < NO ? no0 + nl + r : NO - 1, ng = (n / 32) * 64 + n % 32;
+                            gt += bias[ng];
+                            up += bias[ng + 32];
+                        }
                         if (tail.row_w) { gt *= row_w; up *= row_w; }
                         if (tail.act_limit > 0.f) {
                             gt = fminf(gt, tail.act_limit);
@@ -712,7 +717,7 @@ int qe_gemm_mfma(const void* x, const void* w, const float* bias, void* out, int
     QE_REQUIRE(K % 8 == 0 && K >= 64 && K < (1 << 22), "mfma gemm: K=%d is no multiple of 8 in [64, 2^22)", K);
     QE_REQUIRE(tile == 0 || tile == 512 || tile == 256 || tile == 128 || tile == 64 || tile == 65, "mfma gemm: tile of %d rows", tile);
     if (silu) {
-        QE_REQUIRE(!bias && N % 64 == 0, "mfma gemm: silu-mul takes no bias and gate|up rows in blocks of 32");
+        QE_REQUIRE(N % 64 == 0, "mfma gemm: silu-mul takes gate|up rows in blocks of 32");
         if (dt_o == QE_BF16) return pick_mfma<bf16_t, true>(x, w, bias, out, M, N, K, tile, splits, stream);
         return pick_mfma<float, true>(x, w, bias, out, M, N, K, tile, splits, stream);
     }

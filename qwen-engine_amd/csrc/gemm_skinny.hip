@@ -480,7 +480,13 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(
             if (n >= N) continue;
             float y = v[0][i];
             if (SILU) {
-                y = y / (1.f + __expf(-y)) * v[1][i];
+                float up = v[1][i];
+                if (bias) {                              // (as the rows of W lie)
+                    const int ng = EPI == EPI_SILU_MUL_IL ? (n / 32) * 64 + n % 32 : n;
+                    y += bias[ng];
+                    up += bias[ng + (EPI == EPI_SILU_MUL_IL ? 32 : N)];
+                }
+                y = y / (1.f + __expf(-y)) * up;
             } else if (bias && blockIdx.y == 0) {
                 y += bias[n];
             }
@@ -634,12 +640,11 @@ int qe_gemm_skinny(const void* x, const void* w, const float* bias, void* out, i
         return launch_skinny<EPI_RESIDUAL, float>(x, w, bias, out, M, N, K, 1, norm_w, norm_eps, delta, n_delta, h_out, stream);
     }
     if (epilogue == EPI_SILU_MUL) {
-        QE_REQUIRE(!bias, "skinny gemm: silu-mul takes no bias");
         if (dt_o == QE_BF16) return launch_skinny<EPI_SILU_MUL, bf16_t>(x, w, bias, out, M, N, K, 1, norm_w, norm_eps, delta, n_delta, h_out, stream);
         return launch_skinny<EPI_SILU_MUL, float>(x, w, bias, out, M, N, K, 1, norm_w, norm_eps, delta, n_delta, h_out, stream);
     }
     if (epilogue == EPI_SILU_MUL_IL) {
-        QE_REQUIRE(!bias && N % 32 == 0, "skinny gemm: interleaved silu-mul takes no bias and N in blocks of 32");
+        QE_REQUIRE(N % 32 == 0, "skinny gemm: interleaved silu-mul takes N in blocks of 32");
         if (dt_o == QE_BF16) return launch_skinny<EPI_SILU_MUL_IL, bf16_t>(x, w, bias, out, M, N, K, 1, norm_w, norm_eps, delta, n_delta, h_out, stream);
         return launch_skinny<EPI_SILU_MUL_IL, float>(x, w, bias, out, M, N, K, 1, norm_w, norm_eps, delta, n_delta, h_out, stream);
     }

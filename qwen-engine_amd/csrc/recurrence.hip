@@ -3,15 +3,10 @@
 //   qe_token_shift        n blends of every row with the row of the token before it in its request,
 //                         y_s = x + (x' - x) * mu_s; what lies before a request's rows in this step comes from
 //                         its state row (zeros for a new request), which then takes the request's last row
-//   qe_linear_recurrence  per head, with a state S [D][Dv] in 32-bit:
-//                           mode 0 (one decay per head):  S <- decay_h S + k_t v_t^T;   o_t = S^T q_t
-//                           mode 1 (a decay per key channel, a bonus for the token itself):
-//                                 o_t = (S + diag(u) k_t v_t^T)^T q_t;   S <- diag(w_t) S + k_t v_t^T
-//                                 with w_t = exp(-exp(x_t + w0)) from the projected x_t
-//                           mode 2 (a forget gate per key channel that also decides what is written):
-//                                 S <- diag(f_t) S + (1 - f_t) v_t^T;   o_t = S^T q_t
-//                                 with f_t = l + (1 - l) sigmoid(z_t + b) from the projected z_t
-//   qe_recurrence_single  the same for rows that are each the only row of their request, the norm per head inside
+//   qe_linear_recurrence  per head, with a state S [D][Dv] in 32-bit, the recurrences listed at Rec
+//                         (recurrence_gates.h): one decay a head, a decay per key channel, a forget gate that also decides
+//                         what is written, decays formed beforehand per channel or per row and head, a normaliser beside S
+//   qe_recurrence_single  the same for rows that are each the only row of their request, the norm per head and the gate inside
 //   qe_gated_norm         y = o / rms(o) * weight * act(gate) * scale, the root mean square over each of
 //                         `groups` equal pieces of a row (one: the whole row)
 //
@@ -72,33 +67,37 @@ extern "C" int qe_token_shift(const void* x, const float* mu, int n, float* stat
 #define REC_DG 4
 
 template <typename TA, int DPG, int MODE>
-__global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
-    const TA* __restrict__ q, const TA* __restrict__ k, const TA* __restrict__ v, long row_stride,
-    const float* __restrict__ wx, long w_stride, const float* __restrict__ w0, const float* __restrict__ u,
-    const float* __restrict__ decay, int act_silu, float* __restrict__ state, long state_stride,
-    const int* __restrict__ tok_seq, float* __restrict__ out, int T, int H, int D, int Dv) {
-    // (MODE 2: k holds the forget gate's logits, w0 its bias, u its lower bound; act_silu means q alone)
+__global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(Rec a) {
     const int t0 = blockIdx.x;
+    const int* __restrict__ tok_seq = a.tok_seq;
     const int seq = tok_seq[t0];
     if (t0 > 0 && tok_seq[t0 - 1] == seq) return;          // not a request's first row (the whole block leaves)
-    const int h = blockIdx.y;
+    const int T = a.T, H = a.H, D = a.D, Dv = a.Dv;
+    const int h = blockIdx.y, hk = h / (H / a.Hk);
     const int tid = threadIdx.x, vl = tid & 63, dg = tid >> 6;
     const int col = blockIdx.z * 64 + vl;
     const bool col_ok = col < Dv;
     const int d0 = dg * DPG;
+    const TA* __restrict__ q = (const TA*)a.q + (long)hk * D;
+    const TA* __restrict__ k = (const TA*)a.k + (long)hk * D;
+    const TA* __restrict__ v = (const TA*)a.v + (long)h * Dv;
     constexpr int DP = DPG * REC_DG;                        // channels with the padding
     __shared__ float sq[REC_TB][DP], sk[REC_TB][DP], sw[REC_TB][DP];
     __shared__ float part[REC_TB][REC_DG][64];
+    __shared__ float den[MODE == 5 ? REC_TB : 1][REC_DG];
 
-    float S[DPG], uu[DPG];
-    float* Sp = state + (long)seq * state_stride + ((long)h * D) * Dv + col;
+    float S[DPG], uu[DPG], nn[MODE == 5 ? DPG : 1];
+    float* slot = a.state + (long)seq * a.state_stride;
+    float* Sp = slot + ((long)h * D) * Dv + col;
+    float* np = slot + (long)H * D * Dv + ((long)blockIdx.z * H + h) * D;        // (mode 5: this block's copy of n)
 #pragma unroll
     for (int i = 0; i < DPG; ++i) {
         const int d = d0 + i;
         S[i] = (col_ok && d < D) ? Sp[(long)d * Dv] : 0.f;
-        uu[i] = (MODE == 1 && d < D) ? u[h * D + d] : 0.f;
+        uu[i] = (MODE == 1 && d < D) ? a.u[h * D + d] : 0.f;
+        if (MODE == 5) nn[i] = d < D ? np[d] : 0.f;
     }
-    const float dec = MODE == 0 ? decay[h] : 0.f;
+    const float dec = MODE == 0 ? a.decay[h] : 0.f;
 
     int tb = t0;
     bool more = true;
@@ -110,30 +109,33 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
         __syncthreads();                                     // (the batch before has been read)
         for (int i = tid; i < nb * DP; i += REC_DG * 64) {
             const int tt = i / DP, d = i - tt * DP;
-            float a = 0.f, b = 0.f, c = 0.f;
+            float x = 0.f, y = 0.f, c = 0.f;
             if (d < D) {
-                const long r = (long)(tb + tt) * row_stride + h * D + d;
-                a = Elem<TA>::load(q + r);
-                b = Elem<TA>::load(k + r);
-                if (act_silu) { a = silu_f(a); if (MODE != 2) b = silu_f(b); }
-                if (MODE == 2) { const float z = b + w0[h * D + d]; forget_gate(z, u[h * D + d], c, b); }
-                if (MODE == 1) c = expf(-expf(wx[(long)(tb + tt) * w_stride + h * D + d] + w0[h * D + d]));
+                const long r = (long)(tb + tt) * a.row_stride + d, wr = (long)(tb + tt) * a.w_stride;
+                x = Elem<TA>::load(q + r);
+                y = Elem<TA>::load(k + r);
+                if (a.act_silu) { x = silu_f(x); if (MODE != 2) y = silu_f(y); }
+                x *= a.q_scale;
+                if (MODE == 2) { const float z = y + a.w0[h * D + d]; forget_gate(z, a.u[h * D + d], c, y); }
+                if (MODE == 1) c = expf(-expf(a.wx[wr + h * D + d] + a.w0[h * D + d]));
+                if (MODE == 3) c = a.wx[wr + h * D + d];
+                if (MODE >= 4) { c = a.wx[wr + h]; y *= a.ks[wr + h]; }
             }
-            sq[tt][d] = a; sk[tt][d] = b; sw[tt][d] = c;
+            sq[tt][d] = x; sk[tt][d] = y; sw[tt][d] = c;
         }
         float vv[REC_TB];
 #pragma unroll
         for (int tt = 0; tt < REC_TB; ++tt) {
             vv[tt] = 0.f;
             if (tt < nb && col_ok) {
-                vv[tt] = Elem<TA>::load(v + (long)(tb + tt) * row_stride + (long)h * Dv + col);
-                if (act_silu && MODE != 2) vv[tt] = silu_f(vv[tt]);
+                vv[tt] = Elem<TA>::load(v + (long)(tb + tt) * a.row_stride + col);
+                if (a.act_silu && MODE != 2) vv[tt] = silu_f(vv[tt]);
             }
         }
         __syncthreads();
 #pragma unroll
         for (int tt = 0; tt < REC_TB; ++tt) {
-            float o = 0.f;
+            float o = 0.f, dn = 0.f;
             if (tt < nb) {
                 const float vt = vv[tt];
 #pragma unroll
@@ -142,16 +144,21 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
                     if (MODE == 0) {
                         S[i] = fmaf(dec, S[i], kv);
                         o = fmaf(sq[tt][d0 + i], S[i], o);
-                    } else if (MODE == 2) {
-                        S[i] = fmaf(sw[tt][d0 + i], S[i], kv);
-                        o = fmaf(sq[tt][d0 + i], S[i], o);
-                    } else {
+                    } else if (MODE == 1) {
                         o = fmaf(sq[tt][d0 + i], fmaf(uu[i], kv, S[i]), o);
                         S[i] = fmaf(sw[tt][d0 + i], S[i], kv);
+                    } else {
+                        S[i] = fmaf(sw[tt][d0 + i], S[i], kv);
+                        o = fmaf(sq[tt][d0 + i], S[i], o);
+                    }
+                    if (MODE == 5) {
+                        nn[i] = fmaf(sw[tt][d0 + i], nn[i], sk[tt][d0 + i]);
+                        dn = fmaf(sq[tt][d0 + i], nn[i], dn);
                     }
                 }
             }
             part[tt][dg][vl] = o;
+            if (MODE == 5 && vl == 0) den[tt][dg] = dn;
         }
         __syncthreads();
         for (int i = tid; i < nb * 64; i += REC_DG * 64) {
@@ -160,7 +167,13 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
                 float o = part[tt][0][c];
 #pragma unroll
                 for (int g = 1; g < REC_DG; ++g) o += part[tt][g][c];
-                out[((long)(tb + tt) * H + h) * Dv + blockIdx.z * 64 + c] = o;
+                if (MODE == 5) {
+                    float dn = den[tt][0];
+#pragma unroll
+                    for (int g = 1; g < REC_DG; ++g) dn += den[tt][g];
+                    o /= fmaxf(fabsf(dn), a.fl[(long)(tb + tt) * a.w_stride + h]) + 1e-6f;
+                }
+                a.out[((long)(tb + tt) * H + h) * Dv + blockIdx.z * 64 + c] = o;
             }
         }
         tb += nb;
@@ -169,33 +182,31 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(
     for (int i = 0; i < DPG; ++i) {
         const int d = d0 + i;
         if (col_ok && d < D) Sp[(long)d * Dv] = S[i];
+        if (MODE == 5 && vl == 0 && d < D) np[d] = nn[i];
     }
 }
 
-// q, k: row t at + t * row_stride, H * D numbers; v likewise (v's own pointer), H * Dv numbers.  mode 1: q is what
-// multiplies the state (the receptance), wx float32 [T, w_stride] the decays before their exponentials, w0 and u float32
-// [H * D]; mode 0: decay float32 [H]; mode 2: k the forget gate's logits, w0 their bias, u the gate's lower bound
-// (float32 [H * D]).  act_silu: q, k and v (mode 2: q) pass silu first.  state: row tok_seq[t] at
-// + tok_seq[t] * state_stride, H * D * Dv floats.  out float32 [T, H, Dv].
-extern "C" int qe_linear_recurrence(const void* q, const void* k, const void* v, long row_stride, const float* wx,
-                                    long w_stride, const float* w0, const float* u, const float* decay, int mode,
-                                    int act_silu, float* state, long state_stride, const int* tok_seq, float* out,
-                                    int T, int H, int D, int Dv, int dt_a, hipStream_t stream) {
-    QE_REQUIRE(T >= 0 && H > 0 && D > 0 && Dv > 0, "linear_recurrence: bad sizes");
-    QE_REQUIRE(D <= 256, "linear_recurrence: heads of %d key channels (at most 256)", D);
-    QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "linear_recurrence: mode %d lacks operands", mode);
-    QE_REQUIRE(state_stride >= (long)H * D * Dv, "linear_recurrence: state rows overlap");
-    if (T == 0) return 0;
-    dim3 grid(T, H, (Dv + 63) / 64);
-    const int dpg = D <= 32 ? 8 : (D <= 64 ? 16 : (D <= 128 ? 32 : 64));
-#define QE_LR3(TA_, DPG_, MODE_) linear_recurrence_kernel<TA_, DPG_, MODE_><<<grid, REC_DG * 64, 0, stream>>>(              \
-        (const TA_*)q, (const TA_*)k, (const TA_*)v, row_stride, wx, w_stride, w0, u, decay, act_silu, state, \
-        state_stride, tok_seq, out, T, H, D, Dv)
-#define QE_LR2(TA_, DPG_) do { if (mode == 0) QE_LR3(TA_, DPG_, 0); else if (mode == 1) QE_LR3(TA_, DPG_, 1); else QE_LR3(TA_, DPG_, 2); } while (0)
-#define QE_LR(TA_) do { if (dpg == 8) QE_LR2(TA_, 8); else if (dpg == 16) QE_LR2(TA_, 16); else if (dpg == 32) QE_LR2(TA_, 32); else QE_LR2(TA_, 64); } while (0)
-    if (dt_a == QE_F32) QE_LR(float);
-    else if (dt_a == QE_BF16) QE_LR(bf16_t);
-    else QE_REQUIRE(false, "linear_recurrence: unknown element type %d", dt_a);
+// Row by row; out float32 [T, H, Dv] (norm_w is not looked at).
+extern "C" int qe_linear_recurrence(const Rec* rec, hipStream_t stream) {
+    const Rec& a = *rec;
+    QE_REC_CHECK(a, "linear_recurrence");
+    QE_REQUIRE(a.out, "linear_recurrence: no place for the outputs");
+    if (a.T == 0) return 0;
+    dim3 grid(a.T, a.H, rec_copies(a.Dv));
+    const int dpg = a.D <= 32 ? 8 : (a.D <= 64 ? 16 : (a.D <= 128 ? 32 : 64));
+#define QE_LR3(TA_, DPG_, MODE_) linear_recurrence_kernel<TA_, DPG_, MODE_><<<grid, REC_DG * 64, 0, stream>>>(a)
+#define QE_LR2(TA_, DPG_)                                                                                     \
+    switch (a.mode) {                                                                                         \
+        case 0: QE_LR3(TA_, DPG_, 0); break;                                                                  \
+        case 1: QE_LR3(TA_, DPG_, 1); break;                                                                  \
+        case 2: QE_LR3(TA_, DPG_, 2); break;                                                                  \
+        case 3: QE_LR3(TA_, DPG_, 3); break;                                                                  \
+        case 4: QE_LR3(TA_, DPG_, 4); break;                                                                  \
+        default: QE_LR3(TA_, DPG_, 5);                                                                        \
+    }
+#define QE_LR(TA_) do { if (dpg == 8) QE_LR2(TA_, 8) else if (dpg == 16) QE_LR2(TA_, 16) else if (dpg == 32) QE_LR2(TA_, 32) else QE_LR2(TA_, 64) } while (0)
+    if (a.dt_a == QE_F32) QE_LR(float);
+    else QE_LR(bf16_t);
 #undef QE_LR
 #undef QE_LR2
 #undef QE_LR3
@@ -203,29 +214,28 @@ extern "C" int qe_linear_recurrence(const void* q, const void* k, const void* v,
     return 0;
 }
 
-// ---- single new tokens, the norm per head behind the recurrence inside --------------------------------------------
+// ---- single new tokens, the norm per head and the gate behind the recurrence inside ---------------------------------
 // A block per (row, head); every row is the only row of its request.  A thread holds V neighbouring value columns and
 // every RG-th key channel: its state numbers are all asked for before the gates are formed, so that one trip to memory
 // serves both.  The outputs' shares are added in the order of the row groups; then the head's root mean square, the
-// weight and the rounding.
+// weight, the gate and the rounding.
 #define RS_THREADS 512
 #define RS_HOLD 16       // state pieces a thread asks for ahead
 
-template <typename TA, typename TO, int MODE, int V>
-__global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(
-    const TA* __restrict__ q, const TA* __restrict__ k, const TA* __restrict__ v, long row_stride,
-    const float* __restrict__ wx, long w_stride, const float* __restrict__ w0, const float* __restrict__ u,
-    const float* __restrict__ decay, int act_silu, float* __restrict__ state, long state_stride,
-    const int* __restrict__ tok_seq, const float* __restrict__ weight, float eps, TO* __restrict__ y, int H, int D, int Dv) {
+template <typename TA, int MODE, int V>
+__global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
     extern __shared__ float sm[];                            // q, k, f, bonus of D channels, then RG x Dv shares
-    __shared__ float red[16];
+    __shared__ float red[16], red2[16];
+    const int H = a.H, D = a.D, Dv = a.Dv;
     float* sq = sm, * sk = sm + D, * sf = sm + 2 * D, * sb = sm + 3 * D, * part = sm + 4 * D;
     const long t = blockIdx.x;
-    const int h = blockIdx.y, tid = threadIdx.x;
+    const int h = blockIdx.y, hk = h / (H / a.Hk), tid = threadIdx.x;
     const int cols = Dv / V, RG = RS_THREADS / cols;
     const int rg = tid / cols, col = (tid - rg * cols) * V;
     const bool on = rg < RG;
-    float* Sp = state + (long)tok_seq[t] * state_stride + (long)h * D * Dv;
+    float* slot = a.state + (long)a.tok_seq[t] * a.state_stride;
+    float* Sp = slot + (long)h * D * Dv;
+    const TA* vp = (const TA*)a.v + t * a.row_stride + (long)h * Dv;
     auto load = [&](const float* p, float (&x)[V]) {
         if constexpr (V == 4) Vec4<float>::load(p, x);
         else x[0] = *p;
@@ -239,15 +249,28 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(
 #pragma unroll
         for (int i = 0; i < RS_HOLD; ++i) load(Sp + (long)min(rg + i * RG, D - 1) * Dv + col, S[i]);
     }
+    const float gate0 = a.gate && tid < Dv ? rec_gate(a, t, h * Dv + tid) : 0.f;      // (the first of a thread's columns)
     for (int d = tid; d < D; d += RS_THREADS) {
-        const long at = t * row_stride + h * D + d;
-        float a = Elem<TA>::load(q + at), b = Elem<TA>::load(k + at), f = 0.f;
-        if (act_silu) { a = silu_f(a); if (MODE != 2) b = silu_f(b); }
-        if (MODE == 0) f = decay[h];
-        if (MODE == 1) f = expf(-expf(wx[t * w_stride + h * D + d] + w0[h * D + d]));
-        if (MODE == 2) { const float z = b + w0[h * D + d]; forget_gate(z, u[h * D + d], f, b); }
-        sq[d] = a; sk[d] = b; sf[d] = f;
-        if (MODE == 1) sb[d] = u[h * D + d];
+        const long at = t * a.row_stride + (long)hk * D + d;
+        float x = Elem<TA>::load((const TA*)a.q + at), y = Elem<TA>::load((const TA*)a.k + at), f = 0.f;
+        if (a.act_silu) { x = silu_f(x); if (MODE != 2) y = silu_f(y); }
+        x *= a.q_scale;
+        if (MODE == 0) f = a.decay[h];
+        if (MODE == 1) f = expf(-expf(a.wx[t * a.w_stride + h * D + d] + a.w0[h * D + d]));
+        if (MODE == 2) { const float z = y + a.w0[h * D + d]; forget_gate(z, a.u[h * D + d], f, y); }
+        if (MODE == 3) f = a.wx[t * a.w_stride + h * D + d];
+        if (MODE >= 4) { f = a.wx[t * a.w_stride + h]; y *= a.ks[t * a.w_stride + h]; }
+        sq[d] = x; sk[d] = y; sf[d] = f;
+        if (MODE == 1) sb[d] = a.u[h * D + d];
+    }
+    float dn = 0.f;
+    if (MODE == 5) {                                         // (a thread's own channels: no barrier needed)
+        const float* np = slot + (long)H * D * Dv + (long)h * D;
+        for (int d = tid; d < D; d += RS_THREADS) {
+            const float n = fmaf(sf[d], np[d], sk[d]);
+            dn = fmaf(sq[d], n, dn);
+            sb[d] = n;
+        }
     }
     float vv[V], o[V];
 #pragma unroll
@@ -255,8 +278,8 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(
         o[e] = 0.f;
         vv[e] = 0.f;
         if (on) {
-            vv[e] = Elem<TA>::load(v + t * row_stride + (long)h * Dv + col + e);
-            if (act_silu && MODE != 2) vv[e] = silu_f(vv[e]);
+            vv[e] = Elem<TA>::load(vp + col + e);
+            if (a.act_silu && MODE != 2) vv[e] = silu_f(vv[e]);
         }
     }
     __syncthreads();
@@ -285,45 +308,63 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(
         }
         store(part + rg * Dv + col, o);
     }
+    float inv = 1.f;
+    if (MODE == 5) {
+        const int copies = rec_copies(Dv);
+        for (int d = tid; d < D; d += RS_THREADS)
+            for (int z = 0; z < copies; ++z) slot[(long)H * D * Dv + ((long)z * H + h) * D + d] = sb[d];
+        dn = block_sum(dn, red2);
+        inv = 1.f / (fmaxf(fabsf(dn), a.fl[t * a.w_stride + h]) + 1e-6f);
+    }
     __syncthreads();
     float all = 0.f;
     for (int c = tid; c < Dv; c += RS_THREADS) {
         float x = 0.f;
         for (int i = 0; i < RG; ++i) x += part[i * Dv + c];
+        if (MODE == 5) x *= inv;
         part[c] = x;                                         // (this thread alone reads and writes column c)
         all = fmaf(x, x, all);
     }
-    const float rs = rsqrtf(block_sum(all, red) / (float)Dv + eps);
-    for (int c = tid; c < Dv; c += RS_THREADS)
-        Elem<TO>::store(y + (t * H + h) * Dv + c, part[c] * rs * weight[h * Dv + c]);
+    if (!a.norm_w) {
+        for (int c = tid; c < Dv; c += RS_THREADS) a.out[(t * H + h) * Dv + c] = part[c];
+        return;
+    }
+    const float rs = rsqrtf(block_sum(all, red) / (float)Dv + a.norm_eps) * a.y_scale;
+    for (int c = tid; c < Dv; c += RS_THREADS) {
+        float x = part[c] * rs * a.norm_w[h * Dv + c];
+        if (a.gate) x *= gate_value(c == tid ? gate0 : rec_gate(a, t, h * Dv + c), a.gate_act);
+        rec_store(a, t, h * Dv + c, x);
+    }
 }
 
 extern "C" int qe_recurrence_single_supported(int D, int Dv) {
     return D > 0 && D <= 256 && Dv > 0 && (Dv % 4 == 0 ? Dv / 4 : Dv) <= RS_THREADS;
 }
 
-// As qe_linear_recurrence for rows that are each the only row of their request, with every head's output divided by its
-// root mean square (eps inside) and multiplied by weight (float32 [H * Dv]): y [T, H * Dv] in dt_y.
-extern "C" int qe_recurrence_single(const void* q, const void* k, const void* v, long row_stride, const float* wx, long w_stride,
-                                    const float* w0, const float* u, const float* decay, int mode, int act_silu, float* state,
-                                    long state_stride, const int* tok_seq, const float* weight, float eps, void* y, int T,
-                                    int H, int D, int Dv, int dt_a, int dt_y, hipStream_t stream) {
-    QE_REQUIRE(T >= 0 && H > 0 && H <= 65535, "recurrence_single: bad sizes");
-    QE_REQUIRE(qe_recurrence_single_supported(D, Dv), "recurrence_single: heads of %d x %d", D, Dv);
-    QE_REQUIRE(mode == 0 ? decay != nullptr : (w0 && u && (mode == 2 || (mode == 1 && wx))), "recurrence_single: mode %d lacks operands", mode);
-    QE_REQUIRE(state_stride >= (long)H * D * Dv && weight, "recurrence_single: state rows overlap, or no weight");
-    if (T == 0) return 0;
-    const bool four = Dv % 4 == 0 && state_stride % 4 == 0 && (((unsigned long)state) & 15) == 0;
-    QE_REQUIRE(four || Dv <= RS_THREADS, "recurrence_single: heads of %d x %d", D, Dv);
-    const int cols = four ? Dv / 4 : Dv, RG = RS_THREADS / cols;
-    const size_t lds = (size_t)(4 * D + RG * Dv) * sizeof(float);
-#define QE_RS4(TA_, TO_, M_, V_) recurrence_single_kernel<TA_, TO_, M_, V_><<<dim3(T, H), RS_THREADS, lds, stream>>>((const TA_*)q, (const TA_*)k, (const TA_*)v, row_stride, wx, w_stride, w0, u, decay, act_silu, state, state_stride, tok_seq, weight, eps, (TO_*)y, H, D, Dv)
-#define QE_RS3(TA_, TO_, M_) do { if (four) QE_RS4(TA_, TO_, M_, 4); else QE_RS4(TA_, TO_, M_, 1); } while (0)
-#define QE_RS(TA_, TO_) do { if (mode == 0) QE_RS3(TA_, TO_, 0); else if (mode == 1) QE_RS3(TA_, TO_, 1); else QE_RS3(TA_, TO_, 2); } while (0)
-    if (dt_a == QE_F32 && dt_y == QE_F32) QE_RS(float, float);
-    else if (dt_a == QE_F32 && dt_y == QE_BF16) QE_RS(float, bf16_t);
-    else if (dt_a == QE_BF16 && dt_y == QE_BF16) QE_RS(bf16_t, bf16_t);
-    else QE_REQUIRE(false, "recurrence_single: no kernel from type %d to type %d", dt_a, dt_y);
+// As qe_linear_recurrence for rows that are each the only row of their request; with norm_w the norm and the gate too.
+extern "C" int qe_recurrence_single(const Rec* rec, hipStream_t stream) {
+    const Rec& a = *rec;
+    QE_REC_CHECK(a, "recurrence_single");
+    QE_REQUIRE(qe_recurrence_single_supported(a.D, a.Dv), "recurrence_single: heads of %d x %d", a.D, a.Dv);
+    QE_REQUIRE(a.norm_w || a.out, "recurrence_single: no place for the outputs");
+    if (a.T == 0) return 0;
+    const bool four = a.Dv % 4 == 0 && a.state_stride % 4 == 0 && (((unsigned long)a.state) & 15) == 0;
+    QE_REQUIRE(four || a.Dv <= RS_THREADS, "recurrence_single: heads of %d x %d", a.D, a.Dv);
+    const int cols = four ? a.Dv / 4 : a.Dv, RG = RS_THREADS / cols;
+    const size_t lds = (size_t)(4 * a.D + RG * a.Dv) * sizeof(float);
+#define QE_RS4(TA_, M_, V_) recurrence_single_kernel<TA_, M_, V_><<<dim3(a.T, a.H), RS_THREADS, lds, stream>>>(a)
+#define QE_RS3(TA_, M_) do { if (four) QE_RS4(TA_, M_, 4); else QE_RS4(TA_, M_, 1); } while (0)
+#define QE_RS(TA_)                                  \
+    switch (a.mode) {                               \
+        case 0: QE_RS3(TA_, 0); break;              \
+        case 1: QE_RS3(TA_, 1); break;              \
+        case 2: QE_RS3(TA_, 2); break;              \
+        case 3: QE_RS3(TA_, 3); break;              \
+        case 4: QE_RS3(TA_, 4); break;              \
+        default: QE_RS3(TA_, 5);                    \
+    }
+    if (a.dt_a == QE_F32) QE_RS(float)
+    else QE_RS(bf16_t)
 #undef QE_RS
 #undef QE_RS3
 #undef QE_RS4

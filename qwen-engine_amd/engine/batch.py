@@ -44,3 +44,8 @@ class StepContext:
     # builds once per step and shares between its layers.
     extras: Dict[type, dict] = field(default_factory=dict)
     memo: dict = field(default_factory=dict)
+
+    @property
+    def single_rows(self) -> bool:
+        """Every request of the step brings exactly one token."""
+        return len(self.seqs) == self.num_tokens and all(s.q_len == 1 for s in self.seqs)

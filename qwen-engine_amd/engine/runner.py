@@ -125,7 +125,8 @@ class ModelRunner:
                 self.state.append(None)
             else:
                 # (one slot more than requests: the spare one belongs to the rows that fill a graph up)
-                self.state.append(torch.zeros((max_requests + 1, *need.shape), dtype=torch_dtype(need.dtype), device=dev))
+                dtype = torch.int32 if need.dtype == "int32" else torch_dtype(need.dtype)
+                self.state.append(torch.zeros((max_requests + 1, *need.shape), dtype=dtype, device=dev))
         # per schedule entry: one binding per cache user of its block, in the block's order
         self.bindings = []
         for users in self.plan.entry_users:
@@ -163,6 +164,10 @@ class ModelRunner:
         stateful_ok = all(all(self.plan.user_state[u] is None for u in users) or
                           getattr(model.blocks[e.layer], "graph_safe_with_state", False) is True
                           for users, e in zip(self.plan.entry_users, model.spec.schedule))
+        # (the prologue's users, if it has any, come behind the schedule's entries)
+        for users in self.plan.entry_users[len(model.spec.schedule):]:
+            stateful_ok = stateful_ok and (all(self.plan.user_state[u] is None for u in users) or
+                                           getattr(model.prologue, "graph_safe", False) is True)
         graph_safe = stateful_ok and getattr(model, "graph_safe", True)
         self.use_graphs = (dt == torch.bfloat16 and graph_safe) if use_graphs is None else bool(use_graphs)
         # the part classes that want something prepared for every step (parts.base: step_extras)

@@ -62,14 +62,15 @@ def load_library():
         "qe_attention_prefill_supported": [i32, i32, i32, i32, i32],
         "qe_attention_prefill_rows": [i32, i32],
         "qe_attention_prefill_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, i32, i32,
-                                     i32, vp, i64, vp],
+                                     i32, vp, i64, i64, i32, vp, vp, i64, i32, vp],
         "qe_attention_prefill_plan_segments": [i32, i32, i32],
         "qe_attention_prefill_tiles_run": [vp, i32, i32, vp, i32, vp],
         "qe_attention_prefill_workspace_bytes_for": [i32, i32, i32, i32, i32],
         "qe_attention_prefill_plan": [i32, i32, i32, i32],
         "qe_attention_prefill_plan_uncut_keys": [],
         "qe_attention_prefill_workspace_bytes": [i32, i32, i32, i32, i32, i32],
-        "qe_attention_decode_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, i32, vp, i64, vp],
+        "qe_attention_decode_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, i32, vp, i64,
+                                    i64, i32, vp, vp, i64, i32, vp],
         "qe_attention_decode_fused_run": [vp, vp, vp, vp, i32, vp, vp, vp, i32, vp, vp, vp, vp, f32, vp,
                                           i32, i32, i32, i32, f32, i32, i32, i32, vp, i64, vp],
         "qe_qk_rope_store": [vp, vp, vp, vp, f32, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp],
@@ -77,7 +78,8 @@ def load_library():
         "qe_qk_rope_store_parts_supported": [i32, i32],
         "qe_gemm_partial_preferred": [i32, i32, i32, i32, i32],
         "qe_gemm_branch_splits": [i32, i32, i32, i32, i32],
-        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, vp],
+        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32,
+                         i64, i32, vp, vp, i64, i32, vp],
         "qe_qkv_conv_rope_store": [vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp],
         "qe_scale_f32": [vp, i64, f32, vp],
         "qe_moe_route_biased": [vp, vp, vp, vp, i32, i32, i32, f32, i32, vp, i32, i32, vp],
@@ -90,19 +92,22 @@ def load_library():
         "qe_argmax_static": [vp, vp, i32, i32, vp],
         "qe_sample": [vp, vp, vp, vp, i32, i32, vp],
         "qe_postnorm": [vp, vp, i32, i32, f32, vp, i32, f32, vp, i32, i32, i32, vp],
-        "qe_qkv_norm_store": [vp, i32, vp, vp, i32, f32, i32, i32, f32, vp, vp, i32, vp, vp, i32, vp, vp, vp,
-                              i32, i32, i32, i32, i32, i32, i32, i32, i32, vp],
+        "qe_qkv_norm_store": [vp, i32, vp, vp, i32, f32, i32, i32, f32, vp, vp, i32, vp, vp, i32, i32, f32, vp, vp, vp,
+                              i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp],
         "qe_attention_talk": [vp, vp, i64, f32, vp, vp, vp, vp, i32, vp, i32, vp, i32, vp, i32, i32, i32, i32, i32, i32,
                               f32, i32, i32, vp, i32, vp],
         "qe_attention_talk_splits": [i32, i32],
         "qe_token_shift": [vp, vp, i32, vp, i64, vp, vp, i32, i32, i32, i32, vp],
-        "qe_linear_recurrence_chunked": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, vp, i32, i32, vp, vp, vp, f32, vp, i32,
-                                         i32, i32, i32, i32, vp],
+        "qe_linear_recurrence_chunked": [vp, vp],
         "qe_recurrence_single_supported": [i32, i32],
-        "qe_recurrence_single": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, f32, vp, i32, i32, i32,
-                                 i32, i32, i32, vp],
-        "qe_linear_recurrence": [vp, vp, vp, i64, vp, i64, vp, vp, vp, i32, i32, vp, i64, vp, vp, i32, i32, i32, i32,
-                                 i32, vp],
+        "qe_recurrence_single": [vp, vp],
+        "qe_linear_recurrence": [vp, vp],
+        "qe_memory_gates": [vp, i64, vp, vp, f32, vp, i64, vp, vp, i32, i32, vp, vp, i32, vp],
+        "qe_low_rank_decay": [vp, i64, i32, vp, i32, vp, f32, vp, i32, i32, i32, vp],
+        "qe_conv_steps": [vp, i64, vp, vp, vp, i64, vp, vp, i32, i32, i32, vp, i64, vp, vp, vp, i32, i32, vp, vp, i32, i32, vp],
+        "qe_skip_gate_norm": [vp, vp, i64, vp, vp, i64, vp, f32, vp, i64, i32, i32, i32, i32, i32, i32, vp],
+        "qe_embedding_pairs": [vp, vp, vp, vp, vp, vp, f32, i64, i64, i64, vp, i32, i32, i32, i32, vp],
+        "qe_branch_norm": [vp, vp, i32, f32, i32, vp, f32, f32, vp, i32, vp, f32, vp, i32, i32, i32, vp],
         "qe_gated_norm": [vp, vp, vp, i64, i32, i32, f32, f32, vp, i64, i32, i32, i32, i32, vp],
         "qe_unary": [vp, i32, vp, i32, i64, i32, f32, vp],
         "qe_scaled_sum": [vp, f32, vp, f32, i32, vp, i64, vp],
@@ -221,6 +226,59 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor
     _need(out, "out", torch.float32, (T, H), ids.device)
     _check(lib.qe_embedding(ids.data_ptr(), table.data_ptr(), out.data_ptr(), T, V, H,
                             _DT[table.dtype], _stream()), "embedding")
+    return out
+
+
+def embedding_pairs(ids: torch.Tensor, positions: torch.Tensor, tok_seq: torch.Tensor, last: torch.Tensor, table: torch.Tensor,
+                    pairs: torch.Tensor, scale: float, mul_prev: int, mul_cur: int, single_rows: bool = False) -> torch.Tensor:
+    """out[t] = scale * table[ids[t]] + pairs[(prev * mul_prev + ids[t] * mul_cur) mod B] in 32-bit, pairs [B + 1, H]; prev is the
+    token before in the same request, and a request's first token (position 0) takes row B.  The rows of a request are
+    consecutive; last int32 [slots] holds every request's last token (row tok_seq[t]) and is brought up to date.
+    ``single_rows``: no two rows belong to one request (one launch)."""
+    lib = load_library()
+    _need(ids, "ids", torch.int32, (None,))
+    T, dev = ids.shape[0], ids.device
+    _need(positions, "positions", torch.int32, (T,), dev)
+    _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
+    _need(table, "table", _ACT, (None, None), dev)
+    H = table.shape[1]
+    _need(pairs, "pairs", table.dtype, (None, H), dev)
+    _need(last, "last", torch.int32, None, dev)
+    out = torch.empty((T, H), dtype=torch.float32, device=dev)
+    _check(lib.qe_embedding_pairs(ids.data_ptr(), positions.data_ptr(), tok_seq.data_ptr(), last.data_ptr(), table.data_ptr(),
+                                  pairs.data_ptr(), float(scale), int(mul_prev), int(mul_cur), pairs.shape[0] - 1, out.data_ptr(),
+                                  T, H, int(bool(single_rows)), _DT[table.dtype], _stream()), "embedding_pairs")
+    return out
+
+
+def branch_norm(h: torch.Tensor, branch: torch.Tensor, branch_weight: torch.Tensor, branch_eps: float, mult: float,
+                weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, scale: float = 1.0,
+                rows: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """A branch is normed before it joins the 32-bit stream h [T, H], and the stream behind it:
+      y = scale * (sum of branch)                          branch: [T, H], or float32 [S, T, H] whose parts are added in order
+      h += mult * y / rms(y) * branch_weight               (branch_eps inside the root)
+      out = h / rms(h) * weight                            (eps inside the root; weight None: nothing is returned)
+    With ``rows`` (int32 [R]) only those rows are formed and h stays as it is."""
+    lib = load_library()
+    _need(h, "h", torch.float32, (None, None))
+    T, H = h.shape
+    dev = h.device
+    _need(branch_weight, "branch_weight", torch.float32, (H,), dev)
+    if branch.dim() == 3:
+        _need(branch, "branch", torch.float32, (None, T, H), dev)
+    else:
+        _need(branch, "branch", _ACT, (T, H), dev)
+    n = T
+    if rows is not None:
+        _need(rows, "rows", torch.int32, (None,), dev)
+        n = rows.shape[0]
+    out = None
+    if weight is not None:
+        _need(weight, "weight", torch.float32, (H,), dev)
+        out = torch.empty((n, H), dtype=out_dtype, device=dev)
+    _check(lib.qe_branch_norm(h.data_ptr(), branch.data_ptr(), branch.shape[0] if branch.dim() == 3 else 1, float(scale),
+                              _DT[branch.dtype], branch_weight.data_ptr(), float(branch_eps), float(mult), _ptr(rows), n,
+                              _ptr(weight), float(eps), _ptr(out), _DT[out_dtype], T, H, _stream()), "branch_norm")
     return out
 
 
@@ -414,7 +472,7 @@ def gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
 
     epilogue EPI_RESIDUAL: the product is added into ``out``, the 32-bit stream [M, N].
     epilogue EPI_SILU_MUL: w is [2 N, K] (gate rows, then up rows); the result is
-    silu(x . gate^T) * (x . up^T), [M, N].  EPI_SILU_MUL_IL: the same with the gate and up rows
+    silu(x . gate^T) * (x . up^T), [M, N]; a bias (in w's order of rows, [2 N]) joins before the activation.  EPI_SILU_MUL_IL: the same with the gate and up rows
     interleaved in blocks of 32 (see interleave_gate_up); needs gemm_silu_supported(x, w).
     epilogue EPI_PARTIAL: the product is cut along K into ``splits`` (0: chosen for the shape)
     partial products, returned as float32 [splits, M, N]; their sum over the first index, taken
@@ -455,7 +513,7 @@ def gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
     elif x.dtype == torch.float32 and w.dtype != torch.float32:
         raise KernelError("gemm: 32-bit activations need 32-bit weights")
     if bias is not None:
-        _need(bias, "bias", torch.float32, (N,), x.device)
+        _need(bias, "bias", torch.float32, (w.shape[0],), x.device)
     if epilogue == EPI_RESIDUAL:
         if out is None:
             raise KernelError("gemm: the residual epilogue needs the stream to add into")
@@ -706,14 +764,19 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
               other_tiles: Optional[torch.Tensor] = None, prefill_groups: int = 0,
               max_other_keys: int = 0, prefill_segment_keys: int = -1,
               other_keys_row: Optional[int] = None, shared_keys: Optional[torch.Tensor] = None,
-              keep_first: int = 0, sink: bool = False, chunk: int = 0, softcap: float = 0.0) -> torch.Tensor:
+              keep_first: int = 0, sink=False, chunk: int = 0, softcap: float = 0.0, v_dim: int = 0,
+              gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, Hq, D]; cache [pages, 2, Hkv, P, D] (key tiles [P][D], value tiles transposed [D][P]);
     positions, tok_seq int32 [T]; block_table int32 [B, max_blocks].  Token t sees the keys at
     positions max(0, p - window + 1) .. p of request tok_seq[t] (window 0: all).  The caller
     guarantees that those positions have pages in the table.  With ``keep_first`` the request's first
     keep_first keys are seen as well, wherever the window stands; with ``sink`` the softmax has a 1 added
-    to its denominator (one more entry of score 0 that carries no value).  Both go with uncut walks of the
-    prefill kernel only (no segments of keys).
+    to its denominator (one more entry of score 0 that carries no value); a float32 tensor [Hq] gives that entry's
+    score per head.  Both go with uncut walks of the prefill kernel only (no segments of keys).
+
+    With ``v_dim`` > 0 only the first v_dim numbers of every head's result are written, and ``out`` is [T, Hq * v_dim] (the
+    first columns of wider rows are taken as they are); ``gate`` [T, Hq * v_dim] (likewise), bfloat16 or float32: the result is
+    multiplied by its sigmoid, in 32-bit, before it is rounded.
 
     dec_tokens (int32 rows of q that are the single new token of their request, the largest of
     their positions being max_dec_position) go to the decode kernel where it takes the sizes;
@@ -742,9 +805,30 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
     _need(positions, "positions", torch.int32, (T,), dev)
     _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
     _need(block_table, "block_table", torch.int32, (None, None), dev)
-    if out is None:
-        out = torch.empty_like(q)
-    _need(out, "out", q.dtype, (T, Hq, D), dev)
+    v_dim = int(v_dim)
+    if not 0 <= v_dim <= D:
+        raise KernelError(f"attention: values of {v_dim} numbers in heads of {D}")
+    if v_dim:
+        if out is None:
+            out = torch.empty((T, Hq * v_dim), dtype=q.dtype, device=dev)
+        if out.dtype != q.dtype or out.device != dev:
+            raise KernelError("attention: the result has q's element type")
+        out_stride = _rows_view(out, "out", Hq * v_dim, T)
+    else:
+        if out is None:
+            out = torch.empty_like(q)
+        _need(out, "out", q.dtype, (T, Hq, D), dev)
+        out_stride = Hq * D
+    gate_stride = 0
+    if gate is not None:
+        if gate.dtype not in _ACT or gate.device != dev:
+            raise KernelError("attention: the gate is float32 or bfloat16, on q's device")
+        gate_stride = _rows_view(gate, "gate", Hq * (v_dim or D), T)
+    sinks = None
+    if isinstance(sink, torch.Tensor):
+        _need(sink, "sink", torch.float32, (Hq,), dev)
+        sinks, sink = sink, True
+    tail = (out_stride, v_dim, _ptr(sinks), _ptr(gate), gate_stride, _DT[gate.dtype] if gate is not None else 0)
     if Hq % Hkv:
         raise KernelError(f"attention: {Hq} query heads are no multiple of {Hkv} key/value heads")
     max_blocks = block_table.shape[1]
@@ -767,7 +851,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
         n = T if tokens is None else tokens.shape[0]
         _check(lib.qe_attention(q.data_ptr(), out.data_ptr(), cache.data_ptr(), positions.data_ptr(),
                                 tok_seq.data_ptr(), block_table.data_ptr(), max_blocks, _ptr(tokens), n,
-                                Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap, _DT[q.dtype], _stream()),
+                                Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap, _DT[q.dtype], *tail, _stream()),
                "attention")
 
     if dec_tokens is None and other_tokens is None:
@@ -784,7 +868,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
                                                tok_seq.data_ptr(), block_table.data_ptr(), max_blocks,
                                                _ptr(shared_keys), Hq, Hkv,
                                                D, P, float(scale), int(window), keep_first, sink, softcap, int(max_dec_position),
-                                               DECODE_SPLIT_KEYS, ws.data_ptr(), nbytes, _stream()),
+                                               DECODE_SPLIT_KEYS, ws.data_ptr(), nbytes, *tail, _stream()),
                    "attention (decode)")
         else:
             generic(dec_tokens)
@@ -818,7 +902,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
                                                 positions.data_ptr(), tok_seq.data_ptr(), block_table.data_ptr(),
                                                 max_blocks, Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap,
                                                 int(prefill_groups), seg, max_keys, keys_row, _ptr(ws), nbytes,
-                                                _stream()),
+                                                *tail, _stream()),
                    "attention (prefill)")
         else:
             generic(other_tokens)
@@ -1418,23 +1502,27 @@ def qkv_norm_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, k_dim: 
                    k_weight: Optional[torch.Tensor] = None, qk_eps: float = 0.0, values_from_keys: bool = False,
                    value_norm_eps: Optional[float] = None, v_first: Optional[torch.Tensor] = None,
                    v_blend: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
-                   inv_freq: Optional[torch.Tensor] = None, value_rows: bool = False) -> torch.Tensor:
+                   inv_freq: Optional[torch.Tensor] = None, value_rows: bool = False, rot_pairs: bool = False,
+                   rot_gain: float = 1.0) -> torch.Tensor:
     """From the projected rows qkv [T, Hq k_dim + Hkv k_dim (+ Hkv v_dim)] to q [T, Hq, Dc] and the cache
     [pages, 2, Hkv, P, Dc] (zeros beyond a head's own numbers): q and k normed per head (weights [k_dim]) or
     over the whole projection (weights [Hq k_dim] and [Hkv k_dim]), the values their own projection or the keys
     as projected (``values_from_keys``), each value head divided by its root mean square (``value_norm_eps``),
     then either left in ``v_first`` (float32 [T, Hkv v_dim]; ``v_blend`` None) for later layers or blended with
     it, v <- (1 - v_blend) v + v_blend v_first; the first 2 len(inv_freq) numbers of every q and k head rotated in
-    half-split pairs by positions * inv_freq; k and v written at ``slots`` (page * P + offset; negative: nowhere),
-    value tiles transposed ([Dc][P]) or, with ``value_rows``, as rows ([P][Dc])."""
+    half-split pairs (``rot_pairs``: neighbouring pairs) by positions * inv_freq, sine and cosine times ``rot_gain``; k and v
+    written at ``slots`` (page * P + offset; negative: nowhere),
+    value tiles transposed ([Dc][P]) or, with ``value_rows``, as rows ([P][Dc]).  qkv may be the first columns of wider rows;
+    it has the cache's element type or is float32."""
     lib = load_library()
-    _need(qkv, "qkv", _ACT, (None, None))
+    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.dtype not in _ACT or not qkv.is_cuda:
+        raise KernelError("qkv_norm_store: rows of float32 or bfloat16 on the GPU")
     T, dev = qkv.shape[0], qkv.device
     Hq, Hkv, Dk, Dv = int(num_heads), int(num_kv_heads), int(k_dim), int(v_dim)
     need = Hq * Dk + Hkv * Dk + (0 if values_from_keys else Hkv * Dv)
     if qkv.shape[1] < need:          # (rows may go on behind q | k | v: other outputs of the same product)
         raise KernelError(f"qkv_norm_store: rows of {qkv.shape[1]} numbers, {need} expected")
-    _need(cache, "cache", qkv.dtype, (None, 2, Hkv, None, None), dev)
+    _need(cache, "cache", _ACT if qkv.dtype == torch.float32 else qkv.dtype, (None, 2, Hkv, None, None), dev)
     P, Dc = cache.shape[3], cache.shape[4]
     if qk_norm != QK_NORM_NONE:
         n = (Hq * Dk, Hkv * Dk) if qk_norm == QK_NORM_WHOLE else (Dk, Dk)
@@ -1453,13 +1541,14 @@ def qkv_norm_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, k_dim: 
         _need(inv_freq, "inv_freq", torch.float32, (None,), dev)
         _need(positions, "positions", torch.int32, (T,), dev)
         rot = 2 * inv_freq.shape[0]
-    q = torch.empty((T, Hq, Dc), dtype=qkv.dtype, device=dev)
-    _check(lib.qe_qkv_norm_store(qkv.data_ptr(), qkv.shape[1], _ptr(q_weight), _ptr(k_weight), int(qk_norm), float(qk_eps),
+    q = torch.empty((T, Hq, Dc), dtype=cache.dtype, device=dev)
+    _check(lib.qe_qkv_norm_store(qkv.data_ptr(), qkv.stride(0) if T > 1 else qkv.shape[1], _ptr(q_weight), _ptr(k_weight), int(qk_norm), float(qk_eps),
                                  int(bool(values_from_keys)), int(value_norm_eps is not None),
                                  float(value_norm_eps or 0.0), _ptr(v_blend), _ptr(v_first),
                                  int(v_first is not None and v_blend is None), _ptr(positions), _ptr(inv_freq), rot,
-                                 _ptr(slots), q.data_ptr(), cache.data_ptr(), T, Hq, Hkv, Dk, Dv, Dc, P,
-                                 int(bool(value_rows)), _DT[qkv.dtype], _stream()), "qkv_norm_store")
+                                 int(bool(rot_pairs)), float(rot_gain), _ptr(slots), q.data_ptr(), cache.data_ptr(), T, Hq, Hkv,
+                                 Dk, Dv, Dc, P, int(bool(value_rows)), _DT[qkv.dtype], _DT[cache.dtype], _stream()),
+           "qkv_norm_store")
     return q
 
 
@@ -1565,46 +1654,88 @@ def recurrence_chunks(portions, chunk_len: int):
     return (torch.tensor(chunks, dtype=torch.int32).view(-1, 3), torch.tensor(ports, dtype=torch.int32).view(-1, 3))
 
 
+class _Rec(ctypes.Structure):
+    """The operands of the recurrences' kernels (Rec in csrc/recurrence_gates.h, field by field)."""
+    _fields_ = ([("q", ctypes.c_void_p), ("k", ctypes.c_void_p), ("v", ctypes.c_void_p), ("row_stride", ctypes.c_long),
+                 ("wx", ctypes.c_void_p), ("ks", ctypes.c_void_p), ("fl", ctypes.c_void_p), ("w_stride", ctypes.c_long),
+                 ("w0", ctypes.c_void_p), ("u", ctypes.c_void_p), ("decay", ctypes.c_void_p), ("state", ctypes.c_void_p),
+                 ("state_stride", ctypes.c_long), ("tok_seq", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                 ("norm_w", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y_stride", ctypes.c_long), ("gate", ctypes.c_void_p),
+                 ("gate_stride", ctypes.c_long), ("chunks", ctypes.c_void_p), ("portions", ctypes.c_void_p), ("ws", ctypes.c_void_p)] +
+                [(n, ctypes.c_float) for n in ("norm_eps", "q_scale", "y_scale")] +
+                [(n, ctypes.c_int) for n in ("mode", "act_silu", "dt_a", "dt_y", "dt_g", "gate_act", "T", "H", "Hk", "D", "Dv",
+                                             "n_chunks", "n_portions", "all_single")])
+
+
+def recurrence_state_numbers(heads: int, k_dim: int, v_dim: int, normaliser: bool = False) -> int:
+    """How many 32-bit numbers of state linear_recurrence() keeps per request (with the normaliser beside S: a copy of it per
+    64 value columns)."""
+    return heads * k_dim * (v_dim + ((v_dim + 63) // 64 if normaliser else 0))
+
+
 def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, tok_seq: torch.Tensor,
                       heads: int, decay: Optional[torch.Tensor] = None, decay_x: Optional[torch.Tensor] = None,
                       decay_bias: Optional[torch.Tensor] = None, bonus: Optional[torch.Tensor] = None,
                       silu: bool = False, chunks=None, forget_bias: Optional[torch.Tensor] = None,
                       lower: Optional[torch.Tensor] = None, norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0,
-                      norm_dtype: Optional[torch.dtype] = None, single_rows: bool = False) -> torch.Tensor:
-    """Per head, with a 32-bit state S [D][Dv] per request (state[tok_seq[t]], float32 [slots, >= H D Dv]):
+                      norm_dtype: Optional[torch.dtype] = None, single_rows: bool = False, decays: Optional[torch.Tensor] = None,
+                      steps: Optional[torch.Tensor] = None, normaliser: bool = False, q_scale: float = 1.0, k_heads: int = 0,
+                      gate: Optional[torch.Tensor] = None, gate_act: int = 0, y_scale: float = 1.0,
+                      out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per head, with a 32-bit state S [D][Dv] per request (state[tok_seq[t]], float32 [slots, >= recurrence_state_numbers]):
     with ``decay`` (float32 [H]):  S <- decay_h S + k_t v_t^T, o_t = S^T q_t;
     with ``decay_x`` float32 [T, H D], ``decay_bias`` and ``bonus`` (float32 [H D]):  o_t = (S + diag(bonus) k_t v_t^T)^T q_t,
     then S <- diag(w_t) S + k_t v_t^T with w_t = exp(-exp(decay_x_t + decay_bias)).
     with ``forget_bias`` and ``lower`` (float32 [H D]) k holds the logits of a forget gate f = lower + (1 - lower)
     sigmoid(k + forget_bias):  S <- diag(f_t) S + (1 - f_t) v_t^T, o_t = S^T q_t.
-    q, k [T, H D], v [T, H Dv] (column slices of one wider tensor are taken as they are, all with one row stride);
+    with ``decays`` float32 [T, H D]:  S <- diag(decays_t) S + k_t v_t^T, o_t = S^T q_t.
+    with ``steps`` float32 [T, 2 H] (decays w, key factors c):  S <- w_t S + (c_t k_t) v_t^T, o_t = S^T q_t; with
+    ``normaliser`` steps is [T, 3 H] (and floors b), n <- w_t n + c_t k_t, and o_t is divided by max(|n . q_t|, b_t) + 1e-6.
+    q, k [T, H D] (with ``steps``: ``k_heads`` D, head h using q/k head h // (H / k_heads)), v [T, H Dv] (column slices of one
+    wider tensor are taken as they are, all with one row stride); q is multiplied by ``q_scale``;
     ``silu``: the three (with a forget gate: q) pass silu first.  Returns o float32 [T, H, Dv].
     ``chunks`` (recurrence_chunks() of all rows' portions, on the device): the rows are
     taken chunk by chunk, the chunks in parallel, instead of row by row: for long portions.
     ``norm_weight`` (float32 [H Dv]): every head's o is divided by its root mean square (norm_eps inside) and multiplied
-    by the weight; the result is [T, H Dv] in norm_dtype.  ``single_rows``: no two rows belong to one request (the norm
-    is then part of the one launch)."""
+    by the weight, by act(``gate``) (``gate_act`` GATE_SILU or GATE_SIGMOID; gate [T, H Dv], may be a slice of columns) and by
+    ``y_scale``; the result is [T, H Dv] in norm_dtype (in ``out``, which may be columns of wider rows, if given).
+    ``single_rows``: no two rows belong to one request (everything is then one launch)."""
     lib = load_library()
     T, dev, H = q.shape[0], q.device, int(heads)
+    Hk = int(k_heads) or H
     if q.dtype not in _ACT or k.dtype != q.dtype or v.dtype != q.dtype:
         raise KernelError("linear_recurrence: q, k and v of one element type")
-    D, Dv = q.shape[1] // H, v.shape[1] // H
-    sq, sk, sv = _rows_view(q, "q", H * D, T), _rows_view(k, "k", H * D, T), _rows_view(v, "v", H * Dv, T)
+    D, Dv = q.shape[1] // Hk, v.shape[1] // H
+    sq, sk, sv = _rows_view(q, "q", Hk * D, T), _rows_view(k, "k", Hk * D, T), _rows_view(v, "v", H * Dv, T)
     if T > 1 and not sq == sk == sv:
         raise KernelError("linear_recurrence: q, k and v with different row strides")
+    if T == 1:
+        sq = max(sq, sk, sv)
     _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
-    if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < H * D * Dv or state.stride(1) != 1:
-        raise KernelError("linear_recurrence: the state is float32 [slots, >= H D Dv]")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.device != dev or \
+            state.shape[1] < recurrence_state_numbers(H, D, Dv, normaliser):
+        raise KernelError("linear_recurrence: the state is float32 [slots, >= H D Dv (and the normaliser)]")
     if D < 4:
         chunks = None                # (the chunked kernels read four channels at a time)
     mode, sw = 0, 0
+    wx, ks, fl, w0, u = decay_x, None, None, decay_bias, bonus
     if decay is not None:
         _need(decay, "decay", torch.float32, (H,), dev)
     elif lower is not None:
         mode = 2
         _need(forget_bias, "forget_bias", torch.float32, (H * D,), dev)
         _need(lower, "lower", torch.float32, (H * D,), dev)
-        decay_bias, bonus = forget_bias, lower
+        w0, u = forget_bias, lower
+    elif decays is not None:
+        mode, wx = 3, decays
+        _need(decays, "decays", torch.float32, (T, H * D), dev)
+        sw = H * D
+    elif steps is not None:
+        mode = 5 if normaliser else 4
+        sw = (mode - 2) * H
+        _need(steps, "steps", torch.float32, (T, sw), dev)
+        wx, ks = steps[:, :H], steps[:, H:]
+        fl = steps[:, 2 * H:] if normaliser else None
     else:
         mode = 1
         if decay_x is None or decay_x.dtype != torch.float32:
@@ -1612,46 +1743,157 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         sw = _rows_view(decay_x, "decay_x", H * D, T)
         _need(decay_bias, "decay_bias", torch.float32, (H * D,), dev)
         _need(bonus, "bonus", torch.float32, (H * D,), dev)
-    if norm_weight is not None:
+    normed = norm_weight is not None
+    sg = sy = 0
+    if normed:
         _need(norm_weight, "norm_weight", torch.float32, (H * Dv,), dev)
         norm_dtype = norm_dtype or q.dtype
-        if single_rows and lib.qe_recurrence_single_supported(D, Dv):
-            y = torch.empty((T, H * Dv), dtype=norm_dtype, device=dev)
-            _check(lib.qe_recurrence_single(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw, _ptr(decay_bias),
-                                            _ptr(bonus), _ptr(decay), mode, int(bool(silu)), state.data_ptr(),
-                                            state.stride(0), tok_seq.data_ptr(), norm_weight.data_ptr(), float(norm_eps),
-                                            y.data_ptr(), T, H, D, Dv, _DT[q.dtype], _DT[norm_dtype], _stream()),
-                   "recurrence_single")
-            return y
-    fused_norm = norm_weight is not None and chunks is not None and chunks[0].shape[0] > 0 and Dv <= 128
-    if norm_weight is not None and not fused_norm:
-        o = linear_recurrence(q, k, v, state, tok_seq, heads, decay=decay, decay_x=decay_x,
-                              decay_bias=decay_bias if mode == 1 else None, bonus=bonus if mode == 1 else None, silu=silu,
-                              chunks=chunks, forget_bias=forget_bias, lower=lower)
-        return gated_norm(o.view(T, H * Dv), norm_weight, norm_eps, H, norm_dtype)
+        if gate is not None:
+            if gate.dtype not in _ACT or gate_act not in (GATE_SILU, GATE_SIGMOID):
+                raise KernelError("linear_recurrence: a gate of float32 or bfloat16 with an activation")
+            sg = _rows_view(gate, "gate", H * Dv, T)
+        if out is not None:
+            if out.dtype != norm_dtype or out.device != dev:
+                raise KernelError("linear_recurrence: the result has another element type")
+        else:
+            out = torch.empty((T, H * Dv), dtype=norm_dtype, device=dev)
+        sy = _rows_view(out, "out", H * Dv, T)
+    elif gate is not None or out is not None:
+        raise KernelError("linear_recurrence: a gate, or a place for the result, goes with the norm")
+    use_chunks = chunks is not None and chunks[0].shape[0] > 0
+    single = single_rows and bool(lib.qe_recurrence_single_supported(D, Dv))
+    fused_norm = normed and (single or (use_chunks and Dv <= 128))
+    o = None if fused_norm else torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
+    r = _Rec(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), row_stride=sq, wx=_ptr(wx), ks=_ptr(ks), fl=_ptr(fl), w_stride=sw,
+             w0=_ptr(w0), u=_ptr(u), decay=_ptr(decay), state=state.data_ptr(), state_stride=state.stride(0),
+             tok_seq=tok_seq.data_ptr(), out=_ptr(o), q_scale=float(q_scale), y_scale=float(y_scale), mode=mode,
+             act_silu=int(bool(silu)), dt_a=_DT[q.dtype], T=T, H=H, Hk=Hk, D=D, Dv=Dv)
     if fused_norm:
-        out = torch.empty((T, H * Dv), dtype=norm_dtype, device=dev)
-    else:
-        out = torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
-    if chunks is not None and chunks[0].shape[0]:
+        r.norm_w, r.norm_eps, r.y, r.y_stride, r.dt_y = norm_weight.data_ptr(), float(norm_eps), out.data_ptr(), sy, _DT[out.dtype]
+        if gate is not None:
+            r.gate, r.gate_stride, r.dt_g, r.gate_act = gate.data_ptr(), sg, _DT[gate.dtype], int(gate_act)
+    if single:
+        _check(lib.qe_recurrence_single(ctypes.addressof(r), _stream()), "recurrence_single")
+    elif use_chunks:
         ch, po = chunks
         _need(ch, "chunks", torch.int32, (None, 3), dev)
         _need(po, "portions", torch.int32, (None, 3), dev)
-        all_single = ch.shape[0] == po.shape[0]
-        ws = None if all_single else torch.empty((ch.shape[0] * H * (D * Dv + D),), dtype=torch.float32, device=dev)
-        _check(lib.qe_linear_recurrence_chunked(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw,
-                                                _ptr(decay_bias), _ptr(bonus), _ptr(decay), mode, int(bool(silu)),
-                                                state.data_ptr(), state.stride(0), tok_seq.data_ptr(), ch.data_ptr(),
-                                                ch.shape[0], po.data_ptr(), po.shape[0], int(all_single), _ptr(ws),
-                                                None if fused_norm else out.data_ptr(), _ptr(norm_weight), float(norm_eps),
-                                                out.data_ptr() if fused_norm else None, _DT[out.dtype],
-                                                H, D, Dv, _DT[q.dtype], _stream()), "linear_recurrence (chunked)")
-        return out
-    _check(lib.qe_linear_recurrence(q.data_ptr(), k.data_ptr(), v.data_ptr(), sq, _ptr(decay_x), sw, _ptr(decay_bias),
-                                    _ptr(bonus), _ptr(decay), mode, int(bool(silu)), state.data_ptr(), state.stride(0),
-                                    tok_seq.data_ptr(), out.data_ptr(), T, H, D, Dv, _DT[q.dtype], _stream()),
-           "linear_recurrence")
+        r.n_chunks, r.n_portions, r.all_single = ch.shape[0], po.shape[0], int(ch.shape[0] == po.shape[0])
+        r.chunks, r.portions = ch.data_ptr(), po.data_ptr()
+        ws = None
+        if not r.all_single:
+            ws = torch.empty((ch.shape[0] * H * D * (Dv + (2 if mode == 5 else 1)),), dtype=torch.float32, device=dev)
+            r.ws = ws.data_ptr()
+        _check(lib.qe_linear_recurrence_chunked(ctypes.addressof(r), _stream()), "linear_recurrence (chunked)")
+    else:
+        _check(lib.qe_linear_recurrence(ctypes.addressof(r), _stream()), "linear_recurrence")
+    if not normed:
+        return o
+    if not fused_norm:
+        gated_norm(o.view(T, H * Dv), norm_weight, norm_eps, H, norm_dtype, gate=gate, gate_act=gate_act, scale=float(y_scale), out=out)
     return out
+
+
+def memory_gates(z: torch.Tensor, input_bias: torch.Tensor, forget_bias: torch.Tensor, cap: float, running_max: torch.Tensor,
+                 tok_seq: torch.Tensor, chunks=None) -> torch.Tensor:
+    """The ``steps`` [T, 3 H] of linear_recurrence(normaliser=True) from the logits z float32 [T, 2 H] (input gates, forget gates;
+    columns of wider rows are taken as they are): i = cap tanh((z_i + input_bias) / cap), f = log sigmoid(cap tanh((z_f +
+    forget_bias) / cap)), m_t = max(f + m_(t-1), i); decay exp(f + m_(t-1) - m_t), key factor exp(i - m_t), floor exp(-m_t).
+    running_max float32 [slots, H] (columns of wider rows): m of every request, brought up to date.  ``chunks``: as in
+    linear_recurrence()."""
+    lib = load_library()
+    T, dev = z.shape[0], z.device
+    H = input_bias.shape[0]
+    if z.dtype != torch.float32 or not z.is_cuda:
+        raise KernelError("memory_gates: float32 logits on the GPU")
+    sz = _rows_view(z, "z", 2 * H, T)
+    _need(input_bias, "input_bias", torch.float32, (H,), dev)
+    _need(forget_bias, "forget_bias", torch.float32, (H,), dev)
+    _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
+    if running_max.dtype != torch.float32 or running_max.dim() != 2 or running_max.shape[1] != H or running_max.stride(1) != 1:
+        raise KernelError("memory_gates: the running maximum is float32 [slots, H]")
+    steps = torch.empty((T, 3 * H), dtype=torch.float32, device=dev)
+    ch, po = chunks if chunks is not None else (None, None)
+    _check(lib.qe_memory_gates(z.data_ptr(), sz, input_bias.data_ptr(), forget_bias.data_ptr(), float(cap), running_max.data_ptr(),
+                               running_max.stride(0), tok_seq.data_ptr(), steps.data_ptr(), T, H, _ptr(ch), _ptr(po),
+                               0 if po is None else po.shape[0], _stream()), "memory_gates")
+    return steps
+
+
+def low_rank_decay(low: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
+    """sigmoid(low . w^T + bias)^(1 / tau), float32 [T, N]: low [T, R] (columns of wider rows are taken as they are), w [N, R]."""
+    lib = load_library()
+    T, (N, R) = low.shape[0], w.shape
+    if low.dtype not in _ACT or not low.is_cuda:
+        raise KernelError("low_rank_decay: float32 or bfloat16 rows on the GPU")
+    sl = _rows_view(low, "low", R, T)
+    _need(w, "w", _ACT, (N, R), low.device)
+    _need(bias, "bias", torch.float32, (N,), low.device)
+    out = torch.empty((T, N), dtype=torch.float32, device=low.device)
+    _check(lib.qe_low_rank_decay(low.data_ptr(), sl, _DT[low.dtype], w.data_ptr(), _DT[w.dtype], bias.data_ptr(), float(tau),
+                                 out.data_ptr(), T, N, R, _stream()), "low_rank_decay")
+    return out
+
+
+def conv_steps(x: torch.Tensor, w_t: torch.Tensor, bias: torch.Tensor, state: Optional[torch.Tensor], tok_seq: torch.Tensor,
+               dt: Optional[torch.Tensor] = None, dt_bias: Optional[torch.Tensor] = None, a_log: Optional[torch.Tensor] = None,
+               single_rows: bool = False, chunks=None):
+    """silu(bias + causal convolution over time) of every channel: x [T, C] (columns of wider rows are taken as they are), w_t
+    float32 [taps, C] (the last row is the current token's), state float32 [slots, (taps - 1) C] (columns of wider rows; row
+    tok_seq[t]: the request's last inputs), brought up to date.  With ``dt`` (float32 logits [T, H]): also the step sizes
+    softplus(dt + dt_bias) and the decays exp(-exp(a_log) * step).  Returns (rows [T, C] in x's type, float32 [T, 2 H] = decays,
+    step sizes, or None).  ``single_rows``: no two rows belong to one request (one launch)."""
+    lib = load_library()
+    T, dev = x.shape[0], x.device
+    taps, C = w_t.shape
+    if x.dtype not in _ACT or not x.is_cuda:
+        raise KernelError("conv_steps: float32 or bfloat16 rows on the GPU")
+    sx = _rows_view(x, "x", C, T)
+    _need(w_t, "w_t", torch.float32, (taps, C), dev)
+    _need(bias, "bias", torch.float32, (C,), dev)
+    _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
+    if taps > 1 and (state is None or state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < (taps - 1) * C or
+                     state.stride(1) != 1 or state.device != dev):
+        raise KernelError("conv_steps: the state is float32 [slots, >= (taps - 1) C]")
+    H, sd, steps = 0, 0, None
+    if dt is not None:
+        H = dt_bias.shape[0]
+        if dt.dtype != torch.float32:
+            raise KernelError("conv_steps: float32 step logits")
+        sd = _rows_view(dt, "dt", H, T)
+        _need(dt_bias, "dt_bias", torch.float32, (H,), dev)
+        _need(a_log, "a_log", torch.float32, (H,), dev)
+        steps = torch.empty((T, 2 * H), dtype=torch.float32, device=dev)
+    ch, po = chunks if chunks is not None else (None, None)
+    out = torch.empty((T, C), dtype=x.dtype, device=dev)
+    _check(lib.qe_conv_steps(x.data_ptr(), sx, w_t.data_ptr(), bias.data_ptr(), _ptr(state), 0 if state is None else state.stride(0),
+                             tok_seq.data_ptr(), out.data_ptr(), T, C, taps, _ptr(dt), sd, _ptr(dt_bias), _ptr(a_log), _ptr(steps), H,
+                             int(bool(single_rows)), _ptr(ch), _ptr(po), 0 if po is None else po.shape[0], _DT[x.dtype], _stream()),
+           "conv_steps")
+    return out, steps
+
+
+def skip_gate_norm(o: torch.Tensor, x: torch.Tensor, skip: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float,
+                   groups: int, out_dtype: torch.dtype, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """((o + skip_h x) * silu(z)) divided by the root mean square of each of ``groups`` equal pieces of a row, times the weight:
+    o float32 [T, H, Dv], x and z [T, H Dv] (columns of wider rows are taken as they are), skip float32 [H] -> [T, H Dv]
+    (in ``out``, which may be columns of wider rows, if given)."""
+    lib = load_library()
+    _need(o, "o", torch.float32, (None, None, None))
+    T, H, Dv = o.shape
+    dev = o.device
+    if x.dtype not in _ACT or z.dtype != x.dtype:
+        raise KernelError("skip_gate_norm: x and z of one element type")
+    sx, sz = _rows_view(x, "x", H * Dv, T), _rows_view(z, "z", H * Dv, T)
+    _need(skip, "skip", torch.float32, (H,), dev)
+    _need(weight, "weight", torch.float32, (H * Dv,), dev)
+    y = torch.empty((T, H * Dv), dtype=out_dtype, device=dev) if out is None else out
+    if y.dtype != out_dtype or y.device != dev:
+        raise KernelError("skip_gate_norm: the result has another element type")
+    sy = _rows_view(y, "out", H * Dv, T)
+    _check(lib.qe_skip_gate_norm(o.data_ptr(), x.data_ptr(), sx, skip.data_ptr(), z.data_ptr(), sz, weight.data_ptr(), float(eps),
+                                 y.data_ptr(), sy, T, H, Dv, int(groups), _DT[x.dtype], _DT[out_dtype], _stream()), "skip_gate_norm")
+    return y
 
 
 GATE_NONE, GATE_SILU, GATE_SIGMOID = 0, 1, 2

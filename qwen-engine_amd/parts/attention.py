@@ -450,7 +450,9 @@ class ChunkAttention(PagedAttention):
     attention kernels of PagedAttention with the chunk as their mask (keys and values of different sizes share the
     cache under one head size, ``common_head_dim``), or, with a bias by distance or talking heads, the kernel
     that handles all heads of a token together; then the output projection, whose result stays 32-bit.
-    The values that a layer leaves for later layers of the step travel in ``ctx.memo``."""
+    The values that a layer leaves for later layers of the step travel in ``ctx.memo``.  Without a bias by distance and talking
+    heads it is a projected mixer too (parts.projected): the sink and the output gate are part of the attention kernels.
+    """
     takes_stream = False
     graph_safe = True        # every launch's grid follows the rows alone
 
@@ -474,11 +476,17 @@ class ChunkAttention(PagedAttention):
         self.window = 0
         self.position = build_part(spec.position, hidden_size) if spec.position is not None else None
         self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.q_norm = self.k_norm = None
-        self.blend = self.dist_bias = self.talk = None
+        self.blend = self.dist_bias = self.talk = self.sink = None
+        if self.talks and (spec.head_sink or spec.output_gate):
+            raise ValueError("a bias by distance or talking heads with a sink or an output gate")
 
     @staticmethod
     def _talks(spec) -> bool:
         return bool(spec.distance_bias_rows) or bool(spec.talking_heads)
+
+    @staticmethod
+    def _out_bias(spec) -> bool:
+        return bool(spec.bias if spec.out_bias is None else spec.out_bias)
 
     @staticmethod
     def _cache_head_dim(spec) -> int:
@@ -507,8 +515,12 @@ class ChunkAttention(PagedAttention):
             t[spec.distance_bias_name] = TensorInfo((int(spec.distance_bias_rows), spec.num_heads), "normal", "vector")
         if spec.talking_heads:
             t[spec.talk_name] = TensorInfo((spec.num_heads, spec.num_heads), "normal", "vector")
+        if spec.head_sink:
+            t[spec.sink_name] = TensorInfo((spec.num_heads,), "zeros", "vector")
+        if spec.output_gate:
+            t[spec.gate_name] = TensorInfo((spec.num_heads * spec.v_head_dim, hidden))
         t[no] = TensorInfo((hidden, spec.num_heads * spec.v_head_dim))
-        if spec.bias:
+        if ChunkAttention._out_bias(spec):
             t[no + spec.bias_suffix] = TensorInfo((hidden,), "zeros", "vector")
         return t
 
@@ -521,16 +533,27 @@ class ChunkAttention(PagedAttention):
     def state_need(spec, hidden: int):
         return None
 
-    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+    def _projections(self):
+        """The names of the projections of the mixer's input, in the order of their columns."""
         s = self.spec
-        nq, nk, nv, no = s.names
-        proj = [nq, nk] if s.values_from_keys else [nq, nk, nv]
-        mats = [tensors[n] for n in proj]
-        if len({m.dtype for m in mats}) > 1:
-            mats = [m.float() for m in mats]
-        self.w_qkv = rt.place_matrix(torch.cat(mats, dim=0))
-        if s.bias:
-            self.b_qkv = rt.place_vector(torch.cat([tensors[n + s.bias_suffix].float() for n in proj]))
+        nq, nk, nv, _ = s.names
+        return [nq, nk] + ([] if s.values_from_keys else [nv]) + ([s.gate_name] if s.output_gate else [])
+
+    def inputs(self, tensors: Dict[str, torch.Tensor]):
+        s = self.spec
+        return [(tensors[n], tensors[n + s.bias_suffix] if s.bias and n != s.gate_name else None) for n in self._projections()], []
+
+    def output(self, tensors: Dict[str, torch.Tensor]) -> torch.Tensor:
+        return tensors[self.spec.names[3]]
+
+    @staticmethod
+    def is_projected(spec) -> bool:
+        return not ChunkAttention._talks(spec) and not ChunkAttention._out_bias(spec)
+
+    def load_own(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        s = self.spec
+        nq, nk, _, no = s.names
+        if self._out_bias(s):
             self.b_o = rt.place_vector(tensors[no + s.bias_suffix])
         if s.qk_norm is not None:
             self.q_norm = rt.place_vector(tensors[nq + s.norm_suffix])
@@ -542,51 +565,74 @@ class ChunkAttention(PagedAttention):
                                                                 max_distance=self.chunk - 1 if self.chunk else None))
         if s.talking_heads:
             self.talk = rt.place_vector(tensors[s.talk_name])
-        w_o = tensors[no]
-        if self.talks:               # (that kernel writes a head's own values only)
-            self.w_o = rt.place_matrix(w_o)
-        else:                        # heads of the common size: zero columns beyond a value head's own numbers
-            padded = torch.zeros((self.hidden, self.hq, self.d), dtype=w_o.dtype)
-            padded[:, :, :self.dv] = w_o.view(self.hidden, self.hq, self.dv)
-            self.w_o = rt.place_matrix(padded.view(self.hidden, self.hq * self.d))
+        if s.head_sink:
+            self.sink = rt.place_vector(tensors[s.sink_name])
         if self.position is not None:
             self.position.load({}, rt)
 
-    def forward(self, x: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
-        """x [T, H] in the activation type.  Returns the mixer's output, float32 [T, H]."""
-        if binding.kv is None:
-            raise RuntimeError("attention was given no cache")
+    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        self.load_own(tensors, rt)
+        main, _ = self.inputs(tensors)
+        mats = [m for m, _ in main]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        self.w_qkv = rt.place_matrix(torch.cat(mats, dim=0))
+        if self.spec.bias:
+            self.b_qkv = rt.place_vector(torch.cat([torch.zeros(m.shape[0]) if b is None else b.float() for m, b in main]))
+        self.w_o = rt.place_matrix(self.output(tensors))
+
+    def _store(self, y: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+        """From the projected rows to q [T, Hq, D] and the cache."""
         s = self.spec
-        T, g, cache = x.shape[0], binding.group, binding.kv
-        qkv = ops.gemm(x, self.w_qkv, self.b_qkv)
+        T = y.shape[0]
         v_first = None
         if s.value_blend is not None:
             key = ("chunk_attention.values", self.hkv * self.dv)
             if s.value_blend == "source":
-                v_first = ctx.memo[key] = torch.empty((T, self.hkv * self.dv), dtype=torch.float32, device=x.device)
+                v_first = ctx.memo[key] = torch.empty((T, self.hkv * self.dv), dtype=torch.float32, device=y.device)
             else:
                 v_first = ctx.memo.get(key)
                 if v_first is None:
                     raise RuntimeError("values to blend with: no layer before this one has left any")
         mode = {None: ops.QK_NORM_NONE, "head": ops.QK_NORM_HEAD, "whole": ops.QK_NORM_WHOLE}[s.qk_norm]
-        q = ops.qkv_norm_store(qkv, self.hq, self.hkv, self.dk, self.dv, cache, ctx.slots[g] if binding.write else None,
-                               qk_norm=mode, q_weight=self.q_norm, k_weight=self.k_norm, qk_eps=float(s.qk_norm_eps),
-                               values_from_keys=bool(s.values_from_keys), value_norm_eps=s.value_norm_eps,
-                               v_first=v_first, v_blend=self.blend if s.value_blend == "blend" else None,
-                               positions=ctx.positions,
-                               inv_freq=self.position.inv_freq() if self.position is not None else None,
-                               value_rows=self.talks)
+        pos = self.position
+        return ops.qkv_norm_store(y, self.hq, self.hkv, self.dk, self.dv, binding.kv, ctx.slots[binding.group] if binding.write else None,
+                                  qk_norm=mode, q_weight=self.q_norm, k_weight=self.k_norm, qk_eps=float(s.qk_norm_eps),
+                                  values_from_keys=bool(s.values_from_keys), value_norm_eps=s.value_norm_eps,
+                                  v_first=v_first, v_blend=self.blend if s.value_blend == "blend" else None,
+                                  positions=ctx.positions, inv_freq=pos.inv_freq() if pos is not None else None,
+                                  value_rows=self.talks, rot_pairs=pos is not None and pos.neighbours,
+                                  rot_gain=pos.gain if pos is not None else 1.0)
+
+    def mix(self, y: torch.Tensor, gates, ctx, binding: CacheBinding, out: torch.Tensor, factor: float = 1.0) -> None:
+        """y [T, q | k (| v) (| gate)] -> out [T, Hq * v_head_dim], before the output projection (parts.projected)."""
+        if binding.kv is None:
+            raise RuntimeError("attention was given no cache")
+        if factor != 1.0:
+            raise ValueError("attention leaves its result as it is")
+        q = self._store(y, ctx, binding)
+        n = self.hq * self.dv
+        ex = self._extras(ctx)
+        ops.attention(q, binding.kv, ctx.positions, ctx.tok_seq, ctx.block_tables[binding.group], self.scale, 0,
+                      dec_tokens=ex["dec_tokens"], max_dec_position=ex["max_dec_position"],
+                      other_tokens=ex["other_tokens"],
+                      other_tiles=self._other_tiles(ctx) if ex["other_tokens"] is not None else None,
+                      max_other_keys=ex.get("max_other_keys", 0), other_keys_row=ex.get("other_keys_row"),
+                      shared_keys=ctx.shared_keys, chunk=self.chunk, sink=False if self.sink is None else self.sink,
+                      v_dim=self.dv, gate=y[:, y.shape[1] - n:] if self.spec.output_gate else None, out=out)
+
+    def forward(self, x: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+        """x [T, H] in the activation type.  Returns the mixer's output, float32 [T, H]."""
+        if binding.kv is None:
+            raise RuntimeError("attention was given no cache")
+        y = ops.gemm(x, self.w_qkv, self.b_qkv)
         if self.talks:
-            o = ops.attention_talk(q, cache, ctx.positions, ctx.tok_seq, ctx.block_tables[g], self.scale, self.dk,
+            q = self._store(y, ctx, binding)
+            o = ops.attention_talk(q, binding.kv, ctx.positions, ctx.tok_seq, ctx.block_tables[binding.group], self.scale, self.dk,
                                    self.dv, chunk=self.chunk, bias=self.dist_bias, talk=self.talk)
         else:
-            ex = self._extras(ctx)
-            o = ops.attention(q, cache, ctx.positions, ctx.tok_seq, ctx.block_tables[g], self.scale, 0,
-                              dec_tokens=ex["dec_tokens"], max_dec_position=ex["max_dec_position"],
-                              other_tokens=ex["other_tokens"],
-                              other_tiles=self._other_tiles(ctx) if ex["other_tokens"] is not None else None,
-                              max_other_keys=ex.get("max_other_keys", 0), other_keys_row=ex.get("other_keys_row"),
-                              shared_keys=ctx.shared_keys, chunk=self.chunk).view(T, self.hq * self.d)
+            o = torch.empty((x.shape[0], self.hq * self.dv), dtype=x.dtype, device=x.device)
+            self.mix(y, None, ctx, binding, o)
         return ops.gemm(o, self.w_o, self.b_o, out_dtype=torch.float32)
 
 

@@ -5,8 +5,10 @@ Norm          forward(h, rt, delta=None, rows=None) -> x
               h is the 32-bit residual stream [T, H]; with ``delta`` (a branch output, see
               below) the sum h + delta is normed and written back to h; with ``rows`` only
               those rows are normed.  ``delta`` may be a BranchSum: a branch output with a scale per
-              channel and an average over depth on the way.
+              channel and an average over depth on the way; or a NormedBranch: a branch output that is
+              normed before it is added.
 Mixer         forward(x, ctx, binding) -> y      x, y [T, H] in the activation type
+              forward_scaled(x, ctx, binding) -> (y, s)   (optional) the output is s * y
               cache_need(spec) -> KVNeed | None, state_need(spec, hidden) -> StateNeed | None
 FeedForward   forward(x, ctx) -> y
               A mixer's or feed-forward's y is [T, H] in the activation type, or float32 [S, T, H]:
@@ -14,7 +16,9 @@ FeedForward   forward(x, ctx) -> y
 Position      table() for the fused kernel, or apply(packed, positions, num_q, num_k) in place
               on a [T, Hq + 2 Hkv, D] tensor of q | k | v heads.
 Stream prologue   forward(h, ctx) -> None: changes the 32-bit stream in place right after the
-              embedding (a scale, an added table of positions).
+              embedding (a scale, an added table of positions); or embed(table, ctx, binding) -> h in
+              the place of the embedding.  It may ask for state with state_need(spec, hidden), whose
+              binding comes behind those of the schedule's entries.
 Logit epilogue    forward(logits, ctx) -> logits on the float32 logits [R, V] (a scale, a soft cap).
 
 Few rows (decode): a step is then a chain of short dependent kernels, each of which costs a few
@@ -149,11 +153,29 @@ class BranchSum:
         return d
 
 
+@dataclass
+class NormedBranch:
+    """A branch output that is normed before it joins the stream: h += mult * (scale * parts) / rms * weight.  Handed on in the
+    place of the plain branch output, like BranchSum."""
+    parts: torch.Tensor              # [T, H] in the activation type, or float32 [S, T, H]
+    scale: float
+    weight: torch.Tensor             # float32 [H]
+    eps: float
+    mult: float
+
+    def add(self, h: torch.Tensor, weight: Optional[torch.Tensor], eps: float, dtype: torch.dtype, rows=None):
+        """Into the stream h, with the RMS norm that follows in the same kernel if it has a weight."""
+        from ..kernels import ops
+        return ops.branch_norm(h, self.parts, self.weight, self.eps, self.mult, weight, eps, dtype, scale=self.scale, rows=rows)
+
+
 def add_pending(h: torch.Tensor, pending) -> None:
     """A pending branch output of any form into the stream, by a kernel of its own (for blocks whose first step is not a
     norm of the stream)."""
     from ..kernels import ops
-    if isinstance(pending, BranchSum):
+    if isinstance(pending, NormedBranch):
+        pending.add(h, None, 0.0, torch.float32)
+    elif isinstance(pending, BranchSum):
         ops.stream_norm(h, None, 0.0, torch.float32 if pending.parts is None else pending.parts.dtype, **pending.kernel_args())
     elif pending is not None:
         ops.residual_add(h, pending)
@@ -178,7 +200,7 @@ class StreamInput:
         """True if a product can take the residual sum and the norm as its prologue at all: nothing to
         add, or float32 partial products and a second buffer for the sums."""
         d = self.delta
-        if isinstance(d, BranchSum):
+        if isinstance(d, (BranchSum, NormedBranch)):
             return False
         return d is None or (d.dim() == 3 and d.dtype == torch.float32 and self.stream.spare is not None)
 

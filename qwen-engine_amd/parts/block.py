@@ -8,7 +8,7 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import (BranchSum, CacheBinding, DepthAverage, Runtime, Stream, StreamInput, TensorInfo, add_pending, join_name,
+from .base import (BranchSum, CacheBinding, DepthAverage, NormedBranch, Runtime, Stream, StreamInput, TensorInfo, add_pending, join_name,
                    named_tensors, sub_tensors)
 from ..kernels import ops
 from .registry import build_part, part_class, register_part
@@ -386,7 +386,74 @@ class ScaledPreNormBlock(PreNormBlock):
         return conv.after_norm(norm, x, pending, ctx, next(bind).state)
 
 
+class SandwichBlock:
+    """``SandwichLayerSpec``: a norm before and behind each sublayer, one factor on what joins the stream.  The norm behind a
+    sublayer, the residual sum and the norm before the next sublayer are one kernel: the block hands its branch on as a
+    NormedBranch."""
+
+    def __init__(self, spec, hidden_size: int):
+        self.spec = spec
+        self.hidden = int(hidden_size)
+        self.mult = float(spec.mult)
+        has_ffn = spec.ffn is not None
+        self.mixer_norm, self.mixer, self.mixer_post = (build_part(p, hidden_size) for p in (spec.mixer_norm, spec.mixer, spec.mixer_post))
+        self.ffn_norm, self.ffn, self.ffn_post = ((build_part(p, hidden_size) if has_ffn else None)
+                                                  for p in (spec.ffn_norm, spec.ffn, spec.ffn_post))
+
+    def parts(self):
+        return tuple(p for p in (self.mixer_norm, self.mixer, self.mixer_post, self.ffn_norm, self.ffn, self.ffn_post) if p is not None)
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(p, "graph_safe", True) for p in self.parts())
+
+    @property
+    def graph_safe_with_state(self) -> bool:
+        return getattr(self.mixer, "graph_safe", False) is True
+
+    @staticmethod
+    def _named(spec):
+        subs = [spec.mixer_norm, spec.mixer, spec.mixer_post]
+        if spec.ffn is not None:
+            subs += [spec.ffn_norm, spec.ffn, spec.ffn_post]
+        return list(zip(spec.names, subs))
+
+    @staticmethod
+    def cache_needs(spec, hidden: int):
+        return PreNormBlock.cache_needs(spec, hidden)
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        out: Dict[str, TensorInfo] = {}
+        for name, sub in SandwichBlock._named(spec):
+            for rel, info in part_class(sub.kind).expected_tensors(sub, hidden).items():
+                out[join_name(name, rel)] = info
+        return out
+
+    def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        for (name, sub), part in zip(self._named(self.spec), self.parts()):
+            part.load(named_tensors(tensors, name, type(part).expected_tensors(sub, self.hidden)), rt)
+
+    def _branch(self, parts: torch.Tensor, norm, scale: float = 1.0) -> NormedBranch:
+        return NormedBranch(parts, scale, norm.weight, norm.eps, self.mult)
+
+    def forward(self, h, pending, ctx, bindings):
+        """Returns the block's last branch as a NormedBranch, for the next norm to add."""
+        x = h.h if isinstance(h, Stream) else h
+        n = self.mixer_norm.forward(x, ctx.rt, delta=pending)
+        if hasattr(self.mixer, "forward_scaled"):
+            y, scale = self.mixer.forward_scaled(n, ctx, bindings[0])
+        else:
+            y, scale = self.mixer.forward(n, ctx, bindings[0]), 1.0
+        last = self._branch(y, self.mixer_post, scale)
+        if self.ffn is not None:
+            n = self.ffn_norm.forward(x, ctx.rt, delta=last)
+            last = self._branch(self.ffn.forward(n, ctx), self.ffn_post)
+        return last
+
+
 register_part("prenorm_block", PreNormBlock)
+register_part("sandwich_block", SandwichBlock)
 register_part("scaled_prenorm_block", ScaledPreNormBlock)
 register_part("parallel_block", ParallelBlock)
 register_part("postnorm_block", PostNormBlock)

@@ -1,4 +1,4 @@
-"""Dense gated feed-forward: down(silu(gate x) * up x), no biases
+"""Dense gated feed-forward: down(silu(gate x) * up x), with biases if the spec says so
 (src/models/qwen3/model.py:232-237; silu.mul as src/layers/fused_ops/silumul.py:46-53,
 with the product formed in 32-bit before the one rounding).  gate and up are one
 product with the two weights stacked."""
@@ -20,18 +20,24 @@ class SwiGLU:
         self.hidden = int(hidden_size)
         self.inter = int(spec.intermediate_size)
         self.names = tuple(spec.names)
-        self.w_gu = self.w_down = None
+        self.bias = bool(getattr(spec, "bias", False))
+        self.bias_suffix = getattr(spec, "bias_suffix", ".b")
+        self.w_gu = self.w_down = self.b_gu = self.b_down = None
         self.interleaved = False
 
     @staticmethod
     def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
         i = spec.intermediate_size
         gate, up, down = spec.names
-        return {
+        t = {
             gate: TensorInfo((i, hidden)),
             up: TensorInfo((i, hidden)),
             down: TensorInfo((hidden, i)),
         }
+        if getattr(spec, "bias", False):
+            for name, n in ((gate, i), (up, i), (down, hidden)):
+                t[name + spec.bias_suffix] = TensorInfo((n,), "zeros", "vector")
+        return t
 
     def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
         n_gate, n_up, n_down = self.names
@@ -43,14 +49,19 @@ class SwiGLU:
         self.interleaved = self.inter % 32 == 0
         self.w_gu = rt.place_matrix(ops.interleave_gate_up(g, u) if self.interleaved else torch.cat([g, u], dim=0))
         self.w_down = rt.place_matrix(tensors[n_down])
+        if self.bias:                # (gate's and up's in the order of their rows)
+            bg, bu = (tensors[n + self.bias_suffix].float() for n in (n_gate, n_up))
+            self.b_gu = rt.place_vector(ops.interleave_gate_up(bg.view(-1, 1), bu.view(-1, 1)).view(-1) if self.interleaved
+                                        else torch.cat([bg, bu]))
+            self.b_down = rt.place_vector(tensors[n_down + self.bias_suffix])
 
     def activation(self, x) -> torch.Tensor:
         """silu(gate x) * up x [T, I] in the activation type, for x [T, H] (not a StreamInput)."""
         if self.interleaved and ops.gemm_silu_supported(x, self.w_gu):
-            return ops.gemm(x, self.w_gu, epilogue=ops.EPI_SILU_MUL_IL)
+            return ops.gemm(x, self.w_gu, self.b_gu, epilogue=ops.EPI_SILU_MUL_IL)
         if not self.interleaved and ops.gemm_fused_supported(x, self.w_gu):
-            return ops.gemm(x, self.w_gu, epilogue=ops.EPI_SILU_MUL)
-        return ops.silu_mul(ops.gemm(x, self.w_gu), interleaved=self.interleaved)
+            return ops.gemm(x, self.w_gu, self.b_gu, epilogue=ops.EPI_SILU_MUL)
+        return ops.silu_mul(ops.gemm(x, self.w_gu, self.b_gu), interleaved=self.interleaved)
 
     def forward(self, x, ctx) -> torch.Tensor:
         """Returns the feed-forward output [T, H], or float32 partial products [S, T, H] of it.
@@ -58,21 +69,15 @@ class SwiGLU:
         a = None
         if isinstance(x, StreamInput):
             if x.prefers_prologue(ops, self.w_gu):
-                a = x.gemm(ops, self.w_gu, epilogue=ops.EPI_SILU_MUL_IL if self.interleaved else ops.EPI_SILU_MUL)
+                a = x.gemm(ops, self.w_gu, self.b_gu, epilogue=ops.EPI_SILU_MUL_IL if self.interleaved else ops.EPI_SILU_MUL)
             else:
                 x = x.materialize()
-        if a is not None:
-            pass
-        elif self.interleaved and ops.gemm_silu_supported(x, self.w_gu):
-            a = ops.gemm(x, self.w_gu, epilogue=ops.EPI_SILU_MUL_IL)   # silu.mul in the product's epilogue
-        elif not self.interleaved and ops.gemm_fused_supported(x, self.w_gu):
-            a = ops.gemm(x, self.w_gu, epilogue=ops.EPI_SILU_MUL)
-        else:
-            a = ops.silu_mul(ops.gemm(x, self.w_gu), interleaved=self.interleaved)
+        if a is None:
+            a = self.activation(x)                                     # (silu.mul in the product's epilogue where it can be)
         splits = ops.gemm_branch_splits(a, self.w_down)
         if splits:   # partial products along K, added by the norm that follows
-            return ops.gemm(a, self.w_down, epilogue=ops.EPI_PARTIAL, splits=splits)
-        return ops.gemm(a, self.w_down)
+            return ops.gemm(a, self.w_down, self.b_down, epilogue=ops.EPI_PARTIAL, splits=splits)
+        return ops.gemm(a, self.w_down, self.b_down)
 
 
 class GeluMLP:

@@ -46,6 +46,9 @@ def cache_plan(spec: ModelSpec) -> CachePlan:
         cls = part_class(layer.kind)
         users = list(cls.cache_needs(layer, spec.hidden_size)) if hasattr(cls, "cache_needs") else []
         needs.append((users, entry.cache_from))
+    pro = spec.stream_prologue               # (behind the schedule's entries: what the prologue keeps)
+    if pro is not None and hasattr(part_class(pro.kind), "state_need"):
+        needs.append(([(None, part_class(pro.kind).state_need(pro, spec.hidden_size))], None))
     return plan_cache(needs)
 
 
@@ -74,10 +77,13 @@ class DecoderModel:
         return [p for p in (self.final_norm, self.prologue, self.epilogue) if p is not None]
 
     def all_parts(self):
-        """Every part of the model, the parts inside the blocks included."""
+        """Every part of the model, the parts inside the blocks and inside other parts included."""
+        def inside(part):
+            yield part
+            for p in (part.parts() if hasattr(part, "parts") else ()):
+                yield from inside(p)
         for b in self.blocks:
-            yield b
-            yield from (b.parts() if hasattr(b, "parts") else ())
+            yield from inside(b)
         yield from self._around()
 
     def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
@@ -113,7 +119,8 @@ class DecoderModel:
                     if v.data_ptr() not in seen:
                         seen.add(v.data_ptr())
                         total += v.numel() * v.element_size()
-                elif hasattr(v, "load") and hasattr(v, "expected_tensors"):     # a part inside the part
+                elif getattr(v, "holds_weights", False) or (hasattr(v, "load") and hasattr(v, "expected_tensors")):
+                    # (a part, or what holds weights for it, inside the part)
                     total += held(v)
             return total
 
@@ -132,9 +139,12 @@ class DecoderModel:
     def forward(self, ctx, bindings: List[CacheBinding]) -> torch.Tensor:
         """Runs the tokens of ctx through the schedule; returns float32 logits [R, V]."""
         with ops.one_stream():           # (the whole step runs on the stream that is current now)
-            h = ops.embedding(ctx.token_ids, self.embed)
-            if self.prologue is not None:
-                self.prologue.forward(h, ctx)
+            if hasattr(self.prologue, "embed"):
+                h = self.prologue.embed(self.embed, ctx, bindings[len(self.spec.schedule)][0])
+            else:
+                h = ops.embedding(ctx.token_ids, self.embed)
+                if self.prologue is not None:
+                    self.prologue.forward(h, ctx)
             # (few rows: a second buffer, so that a product can do the residual sum before it, see Stream)
             stream = Stream(h, torch.empty_like(h) if h.shape[0] <= ops.gemm_norm_max_rows() else None)
             pending = None

@@ -7,12 +7,17 @@ from typing import Dict, Optional
 import torch
 
 from ..kernels import ops
-from .base import BranchSum, Runtime, TensorInfo
+from .base import BranchSum, NormedBranch, Runtime, TensorInfo, add_pending
 from .registry import register_part
 
 
 def _norm(h: torch.Tensor, weight: torch.Tensor, eps: float, rt: Runtime, delta, rows, center: bool) -> torch.Tensor:
     """A norm of the stream with whatever is pending before it."""
+    if isinstance(delta, NormedBranch):
+        if not center:
+            return delta.add(h, weight, eps, rt.dtype, rows=rows)
+        add_pending(h, delta)
+        delta = None
     if isinstance(delta, BranchSum):
         return ops.stream_norm(h, weight, eps, rt.dtype, center=center, rows=rows, **delta.kernel_args())
     return ops.rmsnorm(h, weight, eps, rt.dtype, delta=delta, rows=rows, center=center)
@@ -79,12 +84,16 @@ class ScalarRMSNorm:
 class BareRMSNorm(RMSNorm):
     """RMSNorm whose weight tensor carries the part's own name (named "" inside the part)."""
 
+    def __init__(self, spec, size: int):
+        super().__init__(spec, size)
+        self.offset, self.gain = float(getattr(spec, "offset", 0.0)), float(getattr(spec, "gain", 1.0))
+
     @staticmethod
     def expected_tensors(spec, size: int) -> Dict[str, TensorInfo]:
-        return {"": TensorInfo((size,), "ones", "vector")}
+        return {"": TensorInfo((size,), "zeros" if getattr(spec, "offset", 0.0) else "ones", "vector")}
 
     def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
-        self.weight = rt.place_vector(tensors[""])
+        self.weight = rt.place_vector((tensors[""].to(torch.float32) + self.offset) * self.gain)
 
 
 class BareLayerNorm:

@@ -10,12 +10,8 @@ import torch
 from ..cache.plan import StateNeed
 from ..kernels import ops
 from .base import CacheBinding, Runtime, TensorInfo, join_name, named_tensors
+from .projected import InputProducts, OutputProduct, ProjectedMixer
 from .registry import build_part, part_class, register_part
-
-
-def _single_rows(ctx, T: int) -> bool:
-    """True if every request of the step brings exactly one token."""
-    return len(ctx.seqs) == T and all(s.q_len == 1 for s in ctx.seqs)
 
 
 # From this many rows of one request in a step, the recurrences take the step's rows chunk by chunk (the chunks in
@@ -86,7 +82,7 @@ class ShiftedDecayMixer:
         if binding.state is None:
             raise RuntimeError("the recurrence was given no state")
         T, W, st = x.shape[0], self.hidden, binding.state
-        m = ops.token_shift(x, self.mu, st, ctx.tok_seq, single_rows=_single_rows(ctx, T))
+        m = ops.token_shift(x, self.mu, st, ctx.tok_seq, single_rows=ctx.single_rows)
         r, k, v, gate = (ops.gemm(m[i], w) for i, w in enumerate((self.w_r, self.w_k, self.w_v, self.w_g)))
         low = ops.unary(ops.gemm(m[4], self.w_1, out_dtype=torch.float32), ops.UNARY_TANH, out_dtype=ctx.rt.dtype)
         decay_x = ops.gemm(low, self.w_2, out_dtype=torch.float32)      # (exponentials of the decay: in the recurrence, 32-bit)
@@ -196,17 +192,197 @@ class ForgetGateLinearMixer:
         z = ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:], binding.state, ctx.tok_seq, self.h, silu=True,
                                   forget_bias=self.forget_bias, lower=self.lower, chunks=_chunks(ctx, self.h),
                                   norm_weight=self.norm, norm_eps=self.eps, norm_dtype=ctx.rt.dtype,
-                                  single_rows=_single_rows(ctx, T))
+                                  single_rows=ctx.single_rows)
         splits = ops.gemm_branch_splits(z, self.w_o)
         if splits:
             return ops.gemm(z, self.w_o, epilogue=ops.EPI_PARTIAL, splits=splits)
         return ops.gemm(z, self.w_o)
 
 
+class GatedLinearMixer(ProjectedMixer):
+    """``GatedLinearSpec``: the decays come from the low-rank projection in a kernel of their own, the recurrence has the
+    norm per head and the silu gate behind it."""
+
+    def __init__(self, spec, hidden_size: int):
+        self.spec = spec
+        self.hidden = int(hidden_size)
+        self.h, self.d, self.dv, self.rank = int(spec.num_heads), int(spec.head_dim), int(spec.v_head_dim), int(spec.decay_rank)
+        self.tau, self.eps = float(spec.tau), float(spec.norm_eps)
+        self.w_2 = self.b_2 = self.norm = None
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        nk, nv = spec.num_heads * spec.head_dim, spec.num_heads * spec.v_head_dim
+        q, k, v, g, o, norm, a1, a2, a2b = spec.names
+        return {q: TensorInfo((nk, hidden)), k: TensorInfo((nk, hidden)), v: TensorInfo((nv, hidden)), g: TensorInfo((nv, hidden)),
+                o: TensorInfo((hidden, nv)), norm: TensorInfo((int(spec.v_head_dim),), "ones", "vector"),
+                a1: TensorInfo((int(spec.decay_rank), hidden)), a2: TensorInfo((nk, int(spec.decay_rank))),
+                a2b: TensorInfo((nk,), "zeros", "vector")}
+
+    @staticmethod
+    def cache_need(spec):
+        return None
+
+    @staticmethod
+    def state_need(spec, hidden: int) -> Optional[StateNeed]:
+        return StateNeed(shape=(ops.recurrence_state_numbers(spec.num_heads, spec.head_dim, spec.v_head_dim),), dtype="float32")
+
+    def inputs(self, tensors):
+        q, k, v, g, _, _, a1, _, _ = self.spec.names
+        return [(tensors[n], None) for n in (q, k, v, g, a1)], []
+
+    def output(self, tensors):
+        return tensors[self.spec.names[4]]
+
+    def load_own(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        _, _, _, _, _, norm, _, a2, a2b = self.spec.names
+        self.w_2 = rt.place_matrix(tensors[a2])
+        self.b_2 = rt.place_vector(tensors[a2b])
+        self.norm = rt.place_vector(tensors[norm]).repeat(self.h)
+
+    def mix(self, y: torch.Tensor, gates, ctx, binding: CacheBinding, out: torch.Tensor, factor: float = 1.0) -> None:
+        if binding.state is None:
+            raise RuntimeError("the recurrence was given no state")
+        nk, nv = self.h * self.d, self.h * self.dv
+        decays = ops.low_rank_decay(y[:, 2 * nk + 2 * nv:], self.w_2, self.b_2, self.tau)
+        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], binding.state, ctx.tok_seq, self.h, decays=decays,
+                              q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
+                              norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:2 * nk + 2 * nv],
+                              gate_act=ops.GATE_SILU, y_scale=factor, out=out)
+
+
+class MatrixMemoryMixer(ProjectedMixer):
+    """``MatrixMemorySpec``: the two gates' logits stay 32-bit; a kernel turns them into decays, key factors and floors
+    along the running maximum; the recurrence carries its normaliser and has the norm per head and the sigmoid gate behind
+    it.  State: the matrices, the normalisers, the running maxima."""
+
+    def __init__(self, spec, hidden_size: int):
+        self.spec = spec
+        self.hidden = int(hidden_size)
+        self.h, self.d, self.dv = int(spec.num_heads), int(spec.head_dim), int(spec.v_head_dim)
+        self.cap, self.eps = float(spec.gate_cap), float(spec.norm_eps)
+        self.b_i = self.b_f = self.norm = None
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        h, nk, nv = spec.num_heads, spec.num_heads * spec.head_dim, spec.num_heads * spec.v_head_dim
+        q, k, v, g, o, norm, i, ib, f, fb = spec.names
+        return {q: TensorInfo((nk, hidden)), k: TensorInfo((nk, hidden)), v: TensorInfo((nv, hidden)), g: TensorInfo((nv, hidden)),
+                o: TensorInfo((hidden, nv)), norm: TensorInfo((nv,), "ones", "vector"),
+                i: TensorInfo((h, hidden)), ib: TensorInfo((h,), "zeros", "vector"),
+                f: TensorInfo((h, hidden)), fb: TensorInfo((h,), "zeros", "vector")}
+
+    @staticmethod
+    def cache_need(spec):
+        return None
+
+    @staticmethod
+    def state_need(spec, hidden: int) -> Optional[StateNeed]:
+        n = ops.recurrence_state_numbers(spec.num_heads, spec.head_dim, spec.v_head_dim, normaliser=True) + spec.num_heads
+        return StateNeed(shape=((n + 3) // 4 * 4,), dtype="float32")        # (rows of whole 16-byte pieces)
+
+    def inputs(self, tensors):
+        q, k, v, g, _, _, i, _, f, _ = self.spec.names
+        return [(tensors[n], None) for n in (q, k, v, g)], [tensors[i], tensors[f]]
+
+    def output(self, tensors):
+        return tensors[self.spec.names[4]]
+
+    def load_own(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        self.norm, self.b_i, self.b_f = (rt.place_vector(tensors[self.spec.names[n]]) for n in (5, 7, 9))
+
+    def mix(self, y: torch.Tensor, gates, ctx, binding: CacheBinding, out: torch.Tensor, factor: float = 1.0) -> None:
+        st = binding.state
+        if st is None:
+            raise RuntimeError("the recurrence was given no state")
+        nk, nv = self.h * self.d, self.h * self.dv
+        at = ops.recurrence_state_numbers(self.h, self.d, self.dv, normaliser=True)
+        chunks = _chunks(ctx, self.h)
+        steps = ops.memory_gates(gates, self.b_i, self.b_f, self.cap, st[:, at:at + self.h], ctx.tok_seq, chunks=chunks)
+        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], st, ctx.tok_seq, self.h, steps=steps,
+                              normaliser=True, q_scale=self.d ** -0.5, chunks=chunks, norm_weight=self.norm, norm_eps=self.eps,
+                              norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:],
+                              gate_act=ops.GATE_SIGMOID, y_scale=factor, out=out)
+
+
+class StateSpaceMixer(ProjectedMixer):
+    """``StateSpaceSpec`` (Mamba-2): the step sizes' logits stay 32-bit; one kernel convolves x, B and C and forms step sizes and
+    decays, the recurrence runs over them (its keys scaled by the step sizes), one kernel adds the skip, gates and norms.
+    State: the heads' matrices, the convolution's last inputs."""
+
+    def __init__(self, spec, hidden_size: int):
+        self.spec = spec
+        self.hidden = int(hidden_size)
+        self.h, self.dv, self.n, self.groups = int(spec.num_heads), int(spec.head_dim), int(spec.state_dim), int(spec.groups)
+        self.taps, self.norm_groups, self.eps = int(spec.taps), int(spec.norm_groups), float(spec.norm_eps)
+        self.conv_w_t = self.conv_b = self.dt_bias = self.a_log = self.skip = self.norm = None
+
+    @staticmethod
+    def _sizes(spec):
+        """(inner, convolved channels)."""
+        inner = spec.num_heads * spec.head_dim
+        return inner, inner + 2 * spec.groups * spec.state_dim
+
+    @staticmethod
+    def expected_tensors(spec, hidden: int) -> Dict[str, TensorInfo]:
+        inner, C = StateSpaceMixer._sizes(spec)
+        w_in, conv, conv_b, dt_b, a_log, skip, norm, o = spec.names
+        h = spec.num_heads
+        return {w_in: TensorInfo((inner + C + h, hidden)), conv: TensorInfo((C, int(spec.taps)), "normal", "vector"),
+                conv_b: TensorInfo((C,), "zeros", "vector"), dt_b: TensorInfo((h,), "zeros", "vector"),
+                a_log: TensorInfo((h,), "zeros", "vector"), skip: TensorInfo((h,), "ones", "vector"),
+                norm: TensorInfo((inner,), "ones", "vector"), o: TensorInfo((hidden, inner))}
+
+    @staticmethod
+    def cache_need(spec):
+        return None
+
+    @staticmethod
+    def _state_offset(spec) -> int:
+        """Where the convolution's inputs begin in a state row (behind the matrices, at a whole 16-byte piece)."""
+        return (ops.recurrence_state_numbers(spec.num_heads, spec.state_dim, spec.head_dim) + 3) // 4 * 4
+
+    @staticmethod
+    def state_need(spec, hidden: int) -> Optional[StateNeed]:
+        n = StateSpaceMixer._state_offset(spec) + (int(spec.taps) - 1) * StateSpaceMixer._sizes(spec)[1]
+        return StateNeed(shape=((n + 3) // 4 * 4,), dtype="float32")
+
+    def inputs(self, tensors):
+        inner, C = self._sizes(self.spec)
+        w = tensors[self.spec.names[0]]
+        return [(w[:inner + C], None)], [w[inner + C:]]
+
+    def output(self, tensors):
+        return tensors[self.spec.names[7]]
+
+    def load_own(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
+        _, conv, conv_b, dt_b, a_log, skip, norm, _ = self.spec.names
+        self.conv_w_t = rt.place_vector(tensors[conv].t())
+        self.conv_b, self.dt_bias, self.a_log, self.skip, self.norm = (rt.place_vector(tensors[n])
+                                                                       for n in (conv_b, dt_b, a_log, skip, norm))
+
+    def mix(self, y: torch.Tensor, gates, ctx, binding: CacheBinding, out: torch.Tensor, factor: float = 1.0) -> None:
+        st = binding.state
+        if st is None:
+            raise RuntimeError("the recurrence was given no state")
+        if factor != 1.0:
+            raise ValueError("the state space leaves its result as it is")
+        inner, C = self._sizes(self.spec)
+        gn = self.groups * self.n
+        chunks = _chunks(ctx, self.h)
+        xbc, steps = ops.conv_steps(y[:, inner:], self.conv_w_t, self.conv_b, st[:, self._state_offset(self.spec):], ctx.tok_seq,
+                                    dt=gates, dt_bias=self.dt_bias, a_log=self.a_log, single_rows=ctx.single_rows, chunks=chunks)
+        x = xbc[:, :inner]
+        o = ops.linear_recurrence(xbc[:, inner + gn:], xbc[:, inner:inner + gn], x, st, ctx.tok_seq, self.h, steps=steps,
+                                  k_heads=self.groups, chunks=chunks, single_rows=ctx.single_rows)
+        ops.skip_gate_norm(o, x, self.skip, y[:, :inner], self.norm, self.eps, self.norm_groups, ctx.rt.dtype, out=out)
+
+
 class SideBySideMixer:
     """``SideBySideMixerSpec``: two mixers read the same rows; their outputs are added with weights, in 32-bit.  The
     two share the block's one cache binding: the keys and values of the one that has any, the state of the one that
-    has any."""
+    has any.  Two projected mixers (parts.projected) share the products before and behind them: what they leave lies side by
+    side in one row, the right one's part times right_scale / left_scale, and left_scale goes to whoever adds the result."""
 
     def __init__(self, spec, hidden_size: int):
         self.spec = spec
@@ -214,6 +390,18 @@ class SideBySideMixer:
         self.left = build_part(spec.left, hidden_size)
         self.right = build_part(spec.right, hidden_size)
         self.left_scale, self.right_scale = float(spec.left_scale), float(spec.right_scale)
+        self.joint = self.left_scale != 0.0 and self._projected(spec.left) and self._projected(spec.right) and \
+            isinstance(self.right, (GatedLinearMixer, MatrixMemoryMixer))
+        self.products_in: Optional[InputProducts] = None
+        self.products_out: Optional[OutputProduct] = None
+
+    @staticmethod
+    def _projected(spec) -> bool:
+        cls = part_class(spec.kind)
+        return cls.is_projected(spec) if hasattr(cls, "is_projected") else issubclass(cls, ProjectedMixer)
+
+    def parts(self):
+        return (self.left, self.right)
 
     @property
     def graph_safe(self):
@@ -253,16 +441,42 @@ class SideBySideMixer:
         return SideBySideMixer._one(spec, hidden, "state_need")
 
     def load(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
-        for (name, sub), part in zip(self._subs(self.spec), (self.left, self.right)):
-            names = type(part).expected_tensors(sub, self.hidden)
-            part.load(named_tensors(tensors, name, names), rt)
+        held = [named_tensors(tensors, name, type(part).expected_tensors(sub, self.hidden))
+                for (name, sub), part in zip(self._subs(self.spec), (self.left, self.right))]
+        both = list(zip((self.left, self.right), held))
+        if not self.joint:
+            for part, t in both:
+                part.load(t, rt)
+            return
+        for part, t in both:
+            part.load_own(t, rt)
+        self.products_in = InputProducts([part.inputs(t) for part, t in both], rt)
+        self.products_out = OutputProduct([part.output(t) for part, t in both], rt)
+
+    def forward_scaled(self, x: torch.Tensor, ctx, binding: CacheBinding):
+        """(y, s): the output is s * y, y [T, H] or float32 partial products [S, T, H]."""
+        if not self.joint:
+            return self.forward(x, ctx, binding), 1.0
+        ins = self.products_in.run(x, ctx.rt)
+        o = self.products_out.rows(x.shape[0], ctx.rt, x.device)
+        for part, (y, gates), (a, b), factor in zip((self.left, self.right), ins, self.products_out.cols,
+                                                    (1.0, self.right_scale / self.left_scale)):
+            part.mix(y, gates, ctx, binding, o[:, a:b], factor)
+        return self.products_out.run(o), self.left_scale
 
     def forward(self, x: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
-        a = self.left.forward(x, ctx, binding)
-        b = self.right.forward(x, ctx, binding)
+        if self.joint:
+            y, scale = self.forward_scaled(x, ctx, binding)
+            return y if scale == 1.0 else ops.scaled_sum(y, scale, y, 0.0)
+        a, b = (part.forward(x, ctx, binding) for part in (self.left, self.right))
+        if a.dtype != b.dtype or a.shape != b.shape:
+            a, b = (t.float().sum(0) if t.dim() == 3 else t.float() for t in (a, b))
         return ops.scaled_sum(a, self.left_scale, b, self.right_scale)
 
 
+register_part("gated_linear", GatedLinearMixer)
+register_part("matrix_memory", MatrixMemoryMixer)
+register_part("state_space", StateSpaceMixer)
 register_part("shifted_decay", ShiftedDecayMixer)
 register_part("decayed_linear", DecayedLinearMixer)
 register_part("forget_gate_linear", ForgetGateLinearMixer)
