@@ -1,6 +1,6 @@
 // Entry points of attention over the paged cache.
 //
-// qe_attention          any sizes, float32 or bfloat16, one wave per (token, head); for all
+// qe_attention(_tail)   any sizes, float32 or bfloat16, one wave per (token, head); for all
 //                       tokens of the batch or for a list of them
 // qe_attention_decode_* bfloat16 MFMA kernel for tokens that are the single new token of their
 //                       request (see attention_decode.hip)
@@ -120,7 +120,7 @@ extern "C" int qe_attention_prefill_run(const void* q, void* out, const void* ca
 // out_stride, dv, sink_heads, gate, gate_stride, dt_g, here and below: see AttnTail (0, 0, null, null: plain rows of Hq * D
 // numbers, a sink of score 0).  tokens: null for all T rows of q, else n_tokens row indices.  keep_first: the first keys of a request
 // that every later query sees wherever its window stands; sink: a 1 is added to the softmax's denominator.
-extern "C" int qe_attention(const void* q, void* out, const void* cache, const int* positions,
+extern "C" int qe_attention_tail(const void* q, void* out, const void* cache, const int* positions,
                             const int* tok_seq, const int* block_table, int max_blocks, const int* tokens,
                             int n_tokens, int Hq, int Hkv, int D, int P, float scale, int window, int keep_first,
                             int sink, float softcap, int dt_a, long out_stride, int dv, const float* sink_heads,
@@ -133,6 +133,14 @@ extern "C" int qe_attention(const void* q, void* out, const void* cache, const i
     return qe_attention_generic(q, out, cache, positions, tok_seq, block_table, max_blocks, tokens, n_tokens,
                                 Hq, Hkv, D, P, scale, window, keep_first, sink, softcap, dt_a, stream,
                                 make_tail(Hq, D, out, out_stride, dv, sink_heads, gate, gate_stride, dt_g));
+}
+
+// The same with plain rows of Hq * D numbers and a sink, if any, of score 0.
+extern "C" int qe_attention(const void* q, void* out, const void* cache, const int* positions, const int* tok_seq,
+                            const int* block_table, int max_blocks, const int* tokens, int n_tokens, int Hq, int Hkv, int D,
+                            int P, float scale, int window, int keep_first, int sink, float softcap, int dt_a, hipStream_t stream) {
+    return qe_attention_tail(q, out, cache, positions, tok_seq, block_table, max_blocks, tokens, n_tokens, Hq, Hkv, D, P, scale,
+                             window, keep_first, sink, softcap, dt_a, 0, 0, nullptr, nullptr, 0, QE_F32, stream);
 }
 
 extern "C" int qe_attention_decode_supported(int Hq, int Hkv, int D, int P, int dt_a) {

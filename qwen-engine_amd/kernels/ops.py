@@ -78,8 +78,9 @@ def load_library():
         "qe_qk_rope_store_parts_supported": [i32, i32],
         "qe_gemm_partial_preferred": [i32, i32, i32, i32, i32],
         "qe_gemm_branch_splits": [i32, i32, i32, i32, i32],
-        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32,
-                         i64, i32, vp, vp, i64, i32, vp],
+        "qe_attention": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32, vp],
+        "qe_attention_tail": [vp, vp, vp, vp, vp, vp, i32, vp, i32, i32, i32, i32, i32, f32, i32, i32, i32, f32, i32,
+                              i64, i32, vp, vp, i64, i32, vp],
         "qe_qkv_conv_rope_store": [vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp],
         "qe_scale_f32": [vp, i64, f32, vp],
         "qe_moe_route_biased": [vp, vp, vp, vp, i32, i32, i32, f32, i32, vp, i32, i32, vp],
@@ -849,7 +850,7 @@ def attention(q: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor, tok
 
     def generic(tokens):
         n = T if tokens is None else tokens.shape[0]
-        _check(lib.qe_attention(q.data_ptr(), out.data_ptr(), cache.data_ptr(), positions.data_ptr(),
+        _check(lib.qe_attention_tail(q.data_ptr(), out.data_ptr(), cache.data_ptr(), positions.data_ptr(),
                                 tok_seq.data_ptr(), block_table.data_ptr(), max_blocks, _ptr(tokens), n,
                                 Hq, Hkv, D, P, float(scale), int(window), keep_first, sink, softcap, _DT[q.dtype], *tail, _stream()),
                "attention")
