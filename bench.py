@@ -35,10 +35,11 @@ Other sizes and workloads (not what the default line reports):
                             recorded graph of repetitions over weights that do not fit the caches, and its rate
                             against the nominal and the measured peaks (the counterpart of the reference's
                             per-operator benchmarks, src/layers/ops/linear.py:204-249)
-  --design zarorax|nufavik|potatar|safurax|busadra
+  --design zarorax|nufavik|potatar|safurax|busadra|vuzinex
                             another design beside the closest Qwen3 model of equal sizes (safurax: beside the Zarorax
                             model of equal sizes, the engine's other design of latent attention and routed experts;
-                            busadra: beside the Potatar and the Nufavik model of equal sizes, the engine's other designs
+                            vuzinex: beside the Potatar model of equal sizes; busadra: beside the Potatar and the Nufavik model
+                            of equal sizes, the engine's other designs
                             of recurrences and of windowed attention with routed experts) (width, layers, heads, and a
                             feed-forward as wide as the experts a token uses, or of as many weights): prefill (one prompt of --prefill-tokens
                             in one step) and decode (batch 1 and --batch at --context) of both, at the sizes of
@@ -98,7 +99,7 @@ def parse():
                     help="run steps of single new tokens beside a prompt portion as they come, not from a recorded graph")
     ap.add_argument("--requests", type=int, default=None, help="requests of the serving workloads")
     ap.add_argument("--kernels", action="store_true", help="time each kernel of a layer alone over a range of rows")
-    ap.add_argument("--design", default=None, choices=["zarorax", "nufavik", "potatar", "safurax", "busadra"],
+    ap.add_argument("--design", default=None, choices=["zarorax", "nufavik", "potatar", "safurax", "busadra", "vuzinex"],
                     help="measure this design beside the closest Qwen3 model of equal sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="small,medium", help="which of the design's sizes (small, medium), with commas")
     ap.add_argument("--warmup-passes", type=int, default=2,
@@ -491,6 +492,39 @@ def busadra_neighbours(z, layers, vocab):
     return {"potatar": potatar_config(pz, layers, vocab), "nufavik": nufavik_config(nz, layers, vocab)}
 
 
+# Layer sizes for --design vuzinex: those of --design potatar (attention in chunks, recurrences, two mixers side by side),
+# the state space's heads, their size, the state and the groups; the rank of the decays; a feed-forward of three matrices of
+# as many weights as Potatar's two
+VUZINEX_SIZES = {
+    "small": dict(POTATAR_SIZES["small"], ssm_heads=32, ssm_dim=64, state=128, groups=1, taps=4, rank=16),
+    "medium": dict(POTATAR_SIZES["medium"], ssm_heads=64, ssm_dim=64, state=128, groups=1, taps=4, rank=16),
+}
+
+
+def vuzinex_config(z, layers, vocab):
+    """Attention in chunks beside a matrix memory, the state space (without a feed-forward), attention over all keys beside
+    gated linear attention, the state space, in turn."""
+    mlp = {"kind": "dense", "ff": z["ff"] * 2 // 3 // 128 * 128}
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"], "scale": z["dim"] ** -0.5}
+    right = {"heads": z["rec_heads"], "dim": z["rec_dim"], "vdim": z["rec_dim"]}
+    one = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": dict(left, mask={"size": z["chunk"]},
+                                  rot={"base": 1e6, "dims": z["dim"],
+                                       "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 2048}}),
+                     "right": dict(right, gate_cap=15.0), "left_scale": 1.0, "right_scale": 0.5}}
+    two = {"type": "parallel_2", "mlp": mlp,
+           "mixer": {"left": dict(left, rot={"base": 10000.0, "dims": z["dim"],
+                                             "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}),
+                     "right": dict(right, tau=16.0, decay_rank=z["rank"]), "left_scale": 1.0, "right_scale": 0.5}}
+    ssm = {"type": "mamba2", "mlp": None,
+           "mixer": {"heads": z["ssm_heads"], "vdim": z["ssm_dim"], "state": z["state"], "groups": z["groups"], "conv": z["taps"],
+                     "norm_groups": 1}}
+    order = [one, ssm, two, ssm]
+    return {"architecture": "Vuzinex", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-5}, "residual_mult": 0.7,
+            "logit_scale": 0.5, "embedding": {"scale": 8.0, "bigram": {"buckets": 4093, "mul_prev": 31, "mul_cur": 17}},
+            "loop": None, "layers": [order[i % 4] for i in range(layers)]}
+
+
 def design_compare(args) -> int:
     """Prefill and decode of another design beside the Qwen3 model of equal sizes, through the same step
     function.  A "step" is one decode step; the line's value is the design's decode rate at --batch, first size."""
@@ -558,12 +592,19 @@ def design_compare(args) -> int:
     out = {}
     design = args.design
     title = design.capitalize()
-    other, other_title = {"safurax": ("zarorax", "Zarorax"), "busadra": ("potatar", "Potatar and Nufavik")}.get(design, ("qwen3", "Qwen3"))
+    other, other_title = {"safurax": ("zarorax", "Zarorax"), "busadra": ("potatar", "Potatar and Nufavik"),
+                          "vuzinex": ("potatar", "Potatar")}.get(design, ("qwen3", "Qwen3"))
     for name in [n for n in args.design_sizes.split(",") if n]:
         if design == "safurax":
             z = SAFURAX_SIZES[name]
             out[name] = {"sizes": dict(z, layers=layers, vocab=V), design: measure(config_from_dict(safurax_config(z, layers, V))),
                          other: measure(config_from_dict(zarorax_config(z, layers, V)))}
+            print(f"[bench] {name}: {out[name]}", file=sys.stderr, flush=True)
+            continue
+        if design == "vuzinex":
+            z = VUZINEX_SIZES[name]
+            out[name] = {"sizes": dict(z, layers=layers, vocab=V), design: measure(config_from_dict(vuzinex_config(z, layers, V))),
+                         other: measure(config_from_dict(potatar_config(z, layers, V)))}
             print(f"[bench] {name}: {out[name]}", file=sys.stderr, flush=True)
             continue
         if design == "busadra":

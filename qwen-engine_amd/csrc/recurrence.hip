@@ -189,7 +189,7 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(Rec a) {
 // Row by row; out float32 [T, H, Dv] (norm_w is not looked at).
 extern "C" int qe_linear_recurrence(const Rec* rec, hipStream_t stream) {
     const Rec& a = *rec;
-    QE_REC_CHECK(a, "linear_recurrence");
+    QE_REC_CHECK(a, "linear_recurrence", false);
     QE_REQUIRE(a.out, "linear_recurrence: no place for the outputs");
     if (a.T == 0) return 0;
     dim3 grid(a.T, a.H, rec_copies(a.Dv));
@@ -250,6 +250,22 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
         for (int i = 0; i < RS_HOLD; ++i) load(Sp + (long)min(rg + i * RG, D - 1) * Dv + col, S[i]);
     }
     const float gate0 = a.gate && tid < Dv ? rec_gate(a, t, h * Dv + tid) : 0.f;      // (the first of a thread's columns)
+    float keep = 0.f, write = 0.f, floor = 0.f, m_new = 0.f;     // (mode 5: of the row and head)
+    if (MODE == 5) {
+        if (a.z) {
+            float i, f;
+            const float m = slot[a.m_at + h];
+            memory_gates_of(a.z[t * a.z_stride + h] + a.ib[h], a.z[t * a.z_stride + H + h] + a.fb[h], a.cap, i, f);
+            m_new = fmaxf(f + m, i);
+            keep = expf(f + m - m_new);
+            write = expf(i - m_new);
+            floor = expf(-m_new);
+        } else {
+            keep = a.wx[t * a.w_stride + h];
+            write = a.ks[t * a.w_stride + h];
+            floor = a.fl[t * a.w_stride + h];
+        }
+    }
     for (int d = tid; d < D; d += RS_THREADS) {
         const long at = t * a.row_stride + (long)hk * D + d;
         float x = Elem<TA>::load((const TA*)a.q + at), y = Elem<TA>::load((const TA*)a.k + at), f = 0.f;
@@ -258,8 +274,21 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
         if (MODE == 0) f = a.decay[h];
         if (MODE == 1) f = expf(-expf(a.wx[t * a.w_stride + h * D + d] + a.w0[h * D + d]));
         if (MODE == 2) { const float z = y + a.w0[h * D + d]; forget_gate(z, a.u[h * D + d], f, y); }
-        if (MODE == 3) f = a.wx[t * a.w_stride + h * D + d];
-        if (MODE >= 4) { f = a.wx[t * a.w_stride + h]; y *= a.ks[t * a.w_stride + h]; }
+        if (MODE == 3) {
+            if (a.low) {
+                float z = a.b2[h * D + d];
+                for (int r = 0; r < a.rank; ++r) {
+                    const long i = t * a.low_stride + r;
+                    const float l = a.dt_low == QE_F32 ? ((const float*)a.low)[i] : bf16_to_float(((const bf16_t*)a.low)[i]);
+                    z = fmaf(a.w2[(long)r * H * D + h * D + d], l, z);
+                }
+                f = low_rank_decay(z, a.inv_tau);
+            } else {
+                f = a.wx[t * a.w_stride + h * D + d];
+            }
+        }
+        if (MODE == 4) { f = a.wx[t * a.w_stride + h]; y *= a.ks[t * a.w_stride + h]; }
+        if (MODE == 5) { f = keep; y *= write; }
         sq[d] = x; sk[d] = y; sf[d] = f;
         if (MODE == 1) sb[d] = a.u[h * D + d];
     }
@@ -314,7 +343,8 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
         for (int d = tid; d < D; d += RS_THREADS)
             for (int z = 0; z < copies; ++z) slot[(long)H * D * Dv + ((long)z * H + h) * D + d] = sb[d];
         dn = block_sum(dn, red2);
-        inv = 1.f / (fmaxf(fabsf(dn), a.fl[t * a.w_stride + h]) + 1e-6f);
+        inv = 1.f / (fmaxf(fabsf(dn), floor) + 1e-6f);
+        if (a.z && tid == 0) slot[a.m_at + h] = m_new;       // (behind barriers that everyone reached after reading it)
     }
     __syncthreads();
     float all = 0.f;
@@ -344,7 +374,7 @@ extern "C" int qe_recurrence_single_supported(int D, int Dv) {
 // As qe_linear_recurrence for rows that are each the only row of their request; with norm_w the norm and the gate too.
 extern "C" int qe_recurrence_single(const Rec* rec, hipStream_t stream) {
     const Rec& a = *rec;
-    QE_REC_CHECK(a, "recurrence_single");
+    QE_REC_CHECK(a, "recurrence_single", true);
     QE_REQUIRE(qe_recurrence_single_supported(a.D, a.Dv), "recurrence_single: heads of %d x %d", a.D, a.Dv);
     QE_REQUIRE(a.norm_w || a.out, "recurrence_single: no place for the outputs");
     if (a.T == 0) return 0;

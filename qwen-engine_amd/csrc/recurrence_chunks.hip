@@ -10,7 +10,7 @@ int qe_recurrence_chunks_given(const Rec& a, hipStream_t stream);      // modes 
 extern "C" int qe_linear_recurrence_chunked(const Rec* rec, hipStream_t stream) {
     const Rec& a = *rec;
     QE_REQUIRE(a.n_chunks >= 0 && a.n_portions >= 0, "linear_recurrence: bad sizes");
-    QE_REC_CHECK(a, "linear_recurrence");
+    QE_REC_CHECK(a, "linear_recurrence", false);
     QE_REQUIRE(a.D >= 4, "linear_recurrence: heads of %d key channels (4 to 256 in chunks)", a.D);
     if (a.n_chunks == 0) return 0;
     QE_REQUIRE(a.chunks && a.portions && (a.all_single || a.ws), "linear_recurrence: chunks without a workspace");

@@ -13,6 +13,9 @@
 // q is multiplied by q_scale.  act_silu: q, k and v (mode 2: q) pass silu as they are read.
 // A request's state: H * D * Dv numbers; in mode 5 then rec_copies(Dv) equal copies of n [H][D] (a block of value columns
 // reads and writes its own).
+// Where every row is the only row of its request the kernel forms the decays of modes 3 and 5 itself from what they come
+// from: mode 3 from low (dt_low, rank numbers a row), w2 [rank][H * D], b2 and inv_tau (low_rank_decay below); mode 5 from the
+// gates' logits z [T][2 H], ib, fb, cap and the running maxima at state + m_at + h (memory_gates_of below).
 // Results: out float32 [T][H][Dv]; or, with norm_w [H * Dv], every head's o divided by its root mean square (norm_eps
 // inside), times the weight, times act(gate) (gate_act 1 silu, 2 sigmoid; number h * Dv + c of the gate's row), times
 // y_scale, in dt_y at y + t * y_stride + h * Dv.
@@ -40,7 +43,17 @@ struct Rec {
     const int* chunks;
     const int* portions;
     float* ws;
-    float norm_eps, q_scale, y_scale;
+    const void* low;
+    long low_stride;
+    const float* w2;
+    const float* b2;
+    const float* z;
+    long z_stride;
+    const float* ib;
+    const float* fb;
+    long m_at;
+    float norm_eps, q_scale, y_scale, inv_tau, cap;
+    int rank, dt_low;
     int mode, act_silu, dt_a, dt_y, dt_g, gate_act, T, H, Hk, D, Dv, n_chunks, n_portions, all_single;
 };
 
@@ -48,21 +61,21 @@ __host__ __device__ __forceinline__ int rec_copies(int Dv) { return (Dv + 63) / 
 __host__ __device__ __forceinline__ long rec_state_numbers(int mode, int H, int D, int Dv) {
     return (long)H * D * Dv + (mode == 5 ? (long)rec_copies(Dv) * H * D : 0);
 }
-static inline bool rec_operands_ok(const Rec& a) {
+static inline bool rec_operands_ok(const Rec& a, bool single) {
     switch (a.mode) {
         case 0: return a.decay != nullptr;
         case 1: return a.wx && a.w0 && a.u;
         case 2: return a.w0 && a.u;
-        case 3: return a.wx != nullptr;
+        case 3: return a.wx || (single && a.low && a.w2 && a.b2 && a.rank > 0);
         case 4: return a.wx && a.ks;
-        case 5: return a.wx && a.ks && a.fl;
+        case 5: return (a.wx && a.ks && a.fl) || (single && a.z && a.ib && a.fb && a.cap > 0.f);
     }
     return false;
 }
-#define QE_REC_CHECK(a, what)                                                                                            \
+#define QE_REC_CHECK(a, what, single)                                                                                            \
     QE_REQUIRE((a).T >= 0 && (a).H > 0 && (a).H <= 65535 && (a).D > 0 && (a).D <= 256 && (a).Dv > 0, what ": bad sizes (heads of %d x %d)", (a).D, (a).Dv); \
     QE_REQUIRE((a).Hk > 0 && (a).H % (a).Hk == 0 && ((a).mode == 4 || (a).Hk == (a).H), what ": %d heads over %d", (a).H, (a).Hk); \
-    QE_REQUIRE(rec_operands_ok(a), what ": mode %d lacks operands", (a).mode);                                              \
+    QE_REQUIRE(rec_operands_ok(a, single), what ": mode %d lacks operands", (a).mode);                                              \
     QE_REQUIRE((a).state && (a).state_stride >= rec_state_numbers((a).mode, (a).H, (a).D, (a).Dv), what ": state rows overlap"); \
     QE_REQUIRE((a).dt_a == QE_F32 || (a).dt_a == QE_BF16, what ": unknown element type %d", (a).dt_a);                      \
     QE_REQUIRE(!(a).norm_w || ((a).y && (a).y_stride >= (long)(a).H * (a).Dv && ((a).dt_y == QE_F32 || (a).dt_y == QE_BF16)), what ": no place for the normed rows"); \
@@ -93,6 +106,21 @@ __device__ __forceinline__ void forget_gate(float z, float l, float& f, float& k
     sigmoid_both(z, p, n);
     f = fmaf(1.f - l, p, l);
     kf = (1.f - l) * n;
+}
+
+__device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+// The log gates of a matrix memory from their logits (the biases added): i = cap * tanh(zi / cap), f = log sigmoid(cap *
+// tanh(zf / cap)).
+__device__ __forceinline__ void memory_gates_of(float zi, float zf, float cap, float& i, float& f) {
+    i = cap * tanhf(zi / cap);
+    f = log_sigmoid(cap * tanhf(zf / cap));
+}
+// sigmoid(z)^(1 / tau), from the hardware's exponential and logarithm of base 2: the argument of the last exponential is good
+// to some 1e-7 of 1 + |z|, and so is the decay
+__device__ __forceinline__ float low_rank_decay(float z, float inv_tau) {
+    const float l2e = 1.44269504f;
+    const float t = __builtin_amdgcn_exp2f(-fabsf(z) * l2e);
+    return __builtin_amdgcn_exp2f((fminf(z, 0.f) * l2e - __builtin_amdgcn_logf(1.f + t)) * inv_tau);
 }
 
 // what the gate of an output is: act(z), act 1 silu, 2 sigmoid

@@ -10,12 +10,11 @@
 //   qe_skip_gate_norm    y = (o + D_h x) * silu(z), normed in equal groups of a row, times a weight
 #include "recurrence_gates.h"
 
-__device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
-
 // ---- the gates of a matrix memory ------------------------------------------------------------------------------------
 struct MemoryGates {
-    const float* z;              // [T] rows: H input gates, H forget gates
-    long z_stride;
+    const float* z;              // [T] rows: H input gates, H forget gates; parts of them z_part apart, to be added in order
+    long z_stride, z_part;
+    int parts;
     const float* ib;
     const float* fb;
     float cap;
@@ -27,10 +26,11 @@ struct MemoryGates {
     const int* chunks;           // of the chunked recurrence, or null
     const int* portions;
 };
-__device__ __forceinline__ void memory_gates_of(const MemoryGates& a, long t, int h, float& i, float& f) {
+__device__ __forceinline__ void memory_gates_at(const MemoryGates& a, long t, int h, float& i, float& f) {
     const float* z = a.z + t * a.z_stride + h;
-    i = a.cap * tanhf((z[0] + a.ib[h]) / a.cap);
-    f = log_sigmoid(a.cap * tanhf((z[a.H] + a.fb[h]) / a.cap));
+    float zi = z[0], zf = z[a.H];
+    for (int p = 1; p < a.parts; ++p) { zi += z[p * a.z_part]; zf += z[p * a.z_part + a.H]; }
+    memory_gates_of(zi + a.ib[h], zf + a.fb[h], a.cap, i, f);
 }
 __device__ __forceinline__ float memory_gates_step(const MemoryGates& a, long t, int h, float i, float f, float m) {
     const float n = fmaxf(f + m, i);
@@ -49,33 +49,60 @@ __global__ __launch_bounds__(64) void memory_gates_rows_kernel(MemoryGates a) {
         float* ms = a.state + (long)seq * a.state_stride + h;
         float m = *ms, i, f;
         for (int t = t0; t < a.T && a.tok_seq[t] == seq; ++t) {
-            memory_gates_of(a, t, h, i, f);
+            memory_gates_at(a, t, h, i, f);
             m = memory_gates_step(a, t, h, i, f, m);
         }
         *ms = m;
     }
 }
 
-// grid (portions, H), 256 threads: every thread takes a run of neighbouring rows; the running maximum over the runs before
-// it is a scan over pairs (sum of log f, maximum): max(m + sum, maximum), so no sum is ever taken off another
-__global__ __launch_bounds__(256) void memory_gates_portions_kernel(MemoryGates a) {
-    __shared__ float sf[256], sm[256];
-    const int tid = threadIdx.x, h = blockIdx.y;
+// grid (portions, H), 512 threads: every thread takes a run of neighbouring rows; the running maximum over the runs before
+// it is a scan over pairs (sum of log f, maximum): max(m + sum, maximum), so no sum is ever taken off another.  The log gates
+// are formed once, MG_AHEAD rows at a time, and wait in the places of the results.
+#define MG_THREADS 512
+#define MG_AHEAD 4
+__global__ __launch_bounds__(MG_THREADS) void memory_gates_portions_kernel(MemoryGates a) {
+    __shared__ float sf[MG_THREADS], sm[MG_THREADS];
+    const int tid = threadIdx.x, h = blockIdx.y, H = a.H;
     const int* po = a.portions + 3 * blockIdx.x;
     const int* last = a.chunks + 3 * (po[0] + po[1] - 1);
     const long first = po[2];
-    const int n = last[0] + last[1] - (int)first, run = (n + 255) / 256;
+    const int n = last[0] + last[1] - (int)first, run = (n + MG_THREADS - 1) / MG_THREADS;
     const int b = min(tid * run, n), e = min(b + run, n);
-    float F = 0.f, M = -INFINITY, i, f;
-    for (int t = b; t < e; ++t) {
-        memory_gates_of(a, first + t, h, i, f);
-        F += f;
-        M = fmaxf(M + f, i);
+    float* out = a.out + first * 3 * H + h;
+    float* ms = a.state + (long)a.tok_seq[first] * a.state_stride + h;
+    const float m0 = *ms;
+    float F = 0.f, M = -INFINITY;
+    for (int t0 = b; t0 < e; t0 += MG_AHEAD) {
+        float zi[MG_AHEAD], zf[MG_AHEAD];
+#pragma unroll
+        for (int k = 0; k < MG_AHEAD; ++k) {               // (rows beyond the run read its last again)
+            const float* z = a.z + (first + min(t0 + k, e - 1)) * a.z_stride + h;
+            zi[k] = z[0];
+            zf[k] = z[H];
+        }
+        for (int p = 1; p < a.parts; ++p)
+#pragma unroll
+            for (int k = 0; k < MG_AHEAD; ++k) {
+                const float* z = a.z + p * a.z_part + (first + min(t0 + k, e - 1)) * a.z_stride + h;
+                zi[k] += z[0];
+                zf[k] += z[H];
+            }
+#pragma unroll
+        for (int k = 0; k < MG_AHEAD; ++k)
+            if (t0 + k < e) {
+                float i, f;
+                memory_gates_of(zi[k] + a.ib[h], zf[k] + a.fb[h], a.cap, i, f);
+                F += f;
+                M = fmaxf(M + f, i);
+                out[(long)(t0 + k) * 3 * H] = f;
+                out[(long)(t0 + k) * 3 * H + H] = i;
+            }
     }
     sf[tid] = F;
     sm[tid] = M;
     __syncthreads();
-    for (int o = 1; o < 256; o <<= 1) {                    // inclusive: (F1, M1) then (F2, M2) is (F1 + F2, max(M1 + F2, M2))
+    for (int o = 1; o < MG_THREADS; o <<= 1) {             // inclusive: (F1, M1) then (F2, M2) is (F1 + F2, max(M1 + F2, M2))
         float pf = 0.f, pm = -INFINITY;
         if (tid >= o) { pf = sf[tid - o]; pm = sm[tid - o]; }
         __syncthreads();
@@ -87,28 +114,34 @@ __global__ __launch_bounds__(256) void memory_gates_portions_kernel(MemoryGates 
         }
         __syncthreads();
     }
-    float* ms = a.state + (long)a.tok_seq[first] * a.state_stride + h;
-    const float m0 = *ms;
     float m = tid == 0 ? m0 : fmaxf(m0 + sf[tid - 1], sm[tid - 1]);
-    for (int t = b; t < e; ++t) {
-        memory_gates_of(a, first + t, h, i, f);
-        m = memory_gates_step(a, first + t, h, i, f, m);
+    for (int t0 = b; t0 < e; t0 += MG_AHEAD) {
+        float f[MG_AHEAD], i[MG_AHEAD];
+#pragma unroll
+        for (int k = 0; k < MG_AHEAD; ++k) {
+            const float* o = out + (long)min(t0 + k, e - 1) * 3 * H;
+            f[k] = o[0];
+            i[k] = o[H];
+        }
+#pragma unroll
+        for (int k = 0; k < MG_AHEAD; ++k)
+            if (t0 + k < e) m = memory_gates_step(a, first + t0 + k, h, i[k], f[k], m);
     }
-    __syncthreads();                                       // (everyone has read the state)
-    if (e == n && b < e) *ms = m;
+    if (e == n && b < e) *ms = m;                          // (everyone has read it: the scan's barriers)
 }
 
 // chunks and portions (or null, with n_portions 0): as in the chunked recurrence; without them the rows of a request are
 // walked one by one.
-extern "C" int qe_memory_gates(const float* z, long z_stride, const float* ib, const float* fb, float cap, float* state,
+// parts > 1: z is that many tensors of partial products, z_part numbers apart.
+extern "C" int qe_memory_gates(const float* z, long z_stride, int parts, long z_part, const float* ib, const float* fb, float cap, float* state,
                                long state_stride, const int* tok_seq, float* out, int T, int H, const int* chunks,
                                const int* portions, int n_portions, hipStream_t stream) {
-    QE_REQUIRE(T >= 0 && H > 0 && H <= 65535 && cap > 0.f && z_stride >= 2L * H && state_stride >= H, "memory_gates: bad sizes");
+    QE_REQUIRE(T >= 0 && H > 0 && H <= 65535 && cap > 0.f && parts >= 1 && z_stride >= 2L * H && state_stride >= H, "memory_gates: bad sizes");
     if (T == 0) return 0;
-    MemoryGates a{z, z_stride, ib, fb, cap, state, state_stride, tok_seq, out, T, H, chunks, portions};
+    MemoryGates a{z, z_stride, z_part, parts, ib, fb, cap, state, state_stride, tok_seq, out, T, H, chunks, portions};
     if (n_portions > 0) {
         QE_REQUIRE(chunks && portions, "memory_gates: portions without their chunks");
-        memory_gates_portions_kernel<<<dim3(n_portions, H), 256, 0, stream>>>(a);
+        memory_gates_portions_kernel<<<dim3(n_portions, H), MG_THREADS, 0, stream>>>(a);
     } else {
         memory_gates_rows_kernel<<<T, 64, 0, stream>>>(a);
     }
@@ -117,15 +150,19 @@ extern "C" int qe_memory_gates(const float* z, long z_stride, const float* ib, c
 }
 
 // ---- decays through a low rank ---------------------------------------------------------------------------------------
-// A block takes 16 rows x 256 channels; the rows' low numbers pass through shared memory, a thread holds its channel's
-// weights eight at a time.
-#define LR_ROWS 16
-template <typename TL, typename TW>
+// A block takes LR_ROWS rows x 256 channels, a thread a channel; the rows' low numbers pass through shared memory.
+#define LR_ROWS 8
+template <typename TL>
 __global__ __launch_bounds__(256) void low_rank_decay_kernel(const TL* __restrict__ low, long low_stride,
-                                                             const TW* __restrict__ w, const float* __restrict__ bias,
+                                                             const float* __restrict__ w, const float* __restrict__ bias,
                                                              float inv_tau, float* __restrict__ out, int T, int N, int R) {
     extern __shared__ float ls[];                          // [R][LR_ROWS]
-    const int t0 = blockIdx.x * LR_ROWS, c = blockIdx.y * 256 + threadIdx.x;
+    const int t0 = blockIdx.x * LR_ROWS, c = blockIdx.y * 256 + threadIdx.x, cc = min(c, N - 1);
+    constexpr int AHEAD = 16;                              // weights asked for before the rows' numbers are waited for
+    float wv[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) wv[j] = w[(long)min(j, R - 1) * N + cc];
+    const float b = bias[cc];
     for (int i = threadIdx.x; i < LR_ROWS * R; i += 256) {
         const int tt = i / R, r = i - tt * R;
         ls[r * LR_ROWS + tt] = t0 + tt < T ? Elem<TL>::load(low + (long)(t0 + tt) * low_stride + r) : 0.f;
@@ -133,15 +170,15 @@ __global__ __launch_bounds__(256) void low_rank_decay_kernel(const TL* __restric
     __syncthreads();
     if (c >= N) return;
     float acc[LR_ROWS];
-    const float b = bias[c];
 #pragma unroll
-    for (int tt = 0; tt < LR_ROWS; ++tt) acc[tt] = 0.f;
-    for (int r0 = 0; r0 < R; r0 += 8) {
-        float wv[8];
+    for (int tt = 0; tt < LR_ROWS; ++tt) acc[tt] = b;
+    for (int r0 = 0; r0 < R; r0 += AHEAD) {
+        if (r0 > 0) {
 #pragma unroll
-        for (int j = 0; j < 8; ++j) wv[j] = Elem<TW>::load(w + (long)c * R + min(r0 + j, R - 1));
+            for (int j = 0; j < AHEAD; ++j) wv[j] = w[(long)min(r0 + j, R - 1) * N + c];
+        }
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
+        for (int j = 0; j < AHEAD; ++j)
             if (r0 + j < R) {
 #pragma unroll
                 for (int tt = 0; tt < LR_ROWS; ++tt) acc[tt] = fmaf(wv[j], ls[(r0 + j) * LR_ROWS + tt], acc[tt]);
@@ -149,25 +186,19 @@ __global__ __launch_bounds__(256) void low_rank_decay_kernel(const TL* __restric
     }
 #pragma unroll
     for (int tt = 0; tt < LR_ROWS; ++tt)
-        if (t0 + tt < T) out[(long)(t0 + tt) * N + c] = expf(log_sigmoid(acc[tt] + b) * inv_tau);
+        if (t0 + tt < T) out[(long)(t0 + tt) * N + c] = low_rank_decay(acc[tt], inv_tau);
 }
 
-// low [T] rows of R numbers (dt_l), w [N][R] (dt_w), bias [N] -> out float32 [T][N]
-extern "C" int qe_low_rank_decay(const void* low, long low_stride, int dt_l, const void* w, int dt_w, const float* bias,
-                                 float tau, float* out, int T, int N, int R, hipStream_t stream) {
+// low [T] rows of R numbers (dt_l), w [R][N], bias [N] -> out float32 [T][N]
+extern "C" int qe_low_rank_decay(const void* low, long low_stride, int dt_l, const float* w, const float* bias, float tau,
+                                 float* out, int T, int N, int R, hipStream_t stream) {
     QE_REQUIRE(T >= 0 && N > 0 && R > 0 && R <= 1024 && tau > 0.f && low_stride >= R, "low_rank_decay: bad sizes (rank %d)", R);
     if (T == 0) return 0;
     const dim3 grid(qe_cdiv(T, LR_ROWS), qe_cdiv(N, 256));
     const size_t lds = (size_t)R * LR_ROWS * sizeof(float);
-#define QE_LRD(TL_, TW_) do {                                                                                                 \
-        if (lds > 48 * 1024)                                                                                                  \
-            (void)hipFuncSetAttribute((const void*)low_rank_decay_kernel<TL_, TW_>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
-        low_rank_decay_kernel<TL_, TW_><<<grid, 256, lds, stream>>>((const TL_*)low, low_stride, (const TW_*)w, bias, 1.f / tau, out, T, N, R); } while (0)
-    if (dt_l == QE_F32 && dt_w == QE_F32) QE_LRD(float, float);
-    else if (dt_l == QE_F32 && dt_w == QE_BF16) QE_LRD(float, bf16_t);
-    else if (dt_l == QE_BF16 && dt_w == QE_BF16) QE_LRD(bf16_t, bf16_t);
-    else QE_REQUIRE(false, "low_rank_decay: no kernel for rows of type %d and weights of type %d", dt_l, dt_w);
-#undef QE_LRD
+    if (dt_l == QE_F32) low_rank_decay_kernel<float><<<grid, 256, lds, stream>>>((const float*)low, low_stride, w, bias, 1.f / tau, out, T, N, R);
+    else if (dt_l == QE_BF16) low_rank_decay_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)low, low_stride, w, bias, 1.f / tau, out, T, N, R);
+    else QE_REQUIRE(false, "low_rank_decay: unknown element type %d", dt_l);
     QE_LAUNCH_CHECK();
     return 0;
 }
@@ -185,8 +216,9 @@ struct ConvSteps {
     const int* tok_seq;
     void* out;                   // [T][C]
     int T, C, taps;
-    const float* dt;             // [T] rows of H numbers, or null
-    long dt_stride;
+    const float* dt;             // [T] rows of H numbers, or null; parts of them dt_part apart, to be added in order
+    long dt_stride, dt_part;
+    int dt_parts;
     const float* dt_bias;
     const float* A_log;
     float* steps;                // [T][2 H]: decays, dt
@@ -196,7 +228,9 @@ struct ConvSteps {
 #define CS_ROWS 8
 
 __device__ __forceinline__ void conv_step_sizes(const ConvSteps& a, long t, int h) {
-    const float z = a.dt[t * a.dt_stride + h] + a.dt_bias[h];
+    float z = a.dt[t * a.dt_stride + h];
+    for (int p = 1; p < a.dt_parts; ++p) z += a.dt[p * a.dt_part + t * a.dt_stride + h];
+    z += a.dt_bias[h];
     const float dt = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
     a.steps[t * 2 * a.H + h] = expf(-expf(a.A_log[h]) * dt);
     a.steps[t * 2 * a.H + a.H + h] = dt;
@@ -336,7 +370,7 @@ __global__ __launch_bounds__(256) void conv_steps_state_kernel(ConvSteps a, cons
 // w [taps][C], b [C], state rows of (taps - 1) * C numbers; dt (or null): [T] rows of H logits -> steps [T][2 H].
 extern "C" int qe_conv_steps(const void* x, long x_stride, const float* w, const float* b, float* state, long state_stride,
                              const int* tok_seq, void* out, int T, int C, int taps, const float* dt, long dt_stride,
-                             const float* dt_bias, const float* A_log, float* steps, int H, int single_rows,
+                             int dt_parts, long dt_part, const float* dt_bias, const float* A_log, float* steps, int H, int single_rows,
                              const int* chunks, const int* portions, int n_portions, int dt_a, hipStream_t stream) {
     QE_REQUIRE(T >= 0 && C > 0 && taps >= 1 && x_stride >= C, "conv_steps: bad sizes T=%d C=%d taps=%d", T, C, taps);
     QE_REQUIRE(taps == 1 || (state && state_stride >= (long)(taps - 1) * C), "conv_steps: %d taps need a state", taps);
@@ -344,7 +378,7 @@ extern "C" int qe_conv_steps(const void* x, long x_stride, const float* w, const
     QE_REQUIRE(dt_a == QE_F32 || dt_a == QE_BF16, "conv_steps: unknown element type %d", dt_a);
     QE_REQUIRE(n_portions == 0 || (chunks && portions), "conv_steps: portions without their chunks");
     if (T == 0) return 0;
-    ConvSteps a{x, x_stride, w, b, state, state_stride, tok_seq, out, T, C, taps, dt, dt_stride, dt_bias, A_log, steps, H, single_rows};
+    ConvSteps a{x, x_stride, w, b, state, state_stride, tok_seq, out, T, C, taps, dt, dt_stride, dt_part, dt_parts, dt_bias, A_log, steps, H, single_rows};
     const size_t esz = dt_a == QE_BF16 ? 2 : 4;
     const bool four = C % 4 == 0 && x_stride % 4 == 0 && (((unsigned long)x) & (4 * esz - 1)) == 0 && state_stride % 4 == 0 &&
                       (((unsigned long)state) & 15) == 0;

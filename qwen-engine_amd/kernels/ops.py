@@ -103,9 +103,9 @@ def load_library():
         "qe_recurrence_single_supported": [i32, i32],
         "qe_recurrence_single": [vp, vp],
         "qe_linear_recurrence": [vp, vp],
-        "qe_memory_gates": [vp, i64, vp, vp, f32, vp, i64, vp, vp, i32, i32, vp, vp, i32, vp],
-        "qe_low_rank_decay": [vp, i64, i32, vp, i32, vp, f32, vp, i32, i32, i32, vp],
-        "qe_conv_steps": [vp, i64, vp, vp, vp, i64, vp, vp, i32, i32, i32, vp, i64, vp, vp, vp, i32, i32, vp, vp, i32, i32, vp],
+        "qe_memory_gates": [vp, i64, i32, i64, vp, vp, f32, vp, i64, vp, vp, i32, i32, vp, vp, i32, vp],
+        "qe_low_rank_decay": [vp, i64, i32, vp, vp, f32, vp, i32, i32, i32, vp],
+        "qe_conv_steps": [vp, i64, vp, vp, vp, i64, vp, vp, i32, i32, i32, vp, i64, i32, i64, vp, vp, vp, i32, i32, vp, vp, i32, i32, vp],
         "qe_skip_gate_norm": [vp, vp, i64, vp, vp, i64, vp, f32, vp, i64, i32, i32, i32, i32, i32, i32, vp],
         "qe_embedding_pairs": [vp, vp, vp, vp, vp, vp, f32, i64, i64, i64, vp, i32, i32, i32, i32, vp],
         "qe_branch_norm": [vp, vp, i32, f32, i32, vp, f32, f32, vp, i32, vp, f32, vp, i32, i32, i32, vp],
@@ -647,6 +647,12 @@ def gemm_branch_splits(x: torch.Tensor, w: torch.Tensor) -> int:
     if x.dtype not in _DT or w.dtype not in _DT:
         return 0
     return int(lib.qe_gemm_branch_splits(x.shape[0], w.shape[0], x.shape[1], _DT[x.dtype], _DT[w.dtype]))
+
+
+def gemm_splits_supported(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """True if gemm(epilogue=EPI_PARTIAL) takes these operands with any number of splits: bfloat16, more than 64 rows, K a multiple
+    of 8 (64 or more)."""
+    return x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and x.shape[0] > 64 and x.shape[1] % 8 == 0 and x.shape[1] >= 64
 
 
 def gemm_branch_splits_for(rows: int, w: torch.Tensor, x_dtype: torch.dtype) -> int:
@@ -1632,6 +1638,15 @@ def _rows_view(t: torch.Tensor, name: str, n: int, T: int):
     return t.stride(0) if T > 1 else n
 
 
+def _parts_view(t: torch.Tensor, name: str, n: int, T: int):
+    """(row stride, parts, distance of the parts) of [T, n] or partial products [S, T, n]."""
+    if t.dim() == 2:
+        return _rows_view(t, name, n, T), 1, 0
+    if t.dim() != 3 or t.shape[1:] != (T, n) or t.shape[0] < 1 or t.stride(2) != 1:
+        raise KernelError(f"{name} is {tuple(t.shape)} with strides {t.stride()}, expected parts of rows of {n} numbers")
+    return (t.stride(1) if T > 1 else n), t.shape[0], t.stride(0)
+
+
 def recurrence_chunk_len(rows: int, heads: int) -> int:
     """Rows of a chunk of the chunked recurrence, for the longest portion's rows and the heads: the longest of 64, 128 and
     256 that still gives every compute unit a block (the states between chunks cost less the longer the chunks are; a
@@ -1662,9 +1677,12 @@ class _Rec(ctypes.Structure):
                  ("w0", ctypes.c_void_p), ("u", ctypes.c_void_p), ("decay", ctypes.c_void_p), ("state", ctypes.c_void_p),
                  ("state_stride", ctypes.c_long), ("tok_seq", ctypes.c_void_p), ("out", ctypes.c_void_p),
                  ("norm_w", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y_stride", ctypes.c_long), ("gate", ctypes.c_void_p),
-                 ("gate_stride", ctypes.c_long), ("chunks", ctypes.c_void_p), ("portions", ctypes.c_void_p), ("ws", ctypes.c_void_p)] +
-                [(n, ctypes.c_float) for n in ("norm_eps", "q_scale", "y_scale")] +
-                [(n, ctypes.c_int) for n in ("mode", "act_silu", "dt_a", "dt_y", "dt_g", "gate_act", "T", "H", "Hk", "D", "Dv",
+                 ("gate_stride", ctypes.c_long), ("chunks", ctypes.c_void_p), ("portions", ctypes.c_void_p), ("ws", ctypes.c_void_p),
+                 ("low", ctypes.c_void_p), ("low_stride", ctypes.c_long), ("w2", ctypes.c_void_p), ("b2", ctypes.c_void_p),
+                 ("z", ctypes.c_void_p), ("z_stride", ctypes.c_long), ("ib", ctypes.c_void_p), ("fb", ctypes.c_void_p),
+                 ("m_at", ctypes.c_long)] +
+                [(n, ctypes.c_float) for n in ("norm_eps", "q_scale", "y_scale", "inv_tau", "cap")] +
+                [(n, ctypes.c_int) for n in ("rank", "dt_low", "mode", "act_silu", "dt_a", "dt_y", "dt_g", "gate_act", "T", "H", "Hk", "D", "Dv",
                                              "n_chunks", "n_portions", "all_single")])
 
 
@@ -1682,7 +1700,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
                       norm_dtype: Optional[torch.dtype] = None, single_rows: bool = False, decays: Optional[torch.Tensor] = None,
                       steps: Optional[torch.Tensor] = None, normaliser: bool = False, q_scale: float = 1.0, k_heads: int = 0,
                       gate: Optional[torch.Tensor] = None, gate_act: int = 0, y_scale: float = 1.0,
-                      out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      out: Optional[torch.Tensor] = None, low_rank=None, gates=None) -> torch.Tensor:
     """Per head, with a 32-bit state S [D][Dv] per request (state[tok_seq[t]], float32 [slots, >= recurrence_state_numbers]):
     with ``decay`` (float32 [H]):  S <- decay_h S + k_t v_t^T, o_t = S^T q_t;
     with ``decay_x`` float32 [T, H D], ``decay_bias`` and ``bonus`` (float32 [H D]):  o_t = (S + diag(bonus) k_t v_t^T)^T q_t,
@@ -1700,7 +1718,10 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     ``norm_weight`` (float32 [H Dv]): every head's o is divided by its root mean square (norm_eps inside) and multiplied
     by the weight, by act(``gate``) (``gate_act`` GATE_SILU or GATE_SIGMOID; gate [T, H Dv], may be a slice of columns) and by
     ``y_scale``; the result is [T, H Dv] in norm_dtype (in ``out``, which may be columns of wider rows, if given).
-    ``single_rows``: no two rows belong to one request (everything is then one launch)."""
+    ``single_rows``: no two rows belong to one request (everything is then one launch).
+    ``low_rank`` (low, w, bias, tau: what low_rank_decay() takes) stands in the place of ``decays``, ``gates`` (z, input bias, forget
+    bias, cap, place of the running maxima in a state row: what memory_gates() takes) in the place of ``steps`` with
+    ``normaliser``: what they give is formed by that kernel, or, with single rows, on the way."""
     lib = load_library()
     T, dev, H = q.shape[0], q.device, int(heads)
     Hk = int(k_heads) or H
@@ -1718,6 +1739,16 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         raise KernelError("linear_recurrence: the state is float32 [slots, >= H D Dv (and the normaliser)]")
     if D < 4:
         chunks = None                # (the chunked kernels read four channels at a time)
+    single = single_rows and bool(lib.qe_recurrence_single_supported(D, Dv))
+    if low_rank is not None and not single:
+        decays, low_rank = low_rank_decay(*low_rank), None
+    if gates is not None:
+        normaliser = True
+        z, ib, fb, cap, m_at = gates
+        if not 0 <= m_at <= state.shape[1] - H:
+            raise KernelError("linear_recurrence: the running maxima lie in the state row")
+        if not single or z.dim() == 3:
+            steps, gates = memory_gates(z, ib, fb, cap, state[:, m_at:m_at + H], tok_seq, chunks=chunks), None
     mode, sw = 0, 0
     wx, ks, fl, w0, u = decay_x, None, None, decay_bias, bonus
     if decay is not None:
@@ -1727,6 +1758,22 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         _need(forget_bias, "forget_bias", torch.float32, (H * D,), dev)
         _need(lower, "lower", torch.float32, (H * D,), dev)
         w0, u = forget_bias, lower
+    elif low_rank is not None:
+        mode = 3
+        low, w2, b2, tau = low_rank
+        R = w2.shape[0]
+        _need(w2, "w", torch.float32, (R, H * D), dev)
+        _need(b2, "bias", torch.float32, (H * D,), dev)
+        if low.dtype not in _ACT or not low.is_cuda:
+            raise KernelError("linear_recurrence: the low-rank rows are float32 or bfloat16 on the GPU")
+        sl = _rows_view(low, "low", R, T)
+    elif gates is not None:
+        mode = 5
+        if z.dtype != torch.float32 or not z.is_cuda:
+            raise KernelError("linear_recurrence: float32 logits of the gates")
+        sz = _rows_view(z, "z", 2 * H, T)
+        _need(ib, "input bias", torch.float32, (H,), dev)
+        _need(fb, "forget bias", torch.float32, (H,), dev)
     elif decays is not None:
         mode, wx = 3, decays
         _need(decays, "decays", torch.float32, (T, H * D), dev)
@@ -1762,13 +1809,17 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     elif gate is not None or out is not None:
         raise KernelError("linear_recurrence: a gate, or a place for the result, goes with the norm")
     use_chunks = chunks is not None and chunks[0].shape[0] > 0
-    single = single_rows and bool(lib.qe_recurrence_single_supported(D, Dv))
     fused_norm = normed and (single or (use_chunks and Dv <= 128))
     o = None if fused_norm else torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
     r = _Rec(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), row_stride=sq, wx=_ptr(wx), ks=_ptr(ks), fl=_ptr(fl), w_stride=sw,
              w0=_ptr(w0), u=_ptr(u), decay=_ptr(decay), state=state.data_ptr(), state_stride=state.stride(0),
              tok_seq=tok_seq.data_ptr(), out=_ptr(o), q_scale=float(q_scale), y_scale=float(y_scale), mode=mode,
              act_silu=int(bool(silu)), dt_a=_DT[q.dtype], T=T, H=H, Hk=Hk, D=D, Dv=Dv)
+    if low_rank is not None:
+        r.low, r.low_stride, r.dt_low, r.rank = low.data_ptr(), sl, _DT[low.dtype], R
+        r.w2, r.b2, r.inv_tau = w2.data_ptr(), b2.data_ptr(), 1.0 / float(tau)
+    if gates is not None:
+        r.z, r.z_stride, r.ib, r.fb, r.cap, r.m_at = z.data_ptr(), sz, ib.data_ptr(), fb.data_ptr(), float(cap), int(m_at)
     if fused_norm:
         r.norm_w, r.norm_eps, r.y, r.y_stride, r.dt_y = norm_weight.data_ptr(), float(norm_eps), out.data_ptr(), sy, _DT[out.dtype]
         if gate is not None:
@@ -1798,16 +1849,16 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
 def memory_gates(z: torch.Tensor, input_bias: torch.Tensor, forget_bias: torch.Tensor, cap: float, running_max: torch.Tensor,
                  tok_seq: torch.Tensor, chunks=None) -> torch.Tensor:
     """The ``steps`` [T, 3 H] of linear_recurrence(normaliser=True) from the logits z float32 [T, 2 H] (input gates, forget gates;
-    columns of wider rows are taken as they are): i = cap tanh((z_i + input_bias) / cap), f = log sigmoid(cap tanh((z_f +
+    columns of wider rows are taken as they are; or [S, T, 2 H]: partial products to be added in order): i = cap tanh((z_i + input_bias) / cap), f = log sigmoid(cap tanh((z_f +
     forget_bias) / cap)), m_t = max(f + m_(t-1), i); decay exp(f + m_(t-1) - m_t), key factor exp(i - m_t), floor exp(-m_t).
     running_max float32 [slots, H] (columns of wider rows): m of every request, brought up to date.  ``chunks``: as in
     linear_recurrence()."""
     lib = load_library()
-    T, dev = z.shape[0], z.device
+    T, dev = z.shape[-2], z.device
     H = input_bias.shape[0]
     if z.dtype != torch.float32 or not z.is_cuda:
         raise KernelError("memory_gates: float32 logits on the GPU")
-    sz = _rows_view(z, "z", 2 * H, T)
+    sz, parts, part = _parts_view(z, "z", 2 * H, T)
     _need(input_bias, "input_bias", torch.float32, (H,), dev)
     _need(forget_bias, "forget_bias", torch.float32, (H,), dev)
     _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
@@ -1815,24 +1866,25 @@ def memory_gates(z: torch.Tensor, input_bias: torch.Tensor, forget_bias: torch.T
         raise KernelError("memory_gates: the running maximum is float32 [slots, H]")
     steps = torch.empty((T, 3 * H), dtype=torch.float32, device=dev)
     ch, po = chunks if chunks is not None else (None, None)
-    _check(lib.qe_memory_gates(z.data_ptr(), sz, input_bias.data_ptr(), forget_bias.data_ptr(), float(cap), running_max.data_ptr(),
+    _check(lib.qe_memory_gates(z.data_ptr(), sz, parts, part, input_bias.data_ptr(), forget_bias.data_ptr(), float(cap), running_max.data_ptr(),
                                running_max.stride(0), tok_seq.data_ptr(), steps.data_ptr(), T, H, _ptr(ch), _ptr(po),
                                0 if po is None else po.shape[0], _stream()), "memory_gates")
     return steps
 
 
 def low_rank_decay(low: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
-    """sigmoid(low . w^T + bias)^(1 / tau), float32 [T, N]: low [T, R] (columns of wider rows are taken as they are), w [N, R]."""
+    """sigmoid(low . w + bias)^(1 / tau), float32 [T, N]: low [T, R] (columns of wider rows are taken as they are), w float32
+    [R, N]."""
     lib = load_library()
-    T, (N, R) = low.shape[0], w.shape
+    T, (R, N) = low.shape[0], w.shape
     if low.dtype not in _ACT or not low.is_cuda:
         raise KernelError("low_rank_decay: float32 or bfloat16 rows on the GPU")
     sl = _rows_view(low, "low", R, T)
-    _need(w, "w", _ACT, (N, R), low.device)
+    _need(w, "w", torch.float32, (R, N), low.device)
     _need(bias, "bias", torch.float32, (N,), low.device)
     out = torch.empty((T, N), dtype=torch.float32, device=low.device)
-    _check(lib.qe_low_rank_decay(low.data_ptr(), sl, _DT[low.dtype], w.data_ptr(), _DT[w.dtype], bias.data_ptr(), float(tau),
-                                 out.data_ptr(), T, N, R, _stream()), "low_rank_decay")
+    _check(lib.qe_low_rank_decay(low.data_ptr(), sl, _DT[low.dtype], w.data_ptr(), bias.data_ptr(), float(tau), out.data_ptr(), T, N,
+                                 R, _stream()), "low_rank_decay")
     return out
 
 
@@ -1841,7 +1893,8 @@ def conv_steps(x: torch.Tensor, w_t: torch.Tensor, bias: torch.Tensor, state: Op
                single_rows: bool = False, chunks=None):
     """silu(bias + causal convolution over time) of every channel: x [T, C] (columns of wider rows are taken as they are), w_t
     float32 [taps, C] (the last row is the current token's), state float32 [slots, (taps - 1) C] (columns of wider rows; row
-    tok_seq[t]: the request's last inputs), brought up to date.  With ``dt`` (float32 logits [T, H]): also the step sizes
+    tok_seq[t]: the request's last inputs), brought up to date.  With ``dt`` (float32 logits [T, H], or partial products [S, T, H] to be added
+    in order): also the step sizes
     softplus(dt + dt_bias) and the decays exp(-exp(a_log) * step).  Returns (rows [T, C] in x's type, float32 [T, 2 H] = decays,
     step sizes, or None).  ``single_rows``: no two rows belong to one request (one launch)."""
     lib = load_library()
@@ -1856,19 +1909,19 @@ def conv_steps(x: torch.Tensor, w_t: torch.Tensor, bias: torch.Tensor, state: Op
     if taps > 1 and (state is None or state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < (taps - 1) * C or
                      state.stride(1) != 1 or state.device != dev):
         raise KernelError("conv_steps: the state is float32 [slots, >= (taps - 1) C]")
-    H, sd, steps = 0, 0, None
+    H, sd, dp, dpart, steps = 0, 0, 1, 0, None
     if dt is not None:
         H = dt_bias.shape[0]
         if dt.dtype != torch.float32:
             raise KernelError("conv_steps: float32 step logits")
-        sd = _rows_view(dt, "dt", H, T)
+        sd, dp, dpart = _parts_view(dt, "dt", H, T)
         _need(dt_bias, "dt_bias", torch.float32, (H,), dev)
         _need(a_log, "a_log", torch.float32, (H,), dev)
         steps = torch.empty((T, 2 * H), dtype=torch.float32, device=dev)
     ch, po = chunks if chunks is not None else (None, None)
     out = torch.empty((T, C), dtype=x.dtype, device=dev)
     _check(lib.qe_conv_steps(x.data_ptr(), sx, w_t.data_ptr(), bias.data_ptr(), _ptr(state), 0 if state is None else state.stride(0),
-                             tok_seq.data_ptr(), out.data_ptr(), T, C, taps, _ptr(dt), sd, _ptr(dt_bias), _ptr(a_log), _ptr(steps), H,
+                             tok_seq.data_ptr(), out.data_ptr(), T, C, taps, _ptr(dt), sd, dp, dpart, _ptr(dt_bias), _ptr(a_log), _ptr(steps), H,
                              int(bool(single_rows)), _ptr(ch), _ptr(po), 0 if po is None else po.shape[0], _DT[x.dtype], _stream()),
            "conv_steps")
     return out, steps

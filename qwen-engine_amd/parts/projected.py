@@ -6,8 +6,9 @@ A *projected* mixer defines
   output(tensors) -> matrix [H, K]   its output projection
   output_width(spec) -> K
   mix(y, gates, ctx, binding, out, factor)   y [T, n] the first kind's results (columns of wider rows, in the activation
-                                  type or float32), gates float32 [T, n'] the second's (or None); leaves factor * the
-                                  result before the output projection in out [T, K] (columns of wider rows)
+                                  type or float32), gates float32 [T, n'], or [S, T, n'] partial products, the second's (or
+                                  None); leaves factor * the result before the output projection in out [T, K] (columns of
+                                  wider rows)
 """
 from __future__ import annotations
 
@@ -64,8 +65,21 @@ class InputProducts:
             gates = y[:, self.n_main:]
         else:
             y = ops.gemm(x, self._w_main, self._b_main)
-            gates = ops.gemm(x, self._w_gates, out_dtype=torch.float32) if self._w_gates is not None else None
-        return [(y[:, a:b], gates[:, c:d] if d > c else None) for (a, b), (c, d) in zip(self.main_cols, self.gate_cols)]
+            gates = self._few_columns(x) if self._w_gates is not None else None
+        return [(y[:, a:b], gates[..., c:d] if d > c else None) for (a, b), (c, d) in zip(self.main_cols, self.gate_cols)]
+
+
+    def _few_columns(self, x: torch.Tensor) -> torch.Tensor:
+        """The 32-bit results against many rows: a product of so few columns has few tiles, each a walk over all of K, so
+        it is cut along K (in the order of the cuts the consumer adds the parts)."""
+        tiles = -(-x.shape[0] // 64) * -(-self._w_gates.shape[0] // 128)
+        splits = max(1, min(8, 256 // tiles, x.shape[1] // 256))
+        K = x.shape[1]
+        while splits > 1 and (splits - 1) * (-(-(-(-K // splits)) // 64) * 64) >= K:      # (every cut has some of K)
+            splits -= 1
+        if splits > 1 and ops.gemm_splits_supported(x, self._w_gates):
+            return ops.gemm(x, self._w_gates, epilogue=ops.EPI_PARTIAL, splits=splits)
+        return ops.gemm(x, self._w_gates, out_dtype=torch.float32)
 
 
 class OutputProduct:

@@ -200,8 +200,8 @@ class ForgetGateLinearMixer:
 
 
 class GatedLinearMixer(ProjectedMixer):
-    """``GatedLinearSpec``: the decays come from the low-rank projection in a kernel of their own, the recurrence has the
-    norm per head and the silu gate behind it."""
+    """``GatedLinearSpec``: the decays come from the low-rank projection in a kernel of their own (single new tokens: inside the
+    recurrence), the recurrence has the norm per head and the silu gate behind it."""
 
     def __init__(self, spec, hidden_size: int):
         self.spec = spec
@@ -236,7 +236,7 @@ class GatedLinearMixer(ProjectedMixer):
 
     def load_own(self, tensors: Dict[str, torch.Tensor], rt: Runtime) -> None:
         _, _, _, _, _, norm, _, a2, a2b = self.spec.names
-        self.w_2 = rt.place_matrix(tensors[a2])
+        self.w_2 = rt.place_vector(tensors[a2].t())          # [rank, channels], 32-bit: neighbouring channels side by side
         self.b_2 = rt.place_vector(tensors[a2b])
         self.norm = rt.place_vector(tensors[norm]).repeat(self.h)
 
@@ -244,17 +244,16 @@ class GatedLinearMixer(ProjectedMixer):
         if binding.state is None:
             raise RuntimeError("the recurrence was given no state")
         nk, nv = self.h * self.d, self.h * self.dv
-        decays = ops.low_rank_decay(y[:, 2 * nk + 2 * nv:], self.w_2, self.b_2, self.tau)
-        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], binding.state, ctx.tok_seq, self.h, decays=decays,
-                              q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
+        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], binding.state, ctx.tok_seq, self.h,
+                              low_rank=(y[:, 2 * nk + 2 * nv:], self.w_2, self.b_2, self.tau), q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
                               norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:2 * nk + 2 * nv],
                               gate_act=ops.GATE_SILU, y_scale=factor, out=out)
 
 
 class MatrixMemoryMixer(ProjectedMixer):
     """``MatrixMemorySpec``: the two gates' logits stay 32-bit; a kernel turns them into decays, key factors and floors
-    along the running maximum; the recurrence carries its normaliser and has the norm per head and the sigmoid gate behind
-    it.  State: the matrices, the normalisers, the running maxima."""
+    along the running maximum (single new tokens: inside the recurrence); the recurrence carries its normaliser and has the
+    norm per head and the sigmoid gate behind it.  State: the matrices, the normalisers, the running maxima."""
 
     def __init__(self, spec, hidden_size: int):
         self.spec = spec
@@ -297,10 +296,8 @@ class MatrixMemoryMixer(ProjectedMixer):
             raise RuntimeError("the recurrence was given no state")
         nk, nv = self.h * self.d, self.h * self.dv
         at = ops.recurrence_state_numbers(self.h, self.d, self.dv, normaliser=True)
-        chunks = _chunks(ctx, self.h)
-        steps = ops.memory_gates(gates, self.b_i, self.b_f, self.cap, st[:, at:at + self.h], ctx.tok_seq, chunks=chunks)
-        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], st, ctx.tok_seq, self.h, steps=steps,
-                              normaliser=True, q_scale=self.d ** -0.5, chunks=chunks, norm_weight=self.norm, norm_eps=self.eps,
+        ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], st, ctx.tok_seq, self.h,
+                              gates=(gates, self.b_i, self.b_f, self.cap, at), q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
                               norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:],
                               gate_act=ops.GATE_SIGMOID, y_scale=factor, out=out)
 
