@@ -119,7 +119,7 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(Rec a) {
                 if (MODE == 2) { const float z = y + a.w0[h * D + d]; forget_gate(z, a.u[h * D + d], c, y); }
                 if (MODE == 1) c = expf(-expf(a.wx[wr + h * D + d] + a.w0[h * D + d]));
                 if (MODE == 3) c = a.wx[wr + h * D + d];
-                if (MODE >= 4) { c = a.wx[wr + h]; y *= a.ks[wr + h]; }
+                if (MODE >= 4) { c = a.wx[wr + h * a.w_head]; y *= a.ks[wr + h * a.w_head]; }
             }
             sq[tt][d] = x; sk[tt][d] = y; sw[tt][d] = c;
         }
@@ -171,7 +171,7 @@ __global__ __launch_bounds__(REC_DG * 64) void linear_recurrence_kernel(Rec a) {
                     float dn = den[tt][0];
 #pragma unroll
                     for (int g = 1; g < REC_DG; ++g) dn += den[tt][g];
-                    o /= fmaxf(fabsf(dn), a.fl[(long)(tb + tt) * a.w_stride + h]) + 1e-6f;
+                    o /= fmaxf(fabsf(dn), a.fl[(long)(tb + tt) * a.w_stride + h * a.w_head]) + 1e-6f;
                 }
                 a.out[((long)(tb + tt) * H + h) * Dv + blockIdx.z * 64 + c] = o;
             }
@@ -261,9 +261,9 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
             write = expf(i - m_new);
             floor = expf(-m_new);
         } else {
-            keep = a.wx[t * a.w_stride + h];
-            write = a.ks[t * a.w_stride + h];
-            floor = a.fl[t * a.w_stride + h];
+            keep = a.wx[t * a.w_stride + h * a.w_head];
+            write = a.ks[t * a.w_stride + h * a.w_head];
+            floor = a.fl[t * a.w_stride + h * a.w_head];
         }
     }
     for (int d = tid; d < D; d += RS_THREADS) {
@@ -277,17 +277,26 @@ __global__ __launch_bounds__(RS_THREADS) void recurrence_single_kernel(Rec a) {
         if (MODE == 3) {
             if (a.low) {
                 float z = a.b2[h * D + d];
-                for (int r = 0; r < a.rank; ++r) {
-                    const long i = t * a.low_stride + r;
-                    const float l = a.dt_low == QE_F32 ? ((const float*)a.low)[i] : bf16_to_float(((const bf16_t*)a.low)[i]);
-                    z = fmaf(a.w2[(long)r * H * D + h * D + d], l, z);
+                constexpr int N = 16;                        // asked for at a time (beyond the rank: its last again, unused)
+                for (int r0 = 0; r0 < a.rank; r0 += N) {
+                    float w[N], l[N];
+#pragma unroll
+                    for (int j = 0; j < N; ++j) {
+                        const int r = min(r0 + j, a.rank - 1);
+                        const long i = t * a.low_stride + r;
+                        w[j] = a.w2[(long)r * H * D + h * D + d];
+                        l[j] = a.dt_low == QE_F32 ? ((const float*)a.low)[i] : bf16_to_float(((const bf16_t*)a.low)[i]);
+                    }
+#pragma unroll
+                    for (int j = 0; j < N; ++j)
+                        if (r0 + j < a.rank) z = fmaf(w[j], l[j], z);
                 }
                 f = low_rank_decay(z, a.inv_tau);
             } else {
                 f = a.wx[t * a.w_stride + h * D + d];
             }
         }
-        if (MODE == 4) { f = a.wx[t * a.w_stride + h]; y *= a.ks[t * a.w_stride + h]; }
+        if (MODE == 4) { f = a.wx[t * a.w_stride + h * a.w_head]; y *= a.ks[t * a.w_stride + h * a.w_head]; }
         if (MODE == 5) { f = keep; y *= write; }
         sq[d] = x; sk[d] = y; sf[d] = f;
         if (MODE == 1) sb[d] = a.u[h * D + d];

@@ -138,7 +138,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(Rec a) {
     const TA* kc = k + (long)row0 * a.row_stride + (long)hk * D;
     const TA* vc = v + (long)row0 * a.row_stride + (long)h * Dv + (col_ok ? col : 0);
     const float* wc = MODE == 1 || MODE == 3 ? a.wx + (long)row0 * a.w_stride + (long)h * D : nullptr;
-    const long row_scalar = (long)row0 * a.w_stride + h;
+    const long row_scalar = (long)row0 * a.w_stride + h * a.w_head;
     const int stride = (int)a.row_stride, w_stride = (int)a.w_stride;
     auto fetch = [&](int base) {
         const int row = min(base + r, n - 1);

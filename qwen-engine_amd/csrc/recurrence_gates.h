@@ -9,6 +9,7 @@
 //   mode 2: k holds a forget gate's logits, w0 its bias, u its lower bound [H * D]   S <- diag(f) S + (1 - f) v^T   o = S^T q
 //   mode 3: wx [T][H * D] the decays themselves                         S <- diag(w) S + k v^T  o = S^T q
 //   mode 4: wx [T][H] one decay a row and head, ks [T][H] a factor on the key     S <- w S + (ks k) v^T  o = S^T q
+//           (number (t, h) of wx, ks and fl at t * w_stride + h * w_head)
 //   mode 5: as 4, and n <- w n + ks k; o = S^T q / (max(|n . q|, fl) + 1e-6) with fl [T][H]
 // q is multiplied by q_scale.  act_silu: q, k and v (mode 2: q) pass silu as they are read.
 // A request's state: H * D * Dv numbers; in mode 5 then rec_copies(Dv) equal copies of n [H][D] (a block of value columns
@@ -27,7 +28,8 @@ struct Rec {
     const float* wx;
     const float* ks;
     const float* fl;
-    long w_stride;                  // of wx, ks and fl
+    long w_stride;                  // of wx, ks and fl: from row to row
+    long w_head;                    // and (modes 4 and 5) from head to head
     const float* w0;
     const float* u;
     const float* decay;

@@ -21,7 +21,8 @@ struct MemoryGates {
     float* state;                // m of head h at + slot * state_stride + h
     long state_stride;
     const int* tok_seq;
-    float* out;                  // [T][3 H]: decay, key factor, floor
+    float* out;                  // decay, key factor, floor of row t and head h at + k * o_kind + t * o_row + h * o_head
+    long o_kind, o_row, o_head;
     int T, H;
     const int* chunks;           // of the chunked recurrence, or null
     const int* portions;
@@ -31,14 +32,6 @@ __device__ __forceinline__ void memory_gates_at(const MemoryGates& a, long t, in
     float zi = z[0], zf = z[a.H];
     for (int p = 1; p < a.parts; ++p) { zi += z[p * a.z_part]; zf += z[p * a.z_part + a.H]; }
     memory_gates_of(zi + a.ib[h], zf + a.fb[h], a.cap, i, f);
-}
-__device__ __forceinline__ float memory_gates_step(const MemoryGates& a, long t, int h, float i, float f, float m) {
-    const float n = fmaxf(f + m, i);
-    float* o = a.out + t * 3 * a.H + h;
-    o[0] = expf(f + m - n);
-    o[a.H] = expf(i - n);
-    o[2 * a.H] = expf(-n);
-    return n;
 }
 
 // grid (T): the block of a request's first row walks its rows, a thread a head
@@ -50,98 +43,101 @@ __global__ __launch_bounds__(64) void memory_gates_rows_kernel(MemoryGates a) {
         float m = *ms, i, f;
         for (int t = t0; t < a.T && a.tok_seq[t] == seq; ++t) {
             memory_gates_at(a, t, h, i, f);
-            m = memory_gates_step(a, t, h, i, f, m);
+            const float n = fmaxf(f + m, i);
+            float* o = a.out + t * a.o_row + h * a.o_head;
+            o[0] = expf(f + m - n);
+            o[a.o_kind] = expf(i - n);
+            o[2 * a.o_kind] = expf(-n);
+            m = n;
         }
         *ms = m;
     }
 }
 
-// grid (portions, H), 512 threads: every thread takes a run of neighbouring rows; the running maximum over the runs before
-// it is a scan over pairs (sum of log f, maximum): max(m + sum, maximum), so no sum is ever taken off another.  The log gates
-// are formed once, MG_AHEAD rows at a time, and wait in the places of the results.
-#define MG_THREADS 512
-#define MG_AHEAD 4
-__global__ __launch_bounds__(MG_THREADS) void memory_gates_portions_kernel(MemoryGates a) {
-    __shared__ float sf[MG_THREADS], sm[MG_THREADS];
-    const int tid = threadIdx.x, h = blockIdx.y, H = a.H;
+// Many rows: every gate first (log f in the decay's place, i in the key factor's), a thread a row and head ...
+__global__ __launch_bounds__(256) void memory_gates_each_kernel(MemoryGates a) {
+    const int n = blockIdx.x * 256 + threadIdx.x, t = n / a.H, h = n - t * a.H;
+    if (t >= a.T) return;
+    float i, f;
+    memory_gates_at(a, t, h, i, f);
+    float* o = a.out + t * a.o_row + h * a.o_head;
+    o[0] = f;
+    o[a.o_kind] = i;
+}
+
+// ... then the running maximum: grid (portions, H), MG_ROWS neighbouring rows a thread, MG_THREADS of them at a time.  The
+// maximum over what lies before a thread's rows is a scan over pairs (sum of log f, maximum), (F1, M1) then (F2, M2) being
+// (F1 + F2, max(M1 + F2, M2)): no sum is ever taken off another.
+#define MG_THREADS 1024
+#define MG_ROWS 2
+__global__ __launch_bounds__(MG_THREADS) void memory_gates_scan_kernel(MemoryGates a) {
+    __shared__ float wf[MG_THREADS / 64], wm[MG_THREADS / 64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y;
     const int* po = a.portions + 3 * blockIdx.x;
     const int* last = a.chunks + 3 * (po[0] + po[1] - 1);
     const long first = po[2];
-    const int n = last[0] + last[1] - (int)first, run = (n + MG_THREADS - 1) / MG_THREADS;
-    const int b = min(tid * run, n), e = min(b + run, n);
-    float* out = a.out + first * 3 * H + h;
+    const int n = last[0] + last[1] - (int)first;
+    float* out = a.out + first * a.o_row + h * a.o_head;
     float* ms = a.state + (long)a.tok_seq[first] * a.state_stride + h;
-    const float m0 = *ms;
-    float F = 0.f, M = -INFINITY;
-    for (int t0 = b; t0 < e; t0 += MG_AHEAD) {
-        float zi[MG_AHEAD], zf[MG_AHEAD];
+    float m0 = *ms;                                        // the running maximum before the rows of this turn
+    for (int b = 0; b < n; b += MG_THREADS * MG_ROWS) {
+        const int t0 = b + tid * MG_ROWS;
+        float f[MG_ROWS], i[MG_ROWS], F = 0.f, M = -INFINITY;
 #pragma unroll
-        for (int k = 0; k < MG_AHEAD; ++k) {               // (rows beyond the run read its last again)
-            const float* z = a.z + (first + min(t0 + k, e - 1)) * a.z_stride + h;
-            zi[k] = z[0];
-            zf[k] = z[H];
-        }
-        for (int p = 1; p < a.parts; ++p)
-#pragma unroll
-            for (int k = 0; k < MG_AHEAD; ++k) {
-                const float* z = a.z + p * a.z_part + (first + min(t0 + k, e - 1)) * a.z_stride + h;
-                zi[k] += z[0];
-                zf[k] += z[H];
-            }
-#pragma unroll
-        for (int k = 0; k < MG_AHEAD; ++k)
-            if (t0 + k < e) {
-                float i, f;
-                memory_gates_of(zi[k] + a.ib[h], zf[k] + a.fb[h], a.cap, i, f);
-                F += f;
-                M = fmaxf(M + f, i);
-                out[(long)(t0 + k) * 3 * H] = f;
-                out[(long)(t0 + k) * 3 * H + H] = i;
-            }
-    }
-    sf[tid] = F;
-    sm[tid] = M;
-    __syncthreads();
-    for (int o = 1; o < MG_THREADS; o <<= 1) {             // inclusive: (F1, M1) then (F2, M2) is (F1 + F2, max(M1 + F2, M2))
-        float pf = 0.f, pm = -INFINITY;
-        if (tid >= o) { pf = sf[tid - o]; pm = sm[tid - o]; }
-        __syncthreads();
-        if (tid >= o) {
-            M = fmaxf(pm + F, M);
-            F += pf;
-            sf[tid] = F;
-            sm[tid] = M;
-        }
-        __syncthreads();
-    }
-    float m = tid == 0 ? m0 : fmaxf(m0 + sf[tid - 1], sm[tid - 1]);
-    for (int t0 = b; t0 < e; t0 += MG_AHEAD) {
-        float f[MG_AHEAD], i[MG_AHEAD];
-#pragma unroll
-        for (int k = 0; k < MG_AHEAD; ++k) {
-            const float* o = out + (long)min(t0 + k, e - 1) * 3 * H;
+        for (int k = 0; k < MG_ROWS; ++k) {
+            const float* o = out + min(t0 + k, n - 1) * a.o_row;
             f[k] = o[0];
-            i[k] = o[H];
+            i[k] = o[a.o_kind];
         }
 #pragma unroll
-        for (int k = 0; k < MG_AHEAD; ++k)
-            if (t0 + k < e) m = memory_gates_step(a, first + t0 + k, h, i[k], f[k], m);
+        for (int k = 0; k < MG_ROWS; ++k)
+            if (t0 + k < n) { F += f[k]; M = fmaxf(M + f[k], i[k]); }
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {                 // inclusive over the wave
+            const float pf = __shfl_up(F, o, 64), pm = __shfl_up(M, o, 64);
+            if (lane >= o) { M = fmaxf(pm + F, M); F += pf; }
+        }
+        if (lane == 63) { wf[wave] = F; wm[wave] = M; }
+        float eF = __shfl_up(F, 1, 64), eM = __shfl_up(M, 1, 64);      // what lies before this thread's rows in its wave
+        if (lane == 0) { eF = 0.f; eM = -INFINITY; }
+        __syncthreads();
+        float m = m0, all = m0;
+        for (int w = 0; w < MG_THREADS / 64; ++w) {        // the waves before, then all of them
+            if (w == wave) m = all;
+            all = fmaxf(all + wf[w], wm[w]);
+        }
+        m = fmaxf(m + eF, eM);
+        m0 = all;
+#pragma unroll
+        for (int k = 0; k < MG_ROWS; ++k)
+            if (t0 + k < n) {
+                const float x = fmaxf(f[k] + m, i[k]);
+                float* o = out + (t0 + k) * a.o_row;
+                o[0] = expf(f[k] + m - x);
+                o[a.o_kind] = expf(i[k] - x);
+                o[2 * a.o_kind] = expf(-x);
+                m = x;
+            }
+        __syncthreads();                                   // (the waves' pairs have been read)
     }
-    if (e == n && b < e) *ms = m;                          // (everyone has read it: the scan's barriers)
+    if (tid == 0) *ms = m0;
 }
 
-// chunks and portions (or null, with n_portions 0): as in the chunked recurrence; without them the rows of a request are
-// walked one by one.
-// parts > 1: z is that many tensors of partial products, z_part numbers apart.
-extern "C" int qe_memory_gates(const float* z, long z_stride, int parts, long z_part, const float* ib, const float* fb, float cap, float* state,
-                               long state_stride, const int* tok_seq, float* out, int T, int H, const int* chunks,
-                               const int* portions, int n_portions, hipStream_t stream) {
+// out: number (k, t, h) at k * o_kind + t * o_row + h * o_head, k = decay, key factor, floor.  chunks and portions (or null,
+// with n_portions 0): as in the chunked recurrence; without them the rows of a request are walked one by one.  parts > 1: z is
+// that many tensors of partial products, z_part numbers apart.
+extern "C" int qe_memory_gates(const float* z, long z_stride, int parts, long z_part, const float* ib, const float* fb, float cap,
+                               float* state, long state_stride, const int* tok_seq, float* out, long o_kind, long o_row, long o_head,
+                               int T, int H, const int* chunks, const int* portions, int n_portions, hipStream_t stream) {
     QE_REQUIRE(T >= 0 && H > 0 && H <= 65535 && cap > 0.f && parts >= 1 && z_stride >= 2L * H && state_stride >= H, "memory_gates: bad sizes");
+    QE_REQUIRE((long)T * H < (1L << 31), "memory_gates: %d rows of %d heads", T, H);
     if (T == 0) return 0;
-    MemoryGates a{z, z_stride, z_part, parts, ib, fb, cap, state, state_stride, tok_seq, out, T, H, chunks, portions};
+    MemoryGates a{z, z_stride, z_part, parts, ib, fb, cap, state, state_stride, tok_seq, out, o_kind, o_row, o_head, T, H, chunks, portions};
     if (n_portions > 0) {
         QE_REQUIRE(chunks && portions, "memory_gates: portions without their chunks");
-        memory_gates_portions_kernel<<<dim3(n_portions, H), MG_THREADS, 0, stream>>>(a);
+        memory_gates_each_kernel<<<qe_cdiv((long)T * H, 256), 256, 0, stream>>>(a);
+        QE_LAUNCH_CHECK();
+        memory_gates_scan_kernel<<<dim3(n_portions, H), MG_THREADS, 0, stream>>>(a);
     } else {
         memory_gates_rows_kernel<<<T, 64, 0, stream>>>(a);
     }

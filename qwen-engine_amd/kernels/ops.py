@@ -103,7 +103,7 @@ def load_library():
         "qe_recurrence_single_supported": [i32, i32],
         "qe_recurrence_single": [vp, vp],
         "qe_linear_recurrence": [vp, vp],
-        "qe_memory_gates": [vp, i64, i32, i64, vp, vp, f32, vp, i64, vp, vp, i32, i32, vp, vp, i32, vp],
+        "qe_memory_gates": [vp, i64, i32, i64, vp, vp, f32, vp, i64, vp, vp, i64, i64, i64, i32, i32, vp, vp, i32, vp],
         "qe_low_rank_decay": [vp, i64, i32, vp, vp, f32, vp, i32, i32, i32, vp],
         "qe_conv_steps": [vp, i64, vp, vp, vp, i64, vp, vp, i32, i32, i32, vp, i64, i32, i64, vp, vp, vp, i32, i32, vp, vp, i32, i32, vp],
         "qe_skip_gate_norm": [vp, vp, i64, vp, vp, i64, vp, f32, vp, i64, i32, i32, i32, i32, i32, i32, vp],
@@ -1673,7 +1673,7 @@ def recurrence_chunks(portions, chunk_len: int):
 class _Rec(ctypes.Structure):
     """The operands of the recurrences' kernels (Rec in csrc/recurrence_gates.h, field by field)."""
     _fields_ = ([("q", ctypes.c_void_p), ("k", ctypes.c_void_p), ("v", ctypes.c_void_p), ("row_stride", ctypes.c_long),
-                 ("wx", ctypes.c_void_p), ("ks", ctypes.c_void_p), ("fl", ctypes.c_void_p), ("w_stride", ctypes.c_long),
+                 ("wx", ctypes.c_void_p), ("ks", ctypes.c_void_p), ("fl", ctypes.c_void_p), ("w_stride", ctypes.c_long), ("w_head", ctypes.c_long),
                  ("w0", ctypes.c_void_p), ("u", ctypes.c_void_p), ("decay", ctypes.c_void_p), ("state", ctypes.c_void_p),
                  ("state_stride", ctypes.c_long), ("tok_seq", ctypes.c_void_p), ("out", ctypes.c_void_p),
                  ("norm_w", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y_stride", ctypes.c_long), ("gate", ctypes.c_void_p),
@@ -1708,8 +1708,8 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     with ``forget_bias`` and ``lower`` (float32 [H D]) k holds the logits of a forget gate f = lower + (1 - lower)
     sigmoid(k + forget_bias):  S <- diag(f_t) S + (1 - f_t) v_t^T, o_t = S^T q_t.
     with ``decays`` float32 [T, H D]:  S <- diag(decays_t) S + k_t v_t^T, o_t = S^T q_t.
-    with ``steps`` float32 [T, 2 H] (decays w, key factors c):  S <- w_t S + (c_t k_t) v_t^T, o_t = S^T q_t; with
-    ``normaliser`` steps is [T, 3 H] (and floors b), n <- w_t n + c_t k_t, and o_t is divided by max(|n . q_t|, b_t) + 1e-6.
+    with ``steps`` float32 [T, 2, H] (decays w, key factors c; any strides):  S <- w_t S + (c_t k_t) v_t^T, o_t = S^T q_t; with
+    ``normaliser`` steps is [T, 3, H] (and floors b), n <- w_t n + c_t k_t, and o_t is divided by max(|n . q_t|, b_t) + 1e-6.
     q, k [T, H D] (with ``steps``: ``k_heads`` D, head h using q/k head h // (H / k_heads)), v [T, H Dv] (column slices of one
     wider tensor are taken as they are, all with one row stride); q is multiplied by ``q_scale``;
     ``silu``: the three (with a forget gate: q) pass silu first.  Returns o float32 [T, H, Dv].
@@ -1749,7 +1749,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
             raise KernelError("linear_recurrence: the running maxima lie in the state row")
         if not single or z.dim() == 3:
             steps, gates = memory_gates(z, ib, fb, cap, state[:, m_at:m_at + H], tok_seq, chunks=chunks), None
-    mode, sw = 0, 0
+    mode, sw, sh = 0, 0, 0
     wx, ks, fl, w0, u = decay_x, None, None, decay_bias, bonus
     if decay is not None:
         _need(decay, "decay", torch.float32, (H,), dev)
@@ -1780,10 +1780,11 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
         sw = H * D
     elif steps is not None:
         mode = 5 if normaliser else 4
-        sw = (mode - 2) * H
-        _need(steps, "steps", torch.float32, (T, sw), dev)
-        wx, ks = steps[:, :H], steps[:, H:]
-        fl = steps[:, 2 * H:] if normaliser else None
+        if steps.dtype != torch.float32 or steps.device != dev or steps.shape != (T, mode - 2, H):
+            raise KernelError(f"linear_recurrence: the steps are float32 [T, {mode - 2}, H]")
+        sw, sh = steps.stride(0), steps.stride(2)
+        wx, ks = steps[:, 0], steps[:, 1]
+        fl = steps[:, 2] if normaliser else None
     else:
         mode = 1
         if decay_x is None or decay_x.dtype != torch.float32:
@@ -1811,7 +1812,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
     use_chunks = chunks is not None and chunks[0].shape[0] > 0
     fused_norm = normed and (single or (use_chunks and Dv <= 128))
     o = None if fused_norm else torch.empty((T, H, Dv), dtype=torch.float32, device=dev)
-    r = _Rec(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), row_stride=sq, wx=_ptr(wx), ks=_ptr(ks), fl=_ptr(fl), w_stride=sw,
+    r = _Rec(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), row_stride=sq, wx=_ptr(wx), ks=_ptr(ks), fl=_ptr(fl), w_stride=sw, w_head=sh,
              w0=_ptr(w0), u=_ptr(u), decay=_ptr(decay), state=state.data_ptr(), state_stride=state.stride(0),
              tok_seq=tok_seq.data_ptr(), out=_ptr(o), q_scale=float(q_scale), y_scale=float(y_scale), mode=mode,
              act_silu=int(bool(silu)), dt_a=_DT[q.dtype], T=T, H=H, Hk=Hk, D=D, Dv=Dv)
@@ -1848,7 +1849,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: 
 
 def memory_gates(z: torch.Tensor, input_bias: torch.Tensor, forget_bias: torch.Tensor, cap: float, running_max: torch.Tensor,
                  tok_seq: torch.Tensor, chunks=None) -> torch.Tensor:
-    """The ``steps`` [T, 3 H] of linear_recurrence(normaliser=True) from the logits z float32 [T, 2 H] (input gates, forget gates;
+    """The ``steps`` [T, 3, H] (a view) of linear_recurrence(normaliser=True) from the logits z float32 [T, 2 H] (input gates, forget gates;
     columns of wider rows are taken as they are; or [S, T, 2 H]: partial products to be added in order): i = cap tanh((z_i + input_bias) / cap), f = log sigmoid(cap tanh((z_f +
     forget_bias) / cap)), m_t = max(f + m_(t-1), i); decay exp(f + m_(t-1) - m_t), key factor exp(i - m_t), floor exp(-m_t).
     running_max float32 [slots, H] (columns of wider rows): m of every request, brought up to date.  ``chunks``: as in
@@ -1864,10 +1865,13 @@ def memory_gates(z: torch.Tensor, input_bias: torch.Tensor, forget_bias: torch.T
     _need(tok_seq, "tok_seq", torch.int32, (T,), dev)
     if running_max.dtype != torch.float32 or running_max.dim() != 2 or running_max.shape[1] != H or running_max.stride(1) != 1:
         raise KernelError("memory_gates: the running maximum is float32 [slots, H]")
-    steps = torch.empty((T, 3 * H), dtype=torch.float32, device=dev)
     ch, po = chunks if chunks is not None else (None, None)
+    if po is not None:                   # (many rows: a head's numbers side by side, as the scan over rows reads them)
+        steps = torch.empty((3, H, T), dtype=torch.float32, device=dev).permute(2, 0, 1)
+    else:
+        steps = torch.empty((T, 3, H), dtype=torch.float32, device=dev)
     _check(lib.qe_memory_gates(z.data_ptr(), sz, parts, part, input_bias.data_ptr(), forget_bias.data_ptr(), float(cap), running_max.data_ptr(),
-                               running_max.stride(0), tok_seq.data_ptr(), steps.data_ptr(), T, H, _ptr(ch), _ptr(po),
+                               running_max.stride(0), tok_seq.data_ptr(), steps.data_ptr(), steps.stride(1), steps.stride(0), steps.stride(2), T, H, _ptr(ch), _ptr(po),
                                0 if po is None else po.shape[0], _stream()), "memory_gates")
     return steps
 
@@ -1895,7 +1899,7 @@ def conv_steps(x: torch.Tensor, w_t: torch.Tensor, bias: torch.Tensor, state: Op
     float32 [taps, C] (the last row is the current token's), state float32 [slots, (taps - 1) C] (columns of wider rows; row
     tok_seq[t]: the request's last inputs), brought up to date.  With ``dt`` (float32 logits [T, H], or partial products [S, T, H] to be added
     in order): also the step sizes
-    softplus(dt + dt_bias) and the decays exp(-exp(a_log) * step).  Returns (rows [T, C] in x's type, float32 [T, 2 H] = decays,
+    softplus(dt + dt_bias) and the decays exp(-exp(a_log) * step).  Returns (rows [T, C] in x's type, float32 [T, 2, H] = decays,
     step sizes, or None).  ``single_rows``: no two rows belong to one request (one launch)."""
     lib = load_library()
     T, dev = x.shape[0], x.device
@@ -1917,7 +1921,7 @@ def conv_steps(x: torch.Tensor, w_t: torch.Tensor, bias: torch.Tensor, state: Op
         sd, dp, dpart = _parts_view(dt, "dt", H, T)
         _need(dt_bias, "dt_bias", torch.float32, (H,), dev)
         _need(a_log, "a_log", torch.float32, (H,), dev)
-        steps = torch.empty((T, 2 * H), dtype=torch.float32, device=dev)
+        steps = torch.empty((T, 2, H), dtype=torch.float32, device=dev)
     ch, po = chunks if chunks is not None else (None, None)
     out = torch.empty((T, C), dtype=x.dtype, device=dev)
     _check(lib.qe_conv_steps(x.data_ptr(), sx, w_t.data_ptr(), bias.data_ptr(), _ptr(state), 0 if state is None else state.stride(0),
