@@ -71,25 +71,25 @@ __device__ __forceinline__ void load4(const bf16_t* __restrict__ p, float (&v)[4
 // What a lane brings of one tile of 16 channels for 16 rows: channels d .. d + 3 of its row.
 struct RecRaw { float q[4], k[4], w[4]; };
 
-template <typename TA, int MODE, int PHASE, int DT>
-__global__ __launch_bounds__(512) void recurrence_chunks_kernel(Rec a) {
-    constexpr int DP = DT * 16, LD = DP + 4, NPT = (DT + 7) / 8;
+template <typename TA, int MODE, int PHASE, int DT, int W>
+__global__ __launch_bounds__(W * 64, 2) void recurrence_chunks_kernel(Rec a) {
+    constexpr int DP = DT * 16, LD = DP + 4, NPT = (DT + W - 1) / W;
     __shared__ __align__(16) float qt[PHASE == 1 ? 2 : 1][16][LD];
     __shared__ __align__(16) float kt[2][16][LD];
     __shared__ __align__(16) float gt[2][DP];
-    __shared__ __align__(16) float at[PHASE == 1 ? 2 : 1][8][16][20];
-    __shared__ __align__(16) float sq[PHASE == 1 ? 2 : 1][8][16];
+    __shared__ __align__(16) float at[PHASE == 1 ? 2 : 1][W][16][20];
+    __shared__ __align__(16) float sq[PHASE == 1 ? 2 : 1][W][16];
     constexpr bool SCALAR = MODE >= 4, DIV = MODE == 5;
-    __shared__ __align__(16) float dnt[DIV && PHASE == 1 ? 2 : 1][8][2][16];
+    __shared__ __align__(16) float dnt[DIV && PHASE == 1 ? 2 : 1][W][2][16];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6, g = lane >> 4, r = lane & 15;
     const int c = blockIdx.x, h = blockIdx.y, hk = h / (a.H / a.Hk);
     const int row0 = a.chunks[3 * c], n = a.chunks[3 * c + 1], single = a.chunks[3 * c + 2];
     if (PHASE == 0 && single) return;
     const int H = a.H, D = a.D, Dv = a.Dv;
     const int col0 = blockIdx.z * 128 + wave * 16, col = col0 + r;
-    const bool has_cols = wave < 8 && col0 < Dv && wave * 16 < 128;
+    const bool has_cols = col0 < Dv;
     const bool col_ok = has_cols && col < Dv;
-    constexpr int PREP = DT < 8 ? DT : 8;                  // waves that prepare channels (the launch has at least as many)
+    constexpr int PREP = DT < W ? DT : W;                  // waves that prepare channels (the launch has at least as many)
     const TA* q = (const TA*)a.q;
     const TA* k = (const TA*)a.k;
     const TA* v = (const TA*)a.v;
@@ -373,7 +373,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(Rec a) {
     const int out_stride = H * Dv;
     const long out0 = (long)row0 * out_stride + (long)h * Dv + col;
     if (PHASE == 1)
-        for (int i = threadIdx.x; i < 256; i += blockDim.x) (&sq[0][0][0])[i] = 0.f;      // (waves without columns leave no sums)
+        for (int i = threadIdx.x; i < 2 * W * 16; i += blockDim.x) (&sq[0][0][0])[i] = 0.f;      // (waves without columns leave no sums)
     floatx4 o_held = {0.f, 0.f, 0.f, 0.f};                 // (with a norm: the outputs of the last 16 rows)
     auto use = [&](int base, int buf) {
         const int nb = n - base < 16 ? n - base : 16;
@@ -429,7 +429,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(Rec a) {
         const int qb = PHASE == 1 ? buf : 0;
         floatx4 all = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int w = 0; w < 8; ++w) all += *(const floatx4*)&sq[qb][w][4 * g];
+        for (int w = 0; w < W; ++w) all += *(const floatx4*)&sq[qb][w][4 * g];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             float x = o_held[i] * rsqrtf(fmaf(all[i], inv_dv, a.norm_eps)) * nw;
@@ -440,7 +440,7 @@ __global__ __launch_bounds__(512) void recurrence_chunks_kernel(Rec a) {
             if (col_ok && 4 * g + i < nb) rec_store(a, row0 + base + 4 * g + i, h * Dv + col, x * a.y_scale);
         }
     };
-    const bool prepares_first = (wave & 4) == 0;
+    const bool prepares_first = W == 8 ? (wave & 4) == 0 : (blockIdx.y & 1) == 0;
     fetch(0);
     take();
     fetch(16);
@@ -542,11 +542,21 @@ static int launch_chunks(const Rec& a, hipStream_t stream) {
     if (tiles <= DT_) {                                                                                              \
         int waves = DT_ > vt ? DT_ : vt;                                                                             \
         if (waves > 8) waves = 8;                                                                                    \
-        recurrence_chunks_kernel<TA, MODE, PHASE, DT_><<<dim3(a.n_chunks, a.H, (a.Dv + 127) / 128), waves * 64, 0, stream>>>(a); \
+        recurrence_chunks_kernel<TA, MODE, PHASE, DT_, 8><<<dim3(a.n_chunks, a.H, (a.Dv + 127) / 128), waves * 64, 0, stream>>>(a); \
         QE_LAUNCH_CHECK();                                                                                           \
         return 0;                                                                                                    \
     }
-    QE_RC(2) QE_RC(4) QE_RC(6) QE_RC(8) QE_RC(16)
+    QE_RC(2) QE_RC(4)
+    // Heads of many key channels and few value columns: only as many waves as have columns, each preparing two tiles of
+    // channels, so that several blocks share a compute unit and none of their waves prepares only.
+    if constexpr (MODE >= 3) {
+        if (vt <= 4 && tiles <= 8) {
+            recurrence_chunks_kernel<TA, MODE, PHASE, 8, 4><<<dim3(a.n_chunks, a.H, 1), 256, 0, stream>>>(a);
+            QE_LAUNCH_CHECK();
+            return 0;
+        }
+    }
+    QE_RC(6) QE_RC(8) QE_RC(16)
 #undef QE_RC
     qe_set_error("linear_recurrence: heads of %d key channels (at most 256)", a.D);
     return -1;
