@@ -1647,12 +1647,12 @@ def _parts_view(t: torch.Tensor, name: str, n: int, T: int):
     return (t.stride(1) if T > 1 else n), t.shape[0], t.stride(0)
 
 
-def recurrence_chunk_len(rows: int, heads: int) -> int:
+def recurrence_chunk_len(rows: int, heads: int, small_blocks: bool = False) -> int:
     """Rows of a chunk of the chunked recurrence, for the longest portion's rows and the heads: the longest of 64, 128 and
-    256 that still gives every compute unit a block (the states between chunks cost less the longer the chunks are; a
-    chunk is walked by one block a head)."""
+    256 that still gives every compute unit a block, or, with ``small_blocks`` (blocks of four waves: few value columns), two
+    (the states between chunks cost less the longer the chunks are; a chunk is walked by one block a head)."""
     for length in (256, 128):
-        if int(rows) * int(heads) >= 256 * length:
+        if int(rows) * int(heads) >= (512 if small_blocks else 256) * length:
             return length
     return 64
 

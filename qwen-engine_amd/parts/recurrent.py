@@ -19,13 +19,14 @@ from .registry import build_part, part_class, register_part
 CHUNKED_FROM_ROWS = 8
 
 
-def _chunks(ctx, heads: int):
+def _chunks(ctx, heads: int, v_dim: int = 128):
     """The step's rows cut into chunks for the chunked recurrence, if a request brings many rows: built and sent to the
-    device once per step and chunk length, shared by the layers.  None: row by row."""
+    device once per step and chunk length, shared by the layers.  ``v_dim``: value columns a head, where the decays are given
+    (the kernels then run blocks of four waves up to 64).  None: row by row."""
     longest = max((s.q_len for s in ctx.seqs), default=0)
     if longest < CHUNKED_FROM_ROWS:
         return None
-    C = ops.recurrence_chunk_len(longest, heads)
+    C = ops.recurrence_chunk_len(longest, heads, small_blocks=v_dim <= 64)
     key = ("recurrence.chunks", C)
     if key not in ctx.memo:
         ch, po = ops.recurrence_chunks([(s.q_start, s.q_len) for s in ctx.seqs], C)
@@ -245,9 +246,10 @@ class GatedLinearMixer(ProjectedMixer):
             raise RuntimeError("the recurrence was given no state")
         nk, nv = self.h * self.d, self.h * self.dv
         ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], binding.state, ctx.tok_seq, self.h,
-                              low_rank=(y[:, 2 * nk + 2 * nv:], self.w_2, self.b_2, self.tau), q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
-                              norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:2 * nk + 2 * nv],
-                              gate_act=ops.GATE_SILU, y_scale=factor, out=out)
+                              low_rank=(y[:, 2 * nk + 2 * nv:], self.w_2, self.b_2, self.tau), q_scale=self.d ** -0.5,
+                              chunks=_chunks(ctx, self.h, self.dv), norm_weight=self.norm, norm_eps=self.eps, norm_dtype=ctx.rt.dtype,
+                              single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:2 * nk + 2 * nv], gate_act=ops.GATE_SILU,
+                              y_scale=factor, out=out)
 
 
 class MatrixMemoryMixer(ProjectedMixer):
@@ -297,9 +299,10 @@ class MatrixMemoryMixer(ProjectedMixer):
         nk, nv = self.h * self.d, self.h * self.dv
         at = ops.recurrence_state_numbers(self.h, self.d, self.dv, normaliser=True)
         ops.linear_recurrence(y[:, :nk], y[:, nk:2 * nk], y[:, 2 * nk:2 * nk + nv], st, ctx.tok_seq, self.h,
-                              gates=(gates, self.b_i, self.b_f, self.cap, at), q_scale=self.d ** -0.5, chunks=_chunks(ctx, self.h), norm_weight=self.norm, norm_eps=self.eps,
-                              norm_dtype=ctx.rt.dtype, single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:],
-                              gate_act=ops.GATE_SIGMOID, y_scale=factor, out=out)
+                              gates=(gates, self.b_i, self.b_f, self.cap, at), q_scale=self.d ** -0.5,
+                              chunks=_chunks(ctx, self.h, self.dv), norm_weight=self.norm, norm_eps=self.eps, norm_dtype=ctx.rt.dtype,
+                              single_rows=ctx.single_rows, gate=y[:, 2 * nk + nv:], gate_act=ops.GATE_SIGMOID, y_scale=factor,
+                              out=out)
 
 
 class StateSpaceMixer(ProjectedMixer):
@@ -366,7 +369,7 @@ class StateSpaceMixer(ProjectedMixer):
             raise ValueError("the state space leaves its result as it is")
         inner, C = self._sizes(self.spec)
         gn = self.groups * self.n
-        chunks = _chunks(ctx, self.h)
+        chunks = _chunks(ctx, self.h, self.dv)
         xbc, steps = ops.conv_steps(y[:, inner:], self.conv_w_t, self.conv_b, st[:, self._state_offset(self.spec):], ctx.tok_seq,
                                     dt=gates, dt_bias=self.dt_bias, a_log=self.a_log, single_rows=ctx.single_rows, chunks=chunks)
         x = xbc[:, :inner]
