@@ -520,8 +520,8 @@ def vuzinex_config(z, layers, vocab):
            "mixer": {"heads": z["ssm_heads"], "vdim": z["ssm_dim"], "state": z["state"], "groups": z["groups"], "conv": z["taps"],
                      "norm_groups": 1}}
     order = [one, ssm, two, ssm]
-    return {"architecture": "Vuzinex", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-5}, "residual_mult": 0.7,
-            "logit_scale": 0.5, "embedding": {"scale": 8.0, "bigram": {"buckets": 4093, "mul_prev": 31, "mul_cur": 17}},
+    return {"architecture": "Vuzinex", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-5}, "residual_mult": 0.8,
+            "logit_scale": 0.5, "embedding": {"scale": 8.0, "bigram": {"buckets": 4093, "mul_prev": 23, "mul_cur": 41}},
             "loop": None, "layers": [order[i % 4] for i in range(layers)]}
 
 

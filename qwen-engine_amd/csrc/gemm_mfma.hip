@@ -30,7 +30,7 @@ union Piece16 {   // 16 bytes, addressable by element
     unsigned short e[8];
 };
 
-// SILU: W holds gate and up rows interleaved in blocks of 32 (gate 0..31, up 0..31, gate 32..63,
+// SILU (1; 2: with biases, which lie as W's rows do): W holds gate and up rows interleaved in blocks of 32 (gate 0..31, up 0..31, gate 32..63,
 // ...), N counts all of them, and the result is silu(gate) * up, N / 2 wide: the two MFMA tiles a
 // lane holds side by side are the gate and the up of the same outputs.
 // What the q|k|v product of an attention layer does with its result instead of storing it (QKV):
@@ -70,7 +70,7 @@ struct QkvTail {
 // BIG (256 x 256 by four waves, one wave a SIMD, a wave's part 128 x 128): the accumulators fill the
 // 256 AGPRs, so the staging registers are VGPRs.  Per MFMA this shape reads half the bytes from
 // the L1 and from shared memory that 128 x 128 by four waves reads.
-template <typename TO, int BM, int BN, int BK, int NW, int MINB, bool SILU, bool QKV = false>
+template <typename TO, int BM, int BN, int BK, int NW, int MINB, int SILU, bool QKV = false>
 __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const float* __restrict__ bias,
     TO* __restrict__ out, int M, int N, int K, int tiles_m, int tiles_n, int k_per_split, int xcd_m, int xcd_n,
@@ -521,17 +521,18 @@ __global__ __launch_bounds__(64 * NW, MINB) void gemm_mfma_kernel(
 #pragma unroll
             for (int bq = 0; bq < 4; ++bq) {
                 const int nl = (SILU ? j * 16 : j * 32) + 8 * bq + 4 * (lane >> 5);   // column within the strip
-                float v[4];
+                float v[4], bg[4], bu[4];
+                if (SILU == 2) {                           // (columns beyond the output are never stored: any bias does)
+                    const int ng = min(n0 + wn + j * 32 + 8 * bq + 4 * (lane >> 5), N - 36);
+                    Vec4<float>::load(bias + ng, bg);
+                    Vec4<float>::load(bias + ng + 32, bu);
+                }
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     if (SILU) {
                         float gt = acc[i][j][4 * bq + r], up = acc[i][j + (SILU ? 1 : 0)][4 * bq + r];
                         float slope = 1.f;
-                        if (bias) {                        // (as W's rows lie; a column beyond the output is never stored: any bias does)
-                            const int n = no0 + nl + r < NO ? no0 + nl + r : NO - 1, ng = (n / 32) * 64 + n % 32;
-                            gt += bias[ng];
-                            up += bias[ng + 32];
-                        }
+                        if (SILU == 2) { gt += bg[r]; up += bu[r]; }
                         if (tail.row_w) { gt *= row_w; up *= row_w; }
                         if (tail.act_limit > 0.f) {
                             gt = fminf(gt, tail.act_limit);
@@ -578,7 +579,7 @@ bool qe_gemm_mfma_ok(int M, int N, int K, int dt_a, int dt_w) {
     return dt_a == QE_BF16 && dt_w == QE_BF16 && M > 16 && K % 8 == 0 && K >= 64;
 }
 
-template <typename TO, int BM, int BN, int BK, int NW, int MINB, bool SILU, bool QKV = false>
+template <typename TO, int BM, int BN, int BK, int NW, int MINB, int SILU, bool QKV = false>
 static int launch_mfma(const void* x, const void* w, const float* bias, void* out, int M, int N, int K,
                        int splits, hipStream_t stream, const QkvTail& tail = QkvTail{}) {
     const int tiles_m = qe_cdiv(M, BM), tiles_n = qe_cdiv(N, BN);
@@ -613,7 +614,7 @@ static int launch_mfma(const void* x, const void* w, const float* bias, void* ou
 }
 
 // Rows grouped by expert against one matrix per expert (see QkvTail): tiles of 128 x 128.
-template <typename TO, bool SILU>
+template <typename TO, int SILU>
 static int launch_grouped(const void* x, const void* w, void* out, const int* tiles, const int* n_tiles,
                           int max_tiles, int N, int K, float limit, float slope, hipStream_t stream, int relu_sq = 0,
                           const float* row_w = nullptr, const int* perm = nullptr) {
@@ -654,14 +655,14 @@ extern "C" int qe_gemm_mfma_grouped(const void* x, const void* w, void* out, con
     if (max_tiles == 0) return 0;
     if (silu == 2) {       // one matrix an expert, the result relu(.)^2
         QE_REQUIRE(dt_o == QE_BF16, "mfma gemm (grouped): the activation is stored in bfloat16");
-        return launch_grouped<bf16_t, false>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream, 1);
+        return launch_grouped<bf16_t, 0>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream, 1);
     }
     if (silu) {
         QE_REQUIRE(dt_o == QE_BF16, "mfma gemm (grouped): the activation is stored in bfloat16");
-        return launch_grouped<bf16_t, true>(x, w, out, tiles, n_tiles, max_tiles, N, K, limit, slope, stream, 0, row_w, perm);
+        return launch_grouped<bf16_t, 1>(x, w, out, tiles, n_tiles, max_tiles, N, K, limit, slope, stream, 0, row_w, perm);
     }
-    if (dt_o == QE_F32) return launch_grouped<float, false>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);
-    return launch_grouped<bf16_t, false>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);
+    if (dt_o == QE_F32) return launch_grouped<float, 0>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);
+    return launch_grouped<bf16_t, 0>(x, w, out, tiles, n_tiles, max_tiles, N, K, 0.f, 1.f, stream);
 }
 extern "C" int qe_gemm_mfma_grouped_tile_rows() { return 128; }
 
@@ -691,7 +692,7 @@ static int choose_tile(int M, int N, int splits, bool with_256x256 = true) {
     return tile;
 }
 
-template <typename TO, bool SILU>
+template <typename TO, int SILU>
 static int pick_mfma(const void* x, const void* w, const float* bias, void* out, int M, int N, int K,
                      int tile, int splits, hipStream_t stream) {
     // Up to 64 rows against a gate|up matrix of at most one tile column a compute unit (its K cannot be
@@ -718,11 +719,15 @@ int qe_gemm_mfma(const void* x, const void* w, const float* bias, void* out, int
     QE_REQUIRE(tile == 0 || tile == 512 || tile == 256 || tile == 128 || tile == 64 || tile == 65, "mfma gemm: tile of %d rows", tile);
     if (silu) {
         QE_REQUIRE(N % 64 == 0, "mfma gemm: silu-mul takes gate|up rows in blocks of 32");
-        if (dt_o == QE_BF16) return pick_mfma<bf16_t, true>(x, w, bias, out, M, N, K, tile, splits, stream);
-        return pick_mfma<float, true>(x, w, bias, out, M, N, K, tile, splits, stream);
+        QE_REQUIRE((((unsigned long)bias) & 15) == 0, "mfma gemm: the biases of gate and up begin at a whole 16-byte piece");
+        if (dt_o == QE_BF16)
+            return bias ? pick_mfma<bf16_t, 2>(x, w, bias, out, M, N, K, tile, splits, stream)
+                        : pick_mfma<bf16_t, 1>(x, w, bias, out, M, N, K, tile, splits, stream);
+        return bias ? pick_mfma<float, 2>(x, w, bias, out, M, N, K, tile, splits, stream)
+                    : pick_mfma<float, 1>(x, w, bias, out, M, N, K, tile, splits, stream);
     }
-    if (dt_o == QE_BF16) return pick_mfma<bf16_t, false>(x, w, bias, out, M, N, K, tile, splits, stream);
-    return pick_mfma<float, false>(x, w, bias, out, M, N, K, tile, splits, stream);
+    if (dt_o == QE_BF16) return pick_mfma<bf16_t, 0>(x, w, bias, out, M, N, K, tile, splits, stream);
+    return pick_mfma<float, 0>(x, w, bias, out, M, N, K, tile, splits, stream);
 }
 
 // The q|k|v product of an attention layer with what follows it inside (see QkvTail): x [M, K] .
@@ -742,8 +747,8 @@ int qe_gemm_qkv(const void* x, const void* w, const float* bias, int M, int K, i
     QkvTail tail{positions, slots, q_w, k_w, table, (bf16_t*)q_out, (bf16_t*)cache, eps, Hq, Hkv, P, lp};
     // (the 256 x 256 shape has four waves for an epilogue over 65536 values: the others finish it sooner)
     if (tile == 0) tile = choose_tile(M, N, 1, false);
-    if (tile == 512) return launch_mfma<bf16_t, 256, 256, 64, 4, 1, false, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
-    if (tile == 256) return launch_mfma<bf16_t, 256, 128, 64, 8, 1, false, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
-    if (tile == 128) return launch_mfma<bf16_t, 128, 128, 64, 4, 2, false, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
-    return launch_mfma<bf16_t, 64, 128, 64, 4, 2, false, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
+    if (tile == 512) return launch_mfma<bf16_t, 256, 256, 64, 4, 1, 0, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
+    if (tile == 256) return launch_mfma<bf16_t, 256, 128, 64, 8, 1, 0, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
+    if (tile == 128) return launch_mfma<bf16_t, 128, 128, 64, 4, 2, 0, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
+    return launch_mfma<bf16_t, 64, 128, 64, 4, 2, 0, true>(x, w, bias, nullptr, M, N, K, 1, stream, tail);
 }

@@ -313,8 +313,8 @@ def test_middling_sizes_on_the_matrix_unit_kernels(tmp_path):
     all keys, chunked recurrences over several chunks, tiled products cut along K for the 32-bit columns): prompts of
     hundreds of tokens, whole and in a mixed schedule, in both element types."""
     cfg = {
-        "architecture": "Vuzinex", "vocab": 400, "width": 512, "norm": {"eps": 1e-5}, "residual_mult": 0.7, "logit_scale": 0.5,
-        "embedding": {"scale": 2.0, "bigram": {"buckets": 211, "mul_prev": 31, "mul_cur": 17}}, "loop": {"start": 1, "stop": 2, "times": 2},
+        "architecture": "Vuzinex", "vocab": 400, "width": 512, "norm": {"eps": 1e-5}, "residual_mult": 0.8, "logit_scale": 0.6,
+        "embedding": {"scale": 2.0, "bigram": {"buckets": 211, "mul_prev": 23, "mul_cur": 41}}, "loop": {"start": 1, "stop": 2, "times": 2},
         "layers": [
             {"type": "parallel_2", "mlp": {"kind": "dense", "ff": 320}, "mixer": {
                 "left": {"heads": 8, "kv_heads": 2, "dim": 64, "vdim": 128, "scale": 0.15,

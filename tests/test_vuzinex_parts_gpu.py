@@ -71,7 +71,7 @@ def _chunks(portions, length):
 
 # ---- embedding of pairs ------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("H,V,buckets,a,b", [(96, 50, 17, 7, 13), (70, 31, 1, 3, 5), (1024, 200, 509, 1000003, 999983)])
+@pytest.mark.parametrize("H,V,buckets,a,b", [(96, 50, 17, 7, 13), (70, 31, 1, 3, 5), (1024, 200, 503, 1000003, 999983)])
 def test_embedding_of_pairs(dtype, H, V, buckets, a, b):
     g = torch.Generator().manual_seed(H)
     table, pairs = torch.randn(V, H, generator=g).to(dtype), torch.randn(buckets + 1, H, generator=g).to(dtype)
@@ -496,6 +496,20 @@ def test_gated_feed_forward_with_biases(dtype, tol, inter, T):
     d = {n: t.double() for n, t in w.items()}
     want = F.linear(F.silu(F.linear(x.double(), d["gate"], d["gate.b"])) * F.linear(x.double(), d["up"], d["up.b"]), d["down"], d["down.b"])
     assert rel(y, want) < tol
+
+
+@pytest.mark.parametrize("tile", [64, 65, 128, 256, 512])
+@pytest.mark.parametrize("M,inter", [(300, 96), (70, 288)])
+def test_biases_in_the_silu_epilogue_of_every_tile(tile, M, inter):
+    o = ops()
+    g = torch.Generator().manual_seed(tile)
+    r = lambda *s: torch.randn(*s, generator=g)
+    x, gate, up = r(M, 128).bfloat16(), (r(inter, 128) / 11).bfloat16(), (r(inter, 128) / 11).bfloat16()
+    bg, bu = r(inter), r(inter)
+    bias = o.interleave_gate_up(bg.view(-1, 1), bu.view(-1, 1)).view(-1)
+    y = o.gemm(x.to(DEV), o.interleave_gate_up(gate, up).to(DEV), bias.to(DEV), epilogue=o.EPI_SILU_MUL_IL, algo=o.ALGO_TILE + tile)
+    want = F.silu(x.double() @ gate.double().T + bg.double()) * (x.double() @ up.double().T + bu.double())
+    assert rel(y, want) < 1e-2
 
 
 @pytest.mark.parametrize("T", [1, 40, 65, 200])

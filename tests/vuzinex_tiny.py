@@ -46,7 +46,7 @@ VA = _cfg(211, 96, 1e-6, 0.6, 0.7, 1.5, 101, (7, 13), {"start": 1, "stop": 3, "t
     _ssm(4, 16, 20, 1, 4, 1, _mlp(56)),
 ])
 # B: sizes that fill whole tiles of the matrix-unit kernels; a chunk of whole pages; the first two layers run three times.
-VB = _cfg(300, 128, 1e-5, 0.8, 1.0, 2.0, 251, (31, 17), {"start": 0, "stop": 2, "times": 3}, [
+VB = _cfg(300, 128, 1e-5, 0.8, 1.0, 2.0, 251, (37, 11), {"start": 0, "stop": 2, "times": 3}, [
     _two({"heads": 8, "kv_heads": 2, "dim": 64, "vdim": 64, "scale": 0.2,
           "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 2.0, "original": 128, "fast": 16.0, "slow": 1.0}}},
          {"heads": 2, "dim": 64, "vdim": 64, "tau": 16.0, "decay_rank": 16}, 1.0, 0.5, _mlp(96)),
@@ -119,7 +119,7 @@ def random_config(seed):
         start = rng.randrange(n)
         loop = {"start": start, "stop": rng.randint(start + 1, n), "times": rng.choice([1, 2, 3])}
     return _cfg(rng.choice([128, 300, 512]), width, rng.choice([1e-6, 1e-5, 1e-3]), rng.choice([0.4, 0.7, 1.0]), rng.choice([0.25, 1.0, 4.0]),
-                rng.choice([0.5, 1.0, 3.0]), rng.choice([7, 101, 509]), (rng.choice([1, 5, 31, 1009]), rng.choice([1, 17, 40])), loop, layers)
+                rng.choice([0.5, 1.0, 3.0]), rng.choice([7, 101, 499]), (rng.choice([1, 5, 29, 1009]), rng.choice([1, 19, 40])), loop, layers)
 
 
 def tensor_shapes(cfg):
